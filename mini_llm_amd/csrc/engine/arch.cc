@@ -23,6 +23,7 @@ void register_builtin_architectures() {
         register_rekirax();
         register_viladra();
         register_sunulorn();
+        register_zokunex();
         if (const char* env = std::getenv("MINI_LLM_PLUGINS")) {
             std::stringstream ss(env);
             for (std::string path; std::getline(ss, path, ':');)

@@ -12,7 +12,8 @@ extern "C" {
 
 // elementwise.hip
 int mllm_embed(const int* ids, const int* pos, const void* wte, const void* wpe, float* x, int T, int D,
-               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale = 1.f);
+               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale = 1.f, void* copy_bf16 = nullptr);
+int mllm_cast_bf16(const float* x, void* out, size_t n, hipStream_t stream);
 int mllm_depth_mix(float* x, float* kept, size_t stride, int n_old, const float* w, size_t n, hipStream_t stream);
 int mllm_select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream);
 int mllm_reset_state(void* state, size_t slot_bytes, int n_slots, const int* slots, const int* starts, int B,
@@ -71,10 +72,10 @@ int mllm_prefill_attention_bf16(const void* q, int q_stride, int q_col, const vo
 int mllm_rmsnorm(const float* x, int ldx, const int* rows, const float* w, const float* gate, int ldg, void* y, int ldy,
                  int n, int D, int groups, float eps, int out_dtype, int parts, size_t part_stride, hipStream_t stream);
 int mllm_rmsnorm_gate_after(const float* x, int ldx, const float* w, const float* gate, int ldg, void* y, int ldy, int n, int D, int groups,
-                            float eps, int out_dtype, int parts, size_t part_stride, hipStream_t stream);
+                            float eps, int out_dtype, int parts, size_t part_stride, hipStream_t stream, int plain_sigmoid = 0);
 int mllm_softcap(float* x, size_t n, float cap, hipStream_t stream);
-int mllm_rmsnorm_add(float* y, const float* w, const float* scale, float mult, float eps, float* x, int n, int D,
-                     int clear, hipStream_t stream);
+int mllm_norm_add(float* y, const float* w, const float* beta, const float* scale, float mult, float eps, float* x, int n, int D,
+                  int clear, int center, void* copy_bf16, hipStream_t stream);
 int mllm_rmsnorm_add_many(const float* y, size_t y_stride, const float* w, size_t w_stride, int n_in, float mult, float eps,
                           float* x, int n, int D, hipStream_t stream);
 int mllm_glu_clamped(const void* gate, int ldg, const void* up, int ldu, void* out, int ldo, int T, int F, float limit,
@@ -104,9 +105,12 @@ size_t mllm_ssm_scan_workspace_floats(int T, int B, int H, int P, int N);
 // latent_attention.hip
 int mllm_latent_prepare(const float* dq, int ld_dq, int Rq, const float* wq, void* cq, int ld_cq, const float* dkv, int ld_dkv,
                         int R, int Dr, const float* wkv, void* pages, void* vt_pages, int page_size, const int* slots,
-                        const int* positions, int T, float eps, double base, int rot_dims, int dtype, hipStream_t stream);
+                        const int* positions, int T, float eps, double base, int rot_dims, int dtype, hipStream_t stream,
+                        int norm_cols = 0, int half_split = 0);
+int mllm_latent_tile_shape(int R, int Dr, int* R_out, int* E_out);
 int mllm_latent_absorb(const void* q, int ldq, const void* w_uk, int ldw, void* qa, int ldqa, const int* positions, int T, int H,
-                       int Dn, int Dr, int R, double base, int rot_dims, int dtype, hipStream_t stream);
+                       int Dn, int Dr, int R, double base, int rot_dims, int dtype, hipStream_t stream, int q_dtype = -1,
+                       int half_split = 0);
 int mllm_latent_attention(const void* qa, int ldqa, const void* pages, const int* block_tables, int max_blocks,
                           const int* token_seq, const int* positions, int T, int H, int R, int Dr, int page_size, float scale,
                           int window, void* o_lat, int ldo, int dtype, hipStream_t stream);
@@ -115,7 +119,7 @@ int mllm_latent_attention_tiles(const void* qa, const void* k_pages, const void*
                                 int R, int Dr, int page_size, float scale, int window, void* o_lat, int n_rows, int nsplit,
                                 float* partials, int single_tokens, hipStream_t stream);
 int mllm_latent_expand(const void* o_lat, int ldo, const void* w_uv, int ldw, void* out, int ldout, int T, int H, int Dv, int R,
-                       int dtype, hipStream_t stream);
+                       int dtype, hipStream_t stream, const float* gate = nullptr, int ldg = 0);
 
 // scored_attention.hip
 int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, int T, int H, int G, int d, int dv,
@@ -147,12 +151,24 @@ int mllm_lowrank_decay(const float* proj, int ld, int a_col, int rank, const flo
                        int T, int N, hipStream_t stream);
 size_t mllm_hgrn2_workspace_floats(int T, int B, int H, int d, int dv);
 int mllm_hgrn2_chunk();
+// matrix_memory.hip
+int mllm_matrix_memory_chunk();
+int mllm_matrix_memory_copies(int d, int e);
+size_t mllm_matrix_memory_state_floats(int H, int d, int e);
+size_t mllm_matrix_memory_workspace_floats(int T, int B, int H, int d, int e);
+int mllm_matrix_memory(const float* proj, int ld, int q_col, int k_col, int v_col, int g_col, int i_col, int f_col, const float* i_bias,
+                       const float* f_bias, const float* norm_w, float cap, float q_scale, float eps, const int* cu_q, const int* state_slots,
+                       float* state, size_t slot_floats, int T, int B, int n_single, int max_portion, int H, int d, int e, int write,
+                       float* workspace, void* out, int ldo, float* y, int ldy, int dtype, int* needs_norm, hipStream_t stream);
+
 int mllm_concat_cast(const float* a, const float* b, int T, int D, void* out, int dtype, hipStream_t stream);
 int mllm_glu_act(const void* gu, int ld, int T, int F, int act, void* out, int ldo, int dtype, hipStream_t stream);
 
 // moe.hip
 int mllm_moe_act(const void* up, int ldu, const float* logits, int ldl, int E, int ff, int shared_ff, int top, float scale, void* out, int ldo,
-                 float* weights_out, int ldw, int T, int dtype, hipStream_t stream);
+                 float* weights_out, int ldw, int T, int dtype, hipStream_t stream, int up_dtype = -1, int gelu = 0,
+                 const float* correction = nullptr, int identity = 0, const void* h = nullptr, int ldh = 0, int D = 0, float* y = nullptr,
+                 int ldy = 0, int y_add = 0);
 int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int E, int ff, int shared_ff, int top, float scale,
                      int sigmoid_router, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
                      int ldo, int T, int dtype, hipStream_t stream);

@@ -23,11 +23,17 @@ const float* f32_vector(const Params& p, const char* key, int n) {
 // over the page rows with the first kv_rank columns as values, and W_uv expands the result.
 // A mixer without the tensor "dkv.weight" reads pages that another layer's call has written (its execution
 // order entry names that cache, write = false) with its own expansions, queries and window.
-// The turn is the interleaved one: the pair (2i, 2i+1) of the first rot_dims rotated columns at position p
-// by the angle p * rot_base^(-2i / rot_dims).
-// Parameters: heads, plain_dim, rot_dim, value_dim, kv_rank, q_rank, window, scale, rot_base, rot_dims, eps,
-// dtype; tensors dq.weight, dq.norm, uq.weight, [dkv.weight, dkv.norm,] uk.weight (transposed: [kv_rank,
-// heads * plain_dim], the layout in which queries are carried into the latent's space), uv.weight, out.weight.
+// The turn: the pair (2i, 2i+1) of the first rot_dims rotated columns at position p by the angle
+// p * rot_base^(-2i / rot_dims); with half_split the pair (i, i + rot_dims / 2).
+// Without a query latent (q_rank 0) the queries are q = W_q h, and one joined input projection with fp32 results makes
+// everything: in.weight's rows are [W_q | W_dkv | W_g], the last only with `gated`: head h's result is multiplied by
+// sigmoid(W_g h)_h. A latent may be widened with zero columns (rows of zeros in W_dkv, zeros in dkv.norm, zero rows in
+// uk.weight, zero columns in uv.weight) to the sizes of the matrix-core kernels: norm_cols is then its true size, which
+// the norm's mean runs over.
+// Parameters: heads, plain_dim, rot_dim, value_dim, kv_rank, q_rank, window, scale, rot_base, rot_dims, half_split, norm_cols,
+// gated, eps, dtype; tensors dq.weight, dq.norm, uq.weight, [dkv.weight, dkv.norm,] or in.weight, dkv.norm; uk.weight
+// (transposed: [kv_rank, heads * plain_dim], the layout in which queries are carried into the latent's space), uv.weight,
+// out.weight.
 class LatentAttention final : public Mixer {
 public:
     explicit LatentAttention(const Params& p) {
@@ -42,25 +48,39 @@ public:
         sh_.eps = static_cast<float>(p.number("eps"));
         window_ = static_cast<int>(p.number("window", 0));
         scale_ = static_cast<float>(p.number("scale"));
+        sh_.half_split = p.number("half_split", 0) != 0;
+        sh_.norm_cols = static_cast<int>(p.number("norm_cols", 0));
         dtype_ = p.integer("dtype");
-        if (sh_.n_heads < 1 || sh_.plain_dim < 1 || sh_.rot_dim < 0 || sh_.value_dim < 1 || sh_.kv_rank < 1 || sh_.q_rank < 1 || window_ < 0)
+        if (sh_.n_heads < 1 || sh_.plain_dim < 1 || sh_.rot_dim < 0 || sh_.value_dim < 1 || sh_.kv_rank < 1 || sh_.q_rank < 0 || window_ < 0)
             fail("latent_attention: heads and sizes must be positive");
         if (sh_.rot_dim % 2 != 0 || sh_.rot_dims % 2 != 0 || sh_.rot_dims > sh_.rot_dim || sh_.rot_dims < 0)
             fail("latent_attention: %d of %d rotated columns: both must be even, the first at most the second", sh_.rot_dims, sh_.rot_dim);
         const int qd = sh_.n_heads * (sh_.plain_dim + sh_.rot_dim);
-        dq_ = Linear(p.weights("dq.weight"), nullptr);
-        uq_ = Linear(p.weights("uq.weight"), nullptr);
+        q_cols_ = qd;
+        gated_ = p.number("gated", 0) != 0;
+        if (sh_.q_rank > 0) {
+            dq_ = Linear(p.weights("dq.weight"), nullptr);
+            uq_ = Linear(p.weights("uq.weight"), nullptr);
+            if (gated_) fail("latent_attention: a gate goes with queries that have no latent");
+        } else {
+            in_ = Linear(p.weights("in.weight"), nullptr);
+            own_kv_ = true;
+            if (in_.out_features() != qd + sh_.kv_rank + sh_.rot_dim + (gated_ ? sh_.n_heads : 0))
+                fail("latent_attention: the input projection has %d rows, which do not fit %d heads of %d + %d and a latent of %d", in_.out_features(),
+                     sh_.n_heads, sh_.plain_dim, sh_.rot_dim, sh_.kv_rank);
+            dkv_norm_ = f32_vector(p, "dkv.norm", sh_.kv_rank);
+        }
         out_ = Linear(p.weights("out.weight"), nullptr);
         uk_ = p.weights("uk.weight");
         uv_ = p.weights("uv.weight");
-        if (dq_.out_features() != sh_.q_rank || uq_.in_features() != sh_.q_rank || uq_.out_features() != qd)
+        if (sh_.q_rank > 0 && (dq_.out_features() != sh_.q_rank || uq_.in_features() != sh_.q_rank || uq_.out_features() != qd))
             fail("latent_attention: the query projections do not fit %d heads of %d + %d through %d", sh_.n_heads, sh_.plain_dim, sh_.rot_dim, sh_.q_rank);
         if (uk_.cols != static_cast<int64_t>(sh_.n_heads) * sh_.plain_dim || uk_.rows != sh_.kv_rank || uv_.rows != static_cast<int64_t>(sh_.n_heads) * sh_.value_dim ||
             uv_.cols != sh_.kv_rank || uk_.dtype != dtype_ || uv_.dtype != dtype_)
             fail("latent_attention: the key/value expansions do not fit %d heads and a latent of %d", sh_.n_heads, sh_.kv_rank);
         if (out_.in_features() != sh_.n_heads * sh_.value_dim) fail("latent_attention: the out-projection does not take %d heads of %d", sh_.n_heads, sh_.value_dim);
-        dq_norm_ = f32_vector(p, "dq.norm", sh_.q_rank);
-        if (p.weights_or_null("dkv.weight") != nullptr) {
+        if (sh_.q_rank > 0) dq_norm_ = f32_vector(p, "dq.norm", sh_.q_rank);
+        if (sh_.q_rank > 0 && p.weights_or_null("dkv.weight") != nullptr) {
             dkv_ = Linear(p.weights("dkv.weight"), nullptr);
             if (dkv_.out_features() != sh_.kv_rank + sh_.rot_dim || dkv_.in_features() != dq_.in_features())
                 fail("latent_attention: the key/value latent's projection must have %d rows", sh_.kv_rank + sh_.rot_dim);
@@ -70,27 +90,47 @@ public:
     }
     void forward(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
                  hipStream_t s) const override {
+        run(h, step, cache, x, write, arena, s, ADD_RESIDUAL);
+    }
+    void forward_set(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
+                     hipStream_t s) const override {
+        run(h, step, cache, x, write, arena, s, STORE_F32);
+    }
+    void run(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
+             hipStream_t s, int out_epilogue) const {
         const int E = sh_.kv_rank + sh_.rot_dim, T = step.n_tokens, g = cache.group, H = sh_.n_heads;
         if (!cache.has_pages() || cache.k_pages.cols != E) fail("latent_attention needs pages of %d-wide rows", E);
         if (write && !own_kv_) fail("a latent-attention layer without a key/value latent of its own cannot write a cache");
-        Tensor2 dq = arena.tensor(F32, T, sh_.q_rank), cq = arena.tensor(dtype_, T, sh_.q_rank);
         const bool fill = own_kv_ && write;
-        Tensor2 dkv;
-        if (fill) dkv = arena.tensor(F32, T, E);
-        if (T <= tuning().ln_fuse_max_rows) {
-            // few rows: each product normalises the mixer's input itself, and no norm kernel runs
-            h.linear(dq_, dq, STORE_F32, nullptr, arena, s);
-            if (fill) h.linear(dkv_, dkv, STORE_F32, nullptr, arena, s);
-        } else {
-            const Tensor2& in = h.tensor(arena, s);
-            dq_(in, dq, STORE_F32, nullptr, s);
-            if (fill) dkv_(in, dkv, STORE_F32, nullptr, s);
-        }
         LatentPages pages;
         pages.rows = cache.k_pages; pages.latent_t = cache.v_pages; pages.page_size = cache.page_size;
-        latent_prepare(dq, dq_norm_, cq, fill ? &dkv : nullptr, dkv_norm_, fill ? &pages : nullptr, step.slots[g], step.positions, sh_, s);
-        Tensor2 q = arena.tensor(dtype_, T, H * (sh_.plain_dim + sh_.rot_dim));
-        uq_(cq, q, STORE, nullptr, s);
+        Tensor2 q, gate;
+        if (sh_.q_rank == 0) {
+            const int N = in_.out_features(), ld = (N + 7) / 8 * 8;
+            const Tensor2 proj(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N, ld);
+            h.linear(in_, proj, STORE_F32, nullptr, arena, s);
+            float* rows = static_cast<float*>(proj.data);
+            q = Tensor2(rows, F32, T, q_cols_, ld);
+            const Tensor2 dkv(rows + q_cols_, F32, T, E, ld);
+            if (gated_) gate = Tensor2(rows + q_cols_ + E, F32, T, sh_.n_heads, ld);
+            if (fill) latent_prepare(Tensor2(), nullptr, Tensor2(), &dkv, dkv_norm_, &pages, step.slots[g], step.positions, sh_, s);
+        } else {
+            Tensor2 dq = arena.tensor(F32, T, sh_.q_rank), cq = arena.tensor(dtype_, T, sh_.q_rank);
+            Tensor2 dkv;
+            if (fill) dkv = arena.tensor(F32, T, E);
+            if (T <= tuning().ln_fuse_max_rows) {
+                // few rows: each product normalises the mixer's input itself, and no norm kernel runs
+                h.linear(dq_, dq, STORE_F32, nullptr, arena, s);
+                if (fill) h.linear(dkv_, dkv, STORE_F32, nullptr, arena, s);
+            } else {
+                const Tensor2& in = h.tensor(arena, s);
+                dq_(in, dq, STORE_F32, nullptr, s);
+                if (fill) dkv_(in, dkv, STORE_F32, nullptr, s);
+            }
+            latent_prepare(dq, dq_norm_, cq, fill ? &dkv : nullptr, dkv_norm_, fill ? &pages : nullptr, step.slots[g], step.positions, sh_, s);
+            q = arena.tensor(dtype_, T, q_cols_);
+            uq_(cq, q, STORE, nullptr, s);
+        }
         Tensor2 qa = arena.tensor(dtype_, T, H * E);
         latent_absorb(q, uk_, qa, step.positions, sh_, s);
         StageTimes::get().mark("qkv", s);
@@ -105,13 +145,14 @@ public:
         latent_attention(qa, pages, ls, scale_, window_, sh_, o_lat, ws, ws_floats, s);
         StageTimes::get().mark("attention", s);
         Tensor2 o = arena.tensor(dtype_, T, H * sh_.value_dim);
-        latent_expand(o_lat, uv_, o, sh_, s);
-        out_(o, x, ADD_RESIDUAL, nullptr, s);
+        latent_expand(o_lat, uv_, o, sh_, s, gated_ ? &gate : nullptr);
+        out_(o, x, out_epilogue, nullptr, s);
         StageTimes::get().mark("out_proj", s);
     }
     size_t workspace_bytes(int tokens) const override {
         const size_t E = sh_.kv_rank + sh_.rot_dim, H = sh_.n_heads;
-        const size_t per_token = (sh_.q_rank + E) * 4 + (dq_.in_features() + sh_.q_rank + H * (sh_.plain_dim + sh_.rot_dim) + H * E + H * sh_.kv_rank + H * sh_.value_dim) * dtype_size(dtype_);
+        const size_t joined = sh_.q_rank == 0 ? in_.out_features() + 8 : 0;
+        const size_t per_token = (sh_.q_rank + E + joined) * 4 + (in_.in_features() + dq_.in_features() + sh_.q_rank + H * (sh_.plain_dim + sh_.rot_dim) + H * E + H * sh_.kv_rank + H * sh_.value_dim) * dtype_size(dtype_);
         return static_cast<size_t>(tokens) * per_token + (dtype_ == BF16 ? latent_attention_workspace_floats(sh_.kv_rank) * 4 : 0) + 8192;
     }
     CacheNeed cache_need() const override {
@@ -123,8 +164,13 @@ public:
     }
     void reserve(int, hipStream_t s) const override { reserve_linear_scratch(s); }
     void add_cost(StepCost& c) const override {
-        dq_.add_cost(c); uq_.add_cost(c); out_.add_cost(c);
-        if (own_kv_) dkv_.add_cost(c);
+        out_.add_cost(c);
+        if (sh_.q_rank > 0) {
+            dq_.add_cost(c); uq_.add_cost(c);
+            if (own_kv_) dkv_.add_cost(c);
+        } else {
+            in_.add_cost(c);
+        }
         c.weight_bytes += static_cast<double>(uk_.cols + uv_.rows) * sh_.kv_rank * dtype_size(dtype_);
         c.flops_per_token += 2.0 * (uk_.cols + uv_.rows) * sh_.kv_rank;
         c.attention_flops_per_key += 2.0 * sh_.n_heads * (2.0 * sh_.kv_rank + sh_.rot_dim);
@@ -132,10 +178,10 @@ public:
 
 private:
     LatentShape sh_;
-    int window_ = 0, dtype_ = BF16;
+    int window_ = 0, dtype_ = BF16, q_cols_ = 0;
     float scale_ = 1.f;
-    bool own_kv_ = false;
-    Linear dq_, uq_, dkv_, out_;
+    bool own_kv_ = false, gated_ = false;
+    Linear dq_, uq_, dkv_, in_, out_;
     Tensor2 uk_, uv_;
     const float *dq_norm_ = nullptr, *dkv_norm_ = nullptr;
 };

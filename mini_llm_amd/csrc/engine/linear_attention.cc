@@ -146,8 +146,14 @@ private:
 // limit of its own), and with weight_on_input the weight multiplies what the expert READS, y = sum_e expert_e(w_e h):
 // the gate's and the up's products are linear, so the activation scales them before it clamps. With shared_gate the
 // router's matrix has one more row, and the shared expert's result is multiplied by the sigmoid of that logit.
+// With the activation "gelu_erf" an expert is W_down gelu(W_up h) (exact GELU); with the tensor "correction" ([experts +
+// identity]) the experts with the largest score + correction are chosen, weighed by the score alone; with `identity` the
+// router has that many more rows (behind the experts'), and those experts hand on their input h: y = ... + sum w_e h. (These
+// three go with softmax scores and ungated experts.) With the tensor "up_router.weight" (up.weight's rows and behind them
+// the router's, one allocation) steps of few rows run both products as one with fp32 results.
 // Parameters: dtype, experts, ff (an expert's hidden width), top, scale, strings activation, router (softmax);
-// clamped_glu: limit, shared_limit, alpha, weight_on_input, shared_gate; tensors router [experts (+ 1), width],
+// clamped_glu: limit, shared_limit, alpha, weight_on_input, shared_gate; others: identity; tensors router [experts (+ 1 |
+// + identity), width],
 // up.weight [experts * ff + shared_ff (clamped_glu: twice that), width], down.weight [width, experts * ff + shared_ff].
 class RoutedExperts final : public FeedForward {
 public:
@@ -157,7 +163,9 @@ public:
         glu_.scale = scale_ = static_cast<float>(p.number("scale", 1.0));
         const std::string& act = p.string("activation");
         if (act == "clamped_glu") gated_ = true;
-        else if (act != "relu2") fail("routed_experts: unknown activation '%s' (known: relu2, clamped_glu)", act.c_str());
+        else if (act == "gelu_erf") opt_.activation = GELU_ERF;
+        else if (act != "relu2") fail("routed_experts: unknown activation '%s' (known: relu2, gelu_erf, clamped_glu)", act.c_str());
+        opt_.identity = static_cast<int>(p.number("identity", 0));
         if (p.str.count("router")) {
             const std::string& r = p.string("router");
             if (r == "sigmoid") glu_.sigmoid_router = true;
@@ -167,7 +175,9 @@ public:
         up_ = Linear(p.weights("up.weight"), nullptr);
         down_ = Linear(p.weights("down.weight"), nullptr);
         router_ = Linear(p.weights("router"), nullptr);
-        if (E_ < 1 || ff_ < 1 || top_ < 1 || top_ > E_) fail("routed_experts: %d of %d experts of %d do not fit", top_, E_, ff_);
+        if (E_ < 1 || ff_ < 1 || top_ < 1 || opt_.identity < 0 || top_ > E_ + opt_.identity) fail("routed_experts: %d of %d experts of %d do not fit", top_, E_ + opt_.identity, ff_);
+        if (p.weights_or_null("correction") != nullptr) opt_.correction = f32_vector(p, "correction", E_ + opt_.identity, "routed_experts");
+        if (gated_ && (opt_.identity > 0 || opt_.correction != nullptr)) fail("routed_experts: identity experts and a correction go with ungated experts");
         if (gated_) {
             glu_.limit = static_cast<float>(p.number("limit"));
             glu_.alpha = static_cast<float>(p.number("alpha", 1.0));
@@ -181,8 +191,14 @@ public:
         } else if (up_.out_features() < E_ * ff_ || down_.in_features() != up_.out_features()) {
             fail("routed_experts: the joined products' shapes do not fit %d experts of %d", E_, ff_);
         }
-        if (router_.out_features() != E_ + (glu_.shared_gate ? 1 : 0) || router_.in_features() != up_.in_features())
-            fail("routed_experts: the router must be [%d, %d]", E_ + (glu_.shared_gate ? 1 : 0), up_.in_features());
+        const int routes = E_ + opt_.identity + (glu_.shared_gate ? 1 : 0);
+        if (router_.out_features() != routes || router_.in_features() != up_.in_features())
+            fail("routed_experts: the router must be [%d, %d]", routes, up_.in_features());
+        if (p.weights_or_null("up_router.weight") != nullptr) {
+            up_router_ = Linear(p.weights("up_router.weight"), nullptr);
+            if (gated_ || up_router_.out_features() != up_.out_features() + routes || up_router_.in_features() != up_.in_features())
+                fail("routed_experts: 'up_router.weight' must hold up.weight's rows and the router's (ungated experts)");
+        }
         if (down_.out_features() != up_.in_features()) fail("routed_experts: the second products must lead back to the width");
     }
     void forward(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const override {
@@ -194,11 +210,13 @@ public:
     void run(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue) const {
         Pending p;
         first_products(h, step, arena, s, p, false);
+        if (opt_.identity > 0) p.h = h.tensor(arena, s);
         rest(p, step, x, arena, s, out_epilogue);
     }
     bool begin(NormedInput& h, const StepView& step, Arena& arena, hipStream_t s, Pending& pending) const override {
         // (few rows in bfloat16: each of the two products norms its input itself, and no norm kernel runs)
         first_products(h, step, arena, s, pending, dtype_ == BF16 && step.n_tokens <= tuning().ln_fuse_max_rows);
+        if (opt_.identity > 0) pending.h = h.tensor(arena, s);
         return true;
     }
     void finish(const Pending& pending, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const override {
@@ -207,6 +225,15 @@ public:
     // pending.a: the router's logits (fp32), pending.b: the experts' joined first product
     void first_products(NormedInput& h, const StepView& step, Arena& arena, hipStream_t s, Pending& p, bool norm_inside) const {
         const int T = step.n_tokens, N = up_.out_features(), R = router_.out_features();
+        if (up_router_.weight.data != nullptr && T <= tuning().ln_fuse_max_rows) {
+            const int ld = (N + R + 3) / 4 * 4;
+            const Tensor2 both(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N + R, ld);
+            h.linear(up_router_, both, STORE_F32, nullptr, arena, s);
+            p.b = Tensor2(both.data, F32, T, N, ld);
+            p.a = Tensor2(static_cast<float*>(both.data) + N, F32, T, R, ld);
+            StageTimes::get().mark("fc1", s);
+            return;
+        }
         const int lde = (R + 3) / 4 * 4;
         p.a = Tensor2(arena.take(static_cast<size_t>(T) * lde * 4), F32, T, R, lde);
         p.b = arena.tensor(dtype_, T, N);
@@ -228,13 +255,21 @@ public:
             moe_glu_act(p.b, p.a, glu_, act, s);
             down_(act, x, out_epilogue, nullptr, s);
         } else {
-            moe_act(p.b, p.a, ff_, top_, scale_, p.b, nullptr, s);            // in place
-            down_(p.b, x, out_epilogue, nullptr, s);
+            const Tensor2 act = p.b.dtype == dtype_ ? p.b : arena.tensor(dtype_, step.n_tokens, up_.out_features());      // in place
+            MoeOptions o = opt_;
+            if (o.identity > 0) {
+                // the identity experts' share is put into x by the activation, and the second products add to it
+                o.h = p.h; o.y = x; o.y_add = out_epilogue == ADD_RESIDUAL;
+                out_epilogue = ADD_RESIDUAL;
+            }
+            moe_act(p.b, p.a, ff_, top_, scale_, act, nullptr, s, o);
+            down_(act, x, out_epilogue, nullptr, s);
         }
         StageTimes::get().mark("fc2", s);
     }
     size_t workspace_bytes(int tokens) const override {
-        return static_cast<size_t>(tokens) * ((up_.out_features() + down_.in_features() + up_.in_features()) * dtype_size(dtype_) + (E_ + 8) * 4) + 2048;
+        const size_t few = up_router_.weight.data != nullptr ? static_cast<size_t>(std::min(tokens, tuning().ln_fuse_max_rows)) * (up_router_.out_features() + 4) * 4 + 256 : 0;
+        return static_cast<size_t>(tokens) * ((up_.out_features() + down_.in_features() + up_.in_features()) * dtype_size(dtype_) + (E_ + opt_.identity + 8) * 4) + few + 2048;
     }
     void reserve(int, hipStream_t s) const override { reserve_linear_scratch(s); }
     void add_cost(StepCost& c) const override {
@@ -248,7 +283,8 @@ private:
     float scale_ = 1.f;
     bool gated_ = false;
     MoeGlu glu_;
-    Linear up_, down_, router_;
+    MoeOptions opt_;                    // activation, correction, identity experts
+    Linear up_, down_, router_, up_router_;
 };
 
 // What a layer hands on is a weighted sum of the embedding's output and the results of all layers so far: behind the

@@ -151,11 +151,13 @@ Tuning& tuning() {
 // elementwise
 // ---------------------------------------------------------------------------------------------
 void embed(const int* ids, const int* positions, const Tensor2& wte, const Tensor2* wpe, const Tensor2& out,
-           hipStream_t stream, const FedTokens* fed, float scale) {
+           hipStream_t stream, const FedTokens* fed, float scale, const Tensor2* copy) {
     need_dtype(wte, "wte");
     const int T = static_cast<int>(out.rows), D = static_cast<int>(wte.cols);
     if (!wte.contiguous()) fail("embed: wte must be contiguous");
     if (out.dtype != F32 || out.cols != D || !out.contiguous()) fail("embed: out must be contiguous float32 [%d, %d]", T, D);
+    if (copy != nullptr && (copy->dtype != BF16 || !copy->contiguous() || copy->rows != T || copy->cols != D))
+        fail("embed: the copy must be contiguous bfloat16 [%d, %d]", T, D);
     const void* table = nullptr;
     if (wpe != nullptr && wpe->data != nullptr) {
         if (positions == nullptr) fail("embed: positions are needed with a position table");
@@ -166,7 +168,7 @@ void embed(const int* ids, const int* positions, const Tensor2& wte, const Tenso
     const bool feeds = fed != nullptr && fed->src != nullptr;
     if (feeds && (fed->prev == nullptr || fed->n_prev < 1)) fail("embed: fed tokens need the earlier step's sampled tokens");
     check(mllm_embed(ids, table ? positions : nullptr, wte.data, table, static_cast<float*>(out.data), T, D, wte.dtype,
-                     feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, stream, scale), "embed");
+                     feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, stream, scale, copy ? copy->data : nullptr), "embed");
 }
 
 void select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream) {
@@ -220,7 +222,7 @@ static int out_dtype_of(int epilogue, int act_dtype) {
 static void check_linear(int64_t M, int64_t K, int a_dtype, const Tensor2& w, const Tensor2& out, int epilogue,
                          const char* what) {
     need_dtype(w, "w");
-    if (epilogue < STORE || epilogue > STORE_F32) fail("%s: unknown epilogue %d", what, epilogue);
+    if ((epilogue < STORE || epilogue > STORE_F32) && epilogue != RELU2) fail("%s: unknown epilogue %d", what, epilogue);
     if (w.cols != K || w.dtype != a_dtype)
         fail("%s: a is [%lld, %lld] %s, w is [%lld, %lld] %s", what, (long long)M, (long long)K, dtype_name(a_dtype),
              (long long)w.rows, (long long)w.cols, dtype_name(w.dtype));

@@ -23,7 +23,7 @@ enum DType : int { F32 = 0, BF16 = 1 };
 inline size_t dtype_size(int dt) { return dt == F32 ? 4 : 2; }
 const char* dtype_name(int dt);
 
-enum Epilogue : int { STORE = 0, GELU_TANH = 1, GELU_ERF = 2, ADD_RESIDUAL = 3, STORE_F32 = 4 };
+enum Epilogue : int { STORE = 0, GELU_TANH = 1, GELU_ERF = 2, ADD_RESIDUAL = 3, STORE_F32 = 4, RELU2 = 6 };
 // Activations that only the gated feed-forward's kernel knows (glu_act), beside GELU_TANH.
 enum GluActivation : int { GLU_SILU = 5 };
 
@@ -139,9 +139,11 @@ struct FedTokens {
 };
 
 // -- the ops -----------------------------------------------------------------------------------------
-// out[t, :] = scale * wte[ids[t], :] (+ wpe[positions[t], :])
+// out[t, :] = scale * wte[ids[t], :] (+ wpe[positions[t], :]); `copy` (optional): the same rows in bfloat16
 void embed(const int* ids, const int* positions, const Tensor2& wte, const Tensor2* wpe, const Tensor2& out,
-           hipStream_t stream, const FedTokens* fed = nullptr, float scale = 1.f);
+           hipStream_t stream, const FedTokens* fed = nullptr, float scale = 1.f, const Tensor2* copy = nullptr);
+// out = x in bfloat16 (contiguous)
+void cast_stream(const Tensor2& x, const Tensor2& out, hipStream_t stream);
 void select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream);
 void reset_state(void* state, size_t slot_bytes, int n_slots, const int* slots, const int* starts, int n_seqs,
                  hipStream_t stream);
@@ -179,9 +181,12 @@ void rmsnorm(const Tensor2& x, const float* weight, float eps, int groups, const
 void rms_linear(const Tensor2& x, const float* weight, float eps, const Tensor2& w, const float* bias, const Tensor2& out,
                 int epilogue, const int* rows, void* tmp, hipStream_t stream);
 // x += mult * scale * (y / sqrt(mean(y^2) + eps) * weight), row by row (scale: per column, or null);
-// `clear`: y is zero afterwards.
+// `clear`: y is zero afterwards. `copy` (optional, x's shape): the new x in bfloat16.
 void rmsnorm_add(const Tensor2& y, const float* weight, const float* scale, float mult, float eps, const Tensor2& x,
-                 bool clear, hipStream_t stream);
+                 bool clear, hipStream_t stream, const Tensor2* copy = nullptr);
+// The same with a layer norm: x += mult * scale * ((y - mean) / sqrt(var + eps) * gamma + beta) (beta may be null).
+void layernorm_add(const Tensor2& y, const float* gamma, const float* beta, const float* scale, float mult, float eps, const Tensor2& x,
+                   bool clear, hipStream_t stream, const Tensor2* copy = nullptr);
 // out = g sigmoid(alpha g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)
 void glu_clamped(const Tensor2& gate, const Tensor2& up, float limit, float alpha, const Tensor2& out, hipStream_t stream);
 void fill_zero(const Tensor2& x, hipStream_t stream);          // contiguous fp32, by a kernel
@@ -193,6 +198,7 @@ struct StateArgs {
     const int* cu_q = nullptr;         // [B + 1]
     const int* state_slots = nullptr;  // [B], < 0: padding
     int n_seqs = 0, max_q_len = 0;     // max_q_len: the longest portion of the step
+    int n_single = 0;                  // the first n_single sequences bring one token each
     float* state = nullptr;
     size_t slot_floats = 0;
     int n_slots = 0;
@@ -215,7 +221,11 @@ int ssm_scan_parts(int N);
 
 // -- latent attention --------------------------------------------------------------------------------
 struct LatentShape {
-    int n_heads = 0, plain_dim = 0, rot_dim = 0, value_dim = 0, kv_rank = 0, q_rank = 0, rot_dims = 0;
+    int n_heads = 0, plain_dim = 0, rot_dim = 0, value_dim = 0, kv_rank = 0, rot_dims = 0;
+    int q_rank = 0;                    // 0: queries without a latent of their own
+    int norm_cols = 0;                 // columns of the latent that its norm's mean runs over (0: kv_rank; fewer: the latent was
+                                       // widened with zero columns)
+    bool half_split = false;           // rotated pairs are columns i and i + rot_dims / 2 instead of 2i and 2i + 1
     double rot_base = 10000.0;
     float eps = 1e-6f;
 };
@@ -226,10 +236,15 @@ struct LatentPages {
     Tensor2 rows, latent_t;
     int page_size = 0;
 };
-// cq = rmsnorm(dq) * wq; with dkv: page row slots[t] = [rmsnorm(dkv[:, :kv_rank]) * wkv | turned rest]
+// The smallest sizes of the matrix-core kernels that hold a latent of `rank` and a rotated part of `rot` columns (both may
+// come back larger: to be filled with zero columns). False: there are none.
+bool latent_tile_shape(int& rank, int& rot);
+// cq = rmsnorm(dq) * wq (with a query latent, q_rank > 0; otherwise dq and cq are ignored); with dkv: page row slots[t] =
+// [rmsnorm(dkv[:, :kv_rank]) * wkv | turned rest]
 void latent_prepare(const Tensor2& dq, const float* wq, const Tensor2& cq, const Tensor2* dkv, const float* wkv,
                     const LatentPages* pages, const int* slots, const int* positions, const LatentShape& sh, hipStream_t stream);
-// qa[t, h] = [W_uk_h^T q_plain[t, h] | turned q_rot[t, h]]; w_uk is handed over transposed, [kv_rank, heads * plain_dim]
+// qa[t, h] = [W_uk_h^T q_plain[t, h] | turned q_rot[t, h]]; w_uk is handed over transposed, [kv_rank, heads * plain_dim];
+// q in the dtype of w_uk, or fp32
 void latent_absorb(const Tensor2& q, const Tensor2& w_uk, const Tensor2& qa, const int* positions, const LatentShape& sh,
                    hipStream_t stream);
 // The step's sequences, as attention sees them.
@@ -248,8 +263,9 @@ struct LatentStep {
 void latent_attention(const Tensor2& qa, const LatentPages& pages, const LatentStep& step, float scale, int window,
                       const LatentShape& sh, const Tensor2& o_lat, float* workspace, size_t workspace_floats, hipStream_t stream);
 size_t latent_attention_workspace_floats(int kv_rank);
-// out[t, h*value_dim + e] = sum_r w_uv[h*value_dim + e, r] * o_lat[t, h, r]
-void latent_expand(const Tensor2& o_lat, const Tensor2& w_uv, const Tensor2& out, const LatentShape& sh, hipStream_t stream);
+// out[t, h*value_dim + e] = sum_r w_uv[h*value_dim + e, r] * o_lat[t, h, r] (times sigmoid(gate[t, h]): fp32 [T, heads])
+void latent_expand(const Tensor2& o_lat, const Tensor2& w_uv, const Tensor2& out, const LatentShape& sh, hipStream_t stream,
+                   const Tensor2* gate = nullptr);
 
 // -- attention with shaped scores -------------------------------------------------------------------
 // out = in + conv(in): a causal convolution per channel over `taps` inputs (taps [channels, taps], the last tap
@@ -313,6 +329,24 @@ struct ScoredStep {
 void scored_attention(const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, const ScoredStep& step,
                       const ScoredShape& sh, const Tensor2* gate, int gate_col, const Tensor2& out, hipStream_t stream);
 
+// -- matrix memory with exponential gates (mLSTM) ---------------------------------------------------
+// Columns of the joined input projection's fp32 rows, sizes and constants (kernels/matrix_memory.hip has the equations).
+struct MemoryShape {
+    int heads = 0, dim = 0, value_dim = 0;
+    int q_col = 0, k_col = 0, v_col = 0, g_col = 0, i_col = 0, f_col = 0;
+    float cap = 0.f, q_scale = 1.f, eps = 1e-6f;
+    const float *i_bias = nullptr, *f_bias = nullptr;      // [heads]
+    const float* norm = nullptr;                           // [heads * value_dim]
+};
+// out [T, heads * value_dim] (the compute dtype): every head's readout, RMS-normed, weighed and gated. The state of a request
+// (matrix_memory_state_floats floats) starts at st.state. The first st.n_single sequences bring one token each; portions
+// run in chunks side by side, for which `workspace` (matrix_memory_workspace_floats floats) is needed. y (fp32, out's
+// shape): room for heads whose work several workgroups share.
+void matrix_memory(const Tensor2& proj, const MemoryShape& sh, const StateArgs& st, const Tensor2& out, const Tensor2& y, float* workspace,
+                   size_t workspace_floats, hipStream_t stream);
+size_t matrix_memory_state_floats(int heads, int dim, int value_dim);
+size_t matrix_memory_workspace_floats(int tokens, int n_seqs, int heads, int dim, int value_dim);
+
 // -- gated linear recurrence (HGRN2) ----------------------------------------------------------------
 // proj (fp32 rows): raw queries at q_col and raw gates at f_col (heads * dim each), values at v_col (heads * value_dim).
 // y: hgrn2_parts(dim) shares [T, heads * value_dim], y.rows * y.stride floats apart; the state ([heads][dim][value_dim]
@@ -340,9 +374,9 @@ void rotary_rows(const Tensor2& proj, int col0, int n_heads, int dim, int rot_di
 // out[t, c] = sigmoid(w[c, :] . proj[t, a_col : a_col + rank] + bias[c])^(1 / tau): w [N, rank] fp32, out [T, N] fp32.
 void lowrank_decay(const Tensor2& proj, int a_col, const Tensor2& w, const float* bias, float tau, const Tensor2& out, hipStream_t stream);
 // out = rmsnorm(x) * weight * silu(gate[:, gate_col ..]) in `groups` equal parts of the columns, the gate BEHIND the norm
-// (weight [x.cols] or null; gate fp32 rows). Parts as for rmsnorm.
+// (weight [x.cols] or null; gate fp32 rows). Parts as for rmsnorm. plain_sigmoid: sigmoid(gate) in place of silu(gate).
 void rmsnorm_gate_after(const Tensor2& x, const float* weight, float eps, int groups, const Tensor2& gate, int gate_col, const Tensor2& out,
-                        hipStream_t stream, int parts = 1, size_t part_stride = 0);
+                        hipStream_t stream, int parts = 1, size_t part_stride = 0, bool plain_sigmoid = false);
 // x <- cap tanh(x / cap) (contiguous fp32)
 void softcap(const Tensor2& x, float cap, hipStream_t stream);
 // `kept` holds n_old earlier streams of x's shape one behind the other ([>= (n_old + 1) * rows, cols] fp32, contiguous).
@@ -354,8 +388,19 @@ void depth_mix(const Tensor2& x, const Tensor2& kept, int n_old, const float* w,
 // lower index wins a tie), weight_e = scale * score_e for them and 0 for the others. Then
 // out[t, e * ff + j] = weight_e * relu(up[t, e * ff + j])^2 for the E experts of ff columns; the columns behind them (a
 // shared expert's) are relu(.)^2 alone. out may be up. `weights` (optional, [T, E] fp32) receives the weights.
+// The options: GELU_ERF instead of the squared rectified value; `correction` ([E + identity] fp32 on the device): the
+// experts with the largest score + correction are chosen, the score alone stays the weight; the last `identity` columns of
+// the logits are experts that hand on their input: y (fp32, a row per token) is set to (or with y_add grows by) the sum of
+// their weights times h (out's dtype). up may be fp32 where out is bfloat16.
+struct MoeOptions {
+    int activation = RELU2;
+    const float* correction = nullptr;
+    int identity = 0;
+    Tensor2 h, y;
+    bool y_add = false;
+};
 void moe_act(const Tensor2& up, const Tensor2& logits, int ff, int top, float scale, const Tensor2& out, const Tensor2* weights,
-             hipStream_t stream);
+             hipStream_t stream, const MoeOptions& options = MoeOptions());
 // The routed experts' activation for gated, clamped experts (kernels/moe.hip): up [T, 2 (E ff + shared_ff)] with rows
 // [expert: gate | up] ... [shared: gate | up], logits [T, E (+ 1: the shared expert's gate)] fp32, out [T, E ff + shared_ff].
 struct MoeGlu {

@@ -267,7 +267,7 @@ void lowrank_decay(const Tensor2& proj, int a_col, const Tensor2& w, const float
 }
 
 void rmsnorm_gate_after(const Tensor2& x, const float* weight, float eps, int groups, const Tensor2& gate, int gate_col, const Tensor2& out,
-                        hipStream_t stream, int parts, size_t part_stride) {
+                        hipStream_t stream, int parts, size_t part_stride, bool plain_sigmoid) {
     need_f32(x, "rmsnorm_gate_after: x");
     need_f32(gate, "rmsnorm_gate_after: the gate");
     need_act(out, "rmsnorm_gate_after: out");
@@ -275,7 +275,7 @@ void rmsnorm_gate_after(const Tensor2& x, const float* weight, float eps, int gr
     if (out.rows != x.rows || out.cols != x.cols || gate.rows != x.rows || gate_col < 0 || gate_col + x.cols > gate.cols)
         fail("rmsnorm_gate_after: out and the gate's columns must match x [%lld, %lld]", (long long)x.rows, (long long)x.cols);
     check(mllm_rmsnorm_gate_after(static_cast<const float*>(x.data), i32(x.stride), weight, static_cast<const float*>(gate.data) + gate_col, i32(gate.stride),
-                                  out.data, i32(out.stride), i32(x.rows), i32(x.cols), groups, eps, out.dtype, parts, part_stride, stream), "rmsnorm_gate_after");
+                                  out.data, i32(out.stride), i32(x.rows), i32(x.cols), groups, eps, out.dtype, parts, part_stride, stream, plain_sigmoid ? 1 : 0), "rmsnorm_gate_after");
 }
 
 void softcap(const Tensor2& x, float cap, hipStream_t stream) {
@@ -296,23 +296,32 @@ void depth_mix(const Tensor2& x, const Tensor2& kept, int n_old, const float* w,
 }
 
 void moe_act(const Tensor2& up, const Tensor2& logits, int ff, int top, float scale, const Tensor2& out, const Tensor2* weights,
-             hipStream_t stream) {
+             hipStream_t stream, const MoeOptions& o) {
     need_act(up, "moe_act: up");
     need_f32(logits, "moe_act: the router's logits");
-    if (out.dtype != up.dtype || out.rows != up.rows || out.cols != up.cols) fail("moe_act: out must have up's shape and dtype");
-    const int E = i32(logits.cols);
+    if (out.rows != up.rows || out.cols != up.cols || (out.dtype != up.dtype && !(up.dtype == F32 && out.data != up.data)))
+        fail("moe_act: out must have up's shape, and its dtype unless up is float32 and another tensor");
+    if (o.activation != RELU2 && o.activation != GELU_ERF) fail("moe_act: unknown activation %d", o.activation);
+    const int all = i32(logits.cols), E = all - o.identity;
+    if (o.identity < 0) fail("moe_act: %d identity experts", o.identity);
+    if (o.identity > 0) {
+        need_f32(o.y, "moe_act: y");
+        if (o.h.dtype != out.dtype || o.h.rows != up.rows || o.y.rows != up.rows || o.h.cols != o.y.cols) fail("moe_act: the identity experts' input (in out's dtype) and result must have one shape");
+    }
     if (logits.rows != up.rows || E < 1 || ff < 1 || static_cast<int64_t>(E) * ff > up.cols) fail("moe_act: %d experts of %d columns do not fit rows of %lld", E, ff, (long long)up.cols);
-    if (top < 1 || top > E) fail("moe_act: %d of %d experts", top, E);
+    if (top < 1 || top > all) fail("moe_act: %d of %d experts", top, all);
     float* wp = nullptr;
     int ldw = 0;
     if (weights != nullptr) {
         need_f32(*weights, "moe_act: the weights");
-        if (weights->rows != up.rows || weights->cols != E) fail("moe_act: the weights must be [%lld, %d]", (long long)up.rows, E);
+        if (weights->rows != up.rows || weights->cols != all) fail("moe_act: the weights must be [%lld, %d]", (long long)up.rows, all);
         wp = static_cast<float*>(weights->data);
         ldw = i32(weights->stride);
     }
     check(mllm_moe_act(up.data, i32(up.stride), static_cast<const float*>(logits.data), i32(logits.stride), E, ff, i32(up.cols) - E * ff, top, scale,
-                       out.data, i32(out.stride), wp, ldw, i32(up.rows), up.dtype, stream), "moe_act");
+                       out.data, i32(out.stride), wp, ldw, i32(up.rows), out.dtype, stream, up.dtype, o.activation == GELU_ERF ? 1 : 0,
+                       o.correction, o.identity, o.h.data, i32(o.h.stride), i32(o.h.cols), static_cast<float*>(o.y.data), i32(o.y.stride),
+                       o.y_add ? 1 : 0), "moe_act");
 }
 
 void moe_glu_act(const Tensor2& up, const Tensor2& logits, const MoeGlu& m, const Tensor2& out, hipStream_t stream) {

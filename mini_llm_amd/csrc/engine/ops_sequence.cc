@@ -73,15 +73,34 @@ void rms_linear(const Tensor2& x, const float* weight, float eps, const Tensor2&
     linear(h, w, bias, out, epilogue, nullptr, stream);
 }
 
-void rmsnorm_add(const Tensor2& y, const float* weight, const float* scale, float mult, float eps, const Tensor2& x,
-                 bool clear, hipStream_t stream) {
-    need_f32(y, "rmsnorm_add: y");
-    need_f32(x, "rmsnorm_add: x");
-    if (weight == nullptr) fail("rmsnorm_add: the weight is missing");
+static void norm_add(const char* what, const Tensor2& y, const float* weight, const float* beta, const float* scale, float mult, float eps,
+                     const Tensor2& x, bool clear, bool center, const Tensor2* copy, hipStream_t stream) {
+    need_f32(y, what);
+    need_f32(x, what);
+    if (weight == nullptr) fail("%s: the weight is missing", what);
     if (!y.contiguous() || !x.contiguous() || y.rows != x.rows || y.cols != x.cols)
-        fail("rmsnorm_add: x and y must be contiguous float32 of one shape");
-    check(mllm_rmsnorm_add(static_cast<float*>(y.data), weight, scale, mult, eps, static_cast<float*>(x.data), i32(x.rows), i32(x.cols),
-                           clear ? 1 : 0, stream), "rmsnorm_add");
+        fail("%s: x and y must be contiguous float32 of one shape", what);
+    if (copy != nullptr && (copy->dtype != BF16 || copy->data == nullptr || !copy->contiguous() || copy->rows != x.rows || copy->cols != x.cols))
+        fail("%s: the copy must be contiguous bfloat16 of x's shape", what);
+    check(mllm_norm_add(static_cast<float*>(y.data), weight, beta, scale, mult, eps, static_cast<float*>(x.data), i32(x.rows), i32(x.cols),
+                        clear ? 1 : 0, center ? 1 : 0, copy ? copy->data : nullptr, stream), what);
+}
+
+void rmsnorm_add(const Tensor2& y, const float* weight, const float* scale, float mult, float eps, const Tensor2& x,
+                 bool clear, hipStream_t stream, const Tensor2* copy) {
+    norm_add("rmsnorm_add", y, weight, nullptr, scale, mult, eps, x, clear, false, copy, stream);
+}
+
+void layernorm_add(const Tensor2& y, const float* gamma, const float* beta, const float* scale, float mult, float eps, const Tensor2& x,
+                   bool clear, hipStream_t stream, const Tensor2* copy) {
+    norm_add("layernorm_add", y, gamma, beta, scale, mult, eps, x, clear, true, copy, stream);
+}
+
+void cast_stream(const Tensor2& x, const Tensor2& out, hipStream_t stream) {
+    need_f32(x, "cast_stream: x");
+    if (out.dtype != BF16 || !x.contiguous() || !out.contiguous() || out.rows != x.rows || out.cols != x.cols)
+        fail("cast_stream: x must be contiguous float32 and out contiguous bfloat16 of its shape");
+    check(mllm_cast_bf16(static_cast<const float*>(x.data), out.data, static_cast<size_t>(x.rows) * x.cols, stream), "cast_stream");
 }
 
 void glu_clamped(const Tensor2& gate, const Tensor2& up, float limit, float alpha, const Tensor2& out, hipStream_t stream) {
@@ -147,8 +166,43 @@ size_t ssm_scan_workspace_floats(int tokens, int n_seqs, int H, int P, int N) {
     return mllm_ssm_scan_workspace_floats(tokens, n_seqs, H, P, N);
 }
 
+size_t matrix_memory_state_floats(int heads, int dim, int value_dim) { return mllm_matrix_memory_state_floats(heads, dim, value_dim); }
+size_t matrix_memory_workspace_floats(int tokens, int n_seqs, int heads, int dim, int value_dim) {
+    return mllm_matrix_memory_workspace_floats(tokens, n_seqs, heads, dim, value_dim);
+}
+
+void matrix_memory(const Tensor2& proj, const MemoryShape& sh, const StateArgs& st, const Tensor2& out, const Tensor2& y, float* workspace,
+                   size_t workspace_floats, hipStream_t stream) {
+    need_f32(proj, "matrix_memory: the projection");
+    need_act(out, "matrix_memory: out");
+    need_f32(y, "matrix_memory: y");
+    const int H = sh.heads, d = sh.dim, e = sh.value_dim, T = i32(proj.rows);
+    if (H < 1 || d < 1 || e < 1 || !(sh.cap > 0.f)) fail("matrix_memory: heads, sizes and the gates' cap must be positive");
+    auto inside = [&](int col, int64_t n) { return col >= 0 && col + n <= proj.cols; };
+    const int64_t nk = static_cast<int64_t>(H) * d, nv = static_cast<int64_t>(H) * e;
+    if (!inside(sh.q_col, nk) || !inside(sh.k_col, nk) || !inside(sh.v_col, nv) || !inside(sh.g_col, nv) || !inside(sh.i_col, H) || !inside(sh.f_col, H))
+        fail("matrix_memory: the inputs lie outside the projection's rows of %lld", (long long)proj.cols);
+    if (sh.i_bias == nullptr || sh.f_bias == nullptr || sh.norm == nullptr) fail("matrix_memory: the gates' biases and the norm's weight are needed");
+    if (out.rows != T || out.cols != nv || y.rows != T || y.cols != nv) fail("matrix_memory: out and y must be [%d, %lld]", T, (long long)nv);
+    check_state(st, matrix_memory_state_floats(H, d, e), "matrix_memory");
+    if (st.n_single < 0 || st.n_single > st.n_seqs) fail("matrix_memory: %d of %d sequences", st.n_single, st.n_seqs);
+    const int max_portion = st.n_single == st.n_seqs ? 0 : std::max(st.max_q_len, 1);
+    if (workspace != nullptr && workspace_floats < matrix_memory_workspace_floats(T, st.n_seqs, H, d, e))
+        fail("matrix_memory: the workspace holds %zu floats, %zu are needed", workspace_floats, matrix_memory_workspace_floats(T, st.n_seqs, H, d, e));
+    int needs_norm = 0;
+    check(mllm_matrix_memory(static_cast<const float*>(proj.data), i32(proj.stride), sh.q_col, sh.k_col, sh.v_col, sh.g_col, sh.i_col, sh.f_col,
+                             sh.i_bias, sh.f_bias, sh.norm, sh.cap, sh.q_scale, sh.eps, st.cu_q, st.state_slots, st.state, st.slot_floats, T, st.n_seqs,
+                             st.n_single, max_portion, H, d, e, st.write ? 1 : 0, workspace, out.data, i32(out.stride), static_cast<float*>(y.data),
+                             i32(y.stride), out.dtype, &needs_norm, stream), "matrix_memory");
+    // rows whose heads were shared by several workgroups: their norm and gate
+    const int64_t first = (needs_norm & 1) ? 0 : st.n_single, last = (needs_norm & 2) ? T : st.n_single;
+    if (needs_norm != 0 && first < last)
+        rmsnorm_gate_after(y.row_range(first, last - first), sh.norm, sh.eps, H, proj.row_range(first, last - first), sh.g_col,
+                           out.row_range(first, last - first), stream, 1, 0, true);
+}
+
 static void check_shape(const LatentShape& sh, const char* what) {
-    if (sh.n_heads < 1 || sh.plain_dim < 1 || sh.rot_dim < 0 || sh.value_dim < 1 || sh.kv_rank < 1 || sh.q_rank < 1)
+    if (sh.n_heads < 1 || sh.plain_dim < 1 || sh.rot_dim < 0 || sh.value_dim < 1 || sh.kv_rank < 1 || sh.q_rank < 0 || sh.norm_cols < 0 || sh.norm_cols > sh.kv_rank)
         fail("%s: heads and sizes must be positive", what);
     if (sh.rot_dims < 0 || sh.rot_dims % 2 != 0 || sh.rot_dims > sh.rot_dim || sh.rot_dim % 2 != 0 || !(sh.rot_base > 0))
         fail("%s: %d of %d rotary columns (both even) and a positive base are needed", what, sh.rot_dims, sh.rot_dim);
@@ -167,21 +221,36 @@ static void check_pages(const LatentPages& pages, int dtype, const LatentShape& 
 void latent_prepare(const Tensor2& dq, const float* wq, const Tensor2& cq, const Tensor2* dkv, const float* wkv,
                     const LatentPages* pages, const int* slots, const int* positions, const LatentShape& sh, hipStream_t stream) {
     check_shape(sh, "latent_prepare");
-    need_f32(dq, "latent_prepare: the query latent");
-    need_act(cq, "latent_prepare: cq");
-    if (dq.cols != sh.q_rank || cq.cols != sh.q_rank || cq.rows != dq.rows || wq == nullptr)
-        fail("latent_prepare: the query latent must be [T, %d] with its norm weight", sh.q_rank);
+    const bool has_q = sh.q_rank > 0;
+    if (has_q) {
+        need_f32(dq, "latent_prepare: the query latent");
+        need_act(cq, "latent_prepare: cq");
+        if (dq.cols != sh.q_rank || cq.cols != sh.q_rank || cq.rows != dq.rows || wq == nullptr)
+            fail("latent_prepare: the query latent must be [T, %d] with its norm weight", sh.q_rank);
+    } else if (dkv == nullptr) {
+        return;
+    }
+    const int64_t T = has_q ? dq.rows : dkv->rows;
+    const int dtype = has_q ? cq.dtype : pages != nullptr ? pages->rows.dtype : F32;
     if (dkv != nullptr) {
         need_f32(*dkv, "latent_prepare: the key/value latent");
         if (pages == nullptr || slots == nullptr || positions == nullptr || wkv == nullptr) fail("latent_prepare: pages, page rows, positions and the norm weight are needed");
-        if (dkv->cols != sh.kv_rank + sh.rot_dim || dkv->rows != dq.rows) fail("latent_prepare: the key/value latent must be [T, %d]", sh.kv_rank + sh.rot_dim);
-        check_pages(*pages, cq.dtype, sh, "latent_prepare");
+        if (dkv->cols != sh.kv_rank + sh.rot_dim || dkv->rows != T) fail("latent_prepare: the key/value latent must be [T, %d]", sh.kv_rank + sh.rot_dim);
+        check_pages(*pages, dtype, sh, "latent_prepare");
     }
-    check(mllm_latent_prepare(static_cast<const float*>(dq.data), i32(dq.stride), sh.q_rank, wq, cq.data, i32(cq.stride),
+    check(mllm_latent_prepare(has_q ? static_cast<const float*>(dq.data) : nullptr, i32(dq.stride), sh.q_rank, wq, cq.data, i32(cq.stride),
                               dkv ? static_cast<const float*>(dkv->data) : nullptr, dkv ? i32(dkv->stride) : 0, sh.kv_rank, sh.rot_dim, wkv,
                               dkv ? pages->rows.data : nullptr, dkv ? pages->latent_t.data : nullptr, dkv ? pages->page_size : 0, slots, positions,
-                              i32(dq.rows), sh.eps, sh.rot_base, sh.rot_dims, cq.dtype, stream),
+                              i32(T), sh.eps, sh.rot_base, sh.rot_dims, dtype, stream, sh.norm_cols, sh.half_split ? 1 : 0),
           "latent_prepare");
+}
+
+bool latent_tile_shape(int& rank, int& rot) {
+    int R = 0, E = 0;
+    if (mllm_latent_tile_shape(rank, rot, &R, &E) != 0) return false;
+    rank = R;
+    rot = E - R;
+    return true;
 }
 
 void latent_absorb(const Tensor2& q, const Tensor2& w_uk, const Tensor2& qa, const int* positions, const LatentShape& sh,
@@ -190,12 +259,13 @@ void latent_absorb(const Tensor2& q, const Tensor2& w_uk, const Tensor2& qa, con
     need_act(q, "latent_absorb: q");
     const int E = sh.kv_rank + sh.rot_dim;
     if (q.cols != static_cast<int64_t>(sh.n_heads) * (sh.plain_dim + sh.rot_dim)) fail("latent_absorb: q must be [T, %d]", sh.n_heads * (sh.plain_dim + sh.rot_dim));
-    if (w_uk.dtype != q.dtype || w_uk.cols != static_cast<int64_t>(sh.n_heads) * sh.plain_dim || w_uk.rows != sh.kv_rank)
+    if ((w_uk.dtype != q.dtype && q.dtype != F32) || w_uk.cols != static_cast<int64_t>(sh.n_heads) * sh.plain_dim || w_uk.rows != sh.kv_rank)
         fail("latent_absorb: the transposed key expansion must be [%d, %d] %s", sh.kv_rank, sh.n_heads * sh.plain_dim, dtype_name(q.dtype));
-    if (qa.dtype != q.dtype || qa.rows != q.rows || qa.cols != static_cast<int64_t>(sh.n_heads) * E) fail("latent_absorb: qa must be [T, %d]", sh.n_heads * E);
+    if (qa.dtype != w_uk.dtype || qa.rows != q.rows || qa.cols != static_cast<int64_t>(sh.n_heads) * E) fail("latent_absorb: qa must be [T, %d]", sh.n_heads * E);
     if (positions == nullptr) fail("latent_absorb: positions are needed");
     check(mllm_latent_absorb(q.data, i32(q.stride), w_uk.data, i32(w_uk.stride), qa.data, i32(qa.stride), positions, i32(q.rows), sh.n_heads,
-                             sh.plain_dim, sh.rot_dim, sh.kv_rank, sh.rot_base, sh.rot_dims, q.dtype, stream), "latent_absorb");
+                             sh.plain_dim, sh.rot_dim, sh.kv_rank, sh.rot_base, sh.rot_dims, w_uk.dtype, stream, q.dtype, sh.half_split ? 1 : 0),
+          "latent_absorb");
 }
 
 // Rows x splits that a launch with split keys holds at most (its workspace is made for them).
@@ -242,15 +312,19 @@ void latent_attention(const Tensor2& qa, const LatentPages& pages, const LatentS
           "latent_attention");
 }
 
-void latent_expand(const Tensor2& o_lat, const Tensor2& w_uv, const Tensor2& out, const LatentShape& sh, hipStream_t stream) {
+void latent_expand(const Tensor2& o_lat, const Tensor2& w_uv, const Tensor2& out, const LatentShape& sh, hipStream_t stream,
+                   const Tensor2* gate) {
     check_shape(sh, "latent_expand");
     need_act(o_lat, "latent_expand: the attention result");
     if (o_lat.cols != static_cast<int64_t>(sh.n_heads) * sh.kv_rank) fail("latent_expand: the attention result must be [T, %d]", sh.n_heads * sh.kv_rank);
     if (w_uv.dtype != o_lat.dtype || w_uv.rows != static_cast<int64_t>(sh.n_heads) * sh.value_dim || w_uv.cols != sh.kv_rank)
         fail("latent_expand: the value expansion must be [%d, %d] %s", sh.n_heads * sh.value_dim, sh.kv_rank, dtype_name(o_lat.dtype));
     if (out.dtype != o_lat.dtype || out.rows != o_lat.rows || out.cols != w_uv.rows) fail("latent_expand: out must be [T, %lld]", (long long)w_uv.rows);
+    if (gate != nullptr && (gate->dtype != F32 || gate->data == nullptr || gate->rows != o_lat.rows || gate->cols != sh.n_heads))
+        fail("latent_expand: the gate must be float32 [%lld, %d]", (long long)o_lat.rows, sh.n_heads);
     check(mllm_latent_expand(o_lat.data, i32(o_lat.stride), w_uv.data, i32(w_uv.stride), out.data, i32(out.stride), i32(o_lat.rows), sh.n_heads,
-                             sh.value_dim, sh.kv_rank, o_lat.dtype, stream), "latent_expand");
+                             sh.value_dim, sh.kv_rank, o_lat.dtype, stream, gate ? static_cast<const float*>(gate->data) : nullptr,
+                             gate ? i32(gate->stride) : 0), "latent_expand");
 }
 
 }  // namespace minillm

@@ -112,7 +112,7 @@ void Norm::forward_into(const Tensor2&, const int*, const Tensor2&, hipStream_t)
     fail("this kind of norm cannot write into a tensor it is handed");
 }
 
-void Norm::add_scaled(const Tensor2&, const float*, float, const Tensor2&, bool, hipStream_t) const {
+void Norm::add_scaled(const Tensor2&, const float*, float, const Tensor2&, bool, hipStream_t, const Tensor2*) const {
     fail("this kind of norm cannot stand behind a sub-layer (it has no scaled add)");
 }
 
@@ -158,6 +158,11 @@ public:
         void* tmp = arena.take(static_cast<size_t>(out.rows) * size_ * dtype_size(lin.weight.dtype));
         ln_linear(x, gamma_, beta_, eps_, lin.weight, lin.bias, out, epilogue, rows, tmp, kv, s);
         arena.release(mark);
+    }
+    void add_scaled(const Tensor2& y, const float* scale, float mult, const Tensor2& x, bool clear, hipStream_t s,
+                    const Tensor2* copy) const override {
+        if (y.cols != size_) fail("layernorm: rows of %lld, the norm is %d wide", (long long)y.cols, size_);
+        layernorm_add(y, gamma_, beta_, scale, mult, eps_, x, clear, s, copy);
     }
     size_t workspace_bytes(int rows) const override { return static_cast<size_t>(rows) * size_ * dtype_size(dtype) + 256; }
     void add_cost(StepCost& c) const override { c.weight_bytes += 4.0 * size_ * (beta_ ? 2 : 1); }
@@ -283,16 +288,23 @@ public:
         const std::string& act = p.string("activation");
         if (act == "gelu_tanh") act_ = GELU_TANH;
         else if (act == "gelu_erf") act_ = GELU_ERF;
-        else fail("unknown activation '%s' (known: gelu_erf, gelu_tanh)", act.c_str());
+        else if (act == "relu2") act_ = RELU2;
+        else fail("unknown activation '%s' (known: gelu_erf, gelu_tanh, relu2)", act.c_str());
         up_ = Linear(p.weights("up.weight"), p.weights_or_null("up.bias"));
         down_ = Linear(p.weights("down.weight"), p.weights_or_null("down.bias"));
         if (down_.in_features() != up_.out_features()) fail("feed-forward: the two products' shapes do not fit");
     }
     void forward(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const override {
+        run(h, step, x, arena, s, ADD_RESIDUAL);
+    }
+    void forward_set(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const override {
+        run(h, step, x, arena, s, STORE_F32);
+    }
+    void run(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue) const {
         Tensor2 inner = arena.tensor(dtype_, step.n_tokens, up_.out_features());
         h.linear(up_, inner, act_, nullptr, arena, s);
         StageTimes::get().mark("fc1", s);
-        down_(inner, x, ADD_RESIDUAL, nullptr, s);
+        down_(inner, x, out_epilogue, nullptr, s);
         StageTimes::get().mark("fc2", s);
     }
     size_t workspace_bytes(int tokens) const override {
@@ -415,9 +427,11 @@ public:
     int vocab_size() const override { return static_cast<int>(table_.rows); }
     int hidden_size() const override { return static_cast<int>(table_.cols); }
     void forward(const StepView& step, const PositionEncoding* position, const Tensor2& x, hipStream_t s) const override {
-        embed(step.token_ids, step.positions, table_, position ? position->table() : nullptr, x, s, &step.fed, scale_);
+        embed(step.token_ids, step.positions, table_, position ? position->table() : nullptr, x, s, &step.fed, scale_,
+              step.stream_copy.data != nullptr ? &step.stream_copy : nullptr);
     }
     bool resolves_fed_tokens() const override { return true; }
+    bool writes_stream_copy() const override { return true; }
 
 private:
     Tensor2 table_;         // [V, D]
@@ -498,6 +512,7 @@ void register_builtin_parts() {
     register_scored_attention();
     register_recurrent_parts();
     register_linear_attention_parts();
+    register_matrix_memory();
 }
 }  // namespace
 
@@ -643,6 +658,8 @@ size_t DecoderModel::workspace_bytes(int tokens, int n_logits) const {
     const size_t one = stream;
     for (const auto& l : layers)
         if (l->wants_zeroed_rows()) { stream += one; break; }
+    for (const auto& l : layers)
+        if (l->wants_stream_copy()) { stream += one / 2 + 256; break; }
     for (const auto& st : stream_steps) {
         if (st->wants_embedding_output()) { stream += one; break; }
     }
@@ -664,7 +681,14 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
     StageTimes& times = StageTimes::get();
     times.begin_step(step.max_q_len == 1 ? "decode" : (step.n_single > 0 ? "mixed" : "prefill"), step.n_seqs, step.n_tokens, s);
     Tensor2 x = arena.tensor(F32, step.n_tokens, hidden_size());
-    embedding->forward(step, position.get(), x, s);
+    StepView with_rows = step;
+    for (const auto& l : layers) {
+        if (!l->wants_stream_copy()) continue;
+        with_rows.stream_copy = arena.tensor(BF16, step.n_tokens, hidden_size());
+        break;
+    }
+    embedding->forward(with_rows, position.get(), x, s);
+    bool copied = embedding->writes_stream_copy();      // whether the copy, if there is one, equals the stream
     // a stream step that mixes the embedding's output back in later: a copy of it stays for the step
     // (with room behind it for the streams that a stream step keeps for itself during the step)
     Tensor2 x0, x0_and_kept;
@@ -679,7 +703,6 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         break;
     }
     times.mark("embed", s);
-    StepView with_rows = step;
     for (const auto& l : layers) {
         if (!l->wants_zeroed_rows()) continue;
         Tensor2 z = arena.tensor(F32, step.n_tokens, hidden_size());
@@ -696,14 +719,19 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
             const StreamStep& st = *stream_steps[c.before];
             st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, c.pass, with_rows, arena, s);
             arena.release(mark);
+            copied = false;
             times.mark("stream_step", s);
         }
+        const bool reads_copy = layers[c.layer]->wants_stream_copy();
+        if (reads_copy && !copied) cast_stream(x, with_rows.stream_copy, s);
+        copied = reads_copy;                            // such a block keeps it, any other changes the stream alone
         layers[c.layer]->forward(x, with_rows, caches[c.cache], c.write, arena, s);
         if (c.after >= 0) {
             const size_t mark = arena.mark();
             const StreamStep& st = *stream_steps[c.after];
             st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, c.after_pass, with_rows, arena, s);
             arena.release(mark);
+            copied = false;
             times.mark("stream_step_after", s);
         }
     }

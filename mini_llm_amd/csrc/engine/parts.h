@@ -95,6 +95,8 @@ struct StepView {
     const int* logit_rows = nullptr;   // [n_logits]
     float* zeroed_rows = nullptr;      // fp32 [n_tokens, hidden], all zero, if a layer asked for it (Block::wants_zeroed_rows):
                                        // room for a sub-layer's result; whoever uses it leaves it zero again
+    Tensor2 stream_copy;               // the stream in bfloat16 as a block is entered, if a block asked for it
+                                       // (Block::wants_stream_copy)
     int n_groups = 0;
     const int* const* block_tables = nullptr;   // per group [B, max_blocks[g]]
     const int* max_blocks = nullptr;            // per group
@@ -195,6 +197,8 @@ public:
     // true: forward() takes `step.fed` into account itself (one kernel fewer in a decode step); false: the runner
     // writes the fed ids into token_ids with a kernel of its own before the step
     virtual bool resolves_fed_tokens() const { return false; }
+    // true: forward() also writes step.stream_copy where it is there; false: the model casts the stream behind it
+    virtual bool writes_stream_copy() const { return false; }
     virtual void add_cost(StepCost&) const {}
 };
 
@@ -225,9 +229,10 @@ public:
     virtual void linear(const Tensor2& x, const Linear& lin, const Tensor2& out, int epilogue, const int* rows,
                         const KvScatter* kv, Arena& arena, hipStream_t s) const;
     // x += mult * scale * norm(y), row by row (y and x fp32 [rows, size]; scale per column or null); with
-    // `clear`, y is zero afterwards. For arrangements with a norm behind a sub-layer; a norm without it refuses.
+    // `clear`, y is zero afterwards; `copy` (optional) receives the new x in bfloat16. For arrangements with a norm
+    // behind a sub-layer; a norm without it refuses.
     virtual void add_scaled(const Tensor2& y, const float* scale, float mult, const Tensor2& x, bool clear,
-                            hipStream_t s) const;
+                            hipStream_t s, const Tensor2* copy = nullptr) const;
     virtual size_t workspace_bytes(int rows) const = 0;
     virtual void add_cost(StepCost&) const {}
     int dtype = BF16;
@@ -284,7 +289,7 @@ public:
     // arena, in `pending`; finish() does the rest and adds into x, after somebody else may have changed x. What
     // begin() took from the arena must still be there when finish() runs. False from begin(): this kind has no halves,
     // and nothing was done.
-    struct Pending { Tensor2 a, b; };
+    struct Pending { Tensor2 a, b, h; };
     virtual bool begin(NormedInput& h, const StepView& step, Arena& arena, hipStream_t s, Pending& pending) const {
         (void)h; (void)step; (void)arena; (void)s; (void)pending;
         return false;
@@ -307,6 +312,9 @@ public:
     // true: the model keeps one cleared fp32 buffer of the stream's shape for the step (StepView::zeroed_rows),
     // cleared once, instead of every layer clearing one of its own
     virtual bool wants_zeroed_rows() const { return false; }
+    // true: the block's sub-layers read the stream itself, in bfloat16: the model keeps a copy of it for the step
+    // (StepView::stream_copy), and the block leaves the copy equal to the stream it leaves
+    virtual bool wants_stream_copy() const { return false; }
     virtual void reserve(int max_seqs, hipStream_t s) const = 0;
     virtual void add_cost(StepCost&) const = 0;
 };
@@ -385,6 +393,8 @@ void register_recurrent_parts();
 // all streams so far (linear_attention.cc); the arrangement with a norm behind each sub-layer only is registered with
 // the gated parts.
 void register_linear_attention_parts();
+// The matrix memory with exponential gates (matrix_memory.cc).
+void register_matrix_memory();
 
 // One entry of the execution order: which layer runs, on which cache, and whether it writes it.
 struct LayerCall {

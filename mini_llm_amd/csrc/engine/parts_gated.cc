@@ -52,9 +52,10 @@ public:
         rms_linear(x, weight_, eps_, lin.weight, lin.bias, out, epilogue, rows, tmp, s);
         arena.release(mark);
     }
-    void add_scaled(const Tensor2& y, const float* scale, float mult, const Tensor2& x, bool clear, hipStream_t s) const override {
+    void add_scaled(const Tensor2& y, const float* scale, float mult, const Tensor2& x, bool clear, hipStream_t s,
+                    const Tensor2* copy) const override {
         if (y.cols != size_) fail("rmsnorm: rows of %lld, the norm is %d wide", (long long)y.cols, size_);
-        rmsnorm_add(y, weight_, scale, mult, eps_, x, clear, s);
+        rmsnorm_add(y, weight_, scale, mult, eps_, x, clear, s, copy);
     }
     size_t workspace_bytes(int rows) const override { return static_cast<size_t>(rows) * size_ * dtype_size(dtype) + 256; }
     void add_cost(StepCost& c) const override { c.weight_bytes += 4.0 * size_; }
@@ -152,7 +153,9 @@ private:
 // convolution over time on each channel, the last tap the token's own; the last taps - 1 rows of each input are carried
 // per request in the front of the layer's state slot (the mixer's convolution first, then the feed-forward's; the
 // mixer's own state, if it has one, lies behind them). The sub-layer sets an fp32 buffer of the stream's shape and the
-// norm adds from there into the stream. Norms: [norm1] or [norm1, norm2]; parameters: dtype, size (the stream's width).
+// norm adds from there into the stream. A sub-layer without a convolution reads the stream itself (in bfloat16: the copy
+// of it that the norms keep up to date, StepView::stream_copy). Norms: [norm1] or [norm1, norm2]; parameters: dtype, size
+// (the stream's width).
 class PostNormBlock final : public Block {
 public:
     PostNormBlock(std::unique_ptr<Mixer> m, std::unique_ptr<FeedForward> f, std::vector<std::unique_ptr<Norm>> norms, const Params& p)
@@ -199,7 +202,8 @@ public:
                 arena.release(mark);
             }
         }
-        if (fused.data == nullptr) norm1_->add_scaled(y, nullptr, 1.f, x, false, s);
+        const Tensor2* copy = wants_stream_copy() ? &step.stream_copy : nullptr;
+        if (fused.data == nullptr) norm1_->add_scaled(y, nullptr, 1.f, x, false, s, copy);
         StageTimes::get().mark("post_norm", s);
         if (ff_) {
             {
@@ -207,7 +211,7 @@ public:
                 ff_->forward_set(h, step, y, arena, s);
             }
             arena.release(mark);
-            norm2_->add_scaled(y, nullptr, 1.f, x, false, s);
+            norm2_->add_scaled(y, nullptr, 1.f, x, false, s, copy);
             StageTimes::get().mark("post_norm2", s);
         }
         arena.release(outer);
@@ -223,6 +227,7 @@ public:
         if (conv1_bytes_ + conv2_bytes_ > 0) { n.kind |= 2; n.state_bytes += conv1_bytes_ + conv2_bytes_; }
         return n;
     }
+    bool wants_stream_copy() const override { return dtype_ == BF16 && (conv1_.data == nullptr || (ff_ && conv2_.data == nullptr)); }
     void reserve(int max_seqs, hipStream_t s) const override {
         mixer_->reserve(max_seqs, s);
         if (ff_) ff_->reserve(max_seqs, s);
@@ -245,8 +250,9 @@ private:
     Tensor2 input(const Tensor2& x, const Tensor2& conv, size_t state_at, const StepView& step, const CacheView& cache, bool write,
                   Arena& arena, hipStream_t s) const {
         if (conv.data == nullptr) {
-            if (dtype_ != F32) fail("a post-norm block without an input convolution runs in float32 only");
-            return x;
+            if (dtype_ == F32) return x;
+            if (step.stream_copy.data == nullptr) fail("a post-norm block without an input convolution needs the stream's bfloat16 copy");
+            return step.stream_copy;
         }
         if (x.cols != conv.rows) fail("the input convolution has %lld channels, the stream %lld", (long long)conv.rows, (long long)x.cols);
         Tensor2 hc = arena.tensor(dtype_, x.rows, x.cols);

@@ -347,6 +347,41 @@ Tensor2 DeviceTensors::pad_col_blocks(const Tensor2& t, int64_t block, int64_t p
     return Tensor2(base, t.dtype, t.rows, n * padded);
 }
 
+Tensor2 DeviceTensors::pad_row_parts(const Tensor2& t, const std::vector<int64_t>& parts, const std::vector<int64_t>& padded) {
+    int64_t block = 0, out_block = 0;
+    bool ok = !parts.empty() && parts.size() == padded.size() && t.contiguous();
+    for (size_t i = 0; ok && i < parts.size(); ++i) {
+        ok = parts[i] >= 0 && padded[i] >= parts[i];
+        block += parts[i];
+        out_block += padded[i];
+    }
+    if (!ok || block < 1 || t.rows % block != 0) throw WeightsError("pad_row_parts: contiguous rows in whole blocks are needed");
+    const int64_t n = t.rows / block;
+    const size_t row_bytes = static_cast<size_t>(t.cols) * t.esz();
+    char* base = static_cast<char*>(allocate(static_cast<size_t>(n * out_block) * row_bytes, true));
+    for (int64_t b = 0; b < n; ++b) {
+        int64_t from = b * block, to = b * out_block;
+        for (size_t i = 0; i < parts.size(); ++i) {
+            if (parts[i] > 0 && row_bytes > 0 &&
+                hipMemcpy(base + static_cast<size_t>(to) * row_bytes, static_cast<const char*>(t.data) + static_cast<size_t>(from) * row_bytes,
+                          static_cast<size_t>(parts[i]) * row_bytes, hipMemcpyDeviceToDevice) != hipSuccess)
+                throw WeightsError("pad_row_parts: the copy on the device failed");
+            from += parts[i];
+            to += padded[i];
+        }
+    }
+    return Tensor2(base, t.dtype, n * out_block, t.cols);
+}
+
+Tensor2 DeviceTensors::scaled(const Tensor2& v, float factor) {
+    const size_t n = static_cast<size_t>(v.rows) * v.cols;
+    if (v.dtype != F32 || !v.contiguous()) throw WeightsError("scaled: a contiguous float32 vector is needed");
+    std::vector<float> host(n);
+    if (n > 0 && hipMemcpy(host.data(), v.data, n * 4, hipMemcpyDeviceToHost) != hipSuccess) throw WeightsError("scaled: the copy from the device failed");
+    for (float& f : host) f *= factor;
+    return upload(host, 1, static_cast<int64_t>(n), F32);
+}
+
 Tensor2 DeviceTensors::zeros(int64_t n) {
     if (n < 0) throw WeightsError("zeros: a negative size");
     return Tensor2(allocate(static_cast<size_t>(n) * 4, true), F32, 1, n);

@@ -163,6 +163,11 @@ public:
     // as wide as another's, the added ones zero.
     Tensor2 pad_row_blocks(const Tensor2& t, int64_t block, int64_t padded);
     Tensor2 pad_col_blocks(const Tensor2& t, int64_t block, int64_t padded);
+    // The same for blocks made of several parts: a block's part i has parts[i] rows (their sum is the block), each followed by
+    // zero rows up to padded[i].
+    Tensor2 pad_row_parts(const Tensor2& t, const std::vector<int64_t>& parts, const std::vector<int64_t>& padded);
+    // A vector times a number ([1, n] fp32, a copy on the device).
+    Tensor2 scaled(const Tensor2& vector, float factor);
     size_t bytes() const { return bytes_; }
 
 private:

@@ -17,6 +17,7 @@
 #define EPI_GELU_ERF 2      // out[m,n] = gelu_erf(acc + bias)  (activation dtype)
 #define EPI_ADD_RESIDUAL 3  // res[m,n] += acc + bias           (fp32, in place)
 #define EPI_STORE_F32 4     // out[m,n] = acc + bias            (fp32)
+#define EPI_RELU2 6         // out[m,n] = max(acc + bias, 0)^2  (activation dtype; 5 is an activation of the gated kernels)
 
 struct bf16_t {
     uint16_t bits;
@@ -221,6 +222,11 @@ __device__ __forceinline__ float gelu_erf(float v) {
     return 0.5f * v * (1.f + erff(v * 0.70710678118654752440f));
 }
 
+__device__ __forceinline__ float relu2(float v) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+}
+
 // (a 32-bit output takes the full-precision activation: the 32-bit path has no fast approximations)
 template <typename OutT>
 __device__ __forceinline__ void epilogue(int mode, float acc, float bias, void* out, size_t idx) {
@@ -231,6 +237,7 @@ __device__ __forceinline__ void epilogue(int mode, float acc, float bias, void* 
             reinterpret_cast<OutT*>(out)[idx] = from_float<OutT>(sizeof(OutT) == 4 ? gelu_tanh_precise(v) : gelu_tanh(v));
             break;
         case EPI_GELU_ERF: reinterpret_cast<OutT*>(out)[idx] = from_float<OutT>(gelu_erf(v)); break;
+        case EPI_RELU2: reinterpret_cast<OutT*>(out)[idx] = from_float<OutT>(relu2(v)); break;
         case EPI_ADD_RESIDUAL: reinterpret_cast<float*>(out)[idx] += v; break;
         default: reinterpret_cast<float*>(out)[idx] = v; break;
     }

@@ -7,13 +7,14 @@
 // Token + position embedding: x[t,:] = scale * wte[ids[t],:] + wpe[pos[t],:]   (fp32 out)
 // /root/reference/src/kernels/embedding.cu:23-43. wpe may be null (no learned positions).
 // With `src` (optional): where src[t] >= 0, token t's id is prev[src[t]], a token that an earlier step
-// sampled on the device and the host has not read yet; ids[t] is not read then.
+// sampled on the device and the host has not read yet; ids[t] is not read then. With `copy` the row is stored there once
+// more in bfloat16.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void embed_kernel(const int* __restrict__ ids, const int* __restrict__ pos,
                              const T* __restrict__ wte, const T* __restrict__ wpe,
                              float* __restrict__ x, int D, const int* __restrict__ src,
-                             const int* __restrict__ prev, int n_prev, float scale) {
+                             const int* __restrict__ prev, int n_prev, float scale, bf16_t* __restrict__ copy) {
     const int t = blockIdx.x;
     int id = ids[t];
     if (src != nullptr) {
@@ -24,10 +25,23 @@ __global__ void embed_kernel(const int* __restrict__ ids, const int* __restrict_
     float* xr = x + static_cast<size_t>(t) * D;
     if (wpe != nullptr) {
         const T* pe = wpe + static_cast<size_t>(pos[t]) * D;
-        for (int d = threadIdx.x; d < D; d += blockDim.x) xr[d] = to_float(te[d]) * scale + to_float(pe[d]);
+        for (int d = threadIdx.x; d < D; d += blockDim.x) {
+            const float v = to_float(te[d]) * scale + to_float(pe[d]);
+            xr[d] = v;
+            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(v);
+        }
     } else {
-        for (int d = threadIdx.x; d < D; d += blockDim.x) xr[d] = to_float(te[d]) * scale;
+        for (int d = threadIdx.x; d < D; d += blockDim.x) {
+            const float v = to_float(te[d]) * scale;
+            xr[d] = v;
+            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(v);
+        }
     }
+}
+
+__global__ void cast_bf16_kernel(const float* __restrict__ x, bf16_t* __restrict__ out, size_t n) {
+    const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+    if (i < n) out[i] = float_to_bf16(x[i]);
 }
 
 // ---------------------------------------------------------------------------
@@ -253,12 +267,20 @@ int mllm_reset_state(void* state, size_t slot_bytes, int n_slots, const int* slo
 }
 
 int mllm_embed(const int* ids, const int* pos, const void* wte, const void* wpe, float* x, int T, int D,
-               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale) {
+               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale, void* copy_bf16) {
     if (T <= 0) return 0;
+    bf16_t* copy = static_cast<bf16_t*>(copy_bf16);
     if (dtype == MLLM_F32)
-        embed_kernel<float><<<T, 256, 0, stream>>>(ids, pos, (const float*)wte, (const float*)wpe, x, D, src, prev, n_prev, scale);
+        embed_kernel<float><<<T, 256, 0, stream>>>(ids, pos, (const float*)wte, (const float*)wpe, x, D, src, prev, n_prev, scale, copy);
     else
-        embed_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, pos, (const bf16_t*)wte, (const bf16_t*)wpe, x, D, src, prev, n_prev, scale);
+        embed_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, pos, (const bf16_t*)wte, (const bf16_t*)wpe, x, D, src, prev, n_prev, scale, copy);
+    MLLM_LAUNCH_CHECK();
+    return 0;
+}
+
+int mllm_cast_bf16(const float* x, void* out, size_t n, hipStream_t stream) {
+    if (n == 0) return 0;
+    cast_bf16_kernel<<<static_cast<int>((n + 255) / 256), 256, 0, stream>>>(x, static_cast<bf16_t*>(out), n);
     MLLM_LAUNCH_CHECK();
     return 0;
 }

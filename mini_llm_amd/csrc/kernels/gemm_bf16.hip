@@ -46,7 +46,7 @@ __device__ __forceinline__ void store4(void* C, size_t idx, const float (&v)[4],
     float o[4];
 #pragma unroll
     for (int e = 0; e < 4; ++e)
-        o[e] = MODE == EPI_GELU_TANH ? gelu_tanh(v[e]) : MODE == EPI_GELU_ERF ? gelu_erf(v[e]) : v[e];
+        o[e] = MODE == EPI_GELU_TANH ? gelu_tanh(v[e]) : MODE == EPI_GELU_ERF ? gelu_erf(v[e]) : MODE == EPI_RELU2 ? relu2(v[e]) : v[e];
     if (MODE == EPI_ADD_RESIDUAL || MODE == EPI_STORE_F32) {
         float* c = static_cast<float*>(C) + idx;
         if (vec && n_left >= 4) {
@@ -353,7 +353,7 @@ static void launch_tiled(const bf16_t* a, int lda, const bf16_t* w, int ldw, con
 #define TILED(E, MD) gemm_bf16_mfma<WM, WN, TM, TN, BKP, DEPTH, E, MD, KG><<<grid, block, 0, stream>>>(a, lda, w, ldw, bias, C, ldc, M, N, K, tiles_m, tiles_n, xm, xn, kv)
 #define TILED_MODE(MD) case MD: if (edge) TILED(true, MD); else TILED(false, MD); break;
     switch (mode) {
-        TILED_MODE(EPI_STORE) TILED_MODE(EPI_GELU_TANH) TILED_MODE(EPI_GELU_ERF) TILED_MODE(EPI_ADD_RESIDUAL)
+        TILED_MODE(EPI_STORE) TILED_MODE(EPI_GELU_TANH) TILED_MODE(EPI_GELU_ERF) TILED_MODE(EPI_RELU2) TILED_MODE(EPI_ADD_RESIDUAL)
         default: if (edge) TILED(true, EPI_STORE_F32); else TILED(false, EPI_STORE_F32); break;
     }
 #undef TILED_MODE

@@ -12,7 +12,10 @@
 
 namespace {
 
-// Turn of the interleaved pair (u, v) at position p by the angle p * base^(-2i/dims); the angle in double.
+// Turn of the pair (u, v) number i at position p by the angle p * base^(-2i/dims); the angle in double. A pair's columns
+// are 2i and 2i + 1 (interleaved), or i and i + dims / 2 (half != 0).
+__device__ __forceinline__ int pair_first(int i, int half) { return half ? i : 2 * i; }
+__device__ __forceinline__ int pair_second(int i, int half, int dims) { return half ? i + dims / 2 : 2 * i + 1; }
 __device__ __forceinline__ void turn_pair(float u, float v, int pos, int i, double log2_base, int dims, float& a, float& b) {
     const double f = exp2(-2.0 * static_cast<double>(i) / static_cast<double>(dims) * log2_base);
     const double angle = static_cast<double>(pos) * f;
@@ -22,23 +25,27 @@ __device__ __forceinline__ void turn_pair(float u, float v, int pos, int i, doub
 }
 
 // One wavefront per token:
-//   cq[t]  = rmsnorm(dq[t]) * wq                                      (the query latent, activation dtype)
+//   cq[t]  = rmsnorm(dq[t]) * wq                                      (the query latent, activation dtype; dq may be null)
 //   page row slots[t] = [ c = rmsnorm(dkv[t, :R]) * wkv | turned dkv[t, R:R+Dr] ]   (if dkv is given and slot >= 0)
-// The first rot_dims of the Dr columns are turned in interleaved pairs, the rest pass unchanged.
+// The first rot_dims of the Dr columns are turned in pairs, the rest pass unchanged. The mean of c's squares runs over
+// Rn <= R columns (a latent widened with zero columns: the columns behind Rn are zero).
 template <typename T>
 __global__ void __launch_bounds__(64)
 latent_prepare_kernel(const float* __restrict__ dq, int ld_dq, int Rq, const float* __restrict__ wq, T* __restrict__ cq,
                       int ld_cq, const float* __restrict__ dkv, int ld_dkv, int R, int Dr, const float* __restrict__ wkv,
                       T* __restrict__ pages, T* __restrict__ vt_pages, int page_size, const int* __restrict__ slots,
-                      const int* __restrict__ positions, float eps, double log2_base, int rot_dims) {
+                      const int* __restrict__ positions, float eps, double log2_base, int rot_dims, int Rn, int half) {
     const int t = blockIdx.x, lane = threadIdx.x;
     // Up to 8 values a lane of each latent are requested up front, without conditions (a loop of unknown length
     // would wait for every load before it asks for the next); longer latents read the rest in a loop.
-    const float* qrow = dq + static_cast<size_t>(t) * ld_dq;
     const int slot = dkv ? slots[t] : -1;
     const bool fill = dkv != nullptr && slot >= 0;
+    if (dq == nullptr && !fill) return;
+    // (no latent to fill, or none of the query's: the loads below repeat the other's)
+    const float* qrow = dq ? dq + static_cast<size_t>(t) * ld_dq : dkv + static_cast<size_t>(t) * ld_dkv;
     const float* row = fill ? dkv + static_cast<size_t>(t) * ld_dkv : qrow;
-    const int Rk = fill ? R : Rq;                              // (no latent to fill: the loads below repeat the query's)
+    const int Rk = fill ? R : Rq;
+    if (dq == nullptr) { Rq = R; wq = wkv; }
     float qv[8], kv[8], qw[8], kw[8];
 #pragma unroll
     for (int u = 0; u < 8; ++u) {
@@ -48,7 +55,7 @@ latent_prepare_kernel(const float* __restrict__ dq, int ld_dq, int Rq, const flo
         kv[u] = row[ik];
         kw[u] = fill ? wkv[ik] : 0.f;
     }
-    {
+    if (dq != nullptr) {
         float ss = 0.f;
 #pragma unroll
         for (int u = 0; u < 8; ++u) if (lane + 64 * u < Rq) ss += qv[u] * qv[u];
@@ -65,7 +72,7 @@ latent_prepare_kernel(const float* __restrict__ dq, int ld_dq, int Rq, const flo
 #pragma unroll
     for (int u = 0; u < 8; ++u) if (lane + 64 * u < R) ss += kv[u] * kv[u];
     for (int i = lane + 512; i < R; i += 64) ss += row[i] * row[i];
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(R) + eps);
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(Rn) + eps);
     // (vt_pages, optional: the latent once more, transposed page by page, [page][R][page_size], which is the
     // operand shape of the matrix-core kernel's second product)
     T* vt = vt_pages ? vt_pages + static_cast<size_t>(slot / page_size) * page_size * R + slot % page_size : nullptr;
@@ -86,9 +93,10 @@ latent_prepare_kernel(const float* __restrict__ dq, int ld_dq, int Rq, const flo
     const int pos = positions[t];
     for (int i = lane; i < rot_dims / 2; i += 64) {
         float a, b;
-        turn_pair(row[R + 2 * i], row[R + 2 * i + 1], pos, i, log2_base, rot_dims, a, b);
-        o[R + 2 * i] = from_float<T>(a);
-        o[R + 2 * i + 1] = from_float<T>(b);
+        const int u = R + pair_first(i, half), v = R + pair_second(i, half, rot_dims);
+        turn_pair(row[u], row[v], pos, i, log2_base, rot_dims, a, b);
+        o[u] = from_float<T>(a);
+        o[v] = from_float<T>(b);
     }
     for (int i = rot_dims + lane; i < Dr; i += 64) o[R + i] = from_float<T>(row[R + i]);
 }
@@ -98,12 +106,13 @@ latent_prepare_kernel(const float* __restrict__ dq, int ld_dq, int Rq, const flo
 // For 8 tokens and one head a workgroup:
 //   qa[t, h, r] = sum_d q[t, h, d] * w_ukt[r, h*Dn + d]      (thread per r)
 //   qa[t, h, R + i] = the turned rotary part of q[t, h]
-// (Any dtype and sizes; bfloat16 at sizes in steps of 32 goes to head_linear_mfma_kernel.)
-template <typename T>
+// (Any dtype and sizes; bfloat16 at sizes in steps of 32 goes to head_linear_mfma_kernel. The queries may be fp32 rows
+// whatever T is: the input projection's own result.)
+template <typename TQ, typename T>
 __global__ void __launch_bounds__(256)
-latent_absorb_kernel(const T* __restrict__ q, int ldq, const T* __restrict__ w_uk, int ldw, T* __restrict__ qa, int ldqa,
+latent_absorb_kernel(const TQ* __restrict__ q, int ldq, const T* __restrict__ w_uk, int ldw, T* __restrict__ qa, int ldqa,
                      const int* __restrict__ positions, int n_tokens, int H, int Dn, int Dr, int R, double log2_base,
-                     int rot_dims) {
+                     int rot_dims, int half) {
     extern __shared__ float q_s[];                   // [8][Dn]
     const int h = blockIdx.y, t0 = blockIdx.z * 8, E = R + Dr;
     const int nt = min(8, n_tokens - t0);
@@ -128,18 +137,19 @@ latent_absorb_kernel(const T* __restrict__ q, int ldq, const T* __restrict__ w_u
         for (int i = threadIdx.x; i < nt * (Dr / 2 + Dr); i += 256) {
             // the first nt * rot_dims/2 indices turn pairs, the rest copy what is not turned
             const int tt = i / (Dr / 2 + Dr), k = i % (Dr / 2 + Dr);
-            const T* src = q + static_cast<size_t>(t0 + tt) * ldq + h * (Dn + Dr) + Dn;
+            const TQ* src = q + static_cast<size_t>(t0 + tt) * ldq + h * (Dn + Dr) + Dn;
             T* dst = qa + static_cast<size_t>(t0 + tt) * ldqa + h * E + R;
             if (k < Dr / 2) {
                 if (k < rot_dims / 2) {
                     float a, b;
-                    turn_pair(to_float(src[2 * k]), to_float(src[2 * k + 1]), positions[t0 + tt], k, log2_base, rot_dims, a, b);
-                    dst[2 * k] = from_float<T>(a);
-                    dst[2 * k + 1] = from_float<T>(b);
+                    const int u = pair_first(k, half), v = pair_second(k, half, rot_dims);
+                    turn_pair(to_float(src[u]), to_float(src[v]), positions[t0 + tt], k, log2_base, rot_dims, a, b);
+                    dst[u] = from_float<T>(a);
+                    dst[v] = from_float<T>(b);
                 }
             } else {
                 const int c = k - Dr / 2;
-                if (c >= rot_dims) dst[c] = src[c];
+                if (c >= rot_dims) dst[c] = from_float<T>(to_float(src[c]));
             }
         }
     }
@@ -160,16 +170,25 @@ union Frag8 {
 // columns). A workgroup takes 64 tokens, one head and 64 values of n; a wavefront 16 tokens: the weights are the
 // MFMA's A operand, so a lane ends up with four neighbouring n of one token. K is a multiple of 32; rows and head
 // offsets are 16-byte aligned. With `positions`, the workgroups of the first n tile also carry the `tail` columns
-// behind a head's K inputs over to behind its N outputs, the first rot_dims of them turned in interleaved pairs.
+// behind a head's K inputs over to behind its N outputs, the first rot_dims of them turned in pairs. With `gate` (fp32
+// rows of H columns) head h's result is multiplied by sigmoid(gate[t, h]). The inputs are bfloat16 or fp32 rows (TA),
+// which are rounded as they are loaded.
+__device__ __forceinline__ u32x4 operand8(const bf16_t* p) { return *reinterpret_cast<const u32x4*>(p); }
+__device__ __forceinline__ u32x4 operand8(const float* p) {
+    const float4 x = *reinterpret_cast<const float4*>(p), y = *reinterpret_cast<const float4*>(p + 4);
+    return u32x4{pack_bf16x2(x.x, x.y), pack_bf16x2(x.z, x.w), pack_bf16x2(y.x, y.y), pack_bf16x2(y.z, y.w)};
+}
+template <typename TA>
 __global__ void __launch_bounds__(256)
-head_linear_mfma_kernel(const bf16_t* __restrict__ a, int lda, int a_hs, const bf16_t* __restrict__ w, int ldw, int w_head_rows,
+head_linear_mfma_kernel(const TA* __restrict__ a, int lda, int a_hs, const bf16_t* __restrict__ w, int ldw, int w_head_rows,
                         int w_head_cols, bf16_t* __restrict__ out, int ldo, int out_hs, int n_tokens, int N, int K,
-                        const int* __restrict__ positions, int tail, int rot_dims, double log2_base) {
+                        const int* __restrict__ positions, int tail, int rot_dims, double log2_base, int half,
+                        const float* __restrict__ gate, int ldg) {
     const int lane = threadIdx.x % 64, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64);
     const int G = lane / 16, c16 = lane % 16;
     const int h = blockIdx.y, t0 = blockIdx.x * 64, n_base = blockIdx.z * 64;
     const int tok = min(t0 + 16 * wave + c16, n_tokens - 1);
-    const bf16_t* arow = a + static_cast<size_t>(tok) * lda + static_cast<size_t>(h) * a_hs + 8 * G;
+    const TA* arow = a + static_cast<size_t>(tok) * lda + static_cast<size_t>(h) * a_hs + 8 * G;
     const bf16_t* wbase = w + static_cast<size_t>(h) * w_head_rows * ldw + static_cast<size_t>(h) * w_head_cols + 8 * G;
     const bf16_t* wrow[4];
 #pragma unroll
@@ -179,7 +198,7 @@ head_linear_mfma_kernel(const bf16_t* __restrict__ a, int lda, int a_hs, const b
     for (int ct = 0; ct < 4; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int k = 0; k < K; k += 32) {
         Frag8 af, wf[4];
-        af.q = *reinterpret_cast<const u32x4*>(arow + k);
+        af.q = operand8(arow + k);
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) wf[ct].q = *reinterpret_cast<const u32x4*>(wrow[ct] + k);
 #pragma unroll
@@ -187,30 +206,32 @@ head_linear_mfma_kernel(const bf16_t* __restrict__ a, int lda, int a_hs, const b
     }
     if (t0 + 16 * wave + c16 < n_tokens) {
         bf16_t* orow = out + static_cast<size_t>(tok) * ldo + static_cast<size_t>(h) * out_hs;
+        const float g = gate != nullptr ? 1.f / (1.f + expf(-gate[static_cast<size_t>(tok) * ldg + h])) : 1.f;
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) {
             const int n = n_base + 16 * ct + 4 * G;            // acc[ct][r] is output n + r of this lane's token
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-                if (n + r < N) orow[n + r] = float_to_bf16(acc[ct][r]);
+                if (n + r < N) orow[n + r] = float_to_bf16(acc[ct][r] * g);
         }
     }
     if (positions != nullptr && blockIdx.z == 0) {
         const int nt = min(64, n_tokens - t0), per = tail / 2 + tail;
         for (int i = threadIdx.x; i < nt * per; i += 256) {
             const int tt = i / per, k = i % per;
-            const bf16_t* src = a + static_cast<size_t>(t0 + tt) * lda + static_cast<size_t>(h) * a_hs + K;
+            const TA* src = a + static_cast<size_t>(t0 + tt) * lda + static_cast<size_t>(h) * a_hs + K;
             bf16_t* dst = out + static_cast<size_t>(t0 + tt) * ldo + static_cast<size_t>(h) * out_hs + N;
             if (k < tail / 2) {
                 if (k < rot_dims / 2) {
                     float u, v;
-                    turn_pair(to_float(src[2 * k]), to_float(src[2 * k + 1]), positions[t0 + tt], k, log2_base, rot_dims, u, v);
-                    dst[2 * k] = float_to_bf16(u);
-                    dst[2 * k + 1] = float_to_bf16(v);
+                    const int first = pair_first(k, half), second = pair_second(k, half, rot_dims);
+                    turn_pair(to_float(src[first]), to_float(src[second]), positions[t0 + tt], k, log2_base, rot_dims, u, v);
+                    dst[first] = float_to_bf16(u);
+                    dst[second] = float_to_bf16(v);
                 }
             } else {
                 const int c = k - tail / 2;
-                if (c >= rot_dims) dst[c] = src[c];
+                if (c >= rot_dims) dst[c] = float_to_bf16(to_float(src[c]));
             }
         }
     }
@@ -312,12 +333,13 @@ latent_attention_kernel(const T* __restrict__ qa, int ldqa, const T* __restrict_
     }
 }
 
-// Per-head expansion of the attention result: out[t, h*Dv + e] = sum_r w_uv[h*Dv + e, r] * o_lat[t, h, r].
+// Per-head expansion of the attention result: out[t, h*Dv + e] = sum_r w_uv[h*Dv + e, r] * o_lat[t, h, r] (times
+// sigmoid(gate[t, h]) if a gate is given).
 // One wavefront per output column (lanes over r, coalesced weight reads), 8 tokens a pass.
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_expand_kernel(const T* __restrict__ o_lat, int ldo, const T* __restrict__ w_uv, int ldw, T* __restrict__ out, int ldout,
-                     int n_tokens, int H, int Dv, int R) {
+                     int n_tokens, int H, int Dv, int R, const float* __restrict__ gate, int ldg) {
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / MLLM_WAVE), lane = threadIdx.x % MLLM_WAVE;
     const int col = blockIdx.x * 4 + wave;
     if (col >= H * Dv) return;
@@ -336,7 +358,10 @@ latent_expand_kernel(const T* __restrict__ o_lat, int ldo, const T* __restrict__
 #pragma unroll
         for (int tt = 0; tt < 8; ++tt) {
             const float v = wave_sum(acc[tt]);
-            if (lane == 0 && t0 + tt < n_tokens) out[static_cast<size_t>(t0 + tt) * ldout + col] = from_float<T>(v);
+            if (lane == 0 && t0 + tt < n_tokens) {
+                const float g = gate != nullptr ? 1.f / (1.f + expf(-gate[static_cast<size_t>(t0 + tt) * ldg + h])) : 1.f;
+                out[static_cast<size_t>(t0 + tt) * ldout + col] = from_float<T>(v * g);
+            }
         }
     }
 }
@@ -584,50 +609,59 @@ constexpr int MAX_LDS = 160 * 1024;
 
 extern "C" {
 
-// See latent_prepare_kernel. dkv may be null (a layer that reads another layer's pages). -1: an odd rot_dims
-// or one beyond Dr.
+// See latent_prepare_kernel. dkv may be null (a layer that reads another layer's pages), and dq (queries without a latent
+// of their own). norm_cols: the columns of c that its norm's mean runs over (0: R). -1: an odd rot_dims or one beyond Dr.
 int mllm_latent_prepare(const float* dq, int ld_dq, int Rq, const float* wq, void* cq, int ld_cq, const float* dkv, int ld_dkv,
                         int R, int Dr, const float* wkv, void* pages, void* vt_pages, int page_size, const int* slots,
-                        const int* positions, int T, float eps, double base, int rot_dims, int dtype, hipStream_t stream) {
-    if (T <= 0) return 0;
+                        const int* positions, int T, float eps, double base, int rot_dims, int dtype, hipStream_t stream, int norm_cols,
+                        int half_split) {
+    if (T <= 0 || (dq == nullptr && dkv == nullptr)) return 0;
+    if (norm_cols < 0 || norm_cols > R) return -1;
+    const int Rn = norm_cols > 0 ? norm_cols : R;
     if (rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > Dr || !(base > 0) || (vt_pages != nullptr && page_size < 1)) return -1;
     const double l2 = log2(base);
     if (dtype == MLLM_F32)
         latent_prepare_kernel<float><<<T, 64, 0, stream>>>(dq, ld_dq, Rq, wq, static_cast<float*>(cq), ld_cq, dkv, ld_dkv, R, Dr, wkv,
                                                            static_cast<float*>(pages), static_cast<float*>(vt_pages), page_size, slots, positions,
-                                                           eps, l2, rot_dims);
+                                                           eps, l2, rot_dims, Rn, half_split);
     else
         latent_prepare_kernel<bf16_t><<<T, 64, 0, stream>>>(dq, ld_dq, Rq, wq, static_cast<bf16_t*>(cq), ld_cq, dkv, ld_dkv, R, Dr, wkv,
                                                             static_cast<bf16_t*>(pages), static_cast<bf16_t*>(vt_pages), page_size, slots, positions,
-                                                            eps, l2, rot_dims);
+                                                            eps, l2, rot_dims, Rn, half_split);
     MLLM_LAUNCH_CHECK();
     return 0;
 }
 
-// See latent_absorb_kernel; w_uk is the key expansion transposed, [R, H * Dn]. -1: rot_dims odd or beyond Dr, Dr
-// odd; -2: Dn too large for the LDS.
+// See latent_absorb_kernel; w_uk is the key expansion transposed, [R, H * Dn]; q in q_dtype (-1: dtype; fp32 otherwise).
+// -1: rot_dims odd or beyond Dr, Dr odd; -2: Dn too large for the LDS.
 int mllm_latent_absorb(const void* q, int ldq, const void* w_uk, int ldw, void* qa, int ldqa, const int* positions, int T, int H,
-                       int Dn, int Dr, int R, double base, int rot_dims, int dtype, hipStream_t stream) {
+                       int Dn, int Dr, int R, double base, int rot_dims, int dtype, hipStream_t stream, int q_dtype, int half_split) {
     if (T <= 0) return 0;
+    if (q_dtype < 0) q_dtype = dtype;
+    if (q_dtype != dtype && q_dtype != MLLM_F32) return -1;
     if (rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > Dr || Dr % 2 != 0 || !(base > 0)) return -1;
     const double l2 = log2(base);
     const auto aligned16 = [](const void* ptr) { return (reinterpret_cast<uintptr_t>(ptr) & 15) == 0; };
     if (dtype == MLLM_BF16 && Dn % 32 == 0 && ldq % 8 == 0 && (Dn + Dr) % 8 == 0 && ldw % 8 == 0 && aligned16(q) && aligned16(w_uk)) {
-        head_linear_mfma_kernel<<<dim3((T + 63) / 64, H, (R + 63) / 64), 256, 0, stream>>>(
-            static_cast<const bf16_t*>(q), ldq, Dn + Dr, static_cast<const bf16_t*>(w_uk), ldw, 0, Dn, static_cast<bf16_t*>(qa), ldqa, R + Dr,
-            T, R, Dn, positions, Dr, rot_dims, l2);
+#define ABSORB_MFMA(TQ)                                                                                                                \
+    head_linear_mfma_kernel<TQ><<<dim3((T + 63) / 64, H, (R + 63) / 64), 256, 0, stream>>>(                                               \
+        static_cast<const TQ*>(q), ldq, Dn + Dr, static_cast<const bf16_t*>(w_uk), ldw, 0, Dn, static_cast<bf16_t*>(qa), ldqa, R + Dr, T, R, \
+        Dn, positions, Dr, rot_dims, l2, half_split, nullptr, 0)
+        if (q_dtype == MLLM_F32) ABSORB_MFMA(float); else ABSORB_MFMA(bf16_t);
+#undef ABSORB_MFMA
         MLLM_LAUNCH_CHECK();
         return 0;
     }
     const size_t lds = static_cast<size_t>(8) * Dn * sizeof(float);
     if (lds > 64 * 1024) return -2;
     const dim3 grid((R + 255) / 256, H, (T + 7) / 8);
-    if (dtype == MLLM_F32)
-        latent_absorb_kernel<float><<<grid, 256, lds, stream>>>(static_cast<const float*>(q), ldq, static_cast<const float*>(w_uk), ldw,
-                                                                static_cast<float*>(qa), ldqa, positions, T, H, Dn, Dr, R, l2, rot_dims);
-    else
-        latent_absorb_kernel<bf16_t><<<grid, 256, lds, stream>>>(static_cast<const bf16_t*>(q), ldq, static_cast<const bf16_t*>(w_uk), ldw,
-                                                                 static_cast<bf16_t*>(qa), ldqa, positions, T, H, Dn, Dr, R, l2, rot_dims);
+#define ABSORB(TQ, TYPE)                                                                                                                \
+    latent_absorb_kernel<TQ, TYPE><<<grid, 256, lds, stream>>>(static_cast<const TQ*>(q), ldq, static_cast<const TYPE*>(w_uk), ldw,          \
+                                                               static_cast<TYPE*>(qa), ldqa, positions, T, H, Dn, Dr, R, l2, rot_dims, half_split)
+    if (dtype == MLLM_F32) ABSORB(float, float);
+    else if (q_dtype == MLLM_F32) ABSORB(float, bf16_t);
+    else ABSORB(bf16_t, bf16_t);
+#undef ABSORB
     MLLM_LAUNCH_CHECK();
     return 0;
 }
@@ -672,11 +706,21 @@ int mllm_latent_attention(const void* qa, int ldqa, const void* pages, const int
     return 0;
 }
 
+// The smallest sizes the matrix-core kernel is built for that hold a latent of R and a rotated part of Dr columns:
+// R rounded up to *R_out, the whole row to *E_out. -2: none.
+int mllm_latent_tile_shape(int R, int Dr, int* R_out, int* E_out) {
+    static const int shapes[][2] = {{96, 64}, {128, 64}, {128, 96}, {160, 128}, {192, 128}, {288, 256}, {320, 256}, {544, 512}, {576, 512}};
+    for (const auto& s : shapes)
+        if (R <= s[1] && Dr <= s[0] - s[1]) { *E_out = s[0]; *R_out = s[1]; return 0; }
+    return -2;
+}
+
 // The matrix-core kernel (see latent_prefill_kernel): qa [T*H, E] and o_lat [T*H, R] contiguous bfloat16.
 // nsplit > 1: every row's key tiles are shared by nsplit workgroups whose states meet in `partials`
 // (n_rows * nsplit * (R + 2) floats, n_rows = T*H) and are merged by a second kernel. single_tokens != 0: every
 // sequence brings exactly one token (n_tiles_upper is then n_seqs * ceil(H / 64)). n_tiles_upper: an upper bound of sum over sequences of ceil(q_len * H / 64). Returns -2 when the
-// sizes are not ones it is built for (E and R among (128, 96), (96, 64), (160, 128), (288, 256), (544, 512), (576, 512);
+// sizes are not ones it is built for (E and R among (96, 64), (128, 64), (128, 96), (160, 128), (192, 128), (288, 256),
+// (320, 256), (544, 512), (576, 512), see mllm_latent_tile_shape;
 // page sizes 8 to 64, powers of two; a block table that fits the LDS beside the tiles): the caller then runs
 // mllm_latent_attention.
 int mllm_latent_attention_tiles(const void* qa, const void* k_pages, const void* vt_pages, const int* block_tables,
@@ -714,29 +758,30 @@ int mllm_latent_attention_tiles(const void* qa, const void* k_pages, const void*
         }                                                                                                            \
         return 0;                                                                                                    \
     }
-    LP_CASE(4, 6) LP_CASE(3, 4) LP_CASE(5, 8) LP_CASE(9, 16) LP_CASE(17, 32) LP_CASE(18, 32)
+    LP_CASE(3, 4) LP_CASE(4, 4) LP_CASE(4, 6) LP_CASE(5, 8) LP_CASE(6, 8) LP_CASE(9, 16) LP_CASE(10, 16) LP_CASE(17, 32) LP_CASE(18, 32)
 #undef LP_CASE
     return -2;
 }
 
+// See latent_expand_kernel; gate (optional): fp32 rows of H columns, row stride ldg.
 int mllm_latent_expand(const void* o_lat, int ldo, const void* w_uv, int ldw, void* out, int ldout, int T, int H, int Dv, int R,
-                       int dtype, hipStream_t stream) {
+                       int dtype, hipStream_t stream, const float* gate, int ldg) {
     if (T <= 0) return 0;
     if (dtype == MLLM_BF16 && R % 32 == 0 && ldo % 8 == 0 && ldw % 8 == 0 && (reinterpret_cast<uintptr_t>(o_lat) & 15) == 0 &&
         (reinterpret_cast<uintptr_t>(w_uv) & 15) == 0) {
-        head_linear_mfma_kernel<<<dim3((T + 63) / 64, H, (Dv + 63) / 64), 256, 0, stream>>>(
+        head_linear_mfma_kernel<bf16_t><<<dim3((T + 63) / 64, H, (Dv + 63) / 64), 256, 0, stream>>>(
             static_cast<const bf16_t*>(o_lat), ldo, R, static_cast<const bf16_t*>(w_uv), ldw, Dv, 0, static_cast<bf16_t*>(out), ldout, Dv, T, Dv,
-            R, nullptr, 0, 0, 0.0);
+            R, nullptr, 0, 0, 0.0, 0, gate, ldg);
         MLLM_LAUNCH_CHECK();
         return 0;
     }
     const dim3 grid((H * Dv + 3) / 4, std::min((T + 7) / 8, 64));
     if (dtype == MLLM_F32)
         latent_expand_kernel<float><<<grid, 256, 0, stream>>>(static_cast<const float*>(o_lat), ldo, static_cast<const float*>(w_uv), ldw,
-                                                              static_cast<float*>(out), ldout, T, H, Dv, R);
+                                                              static_cast<float*>(out), ldout, T, H, Dv, R, gate, ldg);
     else
         latent_expand_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(o_lat), ldo, static_cast<const bf16_t*>(w_uv), ldw,
-                                                               static_cast<bf16_t*>(out), ldout, T, H, Dv, R);
+                                                               static_cast<bf16_t*>(out), ldout, T, H, Dv, R, gate, ldg);
     MLLM_LAUNCH_CHECK();
     return 0;
 }

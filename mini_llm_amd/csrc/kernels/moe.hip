@@ -3,9 +3,10 @@
 // with fp32 results.
 //
 // The experts' first products are one joined product (rows [expert 0 | expert 1 | ... | shared expert]); the
-// activation kernel squares the rectified values and multiplies every expert's block by the token's weight for that
-// expert (zero for an expert that was not chosen, one for the shared expert), so that the experts' second products are
+// activation kernel applies the activation (squared rectified values, or the exact GELU) and multiplies every expert's
+// block by the token's weight for that expert (zero for an expert that was not chosen, one for the shared expert), so that the experts' second products are
 // one joined product as well: sum_e w_e W_down,e a_e = [W_down,0 | W_down,1 | ...] [w_0 a_0; w_1 a_1; ...].
+// Experts that hand on their input (the identity, times the weight) have no rows; the kernel adds them up by itself.
 // A second kernel serves experts that are gated and clamped, chosen by sigmoid or softmax scores, whose weight may
 // stand on the expert's input, beside a shared expert that a sigmoid of the input scales.
 #include "common.h"
@@ -117,24 +118,51 @@ moe_glu_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ 
 }
 
 // One workgroup per token: the weights from the token's logits, then
-// out[t, e * ff + j] = weight_e * relu(up[t, e * ff + j])^2 for the E experts, and behind them
-// out[t, E * ff + j] = relu(up[t, E * ff + j])^2 for the shared expert's columns (N columns in all).
+// out[t, e * ff + j] = weight_e * act(up[t, e * ff + j]) for the E experts, and behind them
+// out[t, E * ff + j] = act(up[t, E * ff + j]) for the shared expert's columns (N columns in all); act is relu(z)^2, or
+// with GELU the exact GELU. With `correction` (E + identity numbers) the experts with the largest score + correction are
+// chosen, and the score alone is the weight. The last `identity` of the router's outputs are experts that hand on their
+// input: y[t, :] = (the sum of their weights) * h[t, :] (D columns; added to y with y_add).
 // VEC: eight columns a thread at a time (16-byte loads of bfloat16, two of float; ff, N and the strides are then
-// multiples of 8 and the rows aligned). `weights_out` (optional, [T, E]) receives the weights.
-template <typename T, bool VEC>
+// multiples of 8 and the rows aligned). `weights_out` (optional, [T, E + identity]) receives the weights.
+struct MoeChoice {
+    const float* correction;
+    int identity;
+    const void* h;           // [T, ldh], the output's dtype
+    int ldh, D, ldy, y_add;
+    float* y;                // [T, ldy] fp32
+};
+
+template <typename TI, typename T, bool VEC, bool GELU>
 __global__ void __launch_bounds__(256)
-moe_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int N, int top, float scale,
-               T* __restrict__ out, int ldo, float* __restrict__ weights_out, int ldw) {
-    __shared__ float z[MOE_MAX_EXPERTS], wgt[MOE_MAX_EXPERTS];
-    const int t = blockIdx.x, tid = threadIdx.x;
-    if (tid < E) z[tid] = logits[static_cast<size_t>(t) * ldl + tid];
+moe_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int N, int top, float scale,
+               T* __restrict__ out, int ldo, float* __restrict__ weights_out, int ldw, MoeChoice mc) {
+    __shared__ float z[MOE_MAX_EXPERTS], wgt[MOE_MAX_EXPERTS], choice[MOE_MAX_EXPERTS];
+    const int t = blockIdx.x, tid = threadIdx.x, all = E + mc.identity;
+    if (tid < all) z[tid] = logits[static_cast<size_t>(t) * ldl + tid];
     __syncthreads();
-    if (tid < E) {
-        expert_weight(z, wgt, E, top, scale, tid);
-        if (weights_out != nullptr) weights_out[static_cast<size_t>(t) * ldw + tid] = wgt[tid];
+    if (mc.correction == nullptr) {
+        if (tid < all) expert_weight(z, wgt, all, top, scale, tid);
+    } else {
+        float score = 0.f;
+        if (tid < all) {
+            float m = -INFINITY, sum = 0.f;
+            for (int o = 0; o < all; ++o) m = fmaxf(m, z[o]);
+            for (int o = 0; o < all; ++o) sum += expf(z[o] - m);
+            score = expf(z[tid] - m) / sum;
+            choice[tid] = score + mc.correction[tid];
+        }
+        __syncthreads();
+        if (tid < all) {
+            const float mine = choice[tid];
+            int before = 0;
+            for (int o = 0; o < all; ++o) before += (choice[o] > mine || (choice[o] == mine && o < tid)) ? 1 : 0;
+            wgt[tid] = before < top ? scale * score : 0.f;
+        }
     }
     __syncthreads();
-    const T* ur = up + static_cast<size_t>(t) * ldu;
+    if (weights_out != nullptr && tid < all) weights_out[static_cast<size_t>(t) * ldw + tid] = wgt[tid];
+    const TI* ur = up + static_cast<size_t>(t) * ldu;
     T* orow = out + static_cast<size_t>(t) * ldo;
     if (VEC) {
         for (int c = tid * 8; c < N; c += 256 * 8) {
@@ -142,8 +170,14 @@ moe_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ logi
             load8(ur + c, v);
             const int e = c / ff;                       // (ff is a multiple of 8: the eight columns are one expert's)
             const float wt = e < E ? wgt[e] : 1.f;
+            if (GELU) {
+                // (no work for an expert that was not chosen: erf costs more than the rest of the kernel)
 #pragma unroll
-            for (int u = 0; u < 8; ++u) { const float r = fmaxf(v[u], 0.f); v[u] = wt * (r * r); }
+                for (int u = 0; u < 8; ++u) v[u] = wt != 0.f ? wt * gelu_erf(v[u]) : 0.f;
+            } else {
+#pragma unroll
+                for (int u = 0; u < 8; ++u) v[u] = wt * relu2(v[u]);
+            }
             if (sizeof(T) == 2) {
                 uint4 pk;
                 pk.x = pack_bf16x2(v[0], v[1]); pk.y = pack_bf16x2(v[2], v[3]); pk.z = pack_bf16x2(v[4], v[5]); pk.w = pack_bf16x2(v[6], v[7]);
@@ -157,9 +191,16 @@ moe_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ logi
         for (int c = tid; c < N; c += 256) {
             const int e = c / ff;
             const float wt = e < E ? wgt[e] : 1.f;
-            const float r = fmaxf(to_float(ur[c]), 0.f);
-            orow[c] = from_float<T>(wt * (r * r));
+            const float v = to_float(ur[c]);
+            orow[c] = from_float<T>(wt * (GELU ? gelu_erf(v) : relu2(v)));
         }
+    }
+    if (mc.identity > 0) {
+        float w = 0.f;
+        for (int o = E; o < all; ++o) w += wgt[o];
+        const T* hr = static_cast<const T*>(mc.h) + static_cast<size_t>(t) * mc.ldh;
+        float* yr = mc.y + static_cast<size_t>(t) * mc.ldy;
+        for (int c = tid; c < mc.D; c += 256) yr[c] = (mc.y_add ? yr[c] : 0.f) + w * to_float(hr[c]);
     }
 }
 
@@ -167,21 +208,35 @@ moe_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ logi
 
 extern "C" {
 
-// up and out [T, E * ff + shared_ff] in `dtype` (out may be up); logits [T, E] fp32 (row stride ldl); weights_out
-// (optional) [T, E] fp32. -1: more experts than the kernel holds, or a `top` outside 1..E.
+// up [T, E * ff + shared_ff] in up_dtype and out of its shape in `dtype` (out may be up if the dtypes are one; otherwise up is
+// fp32); logits [T, E + identity] fp32 (row stride ldl); weights_out (optional) [T, E + identity] fp32. gelu != 0: the exact
+// GELU in place of the squared rectified value; correction (optional, [E + identity]), identity, h, y: see the kernel.
+// -1: more experts than the kernel holds, or a `top` outside 1..E + identity, or identity experts without h and y.
 int mllm_moe_act(const void* up, int ldu, const float* logits, int ldl, int E, int ff, int shared_ff, int top, float scale, void* out, int ldo,
-                 float* weights_out, int ldw, int T, int dtype, hipStream_t stream) {
+                 float* weights_out, int ldw, int T, int dtype, hipStream_t stream, int up_dtype, int gelu, const float* correction,
+                 int identity, const void* h, int ldh, int D, float* y, int ldy, int y_add) {
     if (T <= 0) return 0;
-    if (E < 1 || E > MOE_MAX_EXPERTS || top < 1 || top > E || ff < 1 || shared_ff < 0 || logits == nullptr) return -1;
+    if (up_dtype < 0) up_dtype = dtype;
+    if (E < 1 || identity < 0 || E + identity > MOE_MAX_EXPERTS || top < 1 || top > E + identity || ff < 1 || shared_ff < 0 || logits == nullptr) return -1;
+    if (identity > 0 && (h == nullptr || y == nullptr || D < 1)) return -1;
+    if (up_dtype != dtype && !(up_dtype == MLLM_F32 && up != out)) return -1;
     const int N = E * ff + shared_ff;
-    const int esz = dtype == MLLM_F32 ? 4 : 2;
-    const bool vec = ff % 8 == 0 && N % 8 == 0 && ldu % 8 == 0 && ldo % 8 == 0 &&
-                     ((reinterpret_cast<uintptr_t>(up) | reinterpret_cast<uintptr_t>(out)) & 15) == 0 && (static_cast<size_t>(ldu) * esz) % 16 == 0;
-#define MOE_ACT(TYPE, VEC)                                                                                                          \
-    moe_act_kernel<TYPE, VEC><<<T, 256, 0, stream>>>(static_cast<const TYPE*>(up), ldu, logits, ldl, E, ff, N, top, scale,           \
-                                                     static_cast<TYPE*>(out), ldo, weights_out, ldw)
-    if (dtype == MLLM_F32) { if (vec) MOE_ACT(float, true); else MOE_ACT(float, false); }
-    else { if (vec) MOE_ACT(bf16_t, true); else MOE_ACT(bf16_t, false); }
+    const int esz = dtype == MLLM_F32 ? 4 : 2, isz = up_dtype == MLLM_F32 ? 4 : 2;
+    const bool vec = ff % 8 == 0 && N % 8 == 0 && ldo % 8 == 0 && ((reinterpret_cast<uintptr_t>(up) | reinterpret_cast<uintptr_t>(out)) & 15) == 0 &&
+                     (static_cast<size_t>(ldu) * isz) % 16 == 0 && (static_cast<size_t>(ldo) * esz) % 16 == 0;
+    const MoeChoice mc{correction, identity, h, ldh, D, ldy, y_add, y};
+#define MOE_ACT(TI, TYPE, VEC, GELU)                                                                                                \
+    moe_act_kernel<TI, TYPE, VEC, GELU><<<T, 256, 0, stream>>>(static_cast<const TI*>(up), ldu, logits, ldl, E, ff, N, top, scale,   \
+                                                               static_cast<TYPE*>(out), ldo, weights_out, ldw, mc)
+#define MOE_ACT_G(TI, TYPE)                                                                                                         \
+    do {                                                                                                                            \
+        if (gelu) { if (vec) MOE_ACT(TI, TYPE, true, true); else MOE_ACT(TI, TYPE, false, true); }                                  \
+        else { if (vec) MOE_ACT(TI, TYPE, true, false); else MOE_ACT(TI, TYPE, false, false); }                                     \
+    } while (0)
+    if (dtype == MLLM_F32) MOE_ACT_G(float, float);
+    else if (up_dtype == MLLM_F32) MOE_ACT_G(float, bf16_t);
+    else MOE_ACT_G(bf16_t, bf16_t);
+#undef MOE_ACT_G
 #undef MOE_ACT
     MLLM_LAUNCH_CHECK();
     return 0;

@@ -1,4 +1,4 @@
-// RMS norms (plain, grouped, gated), the normed and scaled residual add, the clamped gated activation
+// RMS norms (plain, grouped, gated), the normed (RMS or layer norm) and scaled residual add, the clamped gated activation
 // and a fill, for gfx950. Statistics and sums are fp32 whatever the activation dtype.
 #include <algorithm>
 
@@ -63,10 +63,10 @@ rmsnorm_kernel(const float* __restrict__ x, int ldx, const int* __restrict__ row
 }
 
 
-// One wavefront per (row, group): y[r, g*Dg + i] = v_i / sqrt(mean_i(v_i^2) + eps) * w[g*Dg + i] * silu(gate[r, g*Dg + i]),
-// the gate BEHIND the norm (w may be null: no weight). v is the sum of `parts` arrays part_stride floats apart, added
+// One wavefront per (row, group): y[r, g*Dg + i] = v_i / sqrt(mean_i(v_i^2) + eps) * w[g*Dg + i] * silu(gate[r, g*Dg + i])
+// (PLAIN_SIGMOID: sigmoid(gate) instead of silu), the gate BEHIND the norm (w may be null: no weight). v is the sum of `parts` arrays part_stride floats apart, added
 // in the order of their index. The heads of a linear-attention mixer, normed one by one and gated.
-template <typename OutT, int WAVES>
+template <typename OutT, int WAVES, bool PLAIN_SIGMOID>
 __global__ void __launch_bounds__(64 * WAVES)
 rmsnorm_gate_after_kernel(const float* __restrict__ x, int ldx, const float* __restrict__ w, const float* __restrict__ gate, int ldg,
                           OutT* __restrict__ y, int ldy, int n, int D, int groups, float eps, int parts, size_t part_stride) {
@@ -99,13 +99,13 @@ rmsnorm_gate_after_kernel(const float* __restrict__ x, int ldx, const float* __r
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
         const int i = lane + 64 * u;
-        if (i < Dg) yr[i] = from_float<OutT>(v[u] * inv * ww[u] * (z[u] * sigmoid_precise(z[u])));
+        if (i < Dg) yr[i] = from_float<OutT>(v[u] * inv * ww[u] * ((PLAIN_SIGMOID ? 1.f : z[u]) * sigmoid_precise(z[u])));
     }
     for (int i = lane + 256; i < Dg; i += 64) {
         float a = xr[i];
         for (int part = 1; part < parts; ++part) a += xr[part * part_stride + i];
         const float zz = gr[i];
-        yr[i] = from_float<OutT>(a * inv * (w ? w[g * Dg + i] : 1.f) * (zz * sigmoid_precise(zz)));
+        yr[i] = from_float<OutT>(a * inv * (w ? w[g * Dg + i] : 1.f) * ((PLAIN_SIGMOID ? 1.f : zz) * sigmoid_precise(zz)));
     }
 }
 
@@ -115,41 +115,51 @@ __global__ void softcap_kernel(float* __restrict__ x, float cap, size_t n) {
     if (i < n) x[i] = cap * tanhf(x[i] / cap);
 }
 
-// x[r, i] += mult * scale[i] * (y[r, i] / sqrt(mean(y[r]^2) + eps) * w[i]); one wavefront per row.
-// With `clear` the row of y is set to zero behind the read, ready to collect the next sub-layer's output.
-template <int WAVES>
+// x[r, i] += mult * scale[i] * (y[r, i] / sqrt(mean(y[r]^2) + eps) * w[i]); one wavefront per row. CENTER: a layer norm, the
+// row's mean is taken off first (beta[i] is added behind the weight if there is one).
+// With `clear` the row of y is set to zero behind the read, ready to collect the next sub-layer's output. With `copy` the
+// new row of x is stored there once more in bfloat16 (what the next sub-layer reads).
+template <int WAVES, bool CENTER>
 __global__ void __launch_bounds__(64 * WAVES)
-rmsnorm_add_kernel(float* __restrict__ y, const float* __restrict__ w, const float* __restrict__ scale, float mult,
-                   float eps, float* __restrict__ x, int n, int D, int clear) {
+rmsnorm_add_kernel(float* __restrict__ y, const float* __restrict__ w, const float* __restrict__ beta, const float* __restrict__ scale,
+                   float mult, float eps, float* __restrict__ x, int n, int D, int clear, bf16_t* __restrict__ copy) {
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / MLLM_WAVE), lane = threadIdx.x % MLLM_WAVE;
     const int r = blockIdx.x * WAVES + wave;
     if (r >= n) return;
     float* yr = y + static_cast<size_t>(r) * D;
     float* xr = x + static_cast<size_t>(r) * D;
     float v[8];
-    float ss = 0.f;
+    float mean = 0.f;
 #pragma unroll
     for (int u = 0; u < 8; ++u) {
         const int i = lane + 64 * u;
         v[u] = i < D ? yr[i] : 0.f;
-        ss += v[u] * v[u];
+        if (CENTER) mean += v[u];
     }
-    for (int i = lane + 512; i < D; i += 64) ss += yr[i] * yr[i];
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(D) + eps);
+    if (CENTER) {
+        for (int i = lane + 512; i < D; i += 64) mean += yr[i];
+        mean = wave_sum(mean) / static_cast<float>(D);
+    }
+    float ss = 0.f;
 #pragma unroll
     for (int u = 0; u < 8; ++u) {
-        const int i = lane + 64 * u;
-        if (i < D) {
-            const float s = scale ? scale[i] * mult : mult;
-            xr[i] += s * (v[u] * inv * w[i]);
-            if (clear) yr[i] = 0.f;
-        }
+        if (lane + 64 * u < D) { const float a = v[u] - mean; ss += a * a; }
     }
-    for (int i = lane + 512; i < D; i += 64) {
+    for (int i = lane + 512; i < D; i += 64) { const float a = yr[i] - mean; ss += a * a; }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(D) + eps);
+    auto finish = [&](int i, float a) {
         const float s = scale ? scale[i] * mult : mult;
-        xr[i] += s * (yr[i] * inv * w[i]);
+        float o = (a - mean) * inv * w[i];
+        if (CENTER && beta) o += beta[i];
+        const float now = xr[i] + s * o;
+        xr[i] = now;
+        if (copy) copy[static_cast<size_t>(r) * D + i] = float_to_bf16(now);
         if (clear) yr[i] = 0.f;
-    }
+    };
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+        if (lane + 64 * u < D) finish(lane + 64 * u, v[u]);
+    for (int i = lane + 512; i < D; i += 64) finish(i, yr[i]);
 }
 
 // Many short groups (heads of a recurrence: 16 to 128 columns each): LANES = columns / 4 lanes take one (row, group)
@@ -320,10 +330,10 @@ rmsnorm_vec_kernel(const float* __restrict__ x, int ldx, const int* __restrict__
     }
 }
 
-template <int WAVES>
+template <int WAVES, bool CENTER>
 __global__ void __launch_bounds__(64 * WAVES)
-rmsnorm_add_vec_kernel(float* __restrict__ y, const float* __restrict__ w, const float* __restrict__ scale, float mult,
-                       float eps, float* __restrict__ x, int n, int D, int clear) {
+rmsnorm_add_vec_kernel(float* __restrict__ y, const float* __restrict__ w, const float* __restrict__ beta, const float* __restrict__ scale,
+                       float mult, float eps, float* __restrict__ x, int n, int D, int clear, bf16_t* __restrict__ copy) {
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / MLLM_WAVE), lane = threadIdx.x % MLLM_WAVE;
     const int r = blockIdx.x * WAVES + wave;
     if (r >= n) return;
@@ -331,8 +341,9 @@ rmsnorm_add_vec_kernel(float* __restrict__ y, const float* __restrict__ w, const
     float4* xr = reinterpret_cast<float4*>(x + static_cast<size_t>(r) * D);
     const float4* wr = reinterpret_cast<const float4*>(w);
     const float4* sr = reinterpret_cast<const float4*>(scale ? scale : w);
+    const float4* br = reinterpret_cast<const float4*>(CENTER && beta ? beta : w);
     const int nq = D / 4, n_u = (nq + 63) / 64;
-    float4 v[8], xx[8], ww[8], sc[8];
+    float4 v[8], xx[8], ww[8], sc[8], bb[8];
 #pragma unroll
     for (int u = 0; u < 8; ++u)
         if (u < n_u) v[u] = yr[min(lane + 64 * u, nq - 1)];
@@ -343,7 +354,18 @@ rmsnorm_add_vec_kernel(float* __restrict__ y, const float* __restrict__ w, const
             xx[u] = xr[i];
             ww[u] = wr[i];
             sc[u] = sr[i];
+            if (CENTER) bb[u] = br[i];
         }
+    if (CENTER) {
+        float sum = 0.f;
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            if (u < n_u && lane + 64 * u < nq) sum += (v[u].x + v[u].y) + (v[u].z + v[u].w);
+        const float mean = wave_sum(sum) / static_cast<float>(D);
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            if (u < n_u) { v[u].x -= mean; v[u].y -= mean; v[u].z -= mean; v[u].w -= mean; }
+    }
     float ss = 0.f;
 #pragma unroll
     for (int u = 0; u < 8; ++u)
@@ -354,8 +376,16 @@ rmsnorm_add_vec_kernel(float* __restrict__ y, const float* __restrict__ w, const
         const int i = lane + 64 * u;
         if (u < n_u && i < nq) {
             const float4 s4 = scale ? make_float4(sc[u].x * mult, sc[u].y * mult, sc[u].z * mult, sc[u].w * mult) : make_float4(mult, mult, mult, mult);
-            xr[i] = make_float4(xx[u].x + s4.x * (v[u].x * inv * ww[u].x), xx[u].y + s4.y * (v[u].y * inv * ww[u].y),
-                                xx[u].z + s4.z * (v[u].z * inv * ww[u].z), xx[u].w + s4.w * (v[u].w * inv * ww[u].w));
+            float4 o = make_float4(v[u].x * inv * ww[u].x, v[u].y * inv * ww[u].y, v[u].z * inv * ww[u].z, v[u].w * inv * ww[u].w);
+            if (CENTER && beta) { o.x += bb[u].x; o.y += bb[u].y; o.z += bb[u].z; o.w += bb[u].w; }
+            const float4 now = make_float4(xx[u].x + s4.x * o.x, xx[u].y + s4.y * o.y, xx[u].z + s4.z * o.z, xx[u].w + s4.w * o.w);
+            xr[i] = now;
+            if (copy) {
+                uint2 pk;
+                pk.x = pack_bf16x2(now.x, now.y);
+                pk.y = pack_bf16x2(now.z, now.w);
+                *reinterpret_cast<uint2*>(copy + static_cast<size_t>(r) * D + 4 * i) = pk;
+            }
             if (clear) yr[i] = make_float4(0.f, 0.f, 0.f, 0.f);
         }
     }
@@ -429,19 +459,19 @@ int mllm_rmsnorm(const float* x, int ldx, const int* rows, const float* w, const
     return 0;
 }
 
-// y = rmsnorm(x) * w * silu(gate) in `groups` equal parts of the D columns, the gate behind the norm; w ([D]) may be
-// null. x and gate fp32 with row strides ldx / ldg; with parts > 1, x is the sum of `parts` arrays part_stride floats
+// y = rmsnorm(x) * w * silu(gate) (plain_sigmoid != 0: * sigmoid(gate)) in `groups` equal parts of the D columns, the gate
+// behind the norm; w ([D]) may be null. x and gate fp32 with row strides ldx / ldg; with parts > 1, x is the sum of `parts` arrays part_stride floats
 // apart. -1: D is no multiple of groups.
 int mllm_rmsnorm_gate_after(const float* x, int ldx, const float* w, const float* gate, int ldg, void* y, int ldy, int n, int D, int groups,
-                            float eps, int out_dtype, int parts, size_t part_stride, hipStream_t stream) {
+                            float eps, int out_dtype, int parts, size_t part_stride, hipStream_t stream, int plain_sigmoid) {
     if (n <= 0 || D <= 0) return 0;
     if (groups < 1 || D % groups != 0 || parts < 1 || gate == nullptr) return -1;
     const long long pairs = static_cast<long long>(n) * groups;
     const int blocks = static_cast<int>((pairs + 3) / 4);
-    if (out_dtype == MLLM_F32)
-        rmsnorm_gate_after_kernel<float, 4><<<blocks, 256, 0, stream>>>(x, ldx, w, gate, ldg, static_cast<float*>(y), ldy, n, D, groups, eps, parts, part_stride);
-    else
-        rmsnorm_gate_after_kernel<bf16_t, 4><<<blocks, 256, 0, stream>>>(x, ldx, w, gate, ldg, static_cast<bf16_t*>(y), ldy, n, D, groups, eps, parts, part_stride);
+#define RGA(TYPE, PLAIN) rmsnorm_gate_after_kernel<TYPE, 4, PLAIN><<<blocks, 256, 0, stream>>>(x, ldx, w, gate, ldg, static_cast<TYPE*>(y), ldy, n, D, groups, eps, parts, part_stride)
+    if (out_dtype == MLLM_F32) { if (plain_sigmoid) RGA(float, true); else RGA(float, false); }
+    else { if (plain_sigmoid) RGA(bf16_t, true); else RGA(bf16_t, false); }
+#undef RGA
     MLLM_LAUNCH_CHECK();
     return 0;
 }
@@ -455,15 +485,24 @@ int mllm_softcap(float* x, size_t n, float cap, hipStream_t stream) {
     return 0;
 }
 
-int mllm_rmsnorm_add(float* y, const float* w, const float* scale, float mult, float eps, float* x, int n, int D,
-                     int clear, hipStream_t stream) {
+// x += mult * scale * norm(y); center != 0: a layer norm (beta may be null), otherwise an RMS norm. copy_bf16 (optional, [n, D]):
+// the new x in bfloat16.
+int mllm_norm_add(float* y, const float* w, const float* beta, const float* scale, float mult, float eps, float* x, int n, int D,
+                  int clear, int center, void* copy_bf16, hipStream_t stream) {
     if (n <= 0 || D <= 0) return 0;
+    bf16_t* copy = static_cast<bf16_t*>(copy_bf16);
     const bool vec = D % 4 == 0 && D <= 2048 &&
                      ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(scale) |
-                       reinterpret_cast<uintptr_t>(y)) & 15) == 0;
-    if (vec && n >= 512) rmsnorm_add_vec_kernel<8><<<(n + 7) / 8, 512, 0, stream>>>(y, w, scale, mult, eps, x, n, D, clear);
-    else if (vec) rmsnorm_add_vec_kernel<4><<<(n + 3) / 4, 256, 0, stream>>>(y, w, scale, mult, eps, x, n, D, clear);
-    else rmsnorm_add_kernel<4><<<(n + 3) / 4, 256, 0, stream>>>(y, w, scale, mult, eps, x, n, D, clear);
+                       reinterpret_cast<uintptr_t>(beta) | reinterpret_cast<uintptr_t>(copy) | reinterpret_cast<uintptr_t>(y)) & 15) == 0;
+#define NORM_ADD(KERNEL, WAVES)                                                                                                             \
+    do {                                                                                                                                    \
+        if (center) KERNEL<WAVES, true><<<(n + WAVES - 1) / WAVES, 64 * WAVES, 0, stream>>>(y, w, beta, scale, mult, eps, x, n, D, clear, copy); \
+        else KERNEL<WAVES, false><<<(n + WAVES - 1) / WAVES, 64 * WAVES, 0, stream>>>(y, w, beta, scale, mult, eps, x, n, D, clear, copy);   \
+    } while (0)
+    if (vec && n >= 512) NORM_ADD(rmsnorm_add_vec_kernel, 8);
+    else if (vec) NORM_ADD(rmsnorm_add_vec_kernel, 4);
+    else NORM_ADD(rmsnorm_add_kernel, 4);
+#undef NORM_ADD
     MLLM_LAUNCH_CHECK();
     return 0;
 }
