@@ -178,37 +178,39 @@ def feed_forward(h, w, pre, mlp):
 MIXERS = {"mlstm": mlstm_mixer, "latent_attention": latent_attention_mixer}
 
 
-def mixed(x, w, i, lc, cfg):
-    """The stream behind layer i's mixer."""
+def mixed(x, w, i, lc, cfg, seen=lambda x: x):
+    """The stream behind layer i's mixer. `seen`: what a sub-layer sees of the stream (the stream itself; a test may disturb
+    it to learn how much a position's logits move)."""
     eps, L = cfg["norm"]["eps"], "l%d." % i
-    return x + layer_norm(MIXERS[lc["type"]](x, w, L + "mix.", lc["mixer"], eps), w[L + "norm1"], eps)
+    return x + layer_norm(MIXERS[lc["type"]](seen(x), w, L + "mix.", lc["mixer"], eps), w[L + "norm1"], eps)
 
 
-def layer(x, w, i, lc, cfg):
-    x = mixed(x, w, i, lc, cfg)
+def layer(x, w, i, lc, cfg, seen=lambda x: x):
+    x = mixed(x, w, i, lc, cfg, seen)
     if lc.get("mlp") is not None:
-        x = x + layer_norm(feed_forward(x, w, "l%d.mlp." % i, lc["mlp"]), w["l%d.norm2" % i], cfg["norm"]["eps"])
+        x = x + layer_norm(feed_forward(seen(x), w, "l%d.mlp." % i, lc["mlp"]), w["l%d.norm2" % i], cfg["norm"]["eps"])
     return x
 
 
-def streams(cfg, w, tokens: List[int]):
+def streams(cfg, w, tokens: List[int], seen=lambda x: x):
     """The residual stream behind every layer, [layers, T, D]."""
     x = w["embed"][torch.tensor(tokens)]
     out = []
     for i, lc in enumerate(cfg["layers"]):
-        x = layer(x, w, i, lc, cfg)
+        x = layer(x, w, i, lc, cfg, seen)
         out.append(x)
     return torch.stack(out)
 
 
-def logits(cfg, w, tokens: List[int]):
-    x = streams(cfg, w, tokens)[-1]
+def logits(cfg, w, tokens: List[int], seen=lambda x: x):
+    x = streams(cfg, w, tokens, seen)[-1]
     return layer_norm(x, w["final.norm"], cfg["norm"]["eps"]) @ w["head"].T * cfg.get("logit_scale", 1.0)
 
 
-def closest_call(cfg, w, tokens: List[int]):
+def closest_call(cfg, w, tokens: List[int], slight: float = 0.01):
     """Per token the smallest gap between the last chosen and the first rejected choice score over all routed layers
-    (a tiny gap means rounding may choose another expert there)."""
+    (a tiny gap means rounding may choose another expert there); a call between two experts whose weights would both
+    stay below `slight` does not count."""
     x = w["embed"][torch.tensor(tokens)]
     gap = torch.full((len(tokens),), math.inf, dtype=torch.float64)
     for i, lc in enumerate(cfg["layers"]):
@@ -217,9 +219,12 @@ def closest_call(cfg, w, tokens: List[int]):
             r = mlp["router"]
             if r["top"] < r["experts"] + r.get("identity", 0):
                 pre = "l%d.mlp." % i
-                s = router_scores(mixed(x, w, i, lc, cfg), w, pre) + w[pre + "correction"]
-                srt = torch.sort(s, dim=-1, descending=True).values
-                gap = torch.minimum(gap, srt[:, r["top"] - 1] - srt[:, r["top"]])
+                s = router_scores(mixed(x, w, i, lc, cfg), w, pre)
+                srt = torch.sort(s + w[pre + "correction"], dim=-1, descending=True)
+                at = slice(r["top"] - 1, r["top"] + 1)
+                call = srt.values[:, r["top"] - 1] - srt.values[:, r["top"]]
+                matters = torch.gather(s, 1, srt.indices[:, at]).max(dim=1).values >= slight
+                gap = torch.where(matters, torch.minimum(gap, call), gap)
         x = layer(x, w, i, lc, cfg)
     return gap
 
