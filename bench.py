@@ -146,7 +146,33 @@ def sunulorn_config(n_layer, size="gpt2-small", n_positions=1024):
             "vocab_size": 50257, "n_positions": n_positions, "n_layer": n}
 
 
-DESIGNS = {"kugulorn": kugulorn_config, "rekirax": rekirax_config, "viladra": viladra_config, "sunulorn": sunulorn_config}
+def zokunex_config(n_layer, size="gpt2-small", n_positions=1024):
+    """A Zokunex model with as many layers as the GPT-2 configuration `size` has, at the same width, vocabulary and
+    context: two layers of matrix memories (heads of 64 x 64, as many as GPT-2 has) and one of latent attention (as many
+    heads of 64, a latent of up to a third of the width beside 32 rotated columns) in turn; a squared-relu feed-forward of
+    GPT-2's inner width in every third layer, and in the others eight experts that together hold as much, beside two
+    identity experts, two chosen."""
+    full_layers, d, h, f = SIZES[size]
+    n = n_layer or full_layers
+    rank = max(r for r in (64, 128, 256, 512) if r <= max(64, d // 3))      # 256 at 768 and 1,024, 512 at 1,600
+    dense = {"kind": "dense", "ff": f}
+    moe = {"kind": "moe", "router": {"experts": 8, "identity": 2, "top": 2}, "expert": {"ff": f // 8}}
+    layers = []
+    for i in range(n):
+        mlp = dense if i % 3 == 0 else moe
+        if i % 3 < 2:
+            layers.append({"type": "mlstm", "mlp": mlp, "mixer": {"heads": h, "dim": 64, "vdim": 64, "gate_cap": 15.0}})
+        else:
+            layers.append({"type": "latent_attention", "mlp": mlp,
+                           "mixer": {"heads": h, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": rank, "scale": 96 ** -0.5,
+                                     "rot": {"base": 10000.0, "dims": 32}}})
+    return {"architecture": "Zokunex", "vocab": 50257, "width": d, "norm": {"eps": 1e-6}, "logit_scale": 1.0, "layers": layers,
+            # (what the measurement itself reads; the architecture ignores them)
+            "vocab_size": 50257, "n_positions": n_positions, "n_layer": n}
+
+
+DESIGNS = {"kugulorn": kugulorn_config, "rekirax": rekirax_config, "viladra": viladra_config, "sunulorn": sunulorn_config,
+           "zokunex": zokunex_config}
 
 
 def decode_run(model_dir, dtype, batch, prompt_len, steps, warmup, cfg):
@@ -380,10 +406,10 @@ def main():
     ap.add_argument("--config", help="a config.json to measure in place of the GPT-2 sizes (any registered architecture; "
                                      "it names vocab_size and n_positions, or --vocab / --positions do)")
     ap.add_argument("--vocab", type=int, default=0, help="with --config: the vocabulary to draw token ids from")
-    ap.add_argument("--design", default="gpt2", choices=["gpt2", "kugulorn", "rekirax", "viladra", "sunulorn"],
-                    help="kugulorn / rekirax / viladra / sunulorn: a model of that design of about the size --size names (kugulorn_config, "
-                         "rekirax_config, viladra_config, sunulorn_config) through the same measurement; --compare runs it and GPT-2 one after the other")
-    ap.add_argument("--beside", default="gpt2", choices=["gpt2", "kugulorn", "rekirax", "viladra", "sunulorn"],
+    ap.add_argument("--design", default="gpt2", choices=["gpt2", *DESIGNS],
+                    help="kugulorn / rekirax / viladra / sunulorn / zokunex: a model of that design of about the size --size names (kugulorn_config, "
+                         "rekirax_config, viladra_config, sunulorn_config, zokunex_config) through the same measurement; --compare runs it and GPT-2 one after the other")
+    ap.add_argument("--beside", default="gpt2", choices=["gpt2", *DESIGNS],
                     help="with --compare: the design that the --design model is measured beside (default GPT-2)")
     ap.add_argument("--compare", action="store_true",
                     help="prefill (2 x 1,024 tokens) and decode (batch 1, 8, 64) of the --design model (default Kugulorn) and of the GPT-2 model "
