@@ -178,7 +178,9 @@ __device__ __forceinline__ u32x4 operand8(const float* p) {
     const float4 x = *reinterpret_cast<const float4*>(p), y = *reinterpret_cast<const float4*>(p + 4);
     return u32x4{pack_bf16x2(x.x, x.y), pack_bf16x2(x.z, x.w), pack_bf16x2(y.x, y.y), pack_bf16x2(y.z, y.w)};
 }
-template <typename TA>
+// UN steps of the inner loop ask for their operands together (K is a multiple of 32 UN): one step at a time waits a round
+// trip to memory each.
+template <typename TA, int UN>
 __global__ void __launch_bounds__(256)
 head_linear_mfma_kernel(const TA* __restrict__ a, int lda, int a_hs, const bf16_t* __restrict__ w, int ldw, int w_head_rows,
                         int w_head_cols, bf16_t* __restrict__ out, int ldo, int out_hs, int n_tokens, int N, int K,
@@ -196,17 +198,38 @@ head_linear_mfma_kernel(const TA* __restrict__ a, int lda, int a_hs, const bf16_
     f32x4 acc[4];
 #pragma unroll
     for (int ct = 0; ct < 4; ++ct) acc[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < K; k += 32) {
-        Frag8 af, wf[4];
-        af.q = operand8(arow + k);
+    for (int k0 = 0; k0 < K; k0 += 32 * UN) {
+        Frag8 af[UN], wf[UN][4];
 #pragma unroll
-        for (int ct = 0; ct < 4; ++ct) wf[ct].q = *reinterpret_cast<const u32x4*>(wrow[ct] + k);
+        for (int u = 0; u < UN; ++u) {
+            af[u].q = operand8(arow + k0 + 32 * u);
 #pragma unroll
-        for (int ct = 0; ct < 4; ++ct) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ct].v, af.v, acc[ct], 0, 0, 0);
+            for (int ct = 0; ct < 4; ++ct) wf[u][ct].q = *reinterpret_cast<const u32x4*>(wrow[ct] + k0 + 32 * u);
+        }
+        __builtin_amdgcn_sched_barrier(0);              // (left alone the compiler moves each load to its use)
+#pragma unroll
+        for (int u = 0; u < UN; ++u)
+#pragma unroll
+            for (int ct = 0; ct < 4; ++ct) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u][ct].v, af[u].v, acc[ct], 0, 0, 0);
     }
-    if (t0 + 16 * wave + c16 < n_tokens) {
+    const float g = gate != nullptr ? 1.f / (1.f + expf(-gate[static_cast<size_t>(tok) * ldg + h])) : 1.f;
+    if (n_base + 64 <= N && ((ldo | out_hs) & 7) == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0) {
+        // a whole tile: through LDS (this wavefront's own), so that a store instruction covers eight rows of 128 bytes
+        __shared__ __attribute__((aligned(16))) bf16_t tile_s[4][16][72];
+#pragma unroll
+        for (int ct = 0; ct < 4; ++ct)
+            *reinterpret_cast<uint2*>(&tile_s[wave][c16][16 * ct + 4 * G]) =
+                make_uint2(pack_bf16x2(acc[ct][0] * g, acc[ct][1] * g), pack_bf16x2(acc[ct][2] * g, acc[ct][3] * g));
+        wave_lds_sync();
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int r = 8 * u + lane / 8, t = t0 + 16 * wave + r;
+            if (t < n_tokens)
+                *reinterpret_cast<u32x4*>(out + static_cast<size_t>(t) * ldo + static_cast<size_t>(h) * out_hs + n_base + 8 * (lane % 8)) =
+                    *reinterpret_cast<const u32x4*>(&tile_s[wave][r][8 * (lane % 8)]);
+        }
+    } else if (t0 + 16 * wave + c16 < n_tokens) {
         bf16_t* orow = out + static_cast<size_t>(tok) * ldo + static_cast<size_t>(h) * out_hs;
-        const float g = gate != nullptr ? 1.f / (1.f + expf(-gate[static_cast<size_t>(tok) * ldg + h])) : 1.f;
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) {
             const int n = n_base + 16 * ct + 4 * G;            // acc[ct][r] is output n + r of this lane's token
@@ -216,23 +239,22 @@ head_linear_mfma_kernel(const TA* __restrict__ a, int lda, int a_hs, const bf16_
         }
     }
     if (positions != nullptr && blockIdx.z == 0) {
-        const int nt = min(64, n_tokens - t0), per = tail / 2 + tail;
-        for (int i = threadIdx.x; i < nt * per; i += 256) {
-            const int tt = i / per, k = i % per;
+        // (pairs and plain columns in loops of their own: a wavefront that holds both would run the turn for a third of its lanes)
+        const int nt = min(64, n_tokens - t0), pairs = rot_dims / 2, plain = tail - rot_dims;
+        for (int i = threadIdx.x; i < nt * pairs; i += 256) {
+            const int tt = i / pairs, k = i % pairs;
             const TA* src = a + static_cast<size_t>(t0 + tt) * lda + static_cast<size_t>(h) * a_hs + K;
             bf16_t* dst = out + static_cast<size_t>(t0 + tt) * ldo + static_cast<size_t>(h) * out_hs + N;
-            if (k < tail / 2) {
-                if (k < rot_dims / 2) {
-                    float u, v;
-                    const int first = pair_first(k, half), second = pair_second(k, half, rot_dims);
-                    turn_pair(to_float(src[first]), to_float(src[second]), positions[t0 + tt], k, log2_base, rot_dims, u, v);
-                    dst[first] = float_to_bf16(u);
-                    dst[second] = float_to_bf16(v);
-                }
-            } else {
-                const int c = k - tail / 2;
-                if (c >= rot_dims) dst[c] = float_to_bf16(to_float(src[c]));
-            }
+            float u, v;
+            const int first = pair_first(k, half), second = pair_second(k, half, rot_dims);
+            turn_pair(to_float(src[first]), to_float(src[second]), positions[t0 + tt], k, log2_base, rot_dims, u, v);
+            dst[first] = float_to_bf16(u);
+            dst[second] = float_to_bf16(v);
+        }
+        for (int i = threadIdx.x; i < nt * plain; i += 256) {
+            const int tt = i / plain, c = rot_dims + i % plain;
+            out[static_cast<size_t>(t0 + tt) * ldo + static_cast<size_t>(h) * out_hs + N + c] =
+                float_to_bf16(to_float(a[static_cast<size_t>(t0 + tt) * lda + static_cast<size_t>(h) * a_hs + K + c]));
         }
     }
 }
@@ -643,11 +665,12 @@ int mllm_latent_absorb(const void* q, int ldq, const void* w_uk, int ldw, void* 
     const double l2 = log2(base);
     const auto aligned16 = [](const void* ptr) { return (reinterpret_cast<uintptr_t>(ptr) & 15) == 0; };
     if (dtype == MLLM_BF16 && Dn % 32 == 0 && ldq % 8 == 0 && (Dn + Dr) % 8 == 0 && ldw % 8 == 0 && aligned16(q) && aligned16(w_uk)) {
-#define ABSORB_MFMA(TQ)                                                                                                                \
-    head_linear_mfma_kernel<TQ><<<dim3((T + 63) / 64, H, (R + 63) / 64), 256, 0, stream>>>(                                               \
+#define ABSORB_MFMA(TQ, UN)                                                                                                            \
+    head_linear_mfma_kernel<TQ, UN><<<dim3((T + 63) / 64, H, (R + 63) / 64), 256, 0, stream>>>(                                               \
         static_cast<const TQ*>(q), ldq, Dn + Dr, static_cast<const bf16_t*>(w_uk), ldw, 0, Dn, static_cast<bf16_t*>(qa), ldqa, R + Dr, T, R, \
         Dn, positions, Dr, rot_dims, l2, half_split, nullptr, 0)
-        if (q_dtype == MLLM_F32) ABSORB_MFMA(float); else ABSORB_MFMA(bf16_t);
+        if (q_dtype == MLLM_F32) { if (Dn % 64 == 0) ABSORB_MFMA(float, 2); else ABSORB_MFMA(float, 1); }
+        else { if (Dn % 64 == 0) ABSORB_MFMA(bf16_t, 2); else ABSORB_MFMA(bf16_t, 1); }
 #undef ABSORB_MFMA
         MLLM_LAUNCH_CHECK();
         return 0;
@@ -769,9 +792,12 @@ int mllm_latent_expand(const void* o_lat, int ldo, const void* w_uv, int ldw, vo
     if (T <= 0) return 0;
     if (dtype == MLLM_BF16 && R % 32 == 0 && ldo % 8 == 0 && ldw % 8 == 0 && (reinterpret_cast<uintptr_t>(o_lat) & 15) == 0 &&
         (reinterpret_cast<uintptr_t>(w_uv) & 15) == 0) {
-        head_linear_mfma_kernel<bf16_t><<<dim3((T + 63) / 64, H, (Dv + 63) / 64), 256, 0, stream>>>(
-            static_cast<const bf16_t*>(o_lat), ldo, R, static_cast<const bf16_t*>(w_uv), ldw, Dv, 0, static_cast<bf16_t*>(out), ldout, Dv, T, Dv,
-            R, nullptr, 0, 0, 0.0, 0, gate, ldg);
+#define EXPAND_MFMA(UN)                                                                                                                  \
+    head_linear_mfma_kernel<bf16_t, UN><<<dim3((T + 63) / 64, H, (Dv + 63) / 64), 256, 0, stream>>>(                                        \
+        static_cast<const bf16_t*>(o_lat), ldo, R, static_cast<const bf16_t*>(w_uv), ldw, Dv, 0, static_cast<bf16_t*>(out), ldout, Dv, T, Dv, R, \
+        nullptr, 0, 0, 0.0, 0, gate, ldg)
+        if (R % 128 == 0) EXPAND_MFMA(4); else if (R % 64 == 0) EXPAND_MFMA(2); else EXPAND_MFMA(1);
+#undef EXPAND_MFMA
         MLLM_LAUNCH_CHECK();
         return 0;
     }

@@ -61,17 +61,20 @@ __device__ __forceinline__ size_t state_m_at(const MemoryArgs& a, int h, int cop
     return static_cast<size_t>(a.H) * a.d * a.e + static_cast<size_t>(a.H) * a.copies * a.d + static_cast<size_t>(h) * a.copies + copy;
 }
 // workspace per (chunk, head): the memory [d * e], n [d], then [log scale of the chunk's own memory, sum of its f, the
-// request's m in front of the step (a sequence's first chunk only), the m this chunk starts from]
-__host__ __device__ __forceinline__ size_t chunk_floats(int d, int e) { return (static_cast<size_t>(d) * e + d + 4 + 3) / 4 * 4; }
+// request's m in front of the step (a sequence's first chunk only), the m this chunk starts from], and behind that, as
+// doubles, u, its running maximum and F for the chunk's tokens
+__host__ __device__ __forceinline__ size_t chunk_gates_at(int d, int e) { return (static_cast<size_t>(d) * e + d + 4 + 3) / 4 * 4; }
+__host__ __device__ __forceinline__ size_t chunk_floats(int d, int e) { return chunk_gates_at(d, e) + 3 * 2 * MM_CHUNK; }
 __device__ __forceinline__ size_t chunk_scalars_at(int d, int e) { return static_cast<size_t>(d) * e + d; }
 
-// Which sequence (from first_seq on) and which of its chunks is number w: a wavefront looks at 64 sequences at a time.
-// False: there are fewer chunks.
-__device__ __forceinline__ bool find_chunk(const int* __restrict__ cu_q, int first_seq, int n_seqs, int w, int& b, int& chunk, int& first, int& n) {
+// Which sequence (from first_seq on) and which of its chunks is number w, and the sequence's state slot: a wavefront looks
+// at 64 sequences at a time. False: there are fewer chunks.
+__device__ __forceinline__ bool find_chunk(const int* __restrict__ cu_q, const int* __restrict__ state_slots, int first_seq, int n_seqs, int w,
+                                           int& slot, int& chunk, int& first, int& n) {
     const int lane = threadIdx.x % MLLM_WAVE;
     for (int b0 = first_seq; b0 < n_seqs; b0 += MLLM_WAVE) {
         const int mine = min(b0 + lane, n_seqs - 1);
-        const int begin = cu_q[mine], len = cu_q[mine + 1] - begin;
+        const int begin = cu_q[mine], len = cu_q[mine + 1] - begin, its_slot = state_slots[mine];
         const int nc = b0 + lane < n_seqs ? (len + MM_CHUNK - 1) / MM_CHUNK : 0;
         int upto = nc;
 #pragma unroll
@@ -82,11 +85,10 @@ __device__ __forceinline__ bool find_chunk(const int* __restrict__ cu_q, int fir
         const unsigned long long here = __ballot(w < upto);
         if (here != 0) {
             const int l = __ffsll(here) - 1;
-            b = b0 + l;
+            slot = __builtin_amdgcn_readfirstlane(__shfl(its_slot, l, MLLM_WAVE));
             chunk = w - (__shfl(upto, l, MLLM_WAVE) - __shfl(nc, l, MLLM_WAVE));
             first = __shfl(begin, l, MLLM_WAVE) + chunk * MM_CHUNK;
             n = min(MM_CHUNK, __shfl(len, l, MLLM_WAVE) - chunk * MM_CHUNK);
-            b = __builtin_amdgcn_readfirstlane(b);
             chunk = __builtin_amdgcn_readfirstlane(chunk);
             first = __builtin_amdgcn_readfirstlane(first);
             n = __builtin_amdgcn_readfirstlane(n);
@@ -162,6 +164,28 @@ __device__ __forceinline__ void tile_store(float* lds, const float (&v)[16], int
     }
 }
 
+// A lane's operand of a product over 64 key columns, straight from memory: columns 16 kk + 4 G .. + 3 of one row, kk < 4, of
+// which the first `cols` exist (the rest becomes zero in query_finish). Loads without conditions.
+template <bool VEC>
+__device__ __forceinline__ void query_load(float4 (&q4)[4], const float* __restrict__ row, int cols, int G) {
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+        const int col = 16 * kk + 4 * G;
+        if (VEC) q4[kk] = *reinterpret_cast<const float4*>(row + min(col, cols - 4));
+        else q4[kk] = make_float4(row[min(col, cols - 1)], row[min(col + 1, cols - 1)], row[min(col + 2, cols - 1)], row[min(col + 3, cols - 1)]);
+    }
+}
+__device__ __forceinline__ void query_finish(float4 (&q4)[4], float scale, int cols, int G) {
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+        const int col = 16 * kk + 4 * G;
+        q4[kk].x = col < cols ? q4[kk].x * scale : 0.f;
+        q4[kk].y = col + 1 < cols ? q4[kk].y * scale : 0.f;
+        q4[kk].z = col + 2 < cols ? q4[kk].z * scale : 0.f;
+        q4[kk].w = col + 3 < cols ? q4[kk].w * scale : 0.f;
+    }
+}
+
 // A chunk's own memory, 64 x 64 of it a workgroup: grid (chunks, heads, key tiles * value tiles). Four wavefronts of 16
 // key columns each; the products' inner dimension is the chunk's tokens.
 template <bool VEC>
@@ -170,10 +194,8 @@ memory_chunk_kernel(MemoryArgs a, int first_seq, int n_seqs, int value_tiles, fl
     __shared__ __attribute__((aligned(16))) float Ks[MM_CHUNK * MM_STRIDE];
     __shared__ __attribute__((aligned(16))) float Vs[MM_CHUNK * MM_STRIDE];
     __shared__ float weight[MM_CHUNK];
-    int b, chunk, first, n;
-    if (!find_chunk(a.cu_q, first_seq, n_seqs, blockIdx.x, b, chunk, first, n)) return;
-    const int slot = a.state_slots[b];
-    if (slot < 0) return;
+    int slot, chunk, first, n;
+    if (!find_chunk(a.cu_q, a.state_slots, first_seq, n_seqs, blockIdx.x, slot, chunk, first, n) || slot < 0) return;
     const int h = blockIdx.y, kt = blockIdx.z / value_tiles, vt = blockIdx.z % value_tiles;
     const int tid = threadIdx.x, lane = tid % MLLM_WAVE, wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
     const int kc = min(64, a.d - 64 * kt), vc = min(64, a.e - 64 * vt);
@@ -184,13 +206,19 @@ memory_chunk_kernel(MemoryArgs a, int first_seq, int n_seqs, int value_tiles, fl
     if (wave == 0) {
         double F, u;
         chunk_gates(a, h, first, n, lane, F, u);
-        const double U = __shfl(wave_prefix_max(u, lane), MLLM_WAVE - 1, MLLM_WAVE);
+        const double upto = wave_prefix_max(u, lane), U = __shfl(upto, MLLM_WAVE - 1, MLLM_WAVE);
         weight[lane] = expf(static_cast<float>(u - U));
-        if (kt == 0 && vt == 0 && lane == MLLM_WAVE - 1) {
-            float* sc = W + chunk_scalars_at(a.d, a.e);
-            sc[0] = static_cast<float>(U + F);
-            sc[1] = static_cast<float>(F);
-            if (chunk == 0) sc[2] = a.state[static_cast<size_t>(slot) * a.slot_floats + state_m_at(a, h, 0)];
+        if (kt == 0 && vt == 0) {
+            double* gates = reinterpret_cast<double*>(W + chunk_gates_at(a.d, a.e));
+            gates[lane] = u;
+            gates[MM_CHUNK + lane] = upto;
+            gates[2 * MM_CHUNK + lane] = F;
+            if (lane == MLLM_WAVE - 1) {
+                float* sc = W + chunk_scalars_at(a.d, a.e);
+                sc[0] = static_cast<float>(U + F);
+                sc[1] = static_cast<float>(F);
+                if (chunk == 0) sc[2] = a.state[static_cast<size_t>(slot) * a.slot_floats + state_m_at(a, h, 0)];
+            }
         }
     }
     lds_barrier();
@@ -201,12 +229,14 @@ memory_chunk_kernel(MemoryArgs a, int first_seq, int n_seqs, int value_tiles, fl
     f32x4 acc[4];
 #pragma unroll
     for (int t = 0; t < 4; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float key_sum = 0.f;                              // of key column 16 wave + c, over this lane group's tokens
 #pragma unroll
     for (int j = 0; j < 16; ++j) {
         // (which of the 64 tokens a lane group's slot of step j stands for is free, as long as both operands agree;
         // groups four rows apart read conflict-free)
         const int t = (j / 4) * 16 + 4 * G + j % 4;
         const float av = Ks[t * MM_STRIDE + 16 * wave + c];
+        key_sum += av;
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) acc[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(av, Vs[t * MM_STRIDE + 16 * ct + c], acc[ct], 0, 0, 0);
     }
@@ -217,11 +247,8 @@ memory_chunk_kernel(MemoryArgs a, int first_seq, int n_seqs, int value_tiles, fl
             const int i = 16 * wave + 4 * G + r, col = 16 * ct + c;
             if (i < kc && col < vc) W[static_cast<size_t>(64 * kt + i) * a.e + 64 * vt + col] = acc[ct][r];
         }
-    if (vt == 0 && tid < kc) {
-        float s = 0.f;
-        for (int t = 0; t < n; ++t) s += Ks[t * MM_STRIDE + tid];
-        W[static_cast<size_t>(a.d) * a.e + 64 * kt + tid] = s;
-    }
+    key_sum = rows_sum(key_sum);
+    if (vt == 0 && G == 0 && 16 * wave + c < kc) W[static_cast<size_t>(a.d) * a.e + 64 * kt + 16 * wave + c] = key_sum;
 }
 
 // One thread per cell of a head's memory and normaliser: grid (cells of all heads / 256, sequences). In the workspace a
@@ -249,7 +276,7 @@ memory_states_kernel(MemoryArgs a, int first_seq, float* __restrict__ ws) {
     float* W = ws + (static_cast<size_t>(before) * a.H + h) * chunk_floats(a.d, a.e);
     const size_t sc = chunk_scalars_at(a.d, a.e);
     float S = *cell, m = W[sc + 2];
-    constexpr int AHEAD = 8;                           // chunks whose values are asked for together
+    constexpr int AHEAD = 16;                          // chunks whose values are asked for together
     for (int c0 = 0; c0 < nc; c0 += AHEAD) {
         float L[AHEAD], scale[AHEAD], sum_f[AHEAD];
 #pragma unroll
@@ -287,15 +314,13 @@ template <typename T, int NT, bool VEC, bool FUSED>
 __global__ void __launch_bounds__(256)
 memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __restrict__ ws, T* __restrict__ out, int ldo, float* __restrict__ y,
                      int ldy) {
-    __shared__ __attribute__((aligned(16))) float Qs[MM_CHUNK * MM_STRIDE];
     __shared__ __attribute__((aligned(16))) float Ks[MM_CHUNK * MM_STRIDE];       // keys; the weighted scores; the results
     __shared__ __attribute__((aligned(16))) float Bs[MM_CHUNK * MM_STRIDE];       // a tile of the starting memory, then of the values
     __shared__ double u_s[MM_CHUNK], r_s[MM_CHUNK];
     __shared__ float nq_s[MM_CHUNK], start_s[MM_CHUNK], floor_s[MM_CHUNK];
     __shared__ __attribute__((aligned(16))) float n_s[64];
-    int b, chunk, first, n;
-    if (!find_chunk(a.cu_q, first_seq, n_seqs, blockIdx.x, b, chunk, first, n)) return;
-    if (a.state_slots[b] < 0) return;
+    int slot, chunk, first, n;
+    if (!find_chunk(a.cu_q, a.state_slots, first_seq, n_seqs, blockIdx.x, slot, chunk, first, n) || slot < 0) return;
     const int h = blockIdx.y, vt0 = blockIdx.z * NT;
     const int tid = threadIdx.x, lane = tid % MLLM_WAVE, wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
     const int G = lane / 16, c = lane % 16;
@@ -310,44 +335,47 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
 #pragma unroll
         for (int ct = 0; ct < 4; ++ct) o[t][ct] = f32x4{0.f, 0.f, 0.f, 0.f};
     float nq = 0.f;                                  // this lane's share of q_t . n, t = 16 wave + c
+    float vv[16];                                    // the first tile of values: asked for now, used behind the scores
     const int key_tiles = (a.d + 63) / 64;
     for (int kt = 0; kt < key_tiles; ++kt) {
         const int kc = min(64, a.d - 64 * kt);
-        float qv[16], kv[16], sv[16];
-        tile_load<VEC>(qv, rows + a.q_col + h * a.d + 64 * kt, a.ld, n, kc);
+        float kv[16], sv[16];
+        float4 q4[4];                                // this lane's queries: token 16 wave + c, key columns 16 kk + 4 G ..
+        query_load<VEC>(q4, rows + static_cast<size_t>(min(16 * wave + c, n - 1)) * a.ld + a.q_col + h * a.d + 64 * kt, kc, G);
         tile_load<VEC>(kv, rows + a.k_col + h * a.d + 64 * kt, a.ld, n, kc);
         tile_load<VEC>(sv, W + static_cast<size_t>(64 * kt) * a.e + 64 * vt0, a.e, kc, min(64, a.e - 64 * vt0));
         const float nv = W[static_cast<size_t>(a.d) * a.e + 64 * kt + min(tid, kc - 1)];
+        if (kt == key_tiles - 1) tile_load<VEC>(vv, rows + a.v_col + h * a.e + 64 * vt0, a.ld, n, min(64, a.e - 64 * vt0));
         if (kt == 0 && wave == 0) {
-            double F, u;
-            chunk_gates(a, h, first, n, lane, F, u);
+            const double* gates = reinterpret_cast<const double*>(W + chunk_gates_at(a.d, a.e));
+            const double u = gates[lane], upto = gates[MM_CHUNK + lane], F = gates[2 * MM_CHUNK + lane];
             const float m = W[chunk_scalars_at(a.d, a.e) + 3];
-            const double r = fmax(wave_prefix_max(u, lane), static_cast<double>(m));
+            const double r = fmax(upto, static_cast<double>(m));
             u_s[lane] = u;
             r_s[lane] = r;
             start_s[lane] = expf(static_cast<float>(static_cast<double>(m) - r));
             floor_s[lane] = expf(-static_cast<float>(r + F));
         }
         if (kt > 0) lds_barrier();                   // the tiles before are used up
-        tile_store<VEC>(Qs, qv, n, kc, a.q_scale);
         tile_store<VEC>(Ks, kv, n, kc, 1.f);
         tile_store<VEC>(Bs, sv, kc, min(64, a.e - 64 * vt0), 1.f);
         if (tid < 64) n_s[tid] = tid < kc ? nv : 0.f;
+        query_finish(q4, 16 * wave + c < n ? a.q_scale : 0.f, kc, G);
         lds_barrier();
         // (a lane's float4 holds its operand for four steps: which key columns a step's slots stand for is free as long
         // as both operands agree)
 #pragma unroll
         for (int kk = 0; kk < 4; ++kk) {
-            const float4 q4 = *reinterpret_cast<const float4*>(Qs + (16 * wave + c) * MM_STRIDE + 16 * kk + 4 * G);
+            const float4 q = q4[kk];
             const float4 n4 = *reinterpret_cast<const float4*>(n_s + 16 * kk + 4 * G);
-            nq += (q4.x * n4.x + q4.y * n4.y) + (q4.z * n4.z + q4.w * n4.w);
+            nq += (q.x * n4.x + q.y * n4.y) + (q.z * n4.z + q.w * n4.w);
 #pragma unroll
             for (int ct = 0; ct < 4; ++ct) {
                 const float4 k4 = *reinterpret_cast<const float4*>(Ks + (16 * ct + c) * MM_STRIDE + 16 * kk + 4 * G);
-                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4.x, k4.x, p[ct], 0, 0, 0);
-                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4.y, k4.y, p[ct], 0, 0, 0);
-                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4.z, k4.z, p[ct], 0, 0, 0);
-                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4.w, k4.w, p[ct], 0, 0, 0);
+                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.x, k4.x, p[ct], 0, 0, 0);
+                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.y, k4.y, p[ct], 0, 0, 0);
+                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.z, k4.z, p[ct], 0, 0, 0);
+                p[ct] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.w, k4.w, p[ct], 0, 0, 0);
             }
         }
 #pragma unroll
@@ -361,8 +389,7 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
             }
 #pragma unroll
             for (int kk = 0; kk < 4; ++kk) {
-                const float4 q4 = *reinterpret_cast<const float4*>(Qs + (16 * wave + c) * MM_STRIDE + 16 * kk + 4 * G);
-                const float qj[4] = {q4.x, q4.y, q4.z, q4.w};
+                const float qj[4] = {q4[kk].x, q4[kk].y, q4[kk].z, q4[kk].w};
 #pragma unroll
                 for (int j = 0; j < 4; ++j)
 #pragma unroll
@@ -371,8 +398,6 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
             }
         }
     }
-    float vv[16];
-    tile_load<VEC>(vv, rows + a.v_col + h * a.e + 64 * vt0, a.ld, n, min(64, a.e - 64 * vt0));
     nq = rows_sum(nq);                               // the four lane groups' shares
     if (G == 0) nq_s[16 * wave + c] = nq;
     lds_barrier();                                   // keys and memory tiles are used up; nq_s is complete
@@ -429,6 +454,15 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
                 ss[r] += o[t][ct][r] * o[t][ct][r];      // (columns beyond the head's are zero)
             }
     }
+    // (what the end reads from memory is asked for before the sums over the wavefront)
+    float4 gate4[4], norm4;
+    if (VEC && FUSED) {
+        const int col = h * a.e + 64 * vt0 + min(4 * c, min(64, a.e - 64 * vt0) - 4);
+        norm4 = *reinterpret_cast<const float4*>(a.norm_w + col);
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+            gate4[u] = *reinterpret_cast<const float4*>(rows + static_cast<size_t>(min(16 * wave + 4 * u + G, n - 1)) * a.ld + a.g_col + col);
+    }
     float inv[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) inv[r] = FUSED ? 1.f / sqrtf(group_sum<16>(ss[r]) / static_cast<float>(a.e) + a.eps) : 1.f;
@@ -453,8 +487,8 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
                     *reinterpret_cast<float4*>(y + static_cast<size_t>(first + tok) * ldy + col0 + col) = x;
                     continue;
                 }
-                const float4 g = *reinterpret_cast<const float4*>(rows + static_cast<size_t>(tok) * a.ld + a.g_col + col0 + col);
-                const float4 w = *reinterpret_cast<const float4*>(a.norm_w + col0 + col);
+                const float4 g = t == 0 ? gate4[u] : *reinterpret_cast<const float4*>(rows + static_cast<size_t>(tok) * a.ld + a.g_col + col0 + col);
+                const float4 w = t == 0 ? norm4 : *reinterpret_cast<const float4*>(a.norm_w + col0 + col);
                 x.x *= w.x * mm_sigmoid(g.x); x.y *= w.y * mm_sigmoid(g.y); x.z *= w.z * mm_sigmoid(g.z); x.w *= w.w * mm_sigmoid(g.w);
                 T* dst = out + static_cast<size_t>(first + tok) * ldo + col0 + col;
                 if (sizeof(T) == 2) {
@@ -490,6 +524,7 @@ __global__ void __launch_bounds__(256)
 memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float* __restrict__ y, int ldy) {
     extern __shared__ __attribute__((aligned(16))) float mm_smem[];
     constexpr int CW = VEC ? 4 : 1, AHEAD = VEC ? 4 : 8;
+    // (the sequences of single tokens stand in front: sequence b's token is row b)
     const int b = blockIdx.x, h = blockIdx.y, tile = blockIdx.z;
     const int slot = a.state_slots[b];
     if (slot < 0) return;
@@ -500,7 +535,7 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
     float* k_s = q_s + d;
     float* part = k_s + d;                                    // [RG][cols]
     float* red = part + RG * cols;                            // [4]: the wavefronts' shares of n . q
-    const float* row = a.proj + static_cast<size_t>(a.cu_q[b]) * a.ld;
+    const float* row = a.proj + static_cast<size_t>(b) * a.ld;
     float* base = a.state + static_cast<size_t>(slot) * a.slot_floats;
     float* S = base + static_cast<size_t>(h) * d * e + c0;
     float* N = base + state_n_at(a, h, tile);
@@ -511,25 +546,9 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
     float v[CW];
 #pragma unroll
     for (int k = 0; k < CW; ++k) v[k] = row[a.v_col + h * e + c0 + col_c + k];
-    for (int i = tid; i < d; i += 256) {
-        q_s[i] = row[a.q_col + h * d + i] * a.q_scale;
-        k_s[i] = row[a.k_col + h * d + i];
-    }
-    const float ig = mm_log_input(iz, a.i_bias[h], a.cap), fg = mm_log_forget(fz, a.f_bias[h], a.cap);
-    const float m = fmaxf(fg + m_old, ig), keep = expf(fg + m_old - m), take = expf(ig - m);
-    lds_barrier();
-    // the normaliser (its new values are written behind the barrier below: m_old and N are this workgroup's own copy)
-    float nq = 0.f;
-    for (int i = tid; i < d; i += 256) {
-        const float x = keep * N[i] + take * k_s[i];
-        if (a.write) N[i] = x;
-        nq = fmaf(x, q_s[i], nq);
-    }
-    float acc[CW];
-#pragma unroll
-    for (int k = 0; k < CW; ++k) { acc[k] = 0.f; v[k] *= take; }
-    for (int i0 = 0; i0 < d; i0 += RG * AHEAD) {
-        float s[AHEAD][CW];
+    // the first rows of the memory, the normaliser and what the end needs are asked for before anything is waited for
+    float s[AHEAD][CW];
+    auto ask = [&](int i0) {
 #pragma unroll
         for (int u = 0; u < AHEAD; ++u) {
             const float* p = S + static_cast<size_t>(min(i0 + u * RG + min(rg, RG - 1), d - 1)) * e + col_c;
@@ -540,6 +559,29 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
                 s[u][0] = *p;
             }
         }
+    };
+    ask(0);
+    const float n_first = N[min(tid, d - 1)];
+    const float g_first = row[a.g_col + h * e + c0 + min(lane, nc - 1)], w_first = a.norm_w[h * e + c0 + min(lane, nc - 1)];
+    for (int i = tid; i < d; i += 256) {
+        q_s[i] = row[a.q_col + h * d + i] * a.q_scale;
+        k_s[i] = row[a.k_col + h * d + i];
+    }
+    const float ig = mm_log_input(iz, a.i_bias[h], a.cap), fg = mm_log_forget(fz, a.f_bias[h], a.cap);
+    const float m = fmaxf(fg + m_old, ig), keep = expf(fg + m_old - m), take = expf(ig - m);
+    lds_barrier();
+    // the normaliser (its new values are written behind the barrier below: m_old and N are this workgroup's own copy)
+    float nq = 0.f;
+    for (int i = tid; i < d; i += 256) {
+        const float x = keep * (i == tid ? n_first : N[i]) + take * k_s[i];
+        if (a.write) N[i] = x;
+        nq = fmaf(x, q_s[i], nq);
+    }
+    float acc[CW];
+#pragma unroll
+    for (int k = 0; k < CW; ++k) { acc[k] = 0.f; v[k] *= take; }
+    for (int i0 = 0; i0 < d; i0 += RG * AHEAD) {
+        if (i0 > 0) ask(i0);
 #pragma unroll
         for (int u = 0; u < AHEAD; ++u) {
             const int i = i0 + u * RG + rg;
@@ -575,14 +617,14 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
         for (int r = 0; r < RG; ++r) x += part[r * cols + j];
         x /= den;
         if (FUSED) part[j] = x;                                       // (only this lane reads column j)
-        else y[static_cast<size_t>(a.cu_q[b]) * ldy + h * e + c0 + j] = x;
+        else y[static_cast<size_t>(b) * ldy + h * e + c0 + j] = x;
         ss += x * x;
     }
     if (!FUSED) return;
     const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(e) + a.eps);
     for (int j = lane; j < nc; j += MLLM_WAVE) {
-        const float g = row[a.g_col + h * e + j];
-        out[static_cast<size_t>(a.cu_q[b]) * ldo + h * e + j] = from_float<T>(part[j] * inv * a.norm_w[h * e + j] * mm_sigmoid(g));
+        const float g = j == lane ? g_first : row[a.g_col + h * e + j], w = j == lane ? w_first : a.norm_w[h * e + j];
+        out[static_cast<size_t>(b) * ldo + h * e + j] = from_float<T>(part[j] * inv * w * mm_sigmoid(g));
     }
 }
 

@@ -137,43 +137,70 @@ template <typename TI, typename T, bool VEC, bool GELU>
 __global__ void __launch_bounds__(256)
 moe_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int N, int top, float scale,
                T* __restrict__ out, int ldo, float* __restrict__ weights_out, int ldw, MoeChoice mc) {
-    __shared__ float z[MOE_MAX_EXPERTS], wgt[MOE_MAX_EXPERTS], choice[MOE_MAX_EXPERTS];
-    const int t = blockIdx.x, tid = threadIdx.x, all = E + mc.identity;
-    if (tid < all) z[tid] = logits[static_cast<size_t>(t) * ldl + tid];
-    __syncthreads();
-    if (mc.correction == nullptr) {
-        if (tid < all) expert_weight(z, wgt, all, top, scale, tid);
-    } else {
-        float score = 0.f;
-        if (tid < all) {
-            float m = -INFINITY, sum = 0.f;
-            for (int o = 0; o < all; ++o) m = fmaxf(m, z[o]);
-            for (int o = 0; o < all; ++o) sum += expf(z[o] - m);
-            score = expf(z[tid] - m) / sum;
-            choice[tid] = score + mc.correction[tid];
-        }
-        __syncthreads();
-        if (tid < all) {
-            const float mine = choice[tid];
-            int before = 0;
-            for (int o = 0; o < all; ++o) before += (choice[o] > mine || (choice[o] == mine && o < tid)) ? 1 : 0;
-            wgt[tid] = before < top ? scale * score : 0.f;
-        }
-    }
-    __syncthreads();
-    if (weights_out != nullptr && tid < all) weights_out[static_cast<size_t>(t) * ldw + tid] = wgt[tid];
+    // weights: one copy a wavefront where up to 64 experts let every wavefront work them out by itself, without a barrier
+    __shared__ float z[MOE_MAX_EXPERTS], weights[4][MOE_MAX_EXPERTS], choice[MOE_MAX_EXPERTS];
+    const int t = blockIdx.x, tid = threadIdx.x, all = E + mc.identity, lane = tid % MLLM_WAVE;
+    const int wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
     const TI* ur = up + static_cast<size_t>(t) * ldu;
     T* orow = out + static_cast<size_t>(t) * ldo;
+    // the first columns are asked for before the weights are worked out
+    constexpr int AHEAD = 2;
+    float first[AHEAD][8];
     if (VEC) {
-        for (int c = tid * 8; c < N; c += 256 * 8) {
-            float v[8];
-            load8(ur + c, v);
+#pragma unroll
+        for (int u = 0; u < AHEAD; ++u) load8(ur + min(tid * 8 + 2048 * u, N - 8), first[u]);
+    }
+    float* wgt = weights[all <= MLLM_WAVE ? wave : 0];
+    if (all <= MLLM_WAVE) {
+        const float mine = logits[static_cast<size_t>(t) * ldl + min(lane, all - 1)];
+        const float m = wave_max(mine), ex = lane < all ? expf(mine - m) : 0.f;
+        const float score = ex / wave_sum(ex);
+        // (without a correction the order of the scores is that of the logits)
+        const float key = mc.correction != nullptr ? score + mc.correction[min(lane, all - 1)] : mine;
+        int before = 0;
+        for (int o = 0; o < all; ++o) {
+            const float other = row_lane(key, o);
+            before += (other > key || (other == key && o < lane)) ? 1 : 0;
+        }
+        wgt[lane] = before < top ? scale * score : 0.f;
+        wave_lds_sync();
+    } else {
+        if (tid < all) z[tid] = logits[static_cast<size_t>(t) * ldl + tid];
+        __syncthreads();
+        if (mc.correction == nullptr) {
+            if (tid < all) expert_weight(z, wgt, all, top, scale, tid);
+        } else {
+            float score = 0.f;
+            if (tid < all) {
+                float m = -INFINITY, sum = 0.f;
+                for (int o = 0; o < all; ++o) m = fmaxf(m, z[o]);
+                for (int o = 0; o < all; ++o) sum += expf(z[o] - m);
+                score = expf(z[tid] - m) / sum;
+                choice[tid] = score + mc.correction[tid];
+            }
+            __syncthreads();
+            if (tid < all) {
+                const float mine = choice[tid];
+                int before = 0;
+                for (int o = 0; o < all; ++o) before += (choice[o] > mine || (choice[o] == mine && o < tid)) ? 1 : 0;
+                wgt[tid] = before < top ? scale * score : 0.f;
+            }
+        }
+        __syncthreads();
+    }
+    if (weights_out != nullptr && tid < all) weights_out[static_cast<size_t>(t) * ldw + tid] = wgt[tid];
+    if (VEC) {
+        auto columns = [&](int c, float (&v)[8]) {
             const int e = c / ff;                       // (ff is a multiple of 8: the eight columns are one expert's)
             const float wt = e < E ? wgt[e] : 1.f;
             if (GELU) {
-                // (no work for an expert that was not chosen: erf costs more than the rest of the kernel)
+                if (wt != 0.f) {                        // (no erf for an expert that was not chosen)
 #pragma unroll
-                for (int u = 0; u < 8; ++u) v[u] = wt != 0.f ? wt * gelu_erf(v[u]) : 0.f;
+                    for (int u = 0; u < 8; ++u) v[u] = wt * gelu_erf(v[u]);
+                } else {
+#pragma unroll
+                    for (int u = 0; u < 8; ++u) v[u] = 0.f;
+                }
             } else {
 #pragma unroll
                 for (int u = 0; u < 8; ++u) v[u] = wt * relu2(v[u]);
@@ -186,13 +213,21 @@ moe_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ log
                 *reinterpret_cast<float4*>(orow + c) = make_float4(v[0], v[1], v[2], v[3]);
                 *reinterpret_cast<float4*>(orow + c + 4) = make_float4(v[4], v[5], v[6], v[7]);
             }
+        };
+#pragma unroll
+        for (int u = 0; u < AHEAD; ++u)
+            if (tid * 8 + 2048 * u < N) columns(tid * 8 + 2048 * u, first[u]);
+        for (int c = tid * 8 + 2048 * AHEAD; c < N; c += 2048) {
+            float v[8];
+            load8(ur + c, v);
+            columns(c, v);
         }
     } else {
         for (int c = tid; c < N; c += 256) {
             const int e = c / ff;
             const float wt = e < E ? wgt[e] : 1.f;
             const float v = to_float(ur[c]);
-            orow[c] = from_float<T>(wt * (GELU ? gelu_erf(v) : relu2(v)));
+            orow[c] = from_float<T>(wt != 0.f ? wt * (GELU ? gelu_erf(v) : relu2(v)) : 0.f);
         }
     }
     if (mc.identity > 0) {
@@ -200,7 +235,19 @@ moe_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ log
         for (int o = E; o < all; ++o) w += wgt[o];
         const T* hr = static_cast<const T*>(mc.h) + static_cast<size_t>(t) * mc.ldh;
         float* yr = mc.y + static_cast<size_t>(t) * mc.ldy;
-        for (int c = tid; c < mc.D; c += 256) yr[c] = (mc.y_add ? yr[c] : 0.f) + w * to_float(hr[c]);
+        if (((mc.D | mc.ldh | mc.ldy) & 7) == 0 && ((reinterpret_cast<uintptr_t>(mc.h) | reinterpret_cast<uintptr_t>(mc.y)) & 15) == 0) {
+            for (int c = tid * 8; c < mc.D; c += 2048) {
+                float v[8], old[8];
+                load8(hr + c, v);
+                if (mc.y_add) load8(yr + c, old);
+#pragma unroll
+                for (int u = 0; u < 8; ++u) v[u] = (mc.y_add ? old[u] : 0.f) + w * v[u];
+                *reinterpret_cast<float4*>(yr + c) = make_float4(v[0], v[1], v[2], v[3]);
+                *reinterpret_cast<float4*>(yr + c + 4) = make_float4(v[4], v[5], v[6], v[7]);
+            }
+        } else {
+            for (int c = tid; c < mc.D; c += 256) yr[c] = (mc.y_add ? yr[c] : 0.f) + w * to_float(hr[c]);
+        }
     }
 }
 
