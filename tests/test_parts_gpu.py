@@ -45,7 +45,7 @@ def test_layernorm_part(dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("act", ["gelu_tanh", "gelu_erf"])
+@pytest.mark.parametrize("act", ["gelu_tanh", "gelu_erf", "relu2"])
 def test_dense_mlp_part(dtype, act):
     import parts_face as pf
     g = torch.Generator().manual_seed(1)
@@ -57,12 +57,46 @@ def test_dense_mlp_part(dtype, act):
     h = torch.randn(7, 48, generator=g).to(dtype)
     x0 = torch.randn(7, 48, generator=g)
     x = ff.forward(h.to(DEV), x0.clone().to(DEV))
-    fn = P.gelu_tanh if act == "gelu_tanh" else P.gelu_erf
+    fn = {"gelu_tanh": P.gelu_tanh, "gelu_erf": P.gelu_erf, "relu2": lambda z: torch.relu(z) ** 2}[act]
     # (the plain block takes the reference's [in, out] layout)
     w = {"h.0.mlp.c_fc.weight": up.double().T, "h.0.mlp.c_fc.bias": b1.double(),
          "h.0.mlp.c_proj.weight": down.double().T, "h.0.mlp.c_proj.bias": b2.double()}
     ref = x0.double() + P.mlp_block(h.double(), w, 0, fn)
     assert (x.cpu().double() - ref).abs().max() <= TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("joined", [False, True])
+@pytest.mark.parametrize("experts,identity,top,ff,D,T", [(5, 2, 3, 24, 48, 9), (3, 1, 4, 7, 45, 70), (1, 4, 2, 16, 48, 1), (60, 4, 6, 8, 64, 33),
+                                                          (90, 30, 9, 8, 48, 12), (4, 0, 2, 1040, 64, 5)])
+def test_routed_experts_with_a_correction_and_identity_experts(dtype, joined, experts, identity, top, ff, D, T):
+    """Exact-GELU experts chosen by score + correction and weighed by the score, some of which hand on their input: more
+    experts than a wavefront has lanes, sizes that are no multiple of 8, few and many rows, the router's product joined to
+    the experts' first ones or not. The result is added to what the stream holds."""
+    import parts_face as pf
+    import plain_zokunex as pz
+    g = torch.Generator().manual_seed(11)
+    w = {"router": _randn(g, experts + identity, D, std=0.4, dtype=dtype).double(), "correction": _randn(g, experts + identity, std=0.1).double()}
+    for e in range(experts):
+        w[f"e{e}.up"] = _randn(g, ff, D, std=0.15, dtype=dtype).double()
+        w[f"e{e}.down"] = _randn(g, D, ff, std=0.15, dtype=dtype).double()
+    both = torch.cat([w[f"e{e}.up"] for e in range(experts)] + [w["router"]], dim=0).to(dtype).to(DEV).contiguous()
+    down = torch.cat([w[f"e{e}.down"] for e in range(experts)], dim=1).to(dtype).to(DEV).contiguous()
+    params = pf.Params(dtype=pf.DT[dtype], experts=experts, identity=identity, ff=ff, top=top, activation="gelu_erf", up__weight=both[:experts * ff],
+                       router=both[experts * ff:], down__weight=down, correction=w["correction"].float().to(DEV))
+    if joined:
+        params.set("up_router.weight", both)
+    part = pf.FeedForward("routed_experts", params)
+    h = torch.randn(T, D, generator=g).to(dtype)
+    x0 = torch.randn(T, D, generator=g)
+    x = part.forward(h.to(DEV), x0.clone().to(DEV))
+    ref = x0.double() + pz.routed_experts(h.double(), w, "", {"router": {"experts": experts, "identity": identity, "top": top}})
+    err = (x.cpu().double() - ref).abs().amax(dim=1)
+    # (a close call may fall either way by the rounding of the router's product)
+    choice = (pz.router_scores(h.double(), w, "") + w["correction"]).sort(dim=-1, descending=True).values
+    keep = torch.ones(T, dtype=torch.bool) if top >= experts + identity else (choice[:, top - 1] - choice[:, top]) > (1e-5 if dtype == torch.float32 else 2e-4)
+    assert keep.float().mean() > 0.5
+    assert err[keep].max() <= TOL[dtype] * (6 if dtype == torch.bfloat16 else 2), err[keep].max()
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

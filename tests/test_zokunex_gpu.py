@@ -41,7 +41,7 @@ def _families(reqs, seed):
 
 
 SINGLE = ["ONLY_MEMORY", "ONLY_MEMORY_SQUARE", "ONLY_MEMORY_ODD", "ONLY_MEMORY_TILES", "ONLY_MEMORY_SHARED", "ONLY_MEMORY_WIDE",
-          "ONLY_MEMORY_WIDE_ODD", "ONLY_MEMORY_UNALIGNED_KEYS", "ONLY_LATENT", "ONLY_LATENT_NO_TURN", "ONLY_LATENT_TURN_ONLY_LITTLE",
+          "ONLY_MEMORY_WIDE_ODD", "ONLY_MEMORY_UNALIGNED_KEYS", "ONLY_MEMORY_BROAD", "ONLY_LATENT", "ONLY_LATENT_NO_TURN", "ONLY_LATENT_TURN_ONLY_LITTLE",
           "ONLY_LATENT_ONE_HEAD", "ONLY_LATENT_MANY", "ONLY_DENSE", "ONLY_EXPERTS", "EXPERTS_ALL", "EXPERTS_NO_IDENTITY", "ONE_EXPERT",
           "MOSTLY_IDENTITY", "TOP_ONE"]
 

@@ -53,6 +53,7 @@ ONLY_MEMORY_SHARED = model([mlstm(heads=2, dim=160, vdim=256)], width=32)       
 ONLY_MEMORY_WIDE = model([mlstm(heads=1, dim=72, vdim=576)], width=32)                                      # more value tiles than one workgroup takes
 ONLY_MEMORY_WIDE_ODD = model([mlstm(heads=1, dim=9, vdim=331)], width=24)                                   # wide and unaligned
 ONLY_MEMORY_UNALIGNED_KEYS = model([mlstm(heads=1, dim=10, vdim=300)], width=24)                            # aligned values beside unaligned keys
+ONLY_MEMORY_BROAD = model([mlstm(heads=1, dim=8, vdim=8)], width=2056, vocab=64)                              # a stream wider than the norms keep in registers
 ONLY_LATENT = model([latent()])
 ONLY_LATENT_NO_TURN = model([latent(heads=3, dim=24, rot_dim=0, vdim=8, kv_rank=20)], width=48)
 ONLY_LATENT_TURN_ONLY_LITTLE = model([latent(heads=2, dim=40, rot_dim=2, vdim=16, kv_rank=72, base=30.0)], width=32)
