@@ -24,6 +24,7 @@ void register_builtin_architectures() {
         register_viladra();
         register_sunulorn();
         register_zokunex();
+        register_gisedra();
         if (const char* env = std::getenv("MINI_LLM_PLUGINS")) {
             std::stringstream ss(env);
             for (std::string path; std::getline(ss, path, ':');)

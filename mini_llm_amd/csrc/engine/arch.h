@@ -51,8 +51,9 @@ void register_gpt2();              // gpt2.cc
 void register_kugulorn();          // kugulorn.cc
 void register_rekirax();           // rekirax.cc
 void register_viladra();           // viladra.cc
-void register_sunulorn();
-void register_zokunex();          // sunulorn.cc
+void register_sunulorn();          // sunulorn.cc
+void register_zokunex();           // zokunex.cc
+void register_gisedra();           // gisedra.cc
 // Loads a shared library whose initialisers register parts and architectures (dlopen; stays loaded).
 // Also called for every path in the environment variable MINI_LLM_PLUGINS (colon-separated), once.
 void load_plugin(const std::string& path);

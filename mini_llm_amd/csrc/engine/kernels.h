@@ -7,12 +7,14 @@
 #include <stddef.h>
 
 #include "score_shape.h"
+#include "tanh_norm.h"
 
 extern "C" {
 
 // elementwise.hip
 int mllm_embed(const int* ids, const int* pos, const void* wte, const void* wpe, float* x, int T, int D,
-               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale = 1.f, void* copy_bf16 = nullptr);
+               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale = 1.f, void* copy_bf16 = nullptr,
+               MllmTanhNorm next = MllmTanhNorm{nullptr, nullptr, nullptr});
 int mllm_cast_bf16(const float* x, void* out, size_t n, hipStream_t stream);
 int mllm_depth_mix(float* x, float* kept, size_t stride, int n_old, const float* w, size_t n, hipStream_t stream);
 int mllm_select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream);
@@ -125,7 +127,7 @@ int mllm_latent_expand(const void* o_lat, int ldo, const void* w_uv, int ldw, vo
 int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, int T, int H, int G, int d, int dv,
                     int norm_mode, const float* wq, const float* wk, float eps, int rot_dims, double rot_base,
                     const int* positions, const int* slots, void* q_out, int ldq, void* k_pages, void* v_pages, int dtype,
-                    hipStream_t stream, int interleaved = 0);
+                    hipStream_t stream, int interleaved = 0, const float* rot_freqs = nullptr);
 int mllm_scored_attention_rows(const void* q, int ldq, const void* k_pages, const void* v_pages, const int* block_tables,
                                int max_blocks, const int* token_seq, const int* positions, int n_tokens, int H, int G, int d,
                                int dv, int page_size, float scale, float softcap, int window, int chunk, const float* r1,
@@ -170,8 +172,14 @@ int mllm_moe_act(const void* up, int ldu, const float* logits, int ldl, int E, i
                  const float* correction = nullptr, int identity = 0, const void* h = nullptr, int ldh = 0, int D = 0, float* y = nullptr,
                  int ldy = 0, int y_add = 0);
 int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int E, int ff, int shared_ff, int top, float scale,
-                     int sigmoid_router, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
-                     int ldo, int T, int dtype, hipStream_t stream);
+                     int router_kind, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
+                     int ldo, int T, int dtype, hipStream_t stream, float up_shift = 1.f, int up_dtype = -1);
+
+// tanh_norm.hip
+int mllm_tanh_norm(const float* x, int ldx, const int* rows, MllmTanhNorm norm, void* out, int ldo, int n, int D, int dtype, hipStream_t stream);
+int mllm_stream_add(float* x, const float* y, const float* x0, const float* step, int n, int D, MllmStreamAdd add, int precise, hipStream_t stream);
+int mllm_token_gate(const float* z, int ldz, const int* ids, const int* src, const int* prev, int n_prev, const void* table, int ldt, int col0,
+                    int dim, void* out, int ldo, int T, int dtype, hipStream_t stream);
 
 // sampling.hip
 int mllm_argmax_chunks(int V);

@@ -96,8 +96,12 @@ public:
                      hipStream_t s) const override {
         run(h, step, cache, x, write, arena, s, STORE_F32);
     }
+    void forward_through(NormedInput& h, const StepView& step, const CacheView& cache, const StreamAdd& add, bool write, Arena& arena,
+                         hipStream_t s) const override {
+        run(h, step, cache, add.x, write, arena, s, STORE_F32, &add);
+    }
     void run(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
-             hipStream_t s, int out_epilogue) const {
+             hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
         const int E = sh_.kv_rank + sh_.rot_dim, T = step.n_tokens, g = cache.group, H = sh_.n_heads;
         if (!cache.has_pages() || cache.k_pages.cols != E) fail("latent_attention needs pages of %d-wide rows", E);
         if (write && !own_kv_) fail("a latent-attention layer without a key/value latent of its own cannot write a cache");
@@ -146,7 +150,7 @@ public:
         StageTimes::get().mark("attention", s);
         Tensor2 o = arena.tensor(dtype_, T, H * sh_.value_dim);
         latent_expand(o_lat, uv_, o, sh_, s, gated_ ? &gate : nullptr);
-        out_(o, x, out_epilogue, nullptr, s);
+        out_.into(o, x, out_epilogue, add, s);
         StageTimes::get().mark("out_proj", s);
     }
     size_t workspace_bytes(int tokens) const override {

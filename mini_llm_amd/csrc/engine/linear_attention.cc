@@ -68,13 +68,27 @@ public:
                      hipStream_t s) const override {
         run(h, step, cache, x, write, arena, s, STORE_F32);
     }
+    void forward_through(NormedInput& h, const StepView& step, const CacheView& cache, const StreamAdd& add, bool write, Arena& arena,
+                         hipStream_t s) const override {
+        run(h, step, cache, add.x, write, arena, s, STORE_F32, &add);
+    }
     void run(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
-             hipStream_t s, int out_epilogue) const {
-        if (!cache.has_state() || cache.state_bytes < state_floats_ * 4) fail("linear_attention needs a state of %zu floats per request", state_floats_);
-        const int T = step.n_tokens, N = in_.out_features(), ld = (N + 3) / 4 * 4, inner = H_ * dv_;
+             hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
+        const int T = step.n_tokens, N = in_.out_features(), ld = (N + 3) / 4 * 4;
         Tensor2 proj(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N, ld);
         h.linear(in_, proj, STORE_F32, nullptr, arena, s);
         StageTimes::get().mark("in_proj", s);
+        Tensor2 normed = arena.tensor(dtype_, T, H_ * dv_);
+        core(proj, step, cache, normed, write, arena, s);
+        out_.into(normed, x, out_epilogue, add, s);
+        StageTimes::get().mark("out_proj", s);
+    }
+    int core_inputs() const override { return in_.out_features(); }
+    int core_outputs() const override { return out_.in_features(); }
+    void core(const Tensor2& proj, const StepView& step, const CacheView& cache, const Tensor2& normed, bool write, Arena& arena,
+              hipStream_t s) const override {
+        if (!cache.has_state() || cache.state_bytes < state_floats_ * 4) fail("linear_attention needs a state of %zu floats per request", state_floats_);
+        const int T = step.n_tokens, inner = H_ * dv_;
         // queries and keys lie side by side: one turn over 2 * heads heads
         if (rot_dims_ > 0) rotary_rows(proj, 0, 2 * H_, d_, rot_dims_, rot_base_, step.positions, s);
         Tensor2 decay;
@@ -94,10 +108,7 @@ public:
         float* ws = ws_floats ? static_cast<float*>(arena.take(ws_floats * 4)) : nullptr;
         decay_scan(proj, 0, k_col_, v_col_, rank_ > 0 ? &decay : nullptr, head_decay_, q_scale_, k_scale_, st, 0, H_, d_, dv_, y, ws, ws_floats, s);
         StageTimes::get().mark("scan", s);
-        Tensor2 normed = arena.tensor(dtype_, T, inner);
         rmsnorm_gate_after(y, norm_, eps_, H_, proj, g_col_, normed, s, parts, static_cast<size_t>(T) * inner);
-        out_(normed, x, out_epilogue, nullptr, s);
-        StageTimes::get().mark("out_proj", s);
     }
     size_t workspace_bytes(int tokens) const override {
         return static_cast<size_t>(tokens) * ((in_.out_features() + 4) * 4 + (rank_ > 0 ? H_ * d_ * 4 : 0) + hgrn2_parts(d_) * H_ * dv_ * 4 +
@@ -149,8 +160,12 @@ private:
 // With the activation "gelu_erf" an expert is W_down gelu(W_up h) (exact GELU); with the tensor "correction" ([experts +
 // identity]) the experts with the largest score + correction are chosen, weighed by the score alone; with `identity` the
 // router has that many more rows (behind the experts'), and those experts hand on their input h: y = ... + sum w_e h. (These
-// three go with softmax scores and ungated experts.) With the tensor "up_router.weight" (up.weight's rows and behind them
-// the router's, one allocation) steps of few rows run both products as one with fp32 results.
+// three go with softmax scores and ungated experts.)
+// The activation "silu_glu" is the gated one without clamps and shift, W_down (silu(W_gate h) (W_up h)). The router
+// "softmax_chosen" (gated experts) takes the softmax over the chosen experts' logits alone; with "router.bias" ([experts] fp32)
+// the logits are W_r h + bias. With the tensor "up_router.weight" (up.weight's rows and behind them
+// the router's, one allocation) steps of few rows run both products as one with fp32 results (gated experts: [gate | up] rows; with a router bias also
+// "up_router.bias", zeros in front of it).
 // Parameters: dtype, experts, ff (an expert's hidden width), top, scale, strings activation, router (softmax);
 // clamped_glu: limit, shared_limit, alpha, weight_on_input, shared_gate; others: identity; tensors router [experts (+ 1 |
 // + identity), width],
@@ -162,29 +177,32 @@ public:
         glu_.experts = E_ = p.integer("experts"); glu_.ff = ff_ = p.integer("ff"); glu_.top = top_ = p.integer("top");
         glu_.scale = scale_ = static_cast<float>(p.number("scale", 1.0));
         const std::string& act = p.string("activation");
-        if (act == "clamped_glu") gated_ = true;
+        if (act == "clamped_glu" || act == "silu_glu") gated_ = true;
         else if (act == "gelu_erf") opt_.activation = GELU_ERF;
-        else if (act != "relu2") fail("routed_experts: unknown activation '%s' (known: relu2, gelu_erf, clamped_glu)", act.c_str());
+        else if (act != "relu2") fail("routed_experts: unknown activation '%s' (known: relu2, gelu_erf, clamped_glu, silu_glu)", act.c_str());
         opt_.identity = static_cast<int>(p.number("identity", 0));
         if (p.str.count("router")) {
             const std::string& r = p.string("router");
-            if (r == "sigmoid") glu_.sigmoid_router = true;
-            else if (r != "softmax") fail("routed_experts: unknown router '%s' (known: softmax, sigmoid)", r.c_str());
+            if (r == "sigmoid") glu_.router = ROUTER_SIGMOID;
+            else if (r == "softmax_chosen") glu_.router = ROUTER_SOFTMAX_CHOSEN;
+            else if (r != "softmax") fail("routed_experts: unknown router '%s' (known: softmax, sigmoid, softmax_chosen)", r.c_str());
         }
-        if (glu_.sigmoid_router && !gated_) fail("routed_experts: sigmoid scores go with the clamped_glu activation");
+        if (glu_.router != ROUTER_SOFTMAX && !gated_) fail("routed_experts: sigmoid scores and a softmax over the chosen go with gated experts");
         up_ = Linear(p.weights("up.weight"), nullptr);
         down_ = Linear(p.weights("down.weight"), nullptr);
-        router_ = Linear(p.weights("router"), nullptr);
+        router_ = Linear(p.weights("router"), p.weights_or_null("router.bias"));
         if (E_ < 1 || ff_ < 1 || top_ < 1 || opt_.identity < 0 || top_ > E_ + opt_.identity) fail("routed_experts: %d of %d experts of %d do not fit", top_, E_ + opt_.identity, ff_);
         if (p.weights_or_null("correction") != nullptr) opt_.correction = f32_vector(p, "correction", E_ + opt_.identity, "routed_experts");
         if (gated_ && (opt_.identity > 0 || opt_.correction != nullptr)) fail("routed_experts: identity experts and a correction go with ungated experts");
         if (gated_) {
-            glu_.limit = static_cast<float>(p.number("limit"));
+            const bool clamped = act == "clamped_glu";
+            glu_.limit = clamped ? static_cast<float>(p.number("limit")) : INFINITY;
+            glu_.up_shift = clamped ? 1.f : 0.f;
             glu_.alpha = static_cast<float>(p.number("alpha", 1.0));
             glu_.weight_on_input = p.number("weight_on_input", 0) != 0;
             glu_.shared_gate = p.number("shared_gate", 0) != 0;
             glu_.shared_ff = down_.in_features() - E_ * ff_;
-            glu_.shared_limit = glu_.shared_ff > 0 ? static_cast<float>(p.number("shared_limit")) : 0.f;
+            glu_.shared_limit = !clamped ? INFINITY : glu_.shared_ff > 0 ? static_cast<float>(p.number("shared_limit")) : 0.f;
             if (!(glu_.limit > 0.f) || (glu_.shared_ff > 0 && !(glu_.shared_limit > 0.f))) fail("routed_experts: the limits must be positive");
             if (glu_.shared_ff < 0 || up_.out_features() != 2 * down_.in_features() || (glu_.shared_gate && glu_.shared_ff == 0))
                 fail("routed_experts: the joined products' shapes do not fit %d gated experts of %d", E_, ff_);
@@ -195,9 +213,9 @@ public:
         if (router_.out_features() != routes || router_.in_features() != up_.in_features())
             fail("routed_experts: the router must be [%d, %d]", routes, up_.in_features());
         if (p.weights_or_null("up_router.weight") != nullptr) {
-            up_router_ = Linear(p.weights("up_router.weight"), nullptr);
-            if (gated_ || up_router_.out_features() != up_.out_features() + routes || up_router_.in_features() != up_.in_features())
-                fail("routed_experts: 'up_router.weight' must hold up.weight's rows and the router's (ungated experts)");
+            up_router_ = Linear(p.weights("up_router.weight"), p.weights_or_null("up_router.bias"));
+            if ((up_router_.bias != nullptr) != (router_.bias != nullptr) || up_router_.out_features() != up_.out_features() + routes || up_router_.in_features() != up_.in_features())
+                fail("routed_experts: 'up_router.weight' must hold up.weight's rows and the router's, and have a bias if the router has one");
         }
         if (down_.out_features() != up_.in_features()) fail("routed_experts: the second products must lead back to the width");
     }
@@ -207,11 +225,15 @@ public:
     void forward_set(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const override {
         run(h, step, x, arena, s, STORE_F32);
     }
-    void run(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue) const {
+    void forward_through(NormedInput& h, const StepView& step, const StreamAdd& add, Arena& arena, hipStream_t s) const override {
+        if (opt_.identity > 0) { FeedForward::forward_through(h, step, add, arena, s); return; }
+        run(h, step, add.x, arena, s, STORE_F32, &add);
+    }
+    void run(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
         Pending p;
         first_products(h, step, arena, s, p, false);
         if (opt_.identity > 0) p.h = h.tensor(arena, s);
-        rest(p, step, x, arena, s, out_epilogue);
+        rest(p, step, x, arena, s, out_epilogue, add);
     }
     bool begin(NormedInput& h, const StepView& step, Arena& arena, hipStream_t s, Pending& pending) const override {
         // (few rows in bfloat16: each of the two products norms its input itself, and no norm kernel runs)
@@ -249,11 +271,11 @@ public:
         }
         StageTimes::get().mark("fc1", s);
     }
-    void rest(const Pending& p, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue) const {
+    void rest(const Pending& p, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
         if (gated_) {
             Tensor2 act = arena.tensor(dtype_, step.n_tokens, down_.in_features());
             moe_glu_act(p.b, p.a, glu_, act, s);
-            down_(act, x, out_epilogue, nullptr, s);
+            down_.into(act, x, out_epilogue, add, s);
         } else {
             const Tensor2 act = p.b.dtype == dtype_ ? p.b : arena.tensor(dtype_, step.n_tokens, up_.out_features());      // in place
             MoeOptions o = opt_;
@@ -263,7 +285,7 @@ public:
                 out_epilogue = ADD_RESIDUAL;
             }
             moe_act(p.b, p.a, ff_, top_, scale_, act, nullptr, s, o);
-            down_(act, x, out_epilogue, nullptr, s);
+            down_.into(act, x, out_epilogue, add, s);
         }
         StageTimes::get().mark("fc2", s);
     }

@@ -151,7 +151,7 @@ Tuning& tuning() {
 // elementwise
 // ---------------------------------------------------------------------------------------------
 void embed(const int* ids, const int* positions, const Tensor2& wte, const Tensor2* wpe, const Tensor2& out,
-           hipStream_t stream, const FedTokens* fed, float scale, const Tensor2* copy) {
+           hipStream_t stream, const FedTokens* fed, float scale, const Tensor2* copy, const MllmTanhNorm* next) {
     need_dtype(wte, "wte");
     const int T = static_cast<int>(out.rows), D = static_cast<int>(wte.cols);
     if (!wte.contiguous()) fail("embed: wte must be contiguous");
@@ -168,7 +168,8 @@ void embed(const int* ids, const int* positions, const Tensor2& wte, const Tenso
     const bool feeds = fed != nullptr && fed->src != nullptr;
     if (feeds && (fed->prev == nullptr || fed->n_prev < 1)) fail("embed: fed tokens need the earlier step's sampled tokens");
     check(mllm_embed(ids, table ? positions : nullptr, wte.data, table, static_cast<float*>(out.data), T, D, wte.dtype,
-                     feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, stream, scale, copy ? copy->data : nullptr), "embed");
+                     feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, stream, scale, copy ? copy->data : nullptr,
+                     next ? *next : MllmTanhNorm{nullptr, nullptr, nullptr}), "embed");
 }
 
 void select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream) {

@@ -16,6 +16,7 @@
 #include <string>
 
 #include "score_shape.h"
+#include "tanh_norm.h"
 
 namespace minillm {
 
@@ -139,9 +140,10 @@ struct FedTokens {
 };
 
 // -- the ops -----------------------------------------------------------------------------------------
-// out[t, :] = scale * wte[ids[t], :] (+ wpe[positions[t], :]); `copy` (optional): the same rows in bfloat16
+// out[t, :] = scale * wte[ids[t], :] (+ wpe[positions[t], :]); `copy` (optional): the same rows in bfloat16 (behind the norm
+// `next`, if one with a weight is given)
 void embed(const int* ids, const int* positions, const Tensor2& wte, const Tensor2* wpe, const Tensor2& out,
-           hipStream_t stream, const FedTokens* fed = nullptr, float scale = 1.f, const Tensor2* copy = nullptr);
+           hipStream_t stream, const FedTokens* fed = nullptr, float scale = 1.f, const Tensor2* copy = nullptr, const MllmTanhNorm* next = nullptr);
 // out = x in bfloat16 (contiguous)
 void cast_stream(const Tensor2& x, const Tensor2& out, hipStream_t stream);
 void select_tokens(int* ids, const int* src, const int* prev, int n, int n_prev, hipStream_t stream);
@@ -303,6 +305,7 @@ struct ScoredShape {
     int rot_dims = 0;                          // the first rot_dims columns of a head are turned (half-split pairs,
     bool rot_interleaved = false;              // or with rot_interleaved column 2i with column 2i + 1)
     double rot_base = 10000.0;
+    const float* rot_freqs = nullptr;          // angle per position of every pair, two floats each whose sum it is (instead of rot_base)
     // weights without a softmax: a visible key's weight is sigmoid(score + score_bias[h]) (score_bias per head, or
     // null), not normalised over the keys
     bool sigmoid_weights = false;
@@ -403,12 +406,34 @@ void moe_act(const Tensor2& up, const Tensor2& logits, int ff, int top, float sc
              hipStream_t stream, const MoeOptions& options = MoeOptions());
 // The routed experts' activation for gated, clamped experts (kernels/moe.hip): up [T, 2 (E ff + shared_ff)] with rows
 // [expert: gate | up] ... [shared: gate | up], logits [T, E (+ 1: the shared expert's gate)] fp32, out [T, E ff + shared_ff].
+// An expert's hidden values are g sigmoid(alpha g) (u + up_shift) with g and u clamped at the limit (infinite: not clamped).
+// up may be fp32 where out is bfloat16.
+enum RouterKind : int { ROUTER_SOFTMAX = 0, ROUTER_SIGMOID = 1, ROUTER_SOFTMAX_CHOSEN = 2 };
 struct MoeGlu {
     int experts = 0, ff = 0, shared_ff = 0, top = 0;
-    float scale = 1.f, limit = 0.f, shared_limit = 0.f, alpha = 1.f;
-    bool sigmoid_router = false, weight_on_input = false, shared_gate = false;
+    float scale = 1.f, limit = 0.f, shared_limit = 0.f, alpha = 1.f, up_shift = 1.f;
+    int router = ROUTER_SOFTMAX;       // over all experts, each on its own, or over the chosen ones
+    bool weight_on_input = false, shared_gate = false;
 };
 void moe_glu_act(const Tensor2& up, const Tensor2& logits, const MoeGlu& m, const Tensor2& out, hipStream_t stream);
+
+// -- the dynamic tanh norm, things added to the stream ------------------------------------------------
+// out[i, :] = tanh(alpha x[rows ? rows[i] : i, :]) * weight + bias
+void tanh_norm(const Tensor2& x, const MllmTanhNorm& norm, const Tensor2& out, const int* rows, hipStream_t stream);
+// What a sub-layer's result does to the stream: x += norm(y) (norm.weight null: x += y); with `copy` (bfloat16, x's shape)
+// then copy = next(x), or x itself if next.weight is null. `y`: room for the result (fp32, x's shape) where it has to pass
+// through memory.
+struct StreamAdd {
+    MllmTanhNorm norm{nullptr, nullptr, nullptr}, next{nullptr, nullptr, nullptr};
+    Tensor2 x, copy, y;
+};
+// The stream's part of it, for a result that lies in add.y (null data: nothing is added but x0 and step): x += norm(y) + x0
+// + step (x0: x's shape, step: one row [columns], both optional), then the copy. `precise`: the library's tanh.
+void stream_add(const StreamAdd& add, const Tensor2* x0, const float* step, bool precise, hipStream_t stream);
+// The linear map whose result does that, inside the product where the kernels allow.
+void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, const StreamAdd& add, hipStream_t stream);
+// out[t, j] = gelu_tanh(z[t, j]) * table[id of token t, col0 + j] (z fp32; fed tokens as for embed)
+void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Tensor2& table, int col0, const Tensor2& out, hipStream_t stream);
 
 // out = [a | b] row by row in out's dtype (a, b fp32 [T, D])
 void concat_cast(const Tensor2& a, const Tensor2& b, const Tensor2& out, hipStream_t stream);

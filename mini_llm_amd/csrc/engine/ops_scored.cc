@@ -123,7 +123,7 @@ void qk_prepare(const Tensor2& proj, int q_col, int k_col, int v_col, const Scor
         if (sh.norm_mode == 2) fail("qk_prepare: a norm over the whole row needs the keys");
         check(mllm_qk_prepare(static_cast<const float*>(proj.data), i32(proj.stride), q_col, 0, 0, i32(proj.rows), sh.n_heads, 0,
                               sh.dim, sh.value_dim, sh.norm_mode, sh.q_norm, sh.q_norm, sh.eps, sh.rot_dims, sh.rot_base, positions, nullptr, q.data,
-                              i32(q.stride), nullptr, nullptr, q.dtype, stream, sh.rot_interleaved ? 1 : 0), "qk_prepare");
+                              i32(q.stride), nullptr, nullptr, q.dtype, stream, sh.rot_interleaved ? 1 : 0, sh.rot_freqs), "qk_prepare");
         return;
     }
     if (k_pages.dtype != q.dtype || v_pages.dtype != q.dtype || !k_pages.contiguous() || !v_pages.contiguous() || k_pages.cols != nk ||
@@ -136,7 +136,7 @@ void qk_prepare(const Tensor2& proj, int q_col, int k_col, int v_col, const Scor
         fail("qk_prepare: %d turned columns of %d (even, at most the head) and a positive base are needed", sh.rot_dims, sh.dim);
     check(mllm_qk_prepare(static_cast<const float*>(proj.data), i32(proj.stride), q_col, k_col, v_col, i32(proj.rows), sh.n_heads, sh.n_kv_heads,
                           sh.dim, sh.value_dim, sh.norm_mode, sh.q_norm, sh.k_norm, sh.eps, sh.rot_dims, sh.rot_base, positions, slots, q.data,
-                          i32(q.stride), k_pages.data, v_pages.data, q.dtype, stream, sh.rot_interleaved ? 1 : 0), "qk_prepare");
+                          i32(q.stride), k_pages.data, v_pages.data, q.dtype, stream, sh.rot_interleaved ? 1 : 0, sh.rot_freqs), "qk_prepare");
 }
 
 void scored_attention(const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, const ScoredStep& step,
@@ -329,12 +329,65 @@ void moe_glu_act(const Tensor2& up, const Tensor2& logits, const MoeGlu& m, cons
     need_f32(logits, "moe_glu_act: the router's logits");
     const int64_t n = static_cast<int64_t>(m.experts) * m.ff + m.shared_ff;
     if (m.experts < 1 || m.ff < 1 || m.shared_ff < 0 || m.top < 1 || m.top > m.experts) fail("moe_glu_act: %d of %d experts of %d do not fit", m.top, m.experts, m.ff);
-    if (out.dtype != up.dtype || out.rows != up.rows || out.cols != n || up.cols != 2 * n) fail("moe_glu_act: up must be [T, %lld] and out [T, %lld], of one dtype", (long long)(2 * n), (long long)n);
+    if ((out.dtype != up.dtype && up.dtype != F32) || out.rows != up.rows || out.cols != n || up.cols != 2 * n) fail("moe_glu_act: up must be [T, %lld] and out [T, %lld], of one dtype", (long long)(2 * n), (long long)n);
     if (logits.rows != up.rows || logits.cols != m.experts + (m.shared_gate ? 1 : 0)) fail("moe_glu_act: the logits must be [T, %d]", m.experts + (m.shared_gate ? 1 : 0));
     if (out.data == up.data) fail("moe_glu_act: out must not be up");
     check(mllm_moe_glu_act(up.data, i32(up.stride), static_cast<const float*>(logits.data), i32(logits.stride), m.experts, m.ff, m.shared_ff, m.top,
-                           m.scale, m.sigmoid_router ? 1 : 0, m.limit, m.shared_limit, m.alpha, m.weight_on_input ? 1 : 0, m.shared_gate ? 1 : 0,
-                           out.data, i32(out.stride), i32(up.rows), up.dtype, stream), "moe_glu_act");
+                           m.scale, m.router, m.limit, m.shared_limit, m.alpha, m.weight_on_input ? 1 : 0, m.shared_gate ? 1 : 0,
+                           out.data, i32(out.stride), i32(up.rows), out.dtype, stream, m.up_shift, up.dtype), "moe_glu_act");
+}
+
+namespace {
+void check_norm(const MllmTanhNorm& n, const char* what) {
+    if (n.weight != nullptr && (n.alpha == nullptr || n.bias == nullptr)) fail("%s: a tanh norm needs its three tensors", what);
+}
+void check_stream_add(const StreamAdd& add, const char* what) {
+    need_f32(add.x, what);
+    if (!add.x.contiguous()) fail("%s: the stream must be contiguous", what);
+    check_norm(add.norm, what);
+    check_norm(add.next, what);
+    if (add.copy.data != nullptr && (add.copy.dtype != BF16 || add.copy.rows != add.x.rows || add.copy.cols != add.x.cols))
+        fail("%s: the copy must be bfloat16 of the stream's shape", what);
+    if (add.y.data != nullptr && (add.y.dtype != F32 || !add.y.contiguous() || add.y.rows != add.x.rows || add.y.cols != add.x.cols))
+        fail("%s: the result must be contiguous float32 of the stream's shape", what);
+}
+MllmStreamAdd kernel_side(const StreamAdd& add) { return MllmStreamAdd{add.norm, add.next, add.copy.data, i32(add.copy.stride)}; }
+}  // namespace
+
+void tanh_norm(const Tensor2& x, const MllmTanhNorm& norm, const Tensor2& out, const int* rows, hipStream_t stream) {
+    need_f32(x, "tanh_norm: x");
+    need_act(out, "tanh_norm: out");
+    check_norm(norm, "tanh_norm");
+    if (norm.weight == nullptr) fail("tanh_norm: the weight is missing");
+    if (out.cols != x.cols || (rows == nullptr && out.rows != x.rows)) fail("tanh_norm: out must have the input's columns (and rows)");
+    check(mllm_tanh_norm(static_cast<const float*>(x.data), i32(x.stride), rows, norm, out.data, i32(out.stride), i32(out.rows), i32(out.cols), out.dtype,
+                         stream), "tanh_norm");
+}
+
+void stream_add(const StreamAdd& add, const Tensor2* x0, const float* step, bool precise, hipStream_t stream) {
+    check_stream_add(add, "stream_add");
+    if (x0 != nullptr && (x0->dtype != F32 || !x0->contiguous() || x0->rows != add.x.rows || x0->cols != add.x.cols)) fail("stream_add: x0 must have the stream's shape");
+    check(mllm_stream_add(static_cast<float*>(add.x.data), static_cast<const float*>(add.y.data), x0 ? static_cast<const float*>(x0->data) : nullptr, step,
+                          i32(add.x.rows), i32(add.x.cols), kernel_side(add), precise ? 1 : 0, stream), "stream_add");
+}
+
+void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, const StreamAdd& add, hipStream_t stream) {
+    check_stream_add(add, "linear_stream_add");
+    if (add.y.data == nullptr) fail("linear_stream_add: room for the result is needed");
+    linear(a, w, bias, add.y, STORE_F32, nullptr, stream);
+    stream_add(add, nullptr, nullptr, a.dtype == F32, stream);
+}
+
+void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Tensor2& table, int col0, const Tensor2& out, hipStream_t stream) {
+    need_f32(z, "token_gate: z");
+    need_act(table, "token_gate: the table");
+    if (out.dtype != table.dtype || out.rows != z.rows || out.cols != z.cols) fail("token_gate: out must have z's shape and the table's dtype");
+    if (col0 < 0 || col0 + z.cols > table.cols || ids == nullptr) fail("token_gate: columns %d.. of a table of %lld", col0, (long long)table.cols);
+    const bool feeds = fed != nullptr && fed->src != nullptr;
+    if (feeds && (fed->prev == nullptr || fed->n_prev < 1)) fail("token_gate: fed tokens need the earlier step's sampled tokens");
+    check(mllm_token_gate(static_cast<const float*>(z.data), i32(z.stride), ids, feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr,
+                          feeds ? fed->n_prev : 0, table.data, i32(table.stride), col0, i32(z.cols), out.data, i32(out.stride), i32(z.rows), out.dtype,
+                          stream), "token_gate");
 }
 
 void concat_cast(const Tensor2& a, const Tensor2& b, const Tensor2& out, hipStream_t stream) {

@@ -428,7 +428,7 @@ public:
     int hidden_size() const override { return static_cast<int>(table_.cols); }
     void forward(const StepView& step, const PositionEncoding* position, const Tensor2& x, hipStream_t s) const override {
         embed(step.token_ids, step.positions, table_, position ? position->table() : nullptr, x, s, &step.fed, scale_,
-              step.stream_copy.data != nullptr ? &step.stream_copy : nullptr);
+              step.leave.wanted ? &step.stream_copy : nullptr, step.leave.wanted ? &step.leave.norm : nullptr);
     }
     bool resolves_fed_tokens() const override { return true; }
     bool writes_stream_copy() const override { return true; }
@@ -513,6 +513,7 @@ void register_builtin_parts() {
     register_recurrent_parts();
     register_linear_attention_parts();
     register_matrix_memory();
+    register_tanh_norm_parts();
 }
 }  // namespace
 
@@ -687,8 +688,20 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         with_rows.stream_copy = arena.tensor(BF16, step.n_tokens, hidden_size());
         break;
     }
+    // What the block of call i finds in the copy as it is entered, and what is in it now. Whoever runs in front of a block
+    // is told (StepView::leave) and leaves it if it can; otherwise it is made here.
+    using Leave = StepView::Leave;
+    auto wanted_by = [&](size_t i, bool behind_its_step) {
+        Leave w;
+        if (i >= order.size() || (order[i].before >= 0 && !behind_its_step)) return w;
+        const Block& b = *layers[order[i].layer];
+        w.wanted = b.wants_stream_copy();
+        if (w.wanted) b.entry_norm(w.norm);
+        return w;
+    };
+    with_rows.leave = wanted_by(0, false);
     embedding->forward(with_rows, position.get(), x, s);
-    bool copied = embedding->writes_stream_copy();      // whether the copy, if there is one, equals the stream
+    Leave have = embedding->writes_stream_copy() ? with_rows.leave : Leave();
     // a stream step that mixes the embedding's output back in later: a copy of it stays for the step
     // (with room behind it for the streams that a stream step keeps for itself during the step)
     Tensor2 x0, x0_and_kept;
@@ -710,29 +723,39 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         with_rows.zeroed_rows = static_cast<float*>(z.data);
         break;
     }
-    for (const LayerCall& c : order) {
+    for (size_t i = 0; i < order.size(); ++i) {
+        const LayerCall& c = order[i];
         if (c.cache >= static_cast<int>(caches.size()))
             fail("the execution order names cache %d, the step brings %zu caches", c.cache, caches.size());
         times.set_layer(c.layer);
+        auto stream_step = [&](int which, int pass, const char* stage) {
+            const size_t mark = arena.mark();
+            const StreamStep& st = *stream_steps[which];
+            st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, pass, with_rows, arena, s);
+            arena.release(mark);
+            have = st.leaves_copy() ? with_rows.leave : Leave();
+            times.mark(stage, s);
+        };
+        const Leave enters = wanted_by(i, true);
         if (c.before >= 0) {
-            const size_t mark = arena.mark();
-            const StreamStep& st = *stream_steps[c.before];
-            st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, c.pass, with_rows, arena, s);
-            arena.release(mark);
-            copied = false;
-            times.mark("stream_step", s);
+            with_rows.leave = enters;
+            stream_step(c.before, c.pass, "stream_step");
         }
-        const bool reads_copy = layers[c.layer]->wants_stream_copy();
-        if (reads_copy && !copied) cast_stream(x, with_rows.stream_copy, s);
-        copied = reads_copy;                            // such a block keeps it, any other changes the stream alone
-        layers[c.layer]->forward(x, with_rows, caches[c.cache], c.write, arena, s);
+        if (enters.wanted && !have.same(enters)) {
+            if (enters.norm.weight != nullptr) tanh_norm(x, enters.norm, with_rows.stream_copy, nullptr, s);
+            else cast_stream(x, with_rows.stream_copy, s);
+        }
+        const Block& b = *layers[c.layer];
+        with_rows.leave = c.after >= 0 ? Leave() : wanted_by(i + 1, false);
+        b.forward(x, with_rows, caches[c.cache], c.write, arena, s);
+        // (a block that keeps a copy of the stream itself keeps it whether it is asked or not)
+        const bool normed = with_rows.leave.norm.weight != nullptr;
+        have = Leave();
+        if (b.leaves_copy(normed)) have = with_rows.leave;
+        if (b.leaves_copy(false) && !b.leaves_copy(true)) { have = Leave(); have.wanted = true; }
         if (c.after >= 0) {
-            const size_t mark = arena.mark();
-            const StreamStep& st = *stream_steps[c.after];
-            st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, c.after_pass, with_rows, arena, s);
-            arena.release(mark);
-            copied = false;
-            times.mark("stream_step_after", s);
+            with_rows.leave = wanted_by(i + 1, false);
+            stream_step(c.after, c.after_pass, "stream_step_after");
         }
     }
     times.set_layer(-1);

@@ -96,7 +96,13 @@ struct StepView {
     float* zeroed_rows = nullptr;      // fp32 [n_tokens, hidden], all zero, if a layer asked for it (Block::wants_zeroed_rows):
                                        // room for a sub-layer's result; whoever uses it leaves it zero again
     Tensor2 stream_copy;               // the stream in bfloat16 as a block is entered, if a block asked for it
-                                       // (Block::wants_stream_copy)
+                                       // (Block::wants_stream_copy): the stream itself, or the block's entry norm of it
+    // What the part that runs now is asked to leave in stream_copy for the block behind it (parts that can: leaves_copy).
+    struct Leave {
+        bool wanted = false;
+        MllmTanhNorm norm{nullptr, nullptr, nullptr};      // weight null: the stream itself
+        bool same(const Leave& o) const { return wanted == o.wanted && norm.weight == o.norm.weight; }
+    } leave;
     int n_groups = 0;
     const int* const* block_tables = nullptr;   // per group [B, max_blocks[g]]
     const int* max_blocks = nullptr;            // per group
@@ -164,6 +170,11 @@ public:
     const float* bias = nullptr;
     int in_features() const { return static_cast<int>(weight.cols); }
     int out_features() const { return static_cast<int>(weight.rows); }
+    // The same with the result put where a sub-layer's belongs: into `x` by `epilogue`, or (add given) through it.
+    void into(const Tensor2& a, const Tensor2& x, int epilogue, const StreamAdd* add, hipStream_t s) const {
+        if (add != nullptr) linear_stream_add(a, weight, bias, *add, s);
+        else linear(a, weight, bias, x, epilogue, nullptr, s);
+    }
     void add_cost(StepCost& c) const {
         c.weight_bytes += static_cast<double>(weight.rows) * weight.cols * weight.esz() + (bias ? 4.0 * weight.rows : 0.0);
         c.flops_per_token += 2.0 * weight.rows * weight.cols;
@@ -197,7 +208,7 @@ public:
     // true: forward() takes `step.fed` into account itself (one kernel fewer in a decode step); false: the runner
     // writes the fed ids into token_ids with a kernel of its own before the step
     virtual bool resolves_fed_tokens() const { return false; }
-    // true: forward() also writes step.stream_copy where it is there; false: the model casts the stream behind it
+    // true: forward() also writes step.stream_copy as step.leave asks; false: the model makes it behind it
     virtual bool writes_stream_copy() const { return false; }
     virtual void add_cost(StepCost&) const {}
 };
@@ -233,6 +244,9 @@ public:
     // behind a sub-layer; a norm without it refuses.
     virtual void add_scaled(const Tensor2& y, const float* scale, float mult, const Tensor2& x, bool clear,
                             hipStream_t s, const Tensor2* copy = nullptr) const;
+    // True: the norm has no statistics (every value of a row on its own) and `n` is it: what makes or reads the row's
+    // values can apply it in passing.
+    virtual bool pointwise(MllmTanhNorm& n) const { (void)n; return false; }
     virtual size_t workspace_bytes(int rows) const = 0;
     virtual void add_cost(StepCost&) const {}
     int dtype = BF16;
@@ -266,6 +280,23 @@ public:
         fill_zero(x, s);
         forward(h, step, cache, x, write, arena, s);
     }
+    // The same with the output taken into the stream by `add` (a norm without statistics behind the mixer, the next
+    // sub-layer's input): a mixer that ends in a product lets the product do it.
+    virtual void forward_through(NormedInput& h, const StepView& step, const CacheView& cache, const StreamAdd& add, bool write,
+                                 Arena& arena, hipStream_t s) const {
+        forward_set(h, step, cache, add.y, write, arena, s);
+        stream_add(add, nullptr, nullptr, add.copy.data == nullptr, s);
+    }
+    // A mixer between two products, for mixers side by side that share them: core() turns the input projection's fp32 rows
+    // (`proj`, core_inputs() columns) into the rows in front of its output projection (`o`, core_outputs() columns, the
+    // compute dtype). 0 inputs: the mixer has no such middle.
+    virtual int core_inputs() const { return 0; }
+    virtual int core_outputs() const { return 0; }
+    virtual void core(const Tensor2& proj, const StepView& step, const CacheView& cache, const Tensor2& o, bool write, Arena& arena,
+                      hipStream_t s) const {
+        (void)proj; (void)step; (void)cache; (void)o; (void)write; (void)arena; (void)s;
+        fail("this kind of mixer cannot share its products with another");
+    }
     virtual size_t workspace_bytes(int tokens) const = 0;
     virtual CacheNeed cache_need() const = 0;
     // Scratch that the mixer's kernels need on stream `s` for steps of up to max_seqs sequences: taken
@@ -283,6 +314,11 @@ public:
     virtual void forward_set(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s) const {
         fill_zero(x, s);
         forward(h, step, x, arena, s);
+    }
+    // The same with the result taken into the stream by `add`, as for mixers.
+    virtual void forward_through(NormedInput& h, const StepView& step, const StreamAdd& add, Arena& arena, hipStream_t s) const {
+        forward_set(h, step, add.y, arena, s);
+        stream_add(add, nullptr, nullptr, add.copy.data == nullptr, s);
     }
     // The same in two halves, for an arrangement whose sub-layers read ONE stream: begin() does everything that reads
     // the input (the first products, with the norm inside them where the kernels allow) and leaves what it made in the
@@ -315,6 +351,10 @@ public:
     // true: the block's sub-layers read the stream itself, in bfloat16: the model keeps a copy of it for the step
     // (StepView::stream_copy), and the block leaves the copy equal to the stream it leaves
     virtual bool wants_stream_copy() const { return false; }
+    // with wants_stream_copy: true and the norm if the copy is to be the block's first norm of the stream
+    virtual bool entry_norm(MllmTanhNorm& n) const { (void)n; return false; }
+    // true: the block leaves in the copy what StepView::leave asks for (the stream's norm, or the stream itself)
+    virtual bool leaves_copy(bool normed) const { return wants_stream_copy() && !normed; }
     virtual void reserve(int max_seqs, hipStream_t s) const = 0;
     virtual void add_cost(StepCost&) const = 0;
 };
@@ -331,6 +371,7 @@ public:
     virtual size_t workspace_bytes(int tokens) const = 0;
     virtual bool wants_embedding_output() const { return false; }
     virtual int kept_streams() const { return 0; }         // > 0 goes with wants_embedding_output()
+    virtual bool leaves_copy() const { return false; }     // true: it leaves in the copy what StepView::leave asks for
     virtual void reserve(int max_seqs, hipStream_t s) const { (void)max_seqs; (void)s; }
     virtual void add_cost(StepCost&) const {}
 };
@@ -393,6 +434,9 @@ void register_recurrent_parts();
 // all streams so far (linear_attention.cc); the arrangement with a norm behind each sub-layer only is registered with
 // the gated parts.
 void register_linear_attention_parts();
+// The dynamic tanh norm, what is added to the stream between layers: the embedding's output with a vector per pass, a
+// token's own gated input (tanh_norm.cc).
+void register_tanh_norm_parts();
 // The matrix memory with exponential gates (matrix_memory.cc).
 void register_matrix_memory();
 

@@ -72,6 +72,9 @@ private:
 // The sub-layer adds its result into a cleared fp32 buffer of the stream's shape; the norm behind it adds
 // from there into the stream. Norms: [norm1, norm1b] or [norm1, norm1b, norm2, norm2b]; parameters:
 // "size" (the stream's width), "residual_mult" (default 1), tensors "scale1", "scale2" (optional: no scale).
+// Where all norms are without statistics (Norm::pointwise) and nothing scales the results, no norm is a pass of its own:
+// the sub-layer's last product takes its result through the norm into the stream and leaves the next sub-layer's normed
+// input beside it in bfloat16 (in the 32-bit path that input is normed as it is read).
 class SandwichNormBlock final : public Block {
 public:
     SandwichNormBlock(std::unique_ptr<Mixer> m, std::unique_ptr<FeedForward> f, std::vector<std::unique_ptr<Norm>> norms, const Params& p)
@@ -86,9 +89,39 @@ public:
         mult_ = static_cast<float>(p.number("residual_mult", 1.0));
         if (const Tensor2* t = p.weights_or_null("scale1")) scale1_ = checked_scale(*t);
         if (const Tensor2* t = p.weights_or_null("scale2")) scale2_ = checked_scale(*t);
+        pointwise_ = pre1_->pointwise(n_pre1_) && post1_->pointwise(n_post1_) && (!ff_ || (pre2_->pointwise(n_pre2_) && post2_->pointwise(n_post2_))) &&
+                     scale1_.data == nullptr && scale2_.data == nullptr && mult_ == 1.f;
+        dtype_ = pre1_->dtype;
+    }
+    void forward_pointwise(const Tensor2& x, const StepView& step, const CacheView& cache, bool write, Arena& arena, hipStream_t s) const {
+        const size_t outer = arena.mark();
+        const bool copies = dtype_ == BF16;
+        const Tensor2 none;
+        StreamAdd add;
+        add.x = x;
+        add.y = arena.tensor(F32, x.rows, x.cols);        // room for results that a product cannot add by itself
+        const size_t mark = arena.mark();
+        add.norm = n_post1_;
+        add.copy = copies && (ff_ || step.leave.wanted) ? step.stream_copy : none;
+        add.next = ff_ ? n_pre2_ : step.leave.norm;
+        {
+            NormedInput h = copies ? NormedInput(step.stream_copy) : NormedInput(*pre1_, x);
+            mixer_->forward_through(h, step, cache, add, write, arena, s);
+        }
+        arena.release(mark);
+        if (ff_) {
+            add.norm = n_post2_;
+            add.copy = copies && step.leave.wanted ? step.stream_copy : none;
+            add.next = step.leave.norm;
+            NormedInput h = copies ? NormedInput(step.stream_copy) : NormedInput(*pre2_, x);
+            ff_->forward_through(h, step, add, arena, s);
+        }
+        arena.release(outer);
     }
     void forward(const Tensor2& x, const StepView& step, const CacheView& cache, bool write, Arena& arena,
                  hipStream_t s) const override {
+        if (x.cols != size_) fail("a sandwich-norm block of width %d was handed a stream of %lld", size_, (long long)x.cols);
+        if (pointwise_) { forward_pointwise(x, step, cache, write, arena, s); return; }
         const size_t outer = arena.mark();
         // the sub-layer's result: the step's cleared buffer (left cleared again by the norms behind the
         // sub-layers), or one of this layer's own
@@ -101,7 +134,6 @@ public:
             mixer_->forward(h, step, cache, y, write, arena, s);
         }
         arena.release(mark);
-        if (x.cols != size_) fail("a sandwich-norm block of width %d was handed a stream of %lld", size_, (long long)x.cols);
         post1_->add_scaled(y, static_cast<const float*>(scale1_.data), mult_, x, shared || ff_ != nullptr, s);
         StageTimes::get().mark("post_norm", s);
         if (ff_) {
@@ -121,7 +153,10 @@ public:
         return a + static_cast<size_t>(tokens) * size_ * 4 + 1024;
     }
     CacheNeed cache_need() const override { return mixer_->cache_need(); }
-    bool wants_zeroed_rows() const override { return true; }
+    bool wants_zeroed_rows() const override { return !pointwise_; }
+    bool wants_stream_copy() const override { return pointwise_ && dtype_ == BF16; }
+    bool entry_norm(MllmTanhNorm& n) const override { if (pointwise_) n = n_pre1_; return pointwise_; }
+    bool leaves_copy(bool) const override { return wants_stream_copy(); }
     void reserve(int max_seqs, hipStream_t s) const override {
         mixer_->reserve(max_seqs, s);
         if (ff_) ff_->reserve(max_seqs, s);
@@ -143,7 +178,9 @@ private:
     std::unique_ptr<Norm> pre1_, post1_, pre2_, post2_;
     Tensor2 scale1_, scale2_;
     float mult_ = 1.f;
-    int size_ = 0;               // the stream's width
+    int size_ = 0, dtype_ = BF16;      // size: the stream's width
+    bool pointwise_ = false;
+    MllmTanhNorm n_pre1_{}, n_post1_{}, n_pre2_{}, n_post2_{};
 };
 
 

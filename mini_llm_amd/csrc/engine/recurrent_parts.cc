@@ -103,17 +103,34 @@ private:
 // buffer of the stream's shape (Mixer::forward_set). At most one of them may keep pages; their states lie one behind the
 // other in the layer's state slot. Parameters: size, eps; mixers; tensors norm0, norm1, ... and optionally
 // norms (the same weights one behind the other: the norms and the mean then run in one kernel).
+// With the tensors in.weight (the mixers' input projections one below the other) and out.weight (their output projections
+// side by side) there are no norms and the results are added as they are: x += sum_k mixer_k(h). Both products then run
+// once for all mixers, which bring what lies between (Mixer::core). dtype is then needed too.
 class ParallelMixers final : public Mixer {
 public:
     explicit ParallelMixers(const Params& p) : mixers_(p.mixers) {
         size_ = p.integer("size");
         eps_ = static_cast<float>(p.number("eps"));
         if (mixers_.size() < 2) fail("parallel mixers: at least two mixers are needed");
-        int with_pages = 0;
+        joined_ = p.weights_or_null("in.weight") != nullptr;
+        int with_pages = 0, in_cols = 0, out_cols = 0;
         for (size_t k = 0; k < mixers_.size(); ++k) {
             if (!mixers_[k]) fail("parallel mixers: mixer %zu is missing", k);
-            norms_.push_back(f32_vector(p, ("norm" + std::to_string(k)).c_str(), size_, "parallel mixers"));
             if (mixers_[k]->cache_need().kind & 1) with_pages += 1;
+            if (joined_) {
+                if (mixers_[k]->core_inputs() < 1) fail("parallel mixers: mixer %zu cannot share its products", k);
+                in_cols += mixers_[k]->core_inputs();
+                out_cols += mixers_[k]->core_outputs();
+            } else {
+                norms_.push_back(f32_vector(p, ("norm" + std::to_string(k)).c_str(), size_, "parallel mixers"));
+            }
+        }
+        if (joined_) {
+            dtype_ = p.integer("dtype");
+            in_ = Linear(p.weights("in.weight"), nullptr);
+            out_ = Linear(p.weights("out.weight"), nullptr);
+            if (in_.out_features() != in_cols || out_.in_features() != out_cols || out_.out_features() != size_)
+                fail("parallel mixers: the joined products do not fit mixers that take %d columns and make %d", in_cols, out_cols);
         }
         if (with_pages > 1) fail("parallel mixers: only one of the mixers may keep pages");
         // (the weights one behind the other in one tensor: all norms and the mean in one kernel)
@@ -123,27 +140,65 @@ public:
             joined_norms_ = static_cast<const float*>(j->data);
         }
     }
+    // What mixer k sees of the layer's cache; `state_at` moves on behind its state.
+    CacheView share_of(int k, const CacheView& cache, size_t& state_at) const {
+        const CacheNeed need = mixers_[k]->cache_need();
+        CacheView mine = cache;
+        mine.kind = 0;
+        if (need.kind & 1) {
+            if (!cache.has_pages()) fail("parallel mixers: mixer %d needs pages", k);
+            mine.kind |= 1;
+        }
+        if (need.kind & 2) {
+            if (!cache.has_state() || cache.state_bytes < state_at + need.state_bytes) fail("parallel mixers: mixer %d needs %zu bytes of state", k, need.state_bytes);
+            mine.kind |= 2;
+            mine.state = static_cast<char*>(cache.state) + state_at;
+            mine.state_bytes = need.state_bytes;
+            state_at += (need.state_bytes + 15) / 16 * 16;
+        }
+        return mine;
+    }
+    void run_joined(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
+                    hipStream_t s, int out_epilogue, const StreamAdd* add) const {
+        const int T = step.n_tokens, N = in_.out_features(), ld = (N + 3) / 4 * 4, K = out_.in_features();
+        const Tensor2 proj(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N, ld);
+        h.linear(in_, proj, STORE_F32, nullptr, arena, s);
+        StageTimes::get().mark("in_proj", s);
+        const Tensor2 o = arena.tensor(dtype_, T, K);
+        size_t state_at = 0;
+        int col = 0, o_col = 0;
+        for (int k = 0; k < static_cast<int>(mixers_.size()); ++k) {
+            const CacheView mine = share_of(k, cache, state_at);
+            const int n_in = mixers_[k]->core_inputs(), n_out = mixers_[k]->core_outputs();
+            const size_t mark = arena.mark();
+            mixers_[k]->core(Tensor2(static_cast<float*>(proj.data) + col, F32, T, n_in, ld), step, mine,
+                             Tensor2(static_cast<char*>(o.data) + static_cast<size_t>(o_col) * o.esz(), dtype_, T, n_out, K), write, arena, s);
+            arena.release(mark);
+            col += n_in;
+            o_col += n_out;
+        }
+        out_.into(o, x, out_epilogue, add, s);
+        StageTimes::get().mark("out_proj", s);
+    }
+    void forward_set(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
+                     hipStream_t s) const override {
+        if (joined_) run_joined(h, step, cache, x, write, arena, s, STORE_F32, nullptr);
+        else Mixer::forward_set(h, step, cache, x, write, arena, s);
+    }
+    void forward_through(NormedInput& h, const StepView& step, const CacheView& cache, const StreamAdd& add, bool write, Arena& arena,
+                         hipStream_t s) const override {
+        if (joined_) run_joined(h, step, cache, add.x, write, arena, s, STORE_F32, &add);
+        else Mixer::forward_through(h, step, cache, add, write, arena, s);
+    }
     void forward(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
                  hipStream_t s) const override {
+        if (joined_) { run_joined(h, step, cache, x, write, arena, s, ADD_RESIDUAL, nullptr); return; }
         const int n = static_cast<int>(mixers_.size());
         if (x.cols != size_) fail("parallel mixers of width %d were handed a stream of %lld", size_, (long long)x.cols);
         Tensor2 all = arena.tensor(F32, x.rows * n, x.cols);          // (every mixer sets its own share)
         size_t state_at = 0;
         for (int k = 0; k < n; ++k) {
-            const CacheNeed need = mixers_[k]->cache_need();
-            CacheView mine = cache;
-            mine.kind = 0;
-            if (need.kind & 1) {
-                if (!cache.has_pages()) fail("parallel mixers: mixer %d needs pages", k);
-                mine.kind |= 1;
-            }
-            if (need.kind & 2) {
-                if (!cache.has_state() || cache.state_bytes < state_at + need.state_bytes) fail("parallel mixers: mixer %d needs %zu bytes of state", k, need.state_bytes);
-                mine.kind |= 2;
-                mine.state = static_cast<char*>(cache.state) + state_at;
-                mine.state_bytes = need.state_bytes;
-                state_at += (need.state_bytes + 15) / 16 * 16;
-            }
+            const CacheView mine = share_of(k, cache, state_at);
             const size_t mark = arena.mark();
             mixers_[k]->forward_set(h, step, mine, all.row_range(x.rows * k, x.rows), write, arena, s);
             arena.release(mark);
@@ -155,13 +210,14 @@ public:
     size_t workspace_bytes(int tokens) const override {
         size_t most = 0;
         for (const auto& m : mixers_) most = std::max(most, m->workspace_bytes(tokens));
+        if (joined_) most += static_cast<size_t>(tokens) * ((in_.out_features() + 4) * 4 + (out_.in_features() + in_.in_features()) * dtype_size(dtype_));
         return most + static_cast<size_t>(tokens) * size_ * 4 * mixers_.size() + 1024;
     }
     CacheNeed cache_need() const override {
         CacheNeed n;
         for (const auto& m : mixers_) {
             const CacheNeed one = m->cache_need();
-            if (one.kind & 1) { n.n_kv_heads = one.n_kv_heads; n.head_dim = one.head_dim; n.value_dim = one.value_dim; n.window = one.window; }
+            if (one.kind & 1) { n.n_kv_heads = one.n_kv_heads; n.head_dim = one.head_dim; n.value_dim = one.value_dim; n.window = one.window; n.keep_first = one.keep_first; }
             if (one.kind & 2) n.state_bytes += (one.state_bytes + 15) / 16 * 16;
             n.kind |= one.kind;
         }
@@ -170,14 +226,16 @@ public:
     void reserve(int max_seqs, hipStream_t s) const override { for (const auto& m : mixers_) m->reserve(max_seqs, s); }
     void add_cost(StepCost& c) const override {
         for (const auto& m : mixers_) m->add_cost(c);
-        c.weight_bytes += 4.0 * size_ * mixers_.size();
+        if (!joined_) c.weight_bytes += 4.0 * size_ * mixers_.size();
     }
 
 private:
     std::vector<std::shared_ptr<const Mixer>> mixers_;
     std::vector<const float*> norms_;
     const float* joined_norms_ = nullptr;
-    int size_ = 0;
+    bool joined_ = false;              // the mixers share one input and one output product
+    Linear in_, out_;
+    int size_ = 0, dtype_ = BF16;
     float eps_ = 1e-6f;
 };
 

@@ -19,8 +19,9 @@ const float* f32_vector(const Params& p, const char* key, int64_t n) {
 //          RMS-normed (qk_norm "head": per head, one weight [dim] shared by the heads; "row": over all heads at once,
 //          weights as wide as the projections; "none"), then the first rot_dims columns of every head turned by the
 //          token's position (column i pairs with i + rot_dims / 2, or with rot_interleaved column 2i with 2i + 1; angle
-//          p * rot_base^(-2i / rot_dims)); qk_norm "unit_after": every head scaled to unit root mean square BEHIND the
+//          p * rot_base^(-2i / rot_dims), or p times the pair's frequency in the table rot_freqs); qk_norm "unit_after": every head scaled to unit root mean square BEHIND the
 //          turn, without a weight
+//          with qkv_conv ([(heads + kv_heads) * dim + kv_heads * value_dim, taps]) the same over the values too
 //   v      its own projection, or (values_from_keys) the keys as projected (behind the convolution), before norm and turn
 //   score  scale (q . k);  softcap > 0: softcap tanh(score / softcap);  with r1, r2 (one number per head each):
 //          minus r1 ln(1 + r2 (i - j));  or with distance_slope (one number per head): minus slope (i - j)
@@ -37,7 +38,7 @@ const float* f32_vector(const Params& p, const char* key, int64_t n) {
 // Parameters: heads, kv_heads, dim, value_dim, scale, softcap, window, keep_first, chunk, rot_dims, rot_base,
 // rot_interleaved, eps, dtype, values_from_keys, gated, gate_per_head, sigmoid_weights, shared_kv; string qk_norm;
 // tensors in.weight, out.weight, [in.bias, out.bias], [q.norm, k.norm], [r1, r2], [distance_slope], [sink],
-// [score_bias], [qk_conv].
+// [score_bias], [qk_conv | qkv_conv], [rot_freqs] ([rot_dims], two floats a pair whose sum is the frequency).
 class ScoredAttention final : public Mixer {
 public:
     explicit ScoredAttention(const Params& p) {
@@ -93,10 +94,14 @@ public:
         k_col_ = shared_kv_ ? -1 : H * d;
         v_col_ = (values_from_keys_ || shared_kv_) ? -1 : k_col_ + G * d;
         gate_col_ = shared_kv_ ? H * d : k_col_ + G * d + (values_from_keys_ ? 0 : G * dv);
-        if (const Tensor2* c = p.weights_or_null("qk_conv")) {
+        if (p.weights_or_null("rot_freqs") != nullptr) sh_.rot_freqs = f32_vector(p, "rot_freqs", sh_.rot_dims);
+        conv_values_ = p.weights_or_null("qkv_conv") != nullptr;
+        if (conv_values_ && (values_from_keys_ || p.weights_or_null("qk_conv") != nullptr)) fail("scored_attention: one convolution, over values of their own");
+        if (const Tensor2* c = p.weights_or_null(conv_values_ ? "qkv_conv" : "qk_conv")) {
+            const int channels = (H + G) * d + (conv_values_ ? G * dv : 0);
             if (shared_kv_) fail("scored_attention: the convolution runs over queries and keys; a mixer without keys of its own has none");
-            if (c->dtype != F32 || !c->contiguous() || c->rows != static_cast<int64_t>(H + G) * d || c->cols < 1 || c->cols > 16)
-                fail("scored_attention: 'qk_conv' must be contiguous float32 [%d, 1 to 16 taps]", (H + G) * d);
+            if (c->dtype != F32 || !c->contiguous() || c->rows != channels || c->cols < 1 || c->cols > 16)
+                fail("scored_attention: the convolution's taps must be contiguous float32 [%d, 1 to 16 taps]", channels);
             conv_ = *c;
             conv_bytes_ = static_cast<size_t>(c->cols - 1) * c->rows * 4;
         }
@@ -111,17 +116,31 @@ public:
                      hipStream_t s) const override {
         run(h, step, cache, x, write, arena, s, STORE_F32);
     }
+    void forward_through(NormedInput& h, const StepView& step, const CacheView& cache, const StreamAdd& add, bool write, Arena& arena,
+                         hipStream_t s) const override {
+        run(h, step, cache, add.x, write, arena, s, STORE_F32, &add);
+    }
     void run(NormedInput& h, const StepView& step, const CacheView& cache, const Tensor2& x, bool write, Arena& arena,
-             hipStream_t s, int out_epilogue) const {
+             hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
+        const int T = step.n_tokens, N = in_.out_features(), ld = (N + 3) / 4 * 4;
+        Tensor2 proj(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N, ld);
+        h.linear(in_, proj, STORE_F32, nullptr, arena, s);
+        Tensor2 o = arena.tensor(dtype_, T, sh_.n_heads * sh_.value_dim);
+        core(proj, step, cache, o, write, arena, s);
+        out_.into(o, x, out_epilogue, add, s);
+        StageTimes::get().mark("out_proj", s);
+    }
+    int core_inputs() const override { return in_.out_features(); }
+    int core_outputs() const override { return out_.in_features(); }
+    void core(const Tensor2& proj, const StepView& step, const CacheView& cache, const Tensor2& o, bool write, Arena& arena,
+              hipStream_t s) const override {
         if (!cache.has_pages()) fail("scored_attention needs a cache of pages");
         if (write == shared_kv_) fail(shared_kv_ ? "scored_attention without keys of its own reads another call's cache: it cannot write one"
                                                  : "scored_attention writes its own keys and values: it cannot read another call's cache");
-        const int T = step.n_tokens, g = cache.group, N = in_.out_features(), ld = (N + 3) / 4 * 4;
-        Tensor2 proj(arena.take(static_cast<size_t>(T) * ld * 4), F32, T, N, ld);
-        h.linear(in_, proj, STORE_F32, nullptr, arena, s);
+        const int T = step.n_tokens, g = cache.group;
         Tensor2 q = arena.tensor(dtype_, T, sh_.n_heads * sh_.dim);
         if (conv_.data != nullptr) {
-            // the convolution over the projected queries and keys (they lie side by side in front of the rows)
+            // the convolution over the projected queries and keys (and values), which lie side by side in front of the rows
             if (conv_bytes_ > 0 && (!cache.has_state() || cache.state_bytes < conv_bytes_)) fail("scored_attention with a convolution needs %zu bytes of state per request", conv_bytes_);
             const int C = static_cast<int>(conv_.rows);
             Tensor2 qk(arena.take(static_cast<size_t>(T) * C * 4), F32, T, C);
@@ -129,7 +148,9 @@ public:
             st.token_seq = step.token_seq; st.cu_q = step.cu_q; st.state_slots = step.state_slots; st.n_seqs = step.n_seqs;
             st.max_q_len = step.max_q_len; st.state = static_cast<float*>(cache.state); st.slot_floats = cache.slot_bytes / 4;
             st.n_slots = cache.n_slots; st.write = write;
-            conv_residual(Tensor2(proj.data, F32, T, C, ld), conv_, st, qk, s, false);      // (four channels a thread where the sizes allow)
+            conv_residual(Tensor2(proj.data, F32, T, C, proj.stride), conv_, st, qk, s, false);      // (four channels a thread where the sizes allow)
+            // (values outside the convolution are read where the projection left them)
+            if (v_col_ >= 0 && !conv_values_) fail("scored_attention: a convolution over queries and keys goes with values taken from the keys");
             qk_prepare(qk, 0, k_col_, v_col_, sh_, step.positions, step.slots[g], q, cache.k_pages, cache.v_pages, s);
         } else {
             qk_prepare(proj, 0, k_col_, v_col_, sh_, step.positions, step.slots[g], q, cache.k_pages, cache.v_pages, s);
@@ -139,11 +160,8 @@ public:
         st.block_tables = step.block_tables[g]; st.max_blocks = step.max_blocks[g]; st.n_seqs = step.n_seqs; st.max_q_len = step.max_q_len;
         st.max_ctx_len = step.max_ctx_len; st.page_size = cache.page_size; st.token_seq = step.token_seq; st.positions = step.positions;
         st.cu_q = step.cu_q; st.ctx_len = step.ctx_len; st.n_single = step.n_single;
-        Tensor2 o = arena.tensor(dtype_, T, sh_.n_heads * sh_.value_dim);
         scored_attention(q, cache.k_pages, cache.v_pages, st, sh_, gated_ ? &proj : nullptr, gate_col_, o, s);
         StageTimes::get().mark("attention", s);
-        out_(o, x, out_epilogue, nullptr, s);
-        StageTimes::get().mark("out_proj", s);
     }
     size_t workspace_bytes(int tokens) const override {
         return static_cast<size_t>(tokens) * ((in_.out_features() + 4) * 4 + conv_.rows * 4 + (sh_.n_heads * (sh_.dim + sh_.value_dim) + in_.in_features()) * dtype_size(dtype_)) + 4096;
@@ -170,9 +188,9 @@ public:
 private:
     ScoredShape sh_;
     int dtype_ = BF16, k_col_ = 0, v_col_ = 0, gate_col_ = 0;
-    bool values_from_keys_ = false, gated_ = false, shared_kv_ = false;
+    bool values_from_keys_ = false, gated_ = false, shared_kv_ = false, conv_values_ = false;
     Linear in_, out_;
-    Tensor2 conv_;                   // [(heads + kv_heads) * dim, taps], or empty: no convolution
+    Tensor2 conv_;                   // [(heads + kv_heads) * dim (+ kv_heads * value_dim), taps], or empty: no convolution
     size_t conv_bytes_ = 0;
 };
 

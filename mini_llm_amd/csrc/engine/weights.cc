@@ -487,9 +487,10 @@ std::map<std::string, Tensor2> load_tensors(const std::vector<ParamSpec>& specs,
         std::vector<int64_t> shape = s.shape;
         if (!source.generates() && s.free_dim >= 0)
             if (const std::vector<int64_t>* stored = source.shape_of(available.at(s.name))) shape = *stored;
-        if (shape.size() == 1) cols = shape[0];
+        if (shape.empty()) cols = 1;                      // one number
+        else if (shape.size() == 1) cols = shape[0];
         else if (shape.size() == 2) { rows = shape[0]; cols = shape[1]; }
-        else throw WeightsError(where + ": tensor '" + s.name + "' has " + std::to_string(shape.size()) + " dimensions; one or two are expected");
+        else throw WeightsError(where + ": tensor '" + s.name + "' has " + std::to_string(shape.size()) + " dimensions; at most two are expected");
         if (s.add != 0.0)
             for (auto& v : values) v = static_cast<float>(v + s.add);
         const std::vector<float>* src = &values;

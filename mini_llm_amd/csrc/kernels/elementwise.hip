@@ -8,13 +8,13 @@
 // /root/reference/src/kernels/embedding.cu:23-43. wpe may be null (no learned positions).
 // With `src` (optional): where src[t] >= 0, token t's id is prev[src[t]], a token that an earlier step
 // sampled on the device and the host has not read yet; ids[t] is not read then. With `copy` the row is stored there once
-// more in bfloat16.
+// more in bfloat16, behind the norm `next` if it has a weight.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ void embed_kernel(const int* __restrict__ ids, const int* __restrict__ pos,
                              const T* __restrict__ wte, const T* __restrict__ wpe,
                              float* __restrict__ x, int D, const int* __restrict__ src,
-                             const int* __restrict__ prev, int n_prev, float scale, bf16_t* __restrict__ copy) {
+                             const int* __restrict__ prev, int n_prev, float scale, bf16_t* __restrict__ copy, MllmTanhNorm next) {
     const int t = blockIdx.x;
     int id = ids[t];
     if (src != nullptr) {
@@ -28,13 +28,13 @@ __global__ void embed_kernel(const int* __restrict__ ids, const int* __restrict_
         for (int d = threadIdx.x; d < D; d += blockDim.x) {
             const float v = to_float(te[d]) * scale + to_float(pe[d]);
             xr[d] = v;
-            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(v);
+            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(next.weight != nullptr ? fast_tanh(next.alpha[0] * v) * next.weight[d] + next.bias[d] : v);
         }
     } else {
         for (int d = threadIdx.x; d < D; d += blockDim.x) {
             const float v = to_float(te[d]) * scale;
             xr[d] = v;
-            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(v);
+            if (copy) copy[static_cast<size_t>(t) * D + d] = float_to_bf16(next.weight != nullptr ? fast_tanh(next.alpha[0] * v) * next.weight[d] + next.bias[d] : v);
         }
     }
 }
@@ -267,13 +267,13 @@ int mllm_reset_state(void* state, size_t slot_bytes, int n_slots, const int* slo
 }
 
 int mllm_embed(const int* ids, const int* pos, const void* wte, const void* wpe, float* x, int T, int D,
-               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale, void* copy_bf16) {
+               int dtype, const int* src, const int* prev, int n_prev, hipStream_t stream, float scale, void* copy_bf16, MllmTanhNorm next) {
     if (T <= 0) return 0;
     bf16_t* copy = static_cast<bf16_t*>(copy_bf16);
     if (dtype == MLLM_F32)
-        embed_kernel<float><<<T, 256, 0, stream>>>(ids, pos, (const float*)wte, (const float*)wpe, x, D, src, prev, n_prev, scale, copy);
+        embed_kernel<float><<<T, 256, 0, stream>>>(ids, pos, (const float*)wte, (const float*)wpe, x, D, src, prev, n_prev, scale, copy, next);
     else
-        embed_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, pos, (const bf16_t*)wte, (const bf16_t*)wpe, x, D, src, prev, n_prev, scale, copy);
+        embed_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, pos, (const bf16_t*)wte, (const bf16_t*)wpe, x, D, src, prev, n_prev, scale, copy, next);
     MLLM_LAUNCH_CHECK();
     return 0;
 }

@@ -33,54 +33,109 @@ __device__ __forceinline__ void expert_weight(const float* z, float* wgt, int E,
     wgt[e] = before < top ? scale * score : 0.f;
 }
 
-// The same for experts that are gated and clamped: the joined first product's rows are [expert 0: gate | up] ...
+// How scores become weights: a softmax over all experts' logits, every logit's sigmoid on its own, or a softmax over the
+// chosen experts' logits alone.
+enum RouterKind : int { ROUTER_SOFTMAX = 0, ROUTER_SIGMOID = 1, ROUTER_SOFTMAX_CHOSEN = 2 };
+
+// Up to 64 experts: a wavefront works out a token's weights by itself, lane e expert e's (0 for lanes without an expert).
+__device__ __forceinline__ float wave_expert_weight(float mine, int lane, int E, int top, float scale, int kind) {
+    int before = 0;
+    for (int o = 0; o < E; ++o) {
+        const float other = row_lane(mine, o);
+        before += (other > mine || (other == mine && o < lane)) ? 1 : 0;
+    }
+    const bool chosen = lane < E && before < top;
+    if (kind == ROUTER_SIGMOID) return chosen ? scale / (1.f + expf(-mine)) : 0.f;
+    const float m = wave_max(mine);                      // (the largest logit is always chosen)
+    const bool counts = kind == ROUTER_SOFTMAX_CHOSEN ? chosen : lane < E;
+    const float ex = counts ? expf(mine - m) : 0.f, sum = wave_sum(ex);
+    return chosen ? scale * (ex / sum) : 0.f;
+}
+
+// The same for experts that are gated (and clamped): the joined first product's rows are [expert 0: gate | up] ...
 // [expert E-1: gate | up] [shared: gate | up], and with g = min(w G, limit), u = clamp(w U, -limit, limit) (the weight
 // on the expert's INPUT, which a linear map hands on to its result; `weight_on_input` 0: g and u unweighted and the
-// weight on the result) out[t, e * ff + j] = g sigmoid(alpha g) (u + 1), zero for an expert that was not chosen. The
+// weight on the result) out[t, e * ff + j] = g sigmoid(alpha g) (u + up_shift), zero for an expert that was not chosen
+// (whose columns are not read). An infinite limit, alpha 1 and up_shift 0 make it silu(g) u. The
 // shared expert's columns follow, unweighted, with its own limit, times sigmoid(logits[t, E]) if `shared_gate` (the
 // router's product then has one more row). One workgroup per token. VEC: eight columns a thread at a time (16-byte
 // loads of bfloat16, two of float; ff, shared_ff and the strides are then multiples of 8 and the rows aligned), all of
 // one expert.
-template <typename T, bool VEC>
+template <typename TI, typename T, bool VEC>
 __global__ void __launch_bounds__(256)
-moe_glu_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int shared_ff, int top,
-                   float scale, int sigmoid_router, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate,
-                   T* __restrict__ out, int ldo) {
-    __shared__ float z[MOE_MAX_EXPERTS], wgt[MOE_MAX_EXPERTS];
-    __shared__ float sg_s;
-    const int t = blockIdx.x, tid = threadIdx.x;
-    if (tid < E) z[tid] = logits[static_cast<size_t>(t) * ldl + tid];
-    if (tid == 0) sg_s = shared_gate ? 1.f / (1.f + expf(-logits[static_cast<size_t>(t) * ldl + E])) : 1.f;
-    __syncthreads();
-    if (tid < E) expert_weight(z, wgt, E, top, scale, tid, sigmoid_router != 0);
-    __syncthreads();
-    const T* ur = up + static_cast<size_t>(t) * ldu;
+moe_glu_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int shared_ff, int top,
+                   float scale, int router_kind, float limit, float shared_limit, float alpha, float up_shift, int weight_on_input,
+                   int shared_gate, T* __restrict__ out, int ldo) {
+    // weights: one copy a wavefront where up to 64 experts let every wavefront work them out by itself, without a barrier
+    __shared__ float z[MOE_MAX_EXPERTS], weights[4][MOE_MAX_EXPERTS];
+    const int t = blockIdx.x, tid = threadIdx.x, lane = tid % MLLM_WAVE;
+    const int wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
+    const float* lr = logits + static_cast<size_t>(t) * ldl;
+    const float sg = shared_gate ? 1.f / (1.f + expf(-lr[E])) : 1.f;
+    float* wgt = weights[E <= MLLM_WAVE ? wave : 0];
+    if (E <= MLLM_WAVE) {
+        const float mine = lr[min(lane, E - 1)];
+        wgt[lane] = wave_expert_weight(mine, lane, E, top, scale, router_kind);
+        wave_lds_sync();
+    } else {
+        if (tid < E) z[tid] = lr[tid];
+        __syncthreads();
+        if (router_kind == ROUTER_SOFTMAX_CHOSEN) {
+            float* ex = weights[1];
+            if (tid < E) {
+                const float mine = z[tid];
+                float m = -INFINITY;
+                int before = 0;
+                for (int o = 0; o < E; ++o) {
+                    m = fmaxf(m, z[o]);
+                    before += (z[o] > mine || (z[o] == mine && o < tid)) ? 1 : 0;
+                }
+                ex[tid] = before < top ? expf(mine - m) : 0.f;
+            }
+            __syncthreads();
+            if (tid < E) {
+                float sum = 0.f;
+                for (int o = 0; o < E; ++o) sum += ex[o];
+                wgt[tid] = scale * (ex[tid] / sum);
+            }
+        } else if (tid < E) {
+            expert_weight(z, wgt, E, top, scale, tid, router_kind == ROUTER_SIGMOID);
+        }
+        __syncthreads();
+    }
+    const TI* ur = up + static_cast<size_t>(t) * ldu;
     T* orow = out + static_cast<size_t>(t) * ldo;
     const int routed = E * ff, N = routed + shared_ff;
     if (VEC) {
         for (int c = tid * 8; c < N; c += 256 * 8) {
-            float g[8], u[8], lim, w_in = 1.f, w_out = 1.f;
+            float g[8], u[8], lim = limit, w_in = 1.f, w_out = 1.f, y[8];
+            const TI *gp, *upp;
             bool live = true;
             if (c < routed) {
                 const int e = c / ff, j = c - e * ff;
-                load8(ur + static_cast<size_t>(e) * 2 * ff + j, g);
-                load8(ur + static_cast<size_t>(e) * 2 * ff + ff + j, u);
-                lim = limit;
-                live = wgt[e] != 0.f;
-                if (weight_on_input) w_in = wgt[e]; else w_out = wgt[e];
+                gp = ur + static_cast<size_t>(e) * 2 * ff + j;
+                upp = gp + ff;
+                const float we = wgt[e];
+                live = we != 0.f;
+                if (weight_on_input) w_in = we; else w_out = we;
             } else {
-                const int j = c - routed;
-                load8(ur + static_cast<size_t>(routed) * 2 + j, g);
-                load8(ur + static_cast<size_t>(routed) * 2 + shared_ff + j, u);
+                gp = ur + static_cast<size_t>(routed) * 2 + (c - routed);
+                upp = gp + shared_ff;
                 lim = shared_limit;
-                w_out = sg_s;
+                w_out = sg;
             }
-            float y[8];
+            if (live) {
+                load8(gp, g);
+                load8(upp, u);
 #pragma unroll
-            for (int k = 0; k < 8; ++k) {
-                const float gk = fminf(g[k] * w_in, lim), uk = fminf(fmaxf(u[k] * w_in, -lim), lim);
-                const float ex = sizeof(T) == 2 ? __expf(-alpha * gk) : expf(-alpha * gk);
-                y[k] = live ? gk / (1.f + ex) * (uk + 1.f) * w_out : 0.f;
+                for (int k = 0; k < 8; ++k) {
+                    const float gk = fminf(g[k] * w_in, lim), uk = fminf(fmaxf(u[k] * w_in, -lim), lim);
+                    const float ex = sizeof(T) == 2 ? __expf(-alpha * gk) : expf(-alpha * gk);
+                    y[k] = gk / (1.f + ex) * (uk + up_shift) * w_out;
+                }
+            } else {
+#pragma unroll
+                for (int k = 0; k < 8; ++k) y[k] = 0.f;
             }
             if (sizeof(T) == 2) {
                 uint4 pk;
@@ -108,11 +163,11 @@ moe_glu_act_kernel(const T* __restrict__ up, int ldu, const float* __restrict__ 
             g = to_float(ur[static_cast<size_t>(routed) * 2 + j]);
             u = to_float(ur[static_cast<size_t>(routed) * 2 + shared_ff + j]);
             lim = shared_limit;
-            w_out = sg_s;
+            w_out = sg;
         }
         g = fminf(g * w_in, lim);
         u = fminf(fmaxf(u * w_in, -lim), lim);
-        const float y = g / (1.f + expf(-alpha * g)) * (u + 1.f) * w_out;
+        const float y = g / (1.f + expf(-alpha * g)) * (u + up_shift) * w_out;
         orow[c] = from_float<T>(live ? y : 0.f);
     }
 }
@@ -289,23 +344,29 @@ int mllm_moe_act(const void* up, int ldu, const float* logits, int ldl, int E, i
     return 0;
 }
 
-// up [T, 2 (E * ff + shared_ff)] and out [T, E * ff + shared_ff] in `dtype`; logits [T, E (+ 1 with shared_gate)] fp32.
-// -1: more experts than the kernel holds, a `top` outside 1..E, limits that are not positive.
+// up [T, 2 (E * ff + shared_ff)] in up_dtype (`dtype`, or fp32) and out [T, E * ff + shared_ff] in `dtype`; logits [T, E (+ 1
+// with shared_gate)] fp32; router_kind: 0 softmax, 1 sigmoid, 2 softmax over the chosen experts.
+// -1: more experts than the kernel holds, a `top` outside 1..E, limits that are not positive, an unknown router_kind.
 int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int E, int ff, int shared_ff, int top, float scale,
-                     int sigmoid_router, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
-                     int ldo, int T, int dtype, hipStream_t stream) {
+                     int router_kind, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
+                     int ldo, int T, int dtype, hipStream_t stream, float up_shift, int up_dtype) {
     if (T <= 0) return 0;
+    if (up_dtype < 0) up_dtype = dtype;
     if (E < 1 || E > MOE_MAX_EXPERTS || top < 1 || top > E || ff < 1 || shared_ff < 0 || logits == nullptr) return -1;
     if (!(limit > 0.f) || (shared_ff > 0 && !(shared_limit > 0.f)) || (shared_gate && shared_ff == 0)) return -1;
-    const int esz = dtype == MLLM_F32 ? 4 : 2;
-    const bool vec = ff % 8 == 0 && shared_ff % 8 == 0 && ldu % 8 == 0 && ldo % 8 == 0 &&
-                     ((reinterpret_cast<uintptr_t>(up) | reinterpret_cast<uintptr_t>(out)) & 15) == 0 && (static_cast<size_t>(ldu) * esz) % 16 == 0;
-#define MOE_GLU(TYPE, VEC)                                                                                                                     \
-    moe_glu_act_kernel<TYPE, VEC><<<T, 256, 0, stream>>>(static_cast<const TYPE*>(up), ldu, logits, ldl, E, ff, shared_ff, top, scale, sigmoid_router, \
-                                                         limit, shared_limit, alpha, weight_on_input, shared_gate, static_cast<TYPE*>(out), ldo)
-    if (dtype == MLLM_F32) { if (vec) MOE_GLU(float, true); else MOE_GLU(float, false); }
-    else { if (vec) MOE_GLU(bf16_t, true); else MOE_GLU(bf16_t, false); }
+    if (router_kind < ROUTER_SOFTMAX || router_kind > ROUTER_SOFTMAX_CHOSEN || (up_dtype != dtype && up_dtype != MLLM_F32)) return -1;
+    const int isz = up_dtype == MLLM_F32 ? 4 : 2;
+    const bool vec = ff % 8 == 0 && shared_ff % 8 == 0 && ldo % 8 == 0 &&
+                     ((reinterpret_cast<uintptr_t>(up) | reinterpret_cast<uintptr_t>(out)) & 15) == 0 && (static_cast<size_t>(ldu) * isz) % 16 == 0;
+#define MOE_GLU_V(TI, TYPE, VEC)                                                                                                               \
+    moe_glu_act_kernel<TI, TYPE, VEC><<<T, 256, 0, stream>>>(static_cast<const TI*>(up), ldu, logits, ldl, E, ff, shared_ff, top, scale, router_kind, \
+                                                             limit, shared_limit, alpha, up_shift, weight_on_input, shared_gate, static_cast<TYPE*>(out), ldo)
+#define MOE_GLU(TI, TYPE) do { if (vec) MOE_GLU_V(TI, TYPE, true); else MOE_GLU_V(TI, TYPE, false); } while (0)
+    if (dtype == MLLM_F32) MOE_GLU(float, float);
+    else if (up_dtype == MLLM_F32) MOE_GLU(float, bf16_t);
+    else MOE_GLU(bf16_t, bf16_t);
 #undef MOE_GLU
+#undef MOE_GLU_V
     MLLM_LAUNCH_CHECK();
     return 0;
 }

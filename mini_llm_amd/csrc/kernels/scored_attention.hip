@@ -25,6 +25,12 @@ __device__ __forceinline__ int rot_partner(int i, int half, bool interleaved) { 
 __device__ __forceinline__ int rot_pair(int i, int half, bool interleaved) { return interleaved ? i / 2 : (i < half ? i : i - half); }
 __device__ __forceinline__ bool rot_first(int i, int half, bool interleaved) { return interleaved ? (i & 1) == 0 : i < half; }
 
+// The angle per position of pair `i`: rot_base^(-2i / rot_dims), or the table's (two floats a pair, whose sum is the
+// frequency to double precision: frequencies that are scaled or otherwise no power of one base).
+__device__ __forceinline__ double rot_frequency(int i, double base, int rot_dims, const float* __restrict__ table) {
+    return table != nullptr ? static_cast<double>(table[2 * i]) + static_cast<double>(table[2 * i + 1]) : pow(base, -2.0 * i / rot_dims);
+}
+
 // One workgroup per token. proj row (fp32): queries at q_col (H heads of d), keys at k_col (G heads of d), values at
 // v_col (G heads of dv; v_col < 0: the values are the keys as projected, before their norm; then dv == d).
 // LDS: the query and key rows, cos/sin of the token's angles, the inverse root mean squares.
@@ -32,7 +38,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 qk_prepare_kernel(const float* __restrict__ proj, int ld, int q_col, int k_col, int v_col, int H, int G, int d, int dv,
                   int norm_mode, const float* __restrict__ wq, const float* __restrict__ wk, float eps, int rot_dims,
-                  double rot_base, int interleaved, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
+                  double rot_base, const float* __restrict__ rot_freqs, int interleaved, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
                   int ldq, T* __restrict__ k_pages, T* __restrict__ v_pages) {
     extern __shared__ float pr_smem[];
     const int t = blockIdx.x, tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
@@ -47,7 +53,7 @@ qk_prepare_kernel(const float* __restrict__ proj, int ld, int q_col, int k_col, 
     for (int i = tid; i < nk; i += 256) ks[i] = row[k_col + i];
     if (tid < half) {
         // the angle in double, rounded once
-        const double f = pow(rot_base, -2.0 * tid / rot_dims), a = static_cast<double>(positions[t]) * f;
+        const double a = static_cast<double>(positions[t]) * rot_frequency(tid, rot_base, rot_dims, rot_freqs);
         cs[tid] = static_cast<float>(cos(a));
         cs[half + tid] = static_cast<float>(sin(a));
     }
@@ -123,7 +129,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 qk_prepare_heads_kernel(const float* __restrict__ proj, int ld, int q_col, int k_col, int v_col, int n_tokens, int H, int G, int d,
                         int dv, int norm_mode, const float* __restrict__ wq, const float* __restrict__ wk, float eps, int rot_dims,
-                        double rot_base, int interleaved, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
+                        double rot_base, const float* __restrict__ rot_freqs, int interleaved, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
                         int ldq, T* __restrict__ k_pages, T* __restrict__ v_pages) {
     __shared__ float normed_s[4][256];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lane = threadIdx.x % 64;
@@ -181,7 +187,7 @@ qk_prepare_heads_kernel(const float* __restrict__ proj, int ld, int q_col, int k
         if (i < rot_dims) {
             // the angle in double, rounded once
             const int pi = rot_pair(i, half, il);
-            const double a = pos * pow(rot_base, -2.0 * pi / rot_dims);
+            const double a = pos * rot_frequency(pi, rot_base, rot_dims, rot_freqs);
             const float c = static_cast<float>(cos(a)), sn = static_cast<float>(sin(a));
             const float other = mine[rot_partner(i, half, il)];
             val = rot_first(i, half, il) ? val * c - other * sn : val * c + other * sn;
@@ -376,7 +382,7 @@ int mllm_gate_mul(void* x, int ldx, const float* gate, int ldg, int T, int N, in
 int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, int T, int H, int G, int d, int dv,
                     int norm_mode, const float* wq, const float* wk, float eps, int rot_dims, double rot_base,
                     const int* positions, const int* slots, void* q_out, int ldq, void* k_pages, void* v_pages, int dtype,
-                    hipStream_t stream, int interleaved) {
+                    hipStream_t stream, int interleaved, const float* rot_freqs) {
     if (T <= 0) return 0;
     // (G == 0: queries only; the keys and values are another layer's)
     if (H < 1 || G < 0 || d < 1 || dv < 1 || rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > d || rot_dims / 2 > 256) return -1;
@@ -388,11 +394,11 @@ int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, 
         const int blocks = (T * (H + G) + 3) / 4;
         if (dtype == MLLM_F32)
             qk_prepare_heads_kernel<float><<<blocks, 256, 0, stream>>>(proj, ld, q_col, k_col, v_col, T, H, G, d, dv, norm_mode, wq, wk, eps,
-                                                                       rot_dims, rot_base, interleaved, positions, slots, static_cast<float*>(q_out), ldq,
+                                                                       rot_dims, rot_base, rot_freqs, interleaved, positions, slots, static_cast<float*>(q_out), ldq,
                                                                        static_cast<float*>(k_pages), static_cast<float*>(v_pages));
         else
             qk_prepare_heads_kernel<bf16_t><<<blocks, 256, 0, stream>>>(proj, ld, q_col, k_col, v_col, T, H, G, d, dv, norm_mode, wq, wk, eps,
-                                                                        rot_dims, rot_base, interleaved, positions, slots, static_cast<bf16_t*>(q_out), ldq,
+                                                                        rot_dims, rot_base, rot_freqs, interleaved, positions, slots, static_cast<bf16_t*>(q_out), ldq,
                                                                         static_cast<bf16_t*>(k_pages), static_cast<bf16_t*>(v_pages));
         MLLM_LAUNCH_CHECK();
         return 0;
@@ -401,11 +407,11 @@ int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, 
     if (smem > 60 * 1024) return -1;
     if (dtype == MLLM_F32)
         qk_prepare_kernel<float><<<T, 256, smem, stream>>>(proj, ld, q_col, k_col, v_col, H, G, d, dv, norm_mode, wq, wk, eps, rot_dims,
-                                                           rot_base, interleaved, positions, slots, static_cast<float*>(q_out), ldq,
+                                                           rot_base, rot_freqs, interleaved, positions, slots, static_cast<float*>(q_out), ldq,
                                                            static_cast<float*>(k_pages), static_cast<float*>(v_pages));
     else
         qk_prepare_kernel<bf16_t><<<T, 256, smem, stream>>>(proj, ld, q_col, k_col, v_col, H, G, d, dv, norm_mode, wq, wk, eps, rot_dims,
-                                                            rot_base, interleaved, positions, slots, static_cast<bf16_t*>(q_out), ldq,
+                                                            rot_base, rot_freqs, interleaved, positions, slots, static_cast<bf16_t*>(q_out), ldq,
                                                             static_cast<bf16_t*>(k_pages), static_cast<bf16_t*>(v_pages));
     MLLM_LAUNCH_CHECK();
     return 0;
