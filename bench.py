@@ -171,8 +171,41 @@ def zokunex_config(n_layer, size="gpt2-small", n_positions=1024):
             "vocab_size": 50257, "n_positions": n_positions, "n_layer": n}
 
 
+def gisedra_config(n_layer, size="gpt2-small", n_positions=1024):
+    """A Gisedra model whose layers run as often as the GPT-2 configuration `size` has layers, at the same width, vocabulary
+    and context: latent attention (as many heads of 64 as GPT-2 has, a latent of up to a third of the width beside 32 rotated
+    columns, a window of 512) and pairs (attention of heads of 64 over a quarter as many key/value heads, four taps, 32 rotated
+    columns with scaled frequencies, a window of 512 that keeps the first 16 positions; retention of half as many heads of
+    64 x 64) in turn; two of the layers in the middle run twice; sixteen gated experts of which two are chosen, together as
+    large as GPT-2's two feed-forward matrices; 64 columns a token and layer in the second table."""
+    full_layers, d, h, f = SIZES[size]
+    n = n_layer or full_layers
+    distinct = max(n - 2, 2)
+    kv = max(k for k in range(1, max(h // 4, 1) + 1) if h % k == 0)
+    rank = max(r for r in (64, 128, 256, 512) if r <= max(64, d // 3))      # 256 at 768 and 1,024, 512 at 1,600
+    mlp = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": max(32, f // 24 // 32 * 32)}}
+    rh = max(1, h // 2)
+    layers = []
+    for i in range(distinct):
+        if i % 2 == 0:
+            layers.append({"type": "latent_attention", "mlp": mlp,
+                           "mixer": {"heads": h, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": rank, "scale": 96 ** -0.5,
+                                     "rot": {"base": 10000.0, "dims": 32}, "mask": {"size": 512}}})
+        else:
+            layers.append({"type": "parallel", "mlp": mlp, "mixer": {
+                "left": {"heads": h, "kv_heads": kv, "dim": 64, "vdim": 64, "conv": 4, "scale": 0.125, "mask": {"size": 512, "keep_first": 16},
+                         "rot": {"base": 10000.0, "dims": 32, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 512}}},
+                "right": {"heads": rh, "dim": 64, "vdim": 64, "decay": [1.0 - 2.0 ** -(5 + 5 * k / rh) for k in range(rh)]},
+                "left_scale": 0.8, "right_scale": 0.9}})
+    at = distinct // 2
+    return {"architecture": "Gisedra", "vocab": 50257, "width": d, "norm": {"eps": 1e-6}, "token_side": {"dim": 64},
+            "loop": {"start": at - 1, "stop": at + 1, "times": 2}, "layers": layers,
+            # (what the measurement itself reads; the architecture ignores them)
+            "vocab_size": 50257, "n_positions": n_positions, "n_layer": distinct + 2}
+
+
 DESIGNS = {"kugulorn": kugulorn_config, "rekirax": rekirax_config, "viladra": viladra_config, "sunulorn": sunulorn_config,
-           "zokunex": zokunex_config}
+           "zokunex": zokunex_config, "gisedra": gisedra_config}
 
 
 def decode_run(model_dir, dtype, batch, prompt_len, steps, warmup, cfg):
@@ -407,8 +440,8 @@ def main():
                                      "it names vocab_size and n_positions, or --vocab / --positions do)")
     ap.add_argument("--vocab", type=int, default=0, help="with --config: the vocabulary to draw token ids from")
     ap.add_argument("--design", default="gpt2", choices=["gpt2", *DESIGNS],
-                    help="kugulorn / rekirax / viladra / sunulorn / zokunex: a model of that design of about the size --size names (kugulorn_config, "
-                         "rekirax_config, viladra_config, sunulorn_config, zokunex_config) through the same measurement; --compare runs it and GPT-2 one after the other")
+                    help="kugulorn / rekirax / viladra / sunulorn / zokunex / gisedra: a model of that design of about the size --size names (kugulorn_config, "
+                         "rekirax_config, viladra_config, sunulorn_config, zokunex_config, gisedra_config) through the same measurement; --compare runs it and GPT-2 one after the other")
     ap.add_argument("--beside", default="gpt2", choices=["gpt2", *DESIGNS],
                     help="with --compare: the design that the --design model is measured beside (default GPT-2)")
     ap.add_argument("--compare", action="store_true",

@@ -1,0 +1,285 @@
+"""Gisedra through the engine on the GPU against the plain implementation (tests/plain_gisedra.py), in 32-bit and in
+bfloat16: each mechanism alone, whole prompts against token-by-token decoding, portions down to two tokens, mixed
+batches against each request alone, pages and state slots that are used again, keys just inside and just outside every
+window and kept range, the first tokens, states that carry for hundreds of tokens, long decoding, and greedy generation
+through the engine's own entry point and scheduler."""
+import copy
+import tempfile
+
+import pytest
+
+import gisedra_cases as gc
+import plain_gisedra as pg
+import replay_util as ru
+
+pytestmark = pytest.mark.gpu
+DTYPES = ["float32", "bfloat16"]
+
+
+@pytest.fixture(scope="module")
+def dirs(tmp_path_factory):
+    made = {}
+
+    def get(name, seed=3):
+        if name not in made:
+            made[name] = gc.write_case(name, str(tmp_path_factory.mktemp("gisedra_" + name)), seed)
+        return made[name]
+    return get
+
+
+def _runner(model_dir, dtype, n_pages, page=4, max_num_seqs=4):
+    from mini_llm_amd import Runner
+    r = Runner(model_dir=model_dir, dtype=dtype, page_size=page, n_pages=n_pages, max_num_seqs=max_num_seqs)
+    r.poison_cache()               # a stale or unwritten page or slot that is read shows up as NaN
+    return r
+
+
+def _families(reqs, seed):
+    mixed, _ = ru.trace_mixed(reqs, seed=seed, max_live=4, tail=6)
+    return {"whole": ru.trace_whole(reqs), "decode": ru.trace_decode_tail(reqs, tail=11),
+            "chunks": ru.trace_chunks(reqs, seed=seed), "mixed": mixed}
+
+
+SINGLE = [n for n in dir(gc) if n.startswith(("ONLY_", "PAIR_", "EXPERTS_", "ONE_", "TOP_", "MANY_", "SIDE_", "LOOP_"))]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", SINGLE)
+def test_each_mechanism_alone(dirs, name, dtype):
+    cfg, d = getattr(gc, name), dirs(name)
+    reqs = gc.requests(cfg["vocab"], [1, 2, 3, 9, 37, 64, 65], seed=5)
+    mixed, _ = ru.trace_mixed(reqs, seed=3, max_live=4, tail=6)
+    for label, steps in (("whole", ru.trace_whole(reqs)), ("chunks", ru.trace_chunks(reqs, seed=1)),
+                         ("decode", ru.trace_decode_tail(reqs, tail=20)), ("mixed", mixed)):
+        runner = _runner(d, dtype, n_pages=ru.peak_tokens(steps) // 4)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"{name} {label}")
+        assert runner.check() == "" and runner.info()["n_requests"] == 0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["MIXED_A", "MIXED_B", "ODD"])
+@pytest.mark.parametrize("family", ["whole", "decode", "chunks", "mixed"])
+def test_schedule_families_match_plain(dirs, name, family, dtype):
+    """Each request whole; most of it at once and the rest token by token; portions down to two tokens; up to
+    four live requests in mixed batches. The pool holds just the peak of live tokens and there are four state
+    slots for eight requests, so pages and slots are used again (and were filled with NaN before)."""
+    cfg, d = getattr(gc, name), dirs(name)
+    reqs = gc.decisive_requests(d, cfg["vocab"], [1, 2, 3, 4, 5, 29, 64, 71], seed=11)
+    steps = _families(reqs, seed=2)[family]
+    n_pages = ru.peak_tokens(steps) // 4
+    runner = _runner(d, dtype, n_pages)
+    gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"{name} {family}")
+    info = runner.info()
+    assert runner.check() == "" and info["free_pages"] == n_pages and info["n_requests"] == 0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("page", [8, 16, 64])
+@pytest.mark.parametrize("family", ["whole", "decode", "chunks", "mixed"])
+def test_sizes_of_a_larger_models_layers(dirs, family, page, dtype):
+    """Heads of 64 x 64 and 64 x 128, latents of 128 and 224 beside 32 and 64 rotated columns, memories of 64 x 64, at pages
+    of 8 to 64 tokens; prompts of up to 300 tokens (several windows, chunks and key tiles), portions, and mixed batches."""
+    cfg, d = gc.LARGER, dirs("LARGER")
+    reqs = gc.requests(cfg["vocab"], [1, 2, 17, 63, 64, 65, 130, 300], seed=71)
+    steps = _families(reqs, seed=6)[family]
+    runner = _runner(d, dtype, n_pages=-(-ru.peak_tokens(steps) // page), page=page)
+    gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"larger page {page} {family}")
+    assert runner.check() == "" and runner.info()["n_requests"] == 0
+
+
+def test_the_matrix_core_kernels_serve_the_larger_sizes(dirs):
+    """In bfloat16 latents of sizes the tile kernel is not built for are widened with zero columns and no launch goes to the
+    token kernel; the left mixers' prompts run on the matrix-core tiles, not on the row kernel."""
+    from mini_llm_amd.kernels import ops
+    cfg, d = gc.LARGER, dirs("LARGER")
+    reqs = gc.requests(cfg["vocab"], [70, 5], seed=13)
+    steps = ru.trace_decode_tail(reqs, tail=9)
+    runner = _runner(d, "bfloat16", n_pages=32, page=16)
+    ops.reset_seen()
+    gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), "bfloat16", cfg["vocab"], "kernels used")
+    assert ops.seen("latent_tile_launches") > 0 and ops.seen("latent_token_launches") == 0
+    assert ops.seen("prefill_tile_launches") > 0 and ops.seen("generic_attention_launches") == 0
+
+
+@pytest.mark.parametrize("page", [2, 4, 16])
+def test_window_edges_kept_positions_and_page_borders_with_peaked_scores(dirs, page):
+    """Scores scaled so that single keys dominate, over pages of 2, 4 and 16 tokens, windows of 20 and 26 with three kept first
+    positions and hundreds of keys: a window that is one token off, a kept position that is lost, one too many or turned by
+    the wrong angle changes whole rows. Prompts, portions and decoding past the windows."""
+    cfg, d = gc.PEAKED, dirs("PEAKED")
+    reqs = gc.requests(cfg["vocab"], [300, 47, 26, 27, 21, 20, 4, 3], seed=21)
+    mixed, _ = ru.trace_mixed(reqs, seed=7, max_live=4, tail=30)
+    for label, steps in (("whole", ru.trace_whole(reqs)), ("decode", ru.trace_decode_tail(reqs, tail=60)),
+                         ("chunks", ru.trace_chunks(reqs, seed=3, sizes=(2, 5, 3, 16, 70, 7, 2, 20, 26))), ("mixed", mixed)):
+        runner = _runner(d, "float32", n_pages=-(-ru.peak_tokens(steps) // page), page=page)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), "float32", cfg["vocab"], f"peaked page {page} {label}",
+                               tol=gc.TOL_PEAKED)
+        assert runner.check() == ""
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_peaked_scores_on_the_tile_kernels(dirs, dtype):
+    cfg, d = gc.PEAKED_TILES, dirs("PEAKED_TILES")
+    reqs = gc.requests(cfg["vocab"], [300, 130, 64, 71, 46, 7], seed=25)
+    mixed, _ = ru.trace_mixed(reqs, seed=8, max_live=4, tail=6)
+    for label, steps in (("whole", ru.trace_whole(reqs)), ("decode", ru.trace_decode_tail(reqs, tail=80)),
+                         ("chunks", ru.trace_chunks(reqs, seed=5, sizes=(2, 70, 3, 129, 16, 64))), ("mixed", mixed)):
+        runner = _runner(d, dtype, n_pages=-(-ru.peak_tokens(steps) // 16) + 4, page=16)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"peaked tiles {label}")
+
+
+@pytest.mark.parametrize("first", [1, 2, 3, 19, 20, 21, 31, 32, 33, 64])
+def test_portions_at_the_windows_and_chunks_edges(dirs, first):
+    """The first portion ends inside, at and just outside the convolution's reach, the window and the recurrence's chunk; the
+    second is two tokens or a chunk and a bit, and the rest comes token by token: no position's logits move."""
+    cfg, d = gc.PEAKED, dirs("PEAKED")
+    for second in (2, 33):
+        reqs = gc.requests(cfg["vocab"], [first + second + 24], seed=first)
+        toks, steps, at = reqs["r0"], [], 0
+        for n in [first, second] + [1] * 24:
+            steps.append({"step": len(steps), "entries": [{"id": "r0", "tokens": toks[at:at + n], "want": list(range(n))}], "end": []})
+            at += n
+        steps[-1]["end"] = ["r0"]
+        runner = _runner(d, "float32", n_pages=32)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), "float32", cfg["vocab"], f"portions {first} + {second}", tol=gc.TOL_PEAKED)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_memories_that_hardly_decay(dirs, dtype):
+    """Decays of 1, 1 - 2^-11 and 1/2 side by side: what the first tokens wrote carries rows hundreds of tokens later. Whole, in
+    portions of many sizes, decoded, and mixed."""
+    cfg, d = gc.SLOW, dirs("SLOW")
+    reqs = gc.requests(cfg["vocab"], [400, 129, 64, 1, 2], seed=33)
+    mixed, _ = ru.trace_mixed(reqs, seed=9, max_live=4, tail=6, sizes=(2, 70, 3, 129, 16, 64))
+    for label, steps in (("whole", ru.trace_whole(reqs)), ("decode", ru.trace_decode_tail(reqs, tail=60)),
+                         ("chunks", ru.trace_chunks(reqs, seed=5, sizes=(2, 70, 3, 129, 16, 64, 65, 63))), ("mixed", mixed)):
+        runner = _runner(d, dtype, n_pages=ru.peak_tokens(steps) // 4)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"slow {label}")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_prompt_of_a_thousand_tokens(dirs, dtype):
+    """One prompt of 1,100 tokens whole, in portions of hundreds and of two tokens, and with its last tokens one by one."""
+    cfg, d = gc.LARGER, dirs("LARGER")
+    reqs = gc.requests(cfg["vocab"], [1100], seed=81)
+    for label, steps in (("whole", ru.trace_whole(reqs)), ("chunks", ru.trace_chunks(reqs, seed=8, sizes=(300, 2, 129, 64, 401))),
+                         ("decode", ru.trace_decode_tail(reqs, tail=25))):
+        runner = _runner(d, dtype, n_pages=ru.peak_tokens(steps) // 16, page=16)
+        gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], f"long prompt {label}")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding_and_slots_used_again(dirs, dtype):
+    """One state slot and a small pool: three requests one after the other, each a few tokens and then up to 150 one by
+    one, every one of them compared; the slot and the pages are the same ones each time."""
+    cfg, d = gc.MIXED_A, dirs("MIXED_A")
+    reqs = gc.decisive_requests(d, cfg["vocab"], [153, 111, 132], seed=31)
+    steps = ru.trace_decode_tail(reqs, tail=150)
+    runner = _runner(d, dtype, n_pages=48, max_num_seqs=1)
+    gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], "long decoding")
+    assert runner.check() == "" and runner.info()["free_pages"] == 48
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_many_sequences_in_one_step(dirs, dtype):
+    """Seventy requests in one step, some of them single tokens behind their prompts, all with portions of their own length;
+    then steps of seventy single tokens."""
+    cfg, d = gc.MIXED_B, dirs("MIXED_B")
+    reqs = gc.requests(cfg["vocab"], [4 + (7 * i) % 45 for i in range(70)], seed=91)
+    ids = list(reqs)
+    steps = [{"step": 0, "entries": [{"id": r, "tokens": reqs[r][:1], "want": [0]} for r in ids[:5]], "end": []},
+             {"step": 1, "entries": [{"id": r, "tokens": reqs[r][1:2], "want": [0]} for r in ids[:5]] +
+                                    [{"id": r, "tokens": reqs[r][:-2], "want": list(range(len(reqs[r]) - 2))} for r in ids[5:]], "end": []},
+             {"step": 2, "entries": [{"id": r, "tokens": reqs[r][2:-1], "want": list(range(len(reqs[r]) - 3))} for r in ids[:5]] +
+                                    [{"id": r, "tokens": reqs[r][-2:-1], "want": [0]} for r in ids[5:]], "end": []},
+             {"step": 3, "entries": [{"id": r, "tokens": reqs[r][-1:], "want": [0]} for r in ids], "end": ids}]
+    runner = _runner(d, dtype, n_pages=70 * 13, max_num_seqs=70)
+    gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), dtype, cfg["vocab"], "many sequences")
+
+
+def test_batches_of_unequal_requests_equal_each_alone(dirs):
+    """The logits of a position do not depend on what else is in the batch, beyond rounding: the mixed family's
+    rows against the same requests run whole and alone, engine against engine, in bfloat16."""
+    cfg, d = gc.MIXED_B, dirs("MIXED_B")
+    reqs = gc.decisive_requests(d, cfg["vocab"], [3, 50, 18, 64, 7], seed=41)
+    fam = _families(reqs, seed=4)
+    got = {}
+    for family in ("whole", "mixed"):
+        runner = _runner(d, "bfloat16", n_pages=ru.peak_tokens(fam[family]) // 4)
+        got[family] = ru.collect(fam[family], ru.run_in_process(runner, fam[family]), cfg["vocab"])
+    errs = sorted(gc.row_error(got["mixed"][r][p], got["whole"][r][p].astype("float64")) for r in reqs for p in range(len(reqs[r])))
+    print(f"mixed against alone, bfloat16: worst {errs[-1]:.3e}, median {errs[len(errs) // 2]:.3e} of {len(errs)}")
+    assert errs[-1] <= 3e-2 and errs[len(errs) // 2] <= 1e-2
+
+
+def test_residual_stream_after_every_layer(dirs):
+    """Layer by layer: models that stop after 1, 2, ... layers of MIXED_A's list (without the loop, then with it) agree with
+    the plain model's logits, so a fault is pinned to the first layer that shows it."""
+    from mini_llm_amd import write_random_model
+    full = gc.MIXED_A
+    for n in range(1, len(full["layers"]) + 1):
+        cfg = copy.deepcopy(full)
+        cfg["layers"] = cfg["layers"][:n]
+        if n < cfg["loop"]["stop"]:
+            cfg.pop("loop")
+        with tempfile.TemporaryDirectory() as d:
+            write_random_model(cfg, d, 9)
+            reqs = gc.requests(cfg["vocab"], [21], seed=n)
+            steps = ru.trace_chunks(reqs, seed=n, sizes=(5, 2, 9))
+            runner = _runner(d, "float32", n_pages=16)
+            gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), "float32", cfg["vocab"], f"first {n} layers")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_trace_run_program(dirs, tmp_path, dtype):
+    """The mixed family through bin/trace_run as a user drives it (its default page size and four state slots)."""
+    cfg, d = gc.MIXED_A, dirs("MIXED_A")
+    reqs = gc.decisive_requests(d, cfg["vocab"], [2, 33, 64, 5, 70, 21], seed=51)
+    steps, _ = ru.trace_mixed(reqs, seed=5, max_live=4, tail=5)
+    out = ru.run_trace_run(d, dtype, steps, str(tmp_path / "out"), ru.peak_tokens(steps))
+    gc.check_against_plain(d, reqs, steps, out, dtype, cfg["vocab"], "program mixed")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_greedy_generation_through_the_engine(dirs, dtype):
+    """Engine.generate (scheduler, continuous batching, prompt portions of 7 tokens, two requests at a time for
+    five prompts, pages of 4; tokens that the device feeds back reach the token input too) against the plain model's
+    greedy tokens."""
+    from mini_llm_amd import Engine, EngineOptions, SamplingParams
+    d = dirs("MIXED_A" if dtype == "float32" else "UNROUTED")
+    cfg, w = pg.read_model(d)
+    prompts = list(gc.requests(cfg["vocab"], [1, 6, 19, 30, 11], seed=61).values())
+    engine = Engine.from_pretrained(d, dtype=dtype, options=EngineOptions(kv_block_size=4, total_kv_blocks=96, max_batch_num=2,
+                                                                          max_tokens_per_step=16, prefill_chunk=7))
+    outs = engine.generate(prompts, SamplingParams(max_new_tokens=9, ignore_eos=True))
+    for p, o in zip(prompts, outs):
+        assert len(o) == 9
+        if dtype == "float32":
+            assert o == pg.greedy_generate(cfg, w, p, 9)
+        else:
+            # bfloat16 may turn a near-tie: every token must be one the plain model chose or nearly chose
+            ids = list(p)
+            for t in o:
+                row = pg.logits(cfg, w, ids)[-1]
+                assert float(row[t]) >= float(row.max()) - 0.15 * float(row.std()), (o, t)
+                ids.append(t)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_generation_with_preemptions(dirs, dtype):
+    """A pool too small for all requests' growth: some are preempted and recomputed, and generate the tokens they generate
+    in a large pool (a preempted request's states start from zero again)."""
+    from mini_llm_amd import Engine, EngineOptions, SamplingParams
+    d = dirs("MIXED_A")
+    prompts = list(gc.requests(257, [9, 14, 5, 12], seed=65).values())
+    outs = []
+    for blocks in (64, 12):
+        engine = Engine.from_pretrained(d, dtype=dtype, options=EngineOptions(kv_block_size=4, total_kv_blocks=blocks, max_batch_num=4,
+                                                                              max_tokens_per_step=16, prefill_chunk=8))
+        outs.append(engine.generate(prompts, SamplingParams(max_new_tokens=16, ignore_eos=True)))
+        if blocks == 12:
+            assert engine.stats()["preemptions"] > 0
+    if dtype == "float32":
+        assert outs[0] == outs[1]
+    else:
+        assert [len(o) for o in outs[1]] == [16] * 4
