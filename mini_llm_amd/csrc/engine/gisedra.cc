@@ -455,6 +455,11 @@ void gisedra_assemble(const Json& config, const Tensors& t, int dtype, LoadedMod
             p.num["dtype"] = dtype; p.num["eps"] = c.eps; p.num["column"] = static_cast<double>(i * c.side_dim);
             p.tensor["table"] = t.at("side.embed");
             p.tensor["gate.weight"] = t.at(L + "side.gate"); p.tensor["proj.weight"] = t.at(L + "side.proj"); p.tensor["norm.weight"] = t.at(L + "side.norm");
+            if (dtype == BF16 && token_side_fits(D, static_cast<int>(c.side_dim))) {
+                const int64_t dim = token_side_padded(static_cast<int>(c.side_dim));
+                p.tensor["gate.tiles"] = out.store.operand_tiles(t.at(L + "side.gate"), dim, D);
+                p.tensor["proj.tiles"] = out.store.operand_tiles(t.at(L + "side.proj"), D, (dim + 31) / 32 * 32);
+            }
             m.stream_steps.push_back(build_stream_step("token_side", p));          // step i stands behind layer i
         }
     }

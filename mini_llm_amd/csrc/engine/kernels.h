@@ -32,6 +32,8 @@ int mllm_gemm_bf16_plain(const void* A, int lda, const void* W, int ldw, const f
                          int M, int N, int K, int mode, hipStream_t stream);
 int mllm_gemm_bf16(const void* A, int lda, const void* W, int ldw, const float* bias, void* C, int ldc,
                    int M, int N, int K, int mode, void* workspace, size_t workspace_bytes, hipStream_t stream);
+int mllm_gemm_bf16_through(const void* A, int lda, const void* W, int ldw, const float* bias, float* x, int ldx, int M, int N, int K,
+                           MllmStreamAdd add, void* workspace, size_t workspace_bytes, hipStream_t stream);
 int mllm_gemm_bf16_kv(const void* A, int lda, const void* W, int ldw, const float* bias, void* C, int ldc,
                       int M, int N, int K, const int* slots, void* k_pages, void* v_pages, int q_cols, int kv_dim,
                       hipStream_t stream);
@@ -180,6 +182,9 @@ int mllm_tanh_norm(const float* x, int ldx, const int* rows, MllmTanhNorm norm, 
 int mllm_stream_add(float* x, const float* y, const float* x0, const float* step, int n, int D, MllmStreamAdd add, int precise, hipStream_t stream);
 int mllm_token_gate(const float* z, int ldz, const int* ids, const int* src, const int* prev, int n_prev, const void* table, int ldt, int col0,
                     int dim, void* out, int ldo, int T, int dtype, hipStream_t stream);
+int mllm_token_side_fits(int D, int dim);
+int mllm_token_side(float* x, int T, int D, const void* gate, const void* proj, const float* weight, float eps, const int* ids, const int* src,
+                    const int* prev, int n_prev, const void* table, int ldt, int col0, int dim, MllmStreamAdd add, hipStream_t stream);
 
 // sampling.hip
 int mllm_argmax_chunks(int V);

@@ -279,6 +279,25 @@ void linear(const Tensor2& a, const Tensor2& w, const float* bias, const Tensor2
     check(rc, "linear");
 }
 
+void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, const StreamAdd& add, hipStream_t stream) {
+    need_dtype(a, "a");
+    check_stream_add(add, "linear_stream_add");
+    const int64_t M = a.rows, K = a.cols;
+    check_linear(M, K, a.dtype, w, add.x, ADD_RESIDUAL, "linear_stream_add");
+    if (tuning().through_products && a.dtype == BF16 && K % 8 == 0 && a.stride % 8 == 0 && w.stride % 8 == 0 && aligned(a.data, 16) && aligned(w.data, 16)) {
+        void* ws = M <= 256 ? gemm_workspace(stream) : nullptr;
+        const MllmStreamAdd k{add.norm, add.next, add.copy.data, static_cast<int>(add.copy.stride)};
+        const int rc = mllm_gemm_bf16_through(a.data, static_cast<int>(a.stride), w.data, static_cast<int>(w.stride), bias, static_cast<float*>(add.x.data),
+                                              static_cast<int>(add.x.stride), static_cast<int>(M), static_cast<int>(w.rows), static_cast<int>(K), k, ws,
+                                              ws ? GEMM_WORKSPACE_BYTES : 0, stream);
+        if (rc == 0) return;
+        if (rc != -1) check(rc, "linear_stream_add");
+    }
+    if (add.y.data == nullptr) fail("linear_stream_add: these sizes need room for the result");
+    linear(a, w, bias, add.y, STORE_F32, nullptr, stream);
+    stream_add(add, nullptr, nullptr, a.dtype == F32, stream);
+}
+
 void merge_splits(const AttentionSplits& a, const Tensor2& out, hipStream_t stream) {
     if (out.rows != a.n_tokens || out.cols != static_cast<int64_t>(a.n_heads) * a.head_dim)
         fail("merge_splits: out must be [%d, %d]", a.n_tokens, a.n_heads * a.head_dim);

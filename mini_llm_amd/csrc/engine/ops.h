@@ -118,6 +118,7 @@ struct Tuning {
     int ln_fuse_max_rows = 32;                        // rows up to which the norm is fused into the few-row product
     int latent_tiles = 1;                             // 1: latent attention's prompt portions may run on the matrix cores
     int scored_shared_kernels = 1;                    // 1: attention with shaped scores may run on the kernels the plain attention runs on
+    int through_products = 1;                         // 1: a product may take its result into the stream through norms itself
     int halves_max_width = 1024;                      // stream widths up to which a block whose sub-layers read one stream runs the
                                                       // feed-forward's first products, with the norm inside, in front of the mixer
                                                       // (wider: every workgroup of a wide product redoing the norm costs more than the
@@ -430,10 +431,19 @@ struct StreamAdd {
 // The stream's part of it, for a result that lies in add.y (null data: nothing is added but x0 and step): x += norm(y) + x0
 // + step (x0: x's shape, step: one row [columns], both optional), then the copy. `precise`: the library's tanh.
 void stream_add(const StreamAdd& add, const Tensor2* x0, const float* step, bool precise, hipStream_t stream);
-// The linear map whose result does that, inside the product where the kernels allow.
+void check_stream_add(const StreamAdd& add, const char* what);      // (an OpError if it does not fit)
+// The linear map whose result does that, inside the product where the kernels allow (bfloat16; add.y is not written then).
 void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, const StreamAdd& add, hipStream_t stream);
 // out[t, j] = gelu_tanh(z[t, j]) * table[id of token t, col0 + j] (z fp32; fed tokens as for embed)
 void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Tensor2& table, int col0, const Tensor2& out, hipStream_t stream);
+// The whole of it in one kernel, where token_side_fits (bfloat16): with e the columns col0 .. col0 + dim of the token's row of
+// the table, g = gelu_tanh(W_gate x) * e, y = W_proj g, x += y / sqrt(mean(y^2) + eps) * weight, then add's copy (add.x is the
+// stream, add.norm is not used). gate and proj: the maps' bfloat16 tiles in operand order (DeviceTensors::operand_tiles), dim
+// filled up to the next of 16, 32 and 64 rows and to whole tiles of 32 inputs.
+bool token_side_fits(int width, int dim);
+int token_side_padded(int dim);         // 16, 32 or 64
+void token_side(const StreamAdd& add, const Tensor2& gate, const Tensor2& proj, const float* weight, float eps, const int* ids, const FedTokens* fed,
+                const Tensor2& table, int col0, int dim, hipStream_t stream);
 
 // out = [a | b] row by row in out's dtype (a, b fp32 [T, D])
 void concat_cast(const Tensor2& a, const Tensor2& b, const Tensor2& out, hipStream_t stream);

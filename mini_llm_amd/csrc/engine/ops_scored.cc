@@ -337,8 +337,7 @@ void moe_glu_act(const Tensor2& up, const Tensor2& logits, const MoeGlu& m, cons
                            out.data, i32(out.stride), i32(up.rows), out.dtype, stream, m.up_shift, up.dtype), "moe_glu_act");
 }
 
-namespace {
-void check_norm(const MllmTanhNorm& n, const char* what) {
+static void check_norm(const MllmTanhNorm& n, const char* what) {
     if (n.weight != nullptr && (n.alpha == nullptr || n.bias == nullptr)) fail("%s: a tanh norm needs its three tensors", what);
 }
 void check_stream_add(const StreamAdd& add, const char* what) {
@@ -351,8 +350,7 @@ void check_stream_add(const StreamAdd& add, const char* what) {
     if (add.y.data != nullptr && (add.y.dtype != F32 || !add.y.contiguous() || add.y.rows != add.x.rows || add.y.cols != add.x.cols))
         fail("%s: the result must be contiguous float32 of the stream's shape", what);
 }
-MllmStreamAdd kernel_side(const StreamAdd& add) { return MllmStreamAdd{add.norm, add.next, add.copy.data, i32(add.copy.stride)}; }
-}  // namespace
+static MllmStreamAdd kernel_side(const StreamAdd& add) { return MllmStreamAdd{add.norm, add.next, add.copy.data, i32(add.copy.stride)}; }
 
 void tanh_norm(const Tensor2& x, const MllmTanhNorm& norm, const Tensor2& out, const int* rows, hipStream_t stream) {
     need_f32(x, "tanh_norm: x");
@@ -371,13 +369,6 @@ void stream_add(const StreamAdd& add, const Tensor2* x0, const float* step, bool
                           i32(add.x.rows), i32(add.x.cols), kernel_side(add), precise ? 1 : 0, stream), "stream_add");
 }
 
-void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, const StreamAdd& add, hipStream_t stream) {
-    check_stream_add(add, "linear_stream_add");
-    if (add.y.data == nullptr) fail("linear_stream_add: room for the result is needed");
-    linear(a, w, bias, add.y, STORE_F32, nullptr, stream);
-    stream_add(add, nullptr, nullptr, a.dtype == F32, stream);
-}
-
 void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Tensor2& table, int col0, const Tensor2& out, hipStream_t stream) {
     need_f32(z, "token_gate: z");
     need_act(table, "token_gate: the table");
@@ -388,6 +379,25 @@ void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Te
     check(mllm_token_gate(static_cast<const float*>(z.data), i32(z.stride), ids, feeds ? fed->src : nullptr, feeds ? fed->prev : nullptr,
                           feeds ? fed->n_prev : 0, table.data, i32(table.stride), col0, i32(z.cols), out.data, i32(out.stride), i32(z.rows), out.dtype,
                           stream), "token_gate");
+}
+
+bool token_side_fits(int width, int dim) { return mllm_token_side_fits(width, dim) != 0; }
+int token_side_padded(int dim) { return dim <= 16 ? 16 : (dim <= 32 ? 32 : 64); }
+
+void token_side(const StreamAdd& add, const Tensor2& gate, const Tensor2& proj, const float* weight, float eps, const int* ids, const FedTokens* fed,
+                const Tensor2& table, int col0, int dim, hipStream_t stream) {
+    check_stream_add(add, "token_side");
+    const int D = i32(add.x.cols);
+    if (!token_side_fits(D, dim)) fail("token_side: no kernel for a width of %d and %d columns", D, dim);
+    const int64_t rows = token_side_padded(dim), inputs = (rows + 31) / 32;
+    if (gate.dtype != BF16 || proj.dtype != BF16 || !gate.contiguous() || !proj.contiguous() || gate.rows * gate.cols != rows * D ||
+        proj.rows * proj.cols != inputs * 32 * D || weight == nullptr)
+        fail("token_side: the maps' tiles do not fit a width of %d and %d columns", D, dim);
+    if (table.dtype != BF16 || col0 < 0 || col0 + dim > table.cols || ids == nullptr) fail("token_side: columns %d.. of a table of %lld", col0, (long long)table.cols);
+    const bool feeds = fed != nullptr && fed->src != nullptr;
+    if (feeds && (fed->prev == nullptr || fed->n_prev < 1)) fail("token_side: fed tokens need the earlier step's sampled tokens");
+    check(mllm_token_side(static_cast<float*>(add.x.data), i32(add.x.rows), D, gate.data, proj.data, weight, eps, ids, feeds ? fed->src : nullptr,
+                          feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, table.data, i32(table.stride), col0, dim, kernel_side(add), stream), "token_side");
 }
 
 void concat_cast(const Tensor2& a, const Tensor2& b, const Tensor2& out, hipStream_t stream) {

@@ -79,7 +79,8 @@ private:
 // Behind a layer: with e the `dim` columns from column `column` on of the token's row of a second table,
 //   g = gelu_tanh(W_gate x) * e,  y = W_proj g,  x += y / sqrt(mean(y^2) + eps) * weight.
 // Parameters: dtype, column, eps; tensors table [vocab, columns], gate.weight [dim, width], proj.weight [width, dim],
-// norm.weight [width].
+// norm.weight [width]; and, for one kernel that does it all, gate.tiles and proj.tiles (the two maps in operand order, see
+// ops.h).
 class TokenSide final : public StreamStep {
 public:
     explicit TokenSide(const Params& p) : table_(p.weights("table")), gate_(p.weights("gate.weight"), nullptr), proj_(p.weights("proj.weight"), nullptr) {
@@ -90,10 +91,22 @@ public:
         if (proj_.in_features() != dim_ || proj_.out_features() != gate_.in_features()) fail("token_side: the two maps' shapes do not fit");
         if (column_ < 0 || column_ + dim_ > table_.cols || table_.dtype != dtype_) fail("token_side: columns %d to %d of a table of %lld", column_, column_ + dim_, (long long)table_.cols);
         norm_ = f32_vector(p, "norm.weight", proj_.out_features(), "token_side");
+        if (const Tensor2* g = p.weights_or_null("gate.tiles")) {
+            gate_tiles_ = *g;
+            proj_tiles_ = p.weights("proj.tiles");
+            if (dtype_ != BF16 || !token_side_fits(proj_.out_features(), dim_)) fail("token_side: tiles for a width of %d and %d columns: no kernel takes them", proj_.out_features(), dim_);
+        }
     }
     void forward(const Tensor2& x, const Tensor2&, int, const StepView& step, Arena& arena, hipStream_t s) const override {
         const int T = step.n_tokens, ldz = (dim_ + 3) / 4 * 4, ldg = (dim_ + 7) / 8 * 8;
         if (x.cols != proj_.out_features()) fail("token_side of width %d was handed a stream of %lld", proj_.out_features(), (long long)x.cols);
+        if (gate_tiles_.data != nullptr) {
+            StreamAdd add;
+            add.x = x;
+            if (step.leave.wanted) { add.copy = step.stream_copy; add.next = step.leave.norm; }
+            token_side(add, gate_tiles_, proj_tiles_, norm_, eps_, step.token_ids, &step.fed, table_, column_, dim_, s);
+            return;
+        }
         Tensor2 h = x;
         if (dtype_ == BF16) { h = arena.tensor(BF16, T, x.cols); cast_stream(x, h, s); }
         const Tensor2 z(arena.take(static_cast<size_t>(T) * ldz * 4), F32, T, dim_, ldz);
@@ -107,11 +120,12 @@ public:
     size_t workspace_bytes(int tokens) const override {
         return static_cast<size_t>(tokens) * (proj_.out_features() * 6 + (dim_ + 8) * 8) + 2048;
     }
+    bool leaves_copy() const override { return gate_tiles_.data != nullptr; }
     void reserve(int, hipStream_t s) const override { reserve_linear_scratch(s); }
     void add_cost(StepCost& c) const override { gate_.add_cost(c); proj_.add_cost(c); c.weight_bytes += 4.0 * proj_.out_features(); }
 
 private:
-    Tensor2 table_;
+    Tensor2 table_, gate_tiles_, proj_tiles_;
     Linear gate_, proj_;
     const float* norm_ = nullptr;
     int dtype_ = BF16, column_ = 0, dim_ = 0;

@@ -373,6 +373,24 @@ Tensor2 DeviceTensors::pad_row_parts(const Tensor2& t, const std::vector<int64_t
     return Tensor2(base, t.dtype, n * out_block, t.cols);
 }
 
+Tensor2 DeviceTensors::operand_tiles(const Tensor2& t, int64_t rows, int64_t cols) {
+    if (t.dtype != BF16 || !t.contiguous() || rows % 16 != 0 || cols % 32 != 0 || rows < t.rows || cols < t.cols)
+        throw WeightsError("operand_tiles: a contiguous bfloat16 matrix and sizes in whole tiles are needed");
+    std::vector<uint16_t> from(static_cast<size_t>(t.rows) * t.cols), to(static_cast<size_t>(rows) * cols, 0);
+    if (!from.empty() && hipMemcpy(from.data(), t.data, from.size() * 2, hipMemcpyDeviceToHost) != hipSuccess) throw WeightsError("operand_tiles: the copy from the device failed");
+    size_t at = 0;
+    for (int64_t r0 = 0; r0 < rows; r0 += 16)
+        for (int64_t c0 = 0; c0 < cols; c0 += 32)
+            for (int lane = 0; lane < 64; ++lane)
+                for (int i = 0; i < 8; ++i, ++at) {
+                    const int64_t r = r0 + lane % 16, c = c0 + 8 * (lane / 16) + i;
+                    if (r < t.rows && c < t.cols) to[at] = from[static_cast<size_t>(r) * t.cols + c];
+                }
+    void* dev = allocate(to.size() * 2, false);
+    if (!to.empty() && hipMemcpy(dev, to.data(), to.size() * 2, hipMemcpyHostToDevice) != hipSuccess) throw WeightsError("operand_tiles: the copy to the device failed");
+    return Tensor2(dev, BF16, rows, cols);
+}
+
 Tensor2 DeviceTensors::scaled(const Tensor2& v, float factor) {
     const size_t n = static_cast<size_t>(v.rows) * v.cols;
     if (v.dtype != F32 || !v.contiguous()) throw WeightsError("scaled: a contiguous float32 vector is needed");

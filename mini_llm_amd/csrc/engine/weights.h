@@ -166,6 +166,10 @@ public:
     // The same for blocks made of several parts: a block's part i has parts[i] rows (their sum is the block), each followed by
     // zero rows up to padded[i].
     Tensor2 pad_row_parts(const Tensor2& t, const std::vector<int64_t>& parts, const std::vector<int64_t>& padded);
+    // A bfloat16 matrix [rows, cols] as 16 x 32 tiles in the matrix cores' operand order, [rows / 16][cols / 32][lane][8]: lane l holds
+    // row l % 16, columns 8 (l / 16) to 8 (l / 16) + 7 of its tile. Rows and columns are filled up with zeros to `rows` and
+    // `cols` (multiples of 16 and 32).
+    Tensor2 operand_tiles(const Tensor2& t, int64_t rows, int64_t cols);
     // A vector times a number ([1, n] fp32, a copy on the device).
     Tensor2 scaled(const Tensor2& vector, float factor);
     size_t bytes() const { return bytes_; }

@@ -17,6 +17,8 @@
 #define EPI_GELU_ERF 2      // out[m,n] = gelu_erf(acc + bias)  (activation dtype)
 #define EPI_ADD_RESIDUAL 3  // res[m,n] += acc + bias           (fp32, in place)
 #define EPI_STORE_F32 4     // out[m,n] = acc + bias            (fp32)
+#define EPI_THROUGH 7       // x = res[m,n] += norm(acc + bias) (fp32, in place), then a bfloat16 copy of x or of another norm of x
+                            // (tanh_norm.h; only the bfloat16 matrix-core kernels, which take the norms beside the mode)
 #define EPI_RELU2 6         // out[m,n] = max(acc + bias, 0)^2  (activation dtype; 5 is an activation of the gated kernels)
 
 struct bf16_t {
@@ -270,6 +272,11 @@ __device__ __forceinline__ float mllm_shaped_score(float s, const MllmScoreShape
 // The first bias number of head h: r1[h], or the linear bias's slope[h], or 0.
 __device__ __forceinline__ float mllm_bias_r1(const MllmScoreShape& sh, int h) {
     return sh.r1 != nullptr ? sh.r1[h] : (sh.slope != nullptr ? sh.slope[h] : 0.f);
+}
+// The stream's new value x + norm(y) at one column, and what its copy holds of it (norms without a weight: y, x itself).
+struct MllmNormColumn { float w, b; };
+__device__ __forceinline__ float mllm_norm_column(float v, bool has, float alpha, MllmNormColumn c) {
+    return has ? fast_tanh(alpha * v) * c.w + c.b : v;
 }
 #define MLLM_LOG2E 1.44269504088896340736f
 

@@ -40,6 +40,44 @@ struct KvScatter {
     int q_cols, kv_dim;
 };
 
+// What a kernel of one mode takes beside its matrices.
+template <int MODE> struct TiledExtra { typedef KvScatter type; };
+template <> struct TiledExtra<EPI_THROUGH> { typedef MllmStreamAdd type; };
+
+// EPI_THROUGH for 4 consecutive columns of one row: the stream's row at x, columns n..n+3 of which n_left exist.
+__device__ __forceinline__ void through4(float* x, size_t idx, int n, const float (&v)[4], bool vec, int n_left, const MllmStreamAdd& add) {
+    const bool has = add.norm.weight != nullptr, has_next = add.next.weight != nullptr;
+    const float alpha = has ? add.norm.alpha[0] : 0.f, alpha2 = has_next ? add.next.alpha[0] : 0.f;
+    bf16_t* copy = static_cast<bf16_t*>(add.copy);          // (rows as far apart as the stream's)
+    if (vec && n_left >= 4) {
+        const float4 old = *reinterpret_cast<const float4*>(x + idx);
+        float w[4] = {1.f, 1.f, 1.f, 1.f}, b[4] = {0.f, 0.f, 0.f, 0.f};
+        if (has) {
+            const float4 w4 = *reinterpret_cast<const float4*>(add.norm.weight + n), b4 = *reinterpret_cast<const float4*>(add.norm.bias + n);
+            w[0] = w4.x; w[1] = w4.y; w[2] = w4.z; w[3] = w4.w; b[0] = b4.x; b[1] = b4.y; b[2] = b4.z; b[3] = b4.w;
+        }
+        float o[4] = {old.x, old.y, old.z, old.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] += mllm_norm_column(v[e], has, alpha, {w[e], b[e]});
+        *reinterpret_cast<float4*>(x + idx) = make_float4(o[0], o[1], o[2], o[3]);
+        if (copy == nullptr) return;
+        if (has_next) {
+            const float4 w4 = *reinterpret_cast<const float4*>(add.next.weight + n), b4 = *reinterpret_cast<const float4*>(add.next.bias + n);
+            o[0] = mllm_norm_column(o[0], true, alpha2, {w4.x, b4.x}); o[1] = mllm_norm_column(o[1], true, alpha2, {w4.y, b4.y});
+            o[2] = mllm_norm_column(o[2], true, alpha2, {w4.z, b4.z}); o[3] = mllm_norm_column(o[3], true, alpha2, {w4.w, b4.w});
+        }
+        *reinterpret_cast<uint2*>(copy + idx) = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+    } else {
+        for (int e = 0; e < n_left; ++e) {
+            float o = x[idx + e] + mllm_norm_column(v[e], has, alpha, {has ? add.norm.weight[n + e] : 1.f, has ? add.norm.bias[n + e] : 0.f});
+            x[idx + e] = o;
+            if (copy == nullptr) continue;
+            if (has_next) o = mllm_norm_column(o, true, alpha2, {add.next.weight[n + e], add.next.bias[n + e]});
+            copy[idx + e] = float_to_bf16(o);
+        }
+    }
+}
+
 template <int MODE>
 __device__ __forceinline__ void store4(void* C, size_t idx, const float (&v)[4], bool vec, int n_left) {
     // v: 4 consecutive columns of one row, bias already added; n_left: columns that exist (1..4)
@@ -76,7 +114,7 @@ template <int WM, int WN, int TM, int TN, int BKP, int DEPTH, bool EDGE, int MOD
 __global__ void __launch_bounds__(WM * WN * KG * 64)
 gemm_bf16_mfma(const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__ W, int ldw,
                const float* __restrict__ bias, void* __restrict__ C, int ldc, int M, int N, int K,
-               int tiles_m, int tiles_n, int xm, int xn, KvScatter kv) {
+               int tiles_m, int tiles_n, int xm, int xn, typename TiledExtra<MODE>::type kv) {
     // KG groups of WM x WN wavefronts share the tile: a k tile is KG * BKP wide and group g multiplies
     // its g-th part, so a barrier interval covers KG times the depth; the groups' sums meet in LDS.
     constexpr int NT = WM * WN * KG * 64;
@@ -311,8 +349,9 @@ gemm_bf16_mfma(const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__
                     const float4 b = *reinterpret_cast<const float4*>(&bias_s[nb - n0 + c4]);
                     v[0] += b.x; v[1] += b.y; v[2] += b.z; v[3] += b.w;
                 }
-                store4<MODE>(C, static_cast<size_t>(m) * ldc + n, v, vec, n_left);
-                if (MODE == EPI_STORE && kv.slots != nullptr && n >= kv.q_cols) {
+                if constexpr (MODE == EPI_THROUGH) through4(static_cast<float*>(C), static_cast<size_t>(m) * ldc + n, n, v, vec, n_left, kv);
+                else store4<MODE>(C, static_cast<size_t>(m) * ldc + n, v, vec, n_left);
+                if constexpr (MODE == EPI_STORE) if (kv.slots != nullptr && n >= kv.q_cols) {
                     const int slot = kv.slots[m];
                     if (slot >= 0) {
                         // q_cols and kv_dim are multiples of 4: the four columns lie in one of the two parts
@@ -336,7 +375,8 @@ gemm_bf16_mfma(const bf16_t* __restrict__ A, int lda, const bf16_t* __restrict__
 
 template <int WM, int WN, int TM, int TN, int BKP, int DEPTH, int KG = 1>
 static void launch_tiled(const bf16_t* a, int lda, const bf16_t* w, int ldw, const float* bias, void* C, int ldc,
-                         int M, int N, int K, int mode, hipStream_t stream, KvScatter kv = KvScatter{}) {
+                         int M, int N, int K, int mode, hipStream_t stream, KvScatter kv = KvScatter{},
+                         const MllmStreamAdd* through = nullptr) {
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32;
     const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
     // split of the output among the XCDs (xm x xn = 8) that keeps the A rows plus W rows of one XCD smallest
@@ -350,7 +390,13 @@ static void launch_tiled(const bf16_t* a, int lda, const bf16_t* w, int ldw, con
     const int per_xcd = ((tiles_m + xm - 1) / xm) * ((tiles_n + xn - 1) / xn);
     const dim3 grid(per_xcd * N_XCD), block(WM * WN * KG * 64);
     const bool edge = K % (BKP * KG) != 0;      // rows and columns beyond the matrices need no other kernel, see EDGE
-#define TILED(E, MD) gemm_bf16_mfma<WM, WN, TM, TN, BKP, DEPTH, E, MD, KG><<<grid, block, 0, stream>>>(a, lda, w, ldw, bias, C, ldc, M, N, K, tiles_m, tiles_n, xm, xn, kv)
+#define TILED(E, MD) gemm_bf16_mfma<WM, WN, TM, TN, BKP, DEPTH, E, MD, KG><<<grid, block, 0, stream>>>(a, lda, w, ldw, bias, C, ldc, M, N, K, tiles_m, tiles_n, xm, xn, extra)
+    if (mode == EPI_THROUGH) {
+        const MllmStreamAdd extra = *through;
+        if (edge) TILED(true, EPI_THROUGH); else TILED(false, EPI_THROUGH);
+        return;
+    }
+    const KvScatter extra = kv;
 #define TILED_MODE(MD) case MD: if (edge) TILED(true, MD); else TILED(false, MD); break;
     switch (mode) {
         TILED_MODE(EPI_STORE) TILED_MODE(EPI_GELU_TANH) TILED_MODE(EPI_GELU_ERF) TILED_MODE(EPI_RELU2) TILED_MODE(EPI_ADD_RESIDUAL)
@@ -402,7 +448,9 @@ struct SplitStates {
     float4 o[MERGE_MAX_SPLITS][2];        // 8 elements of the unnormalised output
 };
 
-template <int MT, int ASRC, bool SPLIT_K, int U, bool A_TWO = true, int NT = 1>
+struct NoExtra {};
+
+template <int MT, int ASRC, bool SPLIT_K, int U, bool A_TWO = true, int NT = 1, bool THROUGH = false>
 __global__ void __launch_bounds__(ASRC == A_NORMED ? 512 : (ASRC == A_GLOBAL || ASRC == A_MERGED ? 768 : 1024))
 gemm_bf16_skinny(// the first 16 dwords arrive in registers with the wavefront: what the first loads need
                  const bf16_t* __restrict__ W, int ldw, int N, int K, int M, int col_blocks, int row_blocks,
@@ -417,7 +465,10 @@ gemm_bf16_skinny(// the first 16 dwords arrive in registers with the wavefront: 
                  const float* __restrict__ split_o = nullptr, const float* __restrict__ split_ml = nullptr,
                  int n_splits = 1, int a_heads = 1, int a_head_dim = 8,
                  // A_NORMED: != 0: the norm does not centre (RMS norm: x / sqrt(mean(x^2) + eps) * gamma)
-                 int rms = 0) {
+                 int rms = 0,
+                 // THROUGH (mode EPI_THROUGH): the norms the result passes and the copy it leaves
+                 typename std::conditional<THROUGH, MllmStreamAdd, NoExtra>::type add = {}) {
+    static_assert(!THROUGH || (SPLIT_K && MT == 1 && ASRC == A_GLOBAL), "results through norms: split-K kernels of one row tile");
     // NT > 1 (SPLIT_K, MT == 1): the workgroup owns cols_per_wg <= 16 NT columns, NT tiles that share
     // the rows of A, the last one possibly narrower: for products with more than 256 tiles, whose
     // columns are dealt out evenly to 256 workgroups (one per compute unit; a kernel of this size
@@ -490,6 +541,8 @@ gemm_bf16_skinny(// the first 16 dwords arrive in registers with the wavefront: 
     bool ep_ok[NT];
     size_t ep_idx[NT];
     float ep_bias[NT], ep_old[NT];
+    MllmNormColumn ep_norm[NT], ep_next[NT];
+    float ep_alpha = 0.f, ep_alpha2 = 0.f;
 #pragma unroll
     for (int t = 0; t < NT; ++t) { ep_ok[t] = false; ep_idx[t] = 0; ep_bias[t] = 0.f; ep_old[t] = 0.f; }
     if (SPLIT_K && MT == 1 && wave < 4) {
@@ -501,7 +554,16 @@ gemm_bf16_skinny(// the first 16 dwords arrive in registers with the wavefront: 
             ep_ok[t] = m < M && nn < N && ct < cols_per_wg;
             ep_idx[t] = static_cast<size_t>(min(m, M - 1)) * ldc + min(nn, N - 1);
             if (bias) ep_bias[t] = bias[min(nn, N - 1)];
-            if (mode == EPI_ADD_RESIDUAL) ep_old[t] = static_cast<const float*>(C)[ep_idx[t]];
+            if (THROUGH || mode == EPI_ADD_RESIDUAL) ep_old[t] = static_cast<const float*>(C)[ep_idx[t]];
+            if constexpr (THROUGH) {
+                const int nc = min(nn, N - 1);
+                if (add.norm.weight != nullptr) ep_norm[t] = {add.norm.weight[nc], add.norm.bias[nc]};
+                if (add.next.weight != nullptr) ep_next[t] = {add.next.weight[nc], add.next.bias[nc]};
+            }
+        }
+        if constexpr (THROUGH) {
+            if (add.norm.weight != nullptr) ep_alpha = add.norm.alpha[0];
+            if (add.next.weight != nullptr) ep_alpha2 = add.next.alpha[0];
         }
     }
 
@@ -918,7 +980,12 @@ gemm_bf16_skinny(// the first 16 dwords arrive in registers with the wavefront: 
         for (int t = 0; t < NT; ++t) {
             if (ep_ok[t]) {
                 const float r = vt[t] + ep_bias[t];
-                if (mode == EPI_ADD_RESIDUAL) static_cast<float*>(C)[ep_idx[t]] = ep_old[t] + r;
+                if constexpr (THROUGH) {
+                    const float x = ep_old[t] + mllm_norm_column(r, add.norm.weight != nullptr, ep_alpha, ep_norm[t]);
+                    static_cast<float*>(C)[ep_idx[t]] = x;
+                    if (add.copy != nullptr)
+                        static_cast<bf16_t*>(add.copy)[ep_idx[t]] = float_to_bf16(mllm_norm_column(x, add.next.weight != nullptr, ep_alpha2, ep_next[t]));
+                } else if (mode == EPI_ADD_RESIDUAL) static_cast<float*>(C)[ep_idx[t]] = ep_old[t] + r;
                 else epilogue<bf16_t>(mode, r, 0.f, C, ep_idx[t]);
             }
         }
@@ -951,10 +1018,11 @@ template <bool LN_FUSED, bool MERGED = false>
 static int launch_skinny(const void* A, int lda, const bf16_t* W, int ldw, const float* bias, void* C, int ldc,
                          int M, int N, int K, int mode, const float* gamma, const float* beta, float eps,
                          const int* rows, hipStream_t stream, void* workspace = nullptr, size_t workspace_bytes = 0,
-                         MergedA merged = MergedA{}, int rms = 0) {
+                         MergedA merged = MergedA{}, int rms = 0, const MllmStreamAdd* through = nullptr) {
     static_assert(!(LN_FUSED && MERGED), "one source of A");
     const int tiles = (N + 15) / 16;
     const bool split_k = tiles < 1024;
+    if (through != nullptr && (LN_FUSED || MERGED || !split_k)) return -2;
     // Narrow products: 16 rows per workgroup and one workgroup per 16 rows (more workgroups, each
     // reading only its rows). Wide products: every wavefront keeps all rows of its tile in
     // registers (up to 4 accumulators), so the weights are streamed once.
@@ -1036,7 +1104,7 @@ static int launch_skinny(const void* A, int lda, const bf16_t* W, int ldw, const
         if (e != hipSuccess) return static_cast<int>(e);                                               \
         kernel<<<grid, block, staged_bytes, stream>>>(W, ldw, N, K, M, col_blocks, row_blocks, 16, 1, A, lda, mode, \
                                                       bias, C, ldc, gamma, beta, eps, rows, nullptr, nullptr, \
-                                                      nullptr, nullptr, 1, 1, 8, 0);                   \
+                                                      nullptr, nullptr, 1, 1, 8, 0, NoExtra{});                   \
         break;                                                                                         \
     }
         switch (mt) {
@@ -1054,9 +1122,9 @@ static int launch_skinny(const void* A, int lda, const bf16_t* W, int ldw, const
     }
     if (smem > MAX_DYNAMIC_LDS) return -2;
     constexpr int ASRC = LN_FUSED ? A_NORMED : (MERGED ? A_MERGED : A_GLOBAL);
-#define SKINNY_LAUNCH(SPLIT, UV, A2, NTV)                                                              \
+#define SKINNY_KERNEL(SPLIT, UV, A2, NTV, THROUGH, ...)                                                \
     do {                                                                                               \
-        auto kernel = gemm_bf16_skinny<1, ASRC, SPLIT, UV, A2, NTV>;                                   \
+        auto kernel = gemm_bf16_skinny<1, ASRC, SPLIT, UV, A2, NTV, THROUGH>;                          \
         static bool lds_allowed = false;      /* more than 64 KB of dynamic LDS has to be asked for once */ \
         if (!lds_allowed) {                                                                            \
             hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel),                  \
@@ -1067,7 +1135,14 @@ static int launch_skinny(const void* A, int lda, const bf16_t* W, int ldw, const
         kernel<<<grid, block, smem, stream>>>(W, ldw, N, K, M, col_blocks, row_blocks, cols_per_wg, k_parts, A, lda, \
                                               mode, bias, C, ldc, gamma, beta, eps, rows, part_sums,      \
                                               part_counters, merged.split_o, merged.split_ml, merged.n_splits, \
-                                              merged.heads, merged.head_dim, rms);                     \
+                                              merged.heads, merged.head_dim, rms, __VA_ARGS__);        \
+    } while (0)
+#define SKINNY_LAUNCH(SPLIT, UV, A2, NTV)                                                              \
+    do {                                                                                               \
+        if constexpr (ASRC == A_GLOBAL) {                                                              \
+            if (through != nullptr) { SKINNY_KERNEL(SPLIT, UV, A2, NTV, true, *through); break; }      \
+        }                                                                                              \
+        SKINNY_KERNEL(SPLIT, UV, A2, NTV, false, NoExtra{});                                           \
     } while (0)
     if (split_k) {
         // a chunk holds all k blocks of a wavefront when they are at most 3 (4 without the fused
@@ -1122,13 +1197,14 @@ static int launch_skinny(const void* A, int lda, const bf16_t* W, int ldw, const
         return -2;
     }
 #undef SKINNY_LAUNCH
+#undef SKINNY_KERNEL
     return 0;
 }
 
 
 static int gemm_bf16_dispatch(const void* A, int lda, const void* W, int ldw, const float* bias, void* C, int ldc,
                               int M, int N, int K, int mode, hipStream_t stream, KvScatter kv,
-                              void* workspace = nullptr, size_t workspace_bytes = 0) {
+                              void* workspace = nullptr, size_t workspace_bytes = 0, const MllmStreamAdd* through = nullptr) {
     if (M <= 0 || N <= 0) return 0;
     if (K % 8 != 0 || lda % 8 != 0 || ldw % 8 != 0) return -1;
     if ((reinterpret_cast<uintptr_t>(A) & 15) || (reinterpret_cast<uintptr_t>(W) & 15)) return -1;
@@ -1153,10 +1229,10 @@ static int gemm_bf16_dispatch(const void* A, int lda, const void* W, int ldw, co
     };
     const bool few_rows = M <= 16 || (M <= 64 && col_tiles >= 1024) || (M <= 256 && streaming_is_faster());
     if (!scatter && few_rows && launch_skinny<false>(A, lda, w, ldw, bias, C, ldc, M, N, K, mode, nullptr, nullptr,
-                                                    0.f, nullptr, stream, workspace, workspace_bytes) == 0) {
+                                                    0.f, nullptr, stream, workspace, workspace_bytes, MergedA{}, 0, through) == 0) {
         // few rows: weight-streaming kernel
     } else if (M <= 32) {
-        launch_tiled<1, 4, 1, 1, 64, 3>(a, lda, w, ldw, bias, C, ldc, M, N, K, mode, stream, kv);
+        launch_tiled<1, 4, 1, 1, 64, 3>(a, lda, w, ldw, bias, C, ldc, M, N, K, mode, stream, kv, through);
     } else {
         // Tile choice. The compute units run the workgroups in rounds of 256, and a workgroup's time
         // grows with its tile's area, less so for large tiles (they move fewer bytes per flop). So
@@ -1179,7 +1255,7 @@ static int gemm_bf16_dispatch(const void* A, int lda, const void* W, int ldw, co
         // groups of wavefronts per workgroup, each on half of a twice as wide k tile, halve their
         // number (measured at K of 3072 to 6400: 9 to 17 % less time; at K of 768 to 1600: none).
         const bool long_k = K >= 2048;
-#define TILE(...) launch_tiled<__VA_ARGS__>(a, lda, w, ldw, bias, C, ldc, M, N, K, mode, stream, kv)
+#define TILE(...) launch_tiled<__VA_ARGS__>(a, lda, w, ldw, bias, C, ldc, M, N, K, mode, stream, kv, through)
         switch (best) {
             case 0: TILE(2, 4, 2, 2, 64, 4); break;
             case 1: TILE(4, 2, 1, 3, 64, 3); break;
@@ -1209,6 +1285,16 @@ int mllm_gemm_bf16(const void* A, int lda, const void* W, int ldw, const float* 
                               workspace_bytes);
 }
 
+
+// The product whose result is taken into the stream through norms (EPI_THROUGH): x [M, N] fp32 (row stride ldx), add.copy rows as
+// far apart as x's. Workspace as above. -1: as above, or norms whose vectors are not 16-byte aligned.
+int mllm_gemm_bf16_through(const void* A, int lda, const void* W, int ldw, const float* bias, float* x, int ldx, int M, int N, int K,
+                           MllmStreamAdd add, void* workspace, size_t workspace_bytes, hipStream_t stream) {
+    if (add.copy != nullptr && (add.ld_copy != ldx || (reinterpret_cast<uintptr_t>(add.copy) & 7))) return -1;
+    for (const MllmTanhNorm* n : {&add.norm, &add.next})
+        if (n->weight != nullptr && (n->alpha == nullptr || n->bias == nullptr || ((reinterpret_cast<uintptr_t>(n->weight) | reinterpret_cast<uintptr_t>(n->bias)) & 15))) return -1;
+    return gemm_bf16_dispatch(A, lda, W, ldw, bias, x, ldx, M, N, K, EPI_THROUGH, stream, KvScatter{}, workspace, workspace_bytes, &add);
+}
 
 // The plain bf16 store (mode 0) with the key/value scatter of KvScatter fused: C = A W^T + bias, and
 // columns [q_cols, q_cols + kv_dim) / [q_cols + kv_dim, q_cols + 2 kv_dim) of row m also go to row

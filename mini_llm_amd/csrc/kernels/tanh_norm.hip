@@ -91,6 +91,136 @@ token_gate_kernel(const float* __restrict__ z, int ldz, const int* __restrict__ 
     }
 }
 
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+#define SIDE_WAVES 16
+
+// The token's own gated input in one kernel: for every token t of the workgroup's `rows` (up to 16), with e the dim columns
+// from col0 on of the token's table row,
+//   g = gelu_tanh(W_gate x_t) * e,  y = W_proj g,  x_t += y / sqrt(mean(y^2) + eps) * weight,
+// and the copy (add.copy, add.next). Both maps come as 16 x 32 tiles in operand order ([tile of 16 rows][tile of 32 inputs][lane]
+// [8]: lane l holds row l % 16, inputs 8 (l / 16) ..), so a wavefront's load is one kilobyte in a row; both are asked for at the
+// start. The weights are the matrix cores' first operand: a lane then holds four consecutive columns of one token. The inputs of
+// the first map (the stream, rounded to bfloat16) are dealt over the wavefronts, whose sums meet in LDS in the order of their
+// index; of the second the columns are. DT: tiles of 16 over dim; KPW: tiles of 32 over the width a wavefront takes of the
+// first map; CPW: tiles of 16 columns it takes of the second.
+template <int DT, int KPW, int CPW>
+__global__ void __launch_bounds__(SIDE_WAVES * 64)
+token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* __restrict__ gate, const bf16x8* __restrict__ proj,
+                  const float* __restrict__ weight, float eps, const int* __restrict__ ids, const int* __restrict__ src,
+                  const int* __restrict__ prev, int n_prev, const bf16_t* __restrict__ table, int ldt, int col0, int dim, MllmStreamAdd add) {
+    constexpr int DIM = DT * 16, DK = (DIM + 31) / 32, GS = DK * 32 + 8, ZS = DIM + 4;
+    // (wide streams: the second map's tiles are asked for behind the first map's products, whose registers they take)
+    constexpr bool EARLY = KPW * (DT * 4 + 8) + CPW * (DK * 4 + 4) <= 96;
+    __shared__ __attribute__((aligned(16))) float z_s[SIDE_WAVES][ZS * 16];
+    __shared__ __attribute__((aligned(16))) bf16_t g_s[16 * GS];
+    __shared__ float ss_s[SIDE_WAVES][16];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / 64), lane = tid % 64, tok = lane % 16, q = lane / 16;
+    const int first = blockIdx.x * rows, n_rows = min(rows, T - first), KB = D / 32, CB = D / 16;
+    const size_t row_at = static_cast<size_t>(first + min(tok, n_rows - 1)) * D;          // (tokens that are not there: the last one, never stored)
+    // everything the kernel reads is asked for here: the first map's tiles with the stream, then the table's columns, the
+    // second map's tiles and the stream again as the result is laid out
+    bf16x8 wg[KPW][DT];
+    float4 xa[KPW][2];
+#pragma unroll
+    for (int u = 0; u < KPW; ++u) {
+        const int kb = min(wave + SIDE_WAVES * u, KB - 1);
+        xa[u][0] = *reinterpret_cast<const float4*>(x + row_at + kb * 32 + 8 * q);
+        xa[u][1] = *reinterpret_cast<const float4*>(x + row_at + kb * 32 + 8 * q + 4);
+#pragma unroll
+        for (int d = 0; d < DT; ++d) wg[u][d] = gate[(static_cast<size_t>(d) * KB + kb) * 64 + lane];
+    }
+    // thread -> (token, column of dim) for the step between the maps
+    const int e_tok = tid / DIM, e_col = tid % DIM;
+    float e_val = 0.f;
+    {
+        const int t = first + min(min(e_tok, 15), n_rows - 1);
+        int id = ids[t];
+        if (src != nullptr) {
+            const int s = src[t];
+            if (s >= 0 && s < n_prev) id = prev[s];
+        }
+        e_val = to_float(table[static_cast<size_t>(id) * ldt + col0 + min(e_col, dim - 1)]);
+    }
+    bf16x8 wp[CPW][DK];
+    float4 xv[CPW];
+    auto fetch_second = [&]() {
+#pragma unroll
+        for (int c = 0; c < CPW; ++c) {
+            const int cb = min(wave + SIDE_WAVES * c, CB - 1);
+#pragma unroll
+            for (int k = 0; k < DK; ++k) wp[c][k] = proj[(static_cast<size_t>(cb) * DK + k) * 64 + lane];
+            xv[c] = *reinterpret_cast<const float4*>(x + row_at + cb * 16 + 4 * q);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+    };
+    if (EARLY) fetch_second();
+    f32x4 acc[DT];
+#pragma unroll
+    for (int d = 0; d < DT; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int u = 0; u < KPW; ++u) {
+        if (wave + SIDE_WAVES * u >= KB) continue;
+        union { uint32_t w[4]; bf16x8 v; } b;
+        b.w[0] = pack_bf16x2(xa[u][0].x, xa[u][0].y); b.w[1] = pack_bf16x2(xa[u][0].z, xa[u][0].w);
+        b.w[2] = pack_bf16x2(xa[u][1].x, xa[u][1].y); b.w[3] = pack_bf16x2(xa[u][1].z, xa[u][1].w);
+#pragma unroll
+        for (int d = 0; d < DT; ++d) acc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wg[u][d], b.v, acc[d], 0, 0, 0);
+    }
+    // (register r of lane l: column of dim 4 (l / 16) + r, token l % 16)
+#pragma unroll
+    for (int d = 0; d < DT; ++d) *reinterpret_cast<f32x4*>(&z_s[wave][tok * ZS + d * 16 + 4 * q]) = acc[d];
+    if (!EARLY) fetch_second();
+    for (int i = tid; i < 16 * GS; i += SIDE_WAVES * 64) g_s[i] = float_to_bf16(0.f);
+    lds_barrier();
+    if (tid < DIM * 16) {
+        float z = 0.f;
+#pragma unroll
+        for (int w = 0; w < SIDE_WAVES; ++w) z += z_s[w][e_tok * ZS + e_col];
+        if (e_col < dim) g_s[e_tok * GS + e_col] = float_to_bf16(gelu_tanh(z) * e_val);
+    }
+    lds_barrier();
+    bf16x8 gb[DK];
+#pragma unroll
+    for (int k = 0; k < DK; ++k) gb[k] = *reinterpret_cast<const bf16x8*>(g_s + tok * GS + k * 32 + 8 * q);
+    f32x4 y[CPW];
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < CPW; ++c) {
+        y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < DK; ++k) y[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[c][k], gb[k], y[c], 0, 0, 0);
+        if (wave + SIDE_WAVES * c < CB) ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+    }
+    ss = rows_sum(ss);
+    if (lane < 16) ss_s[wave][lane] = ss;
+    lds_barrier();
+    float total = 0.f;
+#pragma unroll
+    for (int w = 0; w < SIDE_WAVES; ++w) total += ss_s[w][tok];
+    const float inv = 1.f / sqrtf(total / static_cast<float>(D) + eps);
+    if (tok >= n_rows) return;
+    const bool has_next = add.next.weight != nullptr;
+    const float alpha = has_next ? add.next.alpha[0] : 0.f;
+#pragma unroll
+    for (int c = 0; c < CPW; ++c) {
+        const int cb = wave + SIDE_WAVES * c;
+        if (cb >= CB) continue;
+        const int n = cb * 16 + 4 * q;
+        const float4 w4 = *reinterpret_cast<const float4*>(weight + n);
+        float o[4] = {xv[c].x + y[c][0] * inv * w4.x, xv[c].y + y[c][1] * inv * w4.y, xv[c].z + y[c][2] * inv * w4.z, xv[c].w + y[c][3] * inv * w4.w};
+        *reinterpret_cast<float4*>(x + row_at + n) = make_float4(o[0], o[1], o[2], o[3]);
+        if (add.copy == nullptr) continue;
+        if (has_next) {
+            const float4 nw = *reinterpret_cast<const float4*>(add.next.weight + n), nb = *reinterpret_cast<const float4*>(add.next.bias + n);
+            o[0] = fast_tanh(alpha * o[0]) * nw.x + nb.x; o[1] = fast_tanh(alpha * o[1]) * nw.y + nb.y;
+            o[2] = fast_tanh(alpha * o[2]) * nw.z + nb.z; o[3] = fast_tanh(alpha * o[3]) * nw.w + nb.w;
+        }
+        *reinterpret_cast<uint2*>(static_cast<bf16_t*>(add.copy) + static_cast<size_t>(first + tok) * add.ld_copy + n) =
+            make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+    }
+}
+
 bool on16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 bool norm_on16(const MllmTanhNorm& n) { return n.weight == nullptr || (on16(n.weight) && on16(n.bias)); }
 
@@ -149,6 +279,34 @@ int mllm_token_gate(const float* z, int ldz, const int* ids, const int* src, con
         token_gate_kernel<float><<<T, threads, 0, stream>>>(z, ldz, ids, src, prev, n_prev, static_cast<const float*>(table), ldt, col0, dim, static_cast<float*>(out), ldo);
     else
         token_gate_kernel<bf16_t><<<T, threads, 0, stream>>>(z, ldz, ids, src, prev, n_prev, static_cast<const bf16_t*>(table), ldt, col0, dim, static_cast<bf16_t*>(out), ldo);
+    MLLM_LAUNCH_CHECK();
+    return 0;
+}
+
+// The sizes token_side_kernel is built for: a width of up to 2,048 in whole tiles of 32, up to 64 columns a token.
+int mllm_token_side_fits(int D, int dim) { return D >= 32 && D % 32 == 0 && D <= 2048 && dim >= 1 && dim <= 64 ? 1 : 0; }
+
+// x fp32 [T, D] contiguous; gate and proj bfloat16 in tiles (see the kernel; dim filled up with zeros to a multiple of 16 in the
+// gate's rows and of 32 in proj's inputs); weight [D]; ids, src, prev, table as for mllm_token_gate. Tokens up to
+// 2,048 take 8 a workgroup, more take 16. -2: sizes the kernel is not built for; -1: operands that are not aligned.
+int mllm_token_side(float* x, int T, int D, const void* gate, const void* proj, const float* weight, float eps, const int* ids, const int* src,
+                    const int* prev, int n_prev, const void* table, int ldt, int col0, int dim, MllmStreamAdd add, hipStream_t stream) {
+    if (T <= 0) return 0;
+    if (!mllm_token_side_fits(D, dim)) return -2;
+    if (ids == nullptr || (src != nullptr && prev == nullptr) || !on16(x) || !on16(gate) || !on16(proj) || !on16(weight) || !norm_on16(add.next) ||
+        (add.copy != nullptr && (add.ld_copy % 4 != 0 || (reinterpret_cast<uintptr_t>(add.copy) & 7))))
+        return -1;
+    const int rows = T <= 2048 ? 8 : 16, blocks = (T + rows - 1) / rows;
+    const int dt = dim <= 16 ? 1 : (dim <= 32 ? 2 : 4), kpw = D <= 512 ? 1 : (D <= 1024 ? 2 : 4);
+#define TOKEN_SIDE(DT, KPW, CPW)                                                                                                        \
+    token_side_kernel<DT, KPW, CPW><<<blocks, SIDE_WAVES * 64, 0, stream>>>(x, T, rows, D, static_cast<const bf16x8*>(gate),              \
+        static_cast<const bf16x8*>(proj), weight, eps, ids, src, prev, n_prev, static_cast<const bf16_t*>(table), ldt, col0, dim, add)
+#define TOKEN_SIDE_D(DT) do { if (kpw == 1) TOKEN_SIDE(DT, 1, 2); else if (kpw == 2) TOKEN_SIDE(DT, 2, 4); else TOKEN_SIDE(DT, 4, 8); } while (0)
+    if (dt == 1) TOKEN_SIDE_D(1);
+    else if (dt == 2) TOKEN_SIDE_D(2);
+    else TOKEN_SIDE_D(4);
+#undef TOKEN_SIDE_D
+#undef TOKEN_SIDE
     MLLM_LAUNCH_CHECK();
     return 0;
 }
