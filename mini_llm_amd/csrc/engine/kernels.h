@@ -158,12 +158,13 @@ int mllm_hgrn2_chunk();
 // matrix_memory.hip
 int mllm_matrix_memory_chunk();
 int mllm_matrix_memory_copies(int d, int e);
-size_t mllm_matrix_memory_state_floats(int H, int d, int e);
+size_t mllm_matrix_memory_state_floats(int H, int d, int e, int retention = 0);
 size_t mllm_matrix_memory_workspace_floats(int T, int B, int H, int d, int e);
 int mllm_matrix_memory(const float* proj, int ld, int q_col, int k_col, int v_col, int g_col, int i_col, int f_col, const float* i_bias,
                        const float* f_bias, const float* norm_w, float cap, float q_scale, float eps, const int* cu_q, const int* state_slots,
                        float* state, size_t slot_floats, int T, int B, int n_single, int max_portion, int H, int d, int e, int write,
-                       float* workspace, void* out, int ldo, float* y, int ldy, int dtype, int* needs_norm, hipStream_t stream);
+                       float* workspace, void* out, int ldo, float* y, int ldy, int dtype, int* needs_norm, hipStream_t stream,
+                       const float* head_decay = nullptr, int silu = 0);
 
 int mllm_concat_cast(const float* a, const float* b, int T, int D, void* out, int dtype, hipStream_t stream);
 int mllm_glu_act(const void* gu, int ld, int T, int F, int act, void* out, int ldo, int dtype, hipStream_t stream);

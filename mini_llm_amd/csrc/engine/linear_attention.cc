@@ -91,6 +91,23 @@ public:
         const int T = step.n_tokens, inner = H_ * dv_;
         // queries and keys lie side by side: one turn over 2 * heads heads
         if (rot_dims_ > 0) rotary_rows(proj, 0, 2 * H_, d_, rot_dims_, rot_base_, step.positions, s);
+        if (head_decay_ != nullptr) {
+            // one fixed decay per head: chunks of products on the fp32 matrix cores, norm and gate inside; single tokens in one
+            // kernel
+            MemoryShape sh;
+            sh.heads = H_; sh.dim = d_; sh.value_dim = dv_; sh.k_col = k_col_; sh.v_col = v_col_; sh.g_col = g_col_;
+            sh.q_scale = q_scale_ * k_scale_; sh.eps = eps_; sh.norm = norm_; sh.head_decay = head_decay_; sh.silu_gate = true;
+            StateArgs st;
+            st.token_seq = step.token_seq; st.cu_q = step.cu_q; st.state_slots = step.state_slots; st.n_seqs = step.n_seqs;
+            st.max_q_len = step.max_q_len; st.n_single = step.n_single; st.state = static_cast<float*>(cache.state);
+            st.slot_floats = cache.slot_bytes / 4; st.n_slots = cache.n_slots; st.write = write;
+            const size_t ws_floats = matrix_memory_workspace_floats(T, step.n_seqs, H_, d_, dv_);
+            float* ws = static_cast<float*>(arena.take(ws_floats * 4));
+            const Tensor2 y = arena.tensor(F32, T, inner);
+            matrix_memory(proj, sh, st, normed, y, ws, ws_floats, s);
+            StageTimes::get().mark("memory", s);
+            return;
+        }
         Tensor2 decay;
         if (rank_ > 0) {
             decay = arena.tensor(F32, T, H_ * d_);
@@ -115,7 +132,8 @@ public:
                                               (H_ * dv_ + in_.in_features()) * dtype_size(dtype_)) +
                // (every sequence of a step adds at most one chunk that is not full; a step holds at most as many
                // sequences as tokens)
-               hgrn2_workspace_floats(tokens, std::min(tokens, 256), H_, d_, dv_) * 4 + 8192;
+               std::max(hgrn2_workspace_floats(tokens, std::min(tokens, 256), H_, d_, dv_),
+                        head_decay_ != nullptr ? matrix_memory_workspace_floats(tokens, std::min(tokens, 256), H_, d_, dv_) : 0) * 4 + 8192;
     }
     CacheNeed cache_need() const override {
         CacheNeed n;

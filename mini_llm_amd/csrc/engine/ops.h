@@ -341,6 +341,10 @@ struct MemoryShape {
     float cap = 0.f, q_scale = 1.f, eps = 1e-6f;
     const float *i_bias = nullptr, *f_bias = nullptr;      // [heads]
     const float* norm = nullptr;                           // [heads * value_dim]
+    // retention instead: S <- decay S + k v^T with one fixed decay per head ([heads] on the device), o = S^T q, no input or
+    // forget gates (i_col, f_col, the biases and cap are not used) and no normaliser; norm may then be null (no weight)
+    const float* head_decay = nullptr;
+    bool silu_gate = false;                                // the output gate is silu(raw) instead of sigmoid(raw)
 };
 // out [T, heads * value_dim] (the compute dtype): every head's readout, RMS-normed, weighed and gated. The state of a request
 // (matrix_memory_state_floats floats) starts at st.state. The first st.n_single sequences bring one token each; portions
@@ -348,7 +352,7 @@ struct MemoryShape {
 // shape): room for heads whose work several workgroups share.
 void matrix_memory(const Tensor2& proj, const MemoryShape& sh, const StateArgs& st, const Tensor2& out, const Tensor2& y, float* workspace,
                    size_t workspace_floats, hipStream_t stream);
-size_t matrix_memory_state_floats(int heads, int dim, int value_dim);
+size_t matrix_memory_state_floats(int heads, int dim, int value_dim, bool retention = false);
 size_t matrix_memory_workspace_floats(int tokens, int n_seqs, int heads, int dim, int value_dim);
 
 // -- gated linear recurrence (HGRN2) ----------------------------------------------------------------

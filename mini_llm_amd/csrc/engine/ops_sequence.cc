@@ -166,7 +166,7 @@ size_t ssm_scan_workspace_floats(int tokens, int n_seqs, int H, int P, int N) {
     return mllm_ssm_scan_workspace_floats(tokens, n_seqs, H, P, N);
 }
 
-size_t matrix_memory_state_floats(int heads, int dim, int value_dim) { return mllm_matrix_memory_state_floats(heads, dim, value_dim); }
+size_t matrix_memory_state_floats(int heads, int dim, int value_dim, bool retention) { return mllm_matrix_memory_state_floats(heads, dim, value_dim, retention ? 1 : 0); }
 size_t matrix_memory_workspace_floats(int tokens, int n_seqs, int heads, int dim, int value_dim) {
     return mllm_matrix_memory_workspace_floats(tokens, n_seqs, heads, dim, value_dim);
 }
@@ -177,14 +177,15 @@ void matrix_memory(const Tensor2& proj, const MemoryShape& sh, const StateArgs& 
     need_act(out, "matrix_memory: out");
     need_f32(y, "matrix_memory: y");
     const int H = sh.heads, d = sh.dim, e = sh.value_dim, T = i32(proj.rows);
-    if (H < 1 || d < 1 || e < 1 || !(sh.cap > 0.f)) fail("matrix_memory: heads, sizes and the gates' cap must be positive");
+    const bool retention = sh.head_decay != nullptr;
+    if (H < 1 || d < 1 || e < 1 || (!retention && !(sh.cap > 0.f))) fail("matrix_memory: heads, sizes and the gates' cap must be positive");
     auto inside = [&](int col, int64_t n) { return col >= 0 && col + n <= proj.cols; };
     const int64_t nk = static_cast<int64_t>(H) * d, nv = static_cast<int64_t>(H) * e;
-    if (!inside(sh.q_col, nk) || !inside(sh.k_col, nk) || !inside(sh.v_col, nv) || !inside(sh.g_col, nv) || !inside(sh.i_col, H) || !inside(sh.f_col, H))
+    if (!inside(sh.q_col, nk) || !inside(sh.k_col, nk) || !inside(sh.v_col, nv) || !inside(sh.g_col, nv) || (!retention && (!inside(sh.i_col, H) || !inside(sh.f_col, H))))
         fail("matrix_memory: the inputs lie outside the projection's rows of %lld", (long long)proj.cols);
-    if (sh.i_bias == nullptr || sh.f_bias == nullptr || sh.norm == nullptr) fail("matrix_memory: the gates' biases and the norm's weight are needed");
+    if (!retention && (sh.i_bias == nullptr || sh.f_bias == nullptr || sh.norm == nullptr)) fail("matrix_memory: the gates' biases and the norm's weight are needed");
     if (out.rows != T || out.cols != nv || y.rows != T || y.cols != nv) fail("matrix_memory: out and y must be [%d, %lld]", T, (long long)nv);
-    check_state(st, matrix_memory_state_floats(H, d, e), "matrix_memory");
+    check_state(st, matrix_memory_state_floats(H, d, e, retention), "matrix_memory");
     if (st.n_single < 0 || st.n_single > st.n_seqs) fail("matrix_memory: %d of %d sequences", st.n_single, st.n_seqs);
     const int max_portion = st.n_single == st.n_seqs ? 0 : std::max(st.max_q_len, 1);
     if (workspace != nullptr && workspace_floats < matrix_memory_workspace_floats(T, st.n_seqs, H, d, e))
@@ -193,12 +194,12 @@ void matrix_memory(const Tensor2& proj, const MemoryShape& sh, const StateArgs& 
     check(mllm_matrix_memory(static_cast<const float*>(proj.data), i32(proj.stride), sh.q_col, sh.k_col, sh.v_col, sh.g_col, sh.i_col, sh.f_col,
                              sh.i_bias, sh.f_bias, sh.norm, sh.cap, sh.q_scale, sh.eps, st.cu_q, st.state_slots, st.state, st.slot_floats, T, st.n_seqs,
                              st.n_single, max_portion, H, d, e, st.write ? 1 : 0, workspace, out.data, i32(out.stride), static_cast<float*>(y.data),
-                             i32(y.stride), out.dtype, &needs_norm, stream), "matrix_memory");
+                             i32(y.stride), out.dtype, &needs_norm, stream, sh.head_decay, sh.silu_gate ? 1 : 0), "matrix_memory");
     // rows whose heads were shared by several workgroups: their norm and gate
     const int64_t first = (needs_norm & 1) ? 0 : st.n_single, last = (needs_norm & 2) ? T : st.n_single;
     if (needs_norm != 0 && first < last)
         rmsnorm_gate_after(y.row_range(first, last - first), sh.norm, sh.eps, H, proj.row_range(first, last - first), sh.g_col,
-                           out.row_range(first, last - first), stream, 1, 0, true);
+                           out.row_range(first, last - first), stream, 1, 0, !sh.silu_gate);
 }
 
 static void check_shape(const LatentShape& sh, const char* what) {

@@ -23,6 +23,10 @@
 // the subtraction.
 //
 // State of a request: S [H][d][e], then n [H][copies][d], then m [H][copies], fp32.
+//
+// The same kernels run retention (head_decay given): S <- decay_h S + k v^T, o = S^T q, no normaliser. With i = 0 and f = log
+// decay_h every u_s = -F_s grows with s, so that r_t = -F_t, the weights inside a chunk are decay^(t - s), the carried memory's
+// decay^(t + 1), and m stays 0; n and m are then neither kept nor read (the state is S alone) and nothing is divided.
 #include "common.h"
 
 #define MM_CHUNK 64
@@ -39,6 +43,8 @@ struct MemoryArgs {
     const float* f_bias;
     const float* norm_w;               // [H * e]
     float cap, q_scale, eps;
+    const float* head_decay;           // [H]: retention with these decays; null: gates from the rows
+    int silu;                          // the output gate is silu(raw) instead of sigmoid(raw)
     const int* cu_q;
     const int* state_slots;
     float* state;
@@ -52,6 +58,9 @@ __device__ __forceinline__ float mm_log_forget(float raw, float bias, float cap)
     const float z = cap * tanhf((raw + bias) / cap);
     return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
 }
+
+__device__ __forceinline__ float mm_gate(const MemoryArgs& a, float z) { return (a.silu ? z : 1.f) * mm_sigmoid(z); }
+__device__ __forceinline__ float mm_norm_weight(const MemoryArgs& a, int col) { return a.norm_w != nullptr ? a.norm_w[col] : 1.f; }
 
 // Where a chunk's or a request's numbers lie.
 __device__ __forceinline__ size_t state_n_at(const MemoryArgs& a, int h, int copy) {
@@ -101,6 +110,12 @@ __device__ __forceinline__ bool find_chunk(const int* __restrict__ cu_q, const i
 
 // The gates of a chunk's tokens, token t in lane t: F_t and u_t = i_t - F_t (tokens beyond n: F stays, u = -inf).
 __device__ __forceinline__ void chunk_gates(const MemoryArgs& a, int h, int first, int n, int lane, double& F, double& u) {
+    if (a.head_decay != nullptr) {
+        const int upto = min(lane + 1, n);
+        F = upto * log(static_cast<double>(a.head_decay[h]));
+        u = lane < n ? -F : -INFINITY;
+        return;
+    }
     const float* row = a.proj + static_cast<size_t>(first + min(lane, n - 1)) * a.ld;
     const float iz = row[a.i_col + h], fz = row[a.f_col + h];
     const float ig = mm_log_input(iz, a.i_bias[h], a.cap);
@@ -217,7 +232,7 @@ memory_chunk_kernel(MemoryArgs a, int first_seq, int n_seqs, int value_tiles, fl
                 float* sc = W + chunk_scalars_at(a.d, a.e);
                 sc[0] = static_cast<float>(U + F);
                 sc[1] = static_cast<float>(F);
-                if (chunk == 0) sc[2] = a.state[static_cast<size_t>(slot) * a.slot_floats + state_m_at(a, h, 0)];
+                if (chunk == 0) sc[2] = a.head_decay != nullptr ? 0.f : a.state[static_cast<size_t>(slot) * a.slot_floats + state_m_at(a, h, 0)];
             }
         }
     }
@@ -263,7 +278,7 @@ memory_states_kernel(MemoryArgs a, int first_seq, float* __restrict__ ws) {
 #pragma unroll
     for (int off = 32; off > 0; off /= 2) before += __shfl_xor(before, off, MLLM_WAVE);
     const int nc = (a.cu_q[b + 1] - a.cu_q[b] + MM_CHUNK - 1) / MM_CHUNK;
-    const long long per_head = static_cast<long long>(a.d) * a.e + a.d;
+    const long long per_head = static_cast<long long>(a.d) * a.e + (a.head_decay != nullptr ? 0 : a.d);
     const long long idx = static_cast<long long>(blockIdx.x) * 256 + threadIdx.x;
     if (idx >= per_head * a.H || nc == 0) return;
     const int h = static_cast<int>(idx / per_head);
@@ -419,7 +434,7 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
             Ps[(4 * G + r) * MM_STRIDE + s] = x;
         }
         start[r] = start_s[t];
-        den[r] = 1.f / (fmaxf(fabsf(group_sum<16>(sum) + start[r] * nq_s[t]), floor_s[t]) + 1e-6f);
+        den[r] = a.head_decay != nullptr ? 1.f : 1.f / (fmaxf(fabsf(group_sum<16>(sum) + start[r] * nq_s[t]), floor_s[t]) + 1e-6f);
     }
     lds_barrier();
     float ss[4] = {0.f, 0.f, 0.f, 0.f};
@@ -458,7 +473,7 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
     float4 gate4[4], norm4;
     if (VEC && FUSED) {
         const int col = h * a.e + 64 * vt0 + min(4 * c, min(64, a.e - 64 * vt0) - 4);
-        norm4 = *reinterpret_cast<const float4*>(a.norm_w + col);
+        norm4 = a.norm_w != nullptr ? *reinterpret_cast<const float4*>(a.norm_w + col) : make_float4(1.f, 1.f, 1.f, 1.f);
 #pragma unroll
         for (int u = 0; u < 4; ++u)
             gate4[u] = *reinterpret_cast<const float4*>(rows + static_cast<size_t>(min(16 * wave + 4 * u + G, n - 1)) * a.ld + a.g_col + col);
@@ -488,8 +503,9 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
                     continue;
                 }
                 const float4 g = t == 0 ? gate4[u] : *reinterpret_cast<const float4*>(rows + static_cast<size_t>(tok) * a.ld + a.g_col + col0 + col);
-                const float4 w = t == 0 ? norm4 : *reinterpret_cast<const float4*>(a.norm_w + col0 + col);
-                x.x *= w.x * mm_sigmoid(g.x); x.y *= w.y * mm_sigmoid(g.y); x.z *= w.z * mm_sigmoid(g.z); x.w *= w.w * mm_sigmoid(g.w);
+                float4 w = norm4;
+                if (t > 0 && a.norm_w != nullptr) w = *reinterpret_cast<const float4*>(a.norm_w + col0 + col);
+                x.x *= w.x * mm_gate(a, g.x); x.y *= w.y * mm_gate(a, g.y); x.z *= w.z * mm_gate(a, g.z); x.w *= w.w * mm_gate(a, g.w);
                 T* dst = out + static_cast<size_t>(first + tok) * ldo + col0 + col;
                 if (sizeof(T) == 2) {
                     uint2 pk;
@@ -507,7 +523,7 @@ memory_output_kernel(MemoryArgs a, int first_seq, int n_seqs, const float* __res
                 const float x = Ps[tt * MM_STRIDE + lane];
                 if (FUSED) {
                     const float g = rows[static_cast<size_t>(tok) * a.ld + a.g_col + col0 + lane];
-                    out[static_cast<size_t>(first + tok) * ldo + col0 + lane] = from_float<T>(x * a.norm_w[col0 + lane] * mm_sigmoid(g));
+                    out[static_cast<size_t>(first + tok) * ldo + col0 + lane] = from_float<T>(x * mm_norm_weight(a, col0 + lane) * mm_gate(a, g));
                 } else {
                     y[static_cast<size_t>(first + tok) * ldy + col0 + lane] = x;
                 }
@@ -539,7 +555,8 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
     float* base = a.state + static_cast<size_t>(slot) * a.slot_floats;
     float* S = base + static_cast<size_t>(h) * d * e + c0;
     float* N = base + state_n_at(a, h, tile);
-    const float iz = row[a.i_col + h], fz = row[a.f_col + h], m_old = base[state_m_at(a, h, tile)];
+    const bool fixed = a.head_decay != nullptr;               // (retention: a decay of the head's own, no normaliser)
+    const float iz = fixed ? 0.f : row[a.i_col + h], fz = fixed ? 0.f : row[a.f_col + h], m_old = fixed ? 0.f : base[state_m_at(a, h, tile)];
     const int rg = tid / groups, col = (tid % groups) * CW;
     const bool active = rg < RG && col < nc;
     const int col_c = min(col, nc - CW);                      // a valid place in any case
@@ -561,18 +578,25 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
         }
     };
     ask(0);
-    const float n_first = N[min(tid, d - 1)];
-    const float g_first = row[a.g_col + h * e + c0 + min(lane, nc - 1)], w_first = a.norm_w[h * e + c0 + min(lane, nc - 1)];
+    const float n_first = fixed ? 0.f : N[min(tid, d - 1)];
+    const float g_first = row[a.g_col + h * e + c0 + min(lane, nc - 1)], w_first = mm_norm_weight(a, h * e + c0 + min(lane, nc - 1));
     for (int i = tid; i < d; i += 256) {
         q_s[i] = row[a.q_col + h * d + i] * a.q_scale;
         k_s[i] = row[a.k_col + h * d + i];
     }
-    const float ig = mm_log_input(iz, a.i_bias[h], a.cap), fg = mm_log_forget(fz, a.f_bias[h], a.cap);
-    const float m = fmaxf(fg + m_old, ig), keep = expf(fg + m_old - m), take = expf(ig - m);
+    float m = 0.f, keep, take = 1.f;
+    if (fixed) {
+        keep = a.head_decay[h];
+    } else {
+        const float ig = mm_log_input(iz, a.i_bias[h], a.cap), fg = mm_log_forget(fz, a.f_bias[h], a.cap);
+        m = fmaxf(fg + m_old, ig);
+        keep = expf(fg + m_old - m);
+        take = expf(ig - m);
+    }
     lds_barrier();
     // the normaliser (its new values are written behind the barrier below: m_old and N are this workgroup's own copy)
     float nq = 0.f;
-    for (int i = tid; i < d; i += 256) {
+    for (int i = fixed ? d : tid; i < d; i += 256) {
         const float x = keep * (i == tid ? n_first : N[i]) + take * k_s[i];
         if (a.write) N[i] = x;
         nq = fmaf(x, q_s[i], nq);
@@ -606,10 +630,10 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
     }
     nq = wave_sum(nq);
     if (lane == 0) red[wave] = nq;
-    if (tid == 0 && a.write) base[state_m_at(a, h, tile)] = m;        // (every wavefront has read m_old: it stands in front of the barrier above)
+    if (tid == 0 && a.write && !fixed) base[state_m_at(a, h, tile)] = m;        // (every wavefront has read m_old: it stands in front of the barrier above)
     lds_barrier();
     if (wave != 0) return;
-    const float den = fmaxf(fabsf((red[0] + red[1]) + (red[2] + red[3])), expf(-m)) + 1e-6f;
+    const float den = fixed ? 1.f : fmaxf(fabsf((red[0] + red[1]) + (red[2] + red[3])), expf(-m)) + 1e-6f;
     // one wavefront finishes: columns lane, lane + 64, ... (FUSED: two passes, the sums kept in LDS)
     float ss = 0.f;
     for (int j = lane; j < nc; j += MLLM_WAVE) {
@@ -623,8 +647,8 @@ memory_single_kernel(MemoryArgs a, int cols, T* __restrict__ out, int ldo, float
     if (!FUSED) return;
     const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(e) + a.eps);
     for (int j = lane; j < nc; j += MLLM_WAVE) {
-        const float g = j == lane ? g_first : row[a.g_col + h * e + j], w = j == lane ? w_first : a.norm_w[h * e + j];
-        out[static_cast<size_t>(b) * ldo + h * e + j] = from_float<T>(part[j] * inv * w * mm_sigmoid(g));
+        const float g = j == lane ? g_first : row[a.g_col + h * e + j], w = j == lane ? w_first : mm_norm_weight(a, h * e + j);
+        out[static_cast<size_t>(b) * ldo + h * e + j] = from_float<T>(part[j] * inv * w * mm_gate(a, g));
     }
 }
 
@@ -642,7 +666,8 @@ int mllm_matrix_memory_copies(int d, int e) {
     if (static_cast<long long>(d) * e <= MM_ONE_WORKGROUP && (e % 4 == 0 ? e <= 1024 : e <= 256)) return 1;
     return (e + 63) / 64;
 }
-size_t mllm_matrix_memory_state_floats(int H, int d, int e) {
+size_t mllm_matrix_memory_state_floats(int H, int d, int e, int retention) {
+    if (retention) return static_cast<size_t>(H) * d * e;
     const size_t copies = mllm_matrix_memory_copies(d, e);
     return static_cast<size_t>(H) * d * e + static_cast<size_t>(H) * copies * (static_cast<size_t>(d) + 1);
 }
@@ -656,22 +681,25 @@ size_t mllm_matrix_memory_workspace_floats(int T, int B, int H, int d, int e) {
 // n_single sequences bring one token each, the others any number; max_portion: the longest portion among those (0: there
 // are none). out [T, H * e] in `dtype`: normed and gated, if *needs_norm comes back 0; otherwise y ([T, ldy] fp32) holds
 // o of those rows that the caller must norm: *needs_norm bit 0 the single tokens' rows, bit 1 the portions' rows.
-// A request's state starts at its slot. -1: sizes or pointers that do not fit; -2: a key width beyond the LDS.
+// A request's state starts at its slot. head_decay ([H], on the device; the i and f columns and biases and cap are then not used)
+// makes it retention, norm_w may be null (no weight), silu: the output gate is silu. -1: sizes or pointers that do not fit; -2: a key width beyond the LDS.
 int mllm_matrix_memory(const float* proj, int ld, int q_col, int k_col, int v_col, int g_col, int i_col, int f_col, const float* i_bias,
                        const float* f_bias, const float* norm_w, float cap, float q_scale, float eps, const int* cu_q, const int* state_slots,
                        float* state, size_t slot_floats, int T, int B, int n_single, int max_portion, int H, int d, int e, int write,
-                       float* workspace, void* out, int ldo, float* y, int ldy, int dtype, int* needs_norm, hipStream_t stream) {
+                       float* workspace, void* out, int ldo, float* y, int ldy, int dtype, int* needs_norm, hipStream_t stream,
+                       const float* head_decay, int silu) {
     *needs_norm = 0;
     bool singles_in_chunks = false;
     if (T <= 0 || B <= 0) return 0;
-    if (H < 1 || d < 1 || e < 1 || !(cap > 0.f) || n_single < 0 || n_single > B || proj == nullptr || i_bias == nullptr || f_bias == nullptr) return -1;
+    if (H < 1 || d < 1 || e < 1 || n_single < 0 || n_single > B || proj == nullptr) return -1;
+    if (head_decay == nullptr && (!(cap > 0.f) || i_bias == nullptr || f_bias == nullptr)) return -1;
     const int copies = mllm_matrix_memory_copies(d, e);
-    const MemoryArgs a{proj, ld, q_col, k_col, v_col, g_col, i_col, f_col, i_bias, f_bias, norm_w, cap, q_scale, eps, cu_q, state_slots,
+    const MemoryArgs a{proj, ld, q_col, k_col, v_col, g_col, i_col, f_col, i_bias, f_bias, norm_w, cap, q_scale, eps, head_decay, silu, cu_q, state_slots,
                        state, slot_floats, H, d, e, copies, write};
     const auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
     // (16-byte accesses: every row and head starts on a multiple of 4 floats; bfloat16 rows on 8 bytes)
     const bool vec = d % 4 == 0 && e % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && v_col % 4 == 0 && g_col % 4 == 0 && ldo % 4 == 0 &&
-                     ldy % 4 == 0 && slot_floats % 4 == 0 && a16(proj) && a16(state) && a16(workspace) && a16(out) && a16(y) && a16(norm_w);
+                     ldy % 4 == 0 && slot_floats % 4 == 0 && a16(proj) && a16(state) && a16(workspace) && a16(out) && a16(y) && (norm_w == nullptr || a16(norm_w));
     if (n_single > 0) {
         const bool fused = copies == 1;
         const bool v4 = vec && (!fused || e <= 1024);
