@@ -178,6 +178,10 @@ int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int 
                      int router_kind, float limit, float shared_limit, float alpha, int weight_on_input, int shared_gate, void* out,
                      int ldo, int T, int dtype, hipStream_t stream, float up_shift = 1.f, int up_dtype = -1);
 
+int mllm_moe_grouped_glu(const void* h, int ldh, const float* logits, int ldl, int T, int D, int E, int ff, int top, float scale, int router_kind,
+                         float limit, float alpha, float up_shift, const void* up, int ldu, const void* down, int ldd, int* counts, int* lists,
+                         float* weights, void* act, float* y, float* x, int add_to, MllmStreamAdd add, hipStream_t stream);
+
 // tanh_norm.hip
 int mllm_tanh_norm(const float* x, int ldx, const int* rows, MllmTanhNorm norm, void* out, int ldo, int n, int D, int dtype, hipStream_t stream);
 int mllm_stream_add(float* x, const float* y, const float* x0, const float* step, int n, int D, MllmStreamAdd add, int precise, hipStream_t stream);

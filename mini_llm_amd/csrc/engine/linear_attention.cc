@@ -248,6 +248,19 @@ public:
         run(h, step, add.x, arena, s, STORE_F32, &add);
     }
     void run(NormedInput& h, const StepView& step, const Tensor2& x, Arena& arena, hipStream_t s, int out_epilogue, const StreamAdd* add = nullptr) const {
+        if (gated_ && dtype_ == BF16 && moe_grouped_fits(step.n_tokens, up_.in_features(), glu_)) {
+            // many tokens, few experts each: the router's product, then every expert on its own tokens
+            const Tensor2& in = h.tensor(arena, s);
+            const int T = step.n_tokens, R = router_.out_features(), lde = (R + 3) / 4 * 4;
+            const Tensor2 z(arena.take(static_cast<size_t>(T) * lde * 4), F32, T, R, lde);
+            router_(in, z, STORE_F32, nullptr, s);
+            StageTimes::get().mark("router", s);
+            void* room = arena.take(moe_grouped_bytes(T, up_.in_features(), glu_));
+            if (moe_grouped(in, z, glu_, up_.weight, down_.weight, x, out_epilogue == ADD_RESIDUAL, add, room, s)) {
+                StageTimes::get().mark("experts", s);
+                return;
+            }
+        }
         Pending p;
         first_products(h, step, arena, s, p, false);
         if (opt_.identity > 0) p.h = h.tensor(arena, s);
@@ -309,9 +322,17 @@ public:
     }
     size_t workspace_bytes(int tokens) const override {
         const size_t few = up_router_.weight.data != nullptr ? static_cast<size_t>(std::min(tokens, tuning().ln_fuse_max_rows)) * (up_router_.out_features() + 4) * 4 + 256 : 0;
-        return static_cast<size_t>(tokens) * ((up_.out_features() + down_.in_features() + up_.in_features()) * dtype_size(dtype_) + (E_ + opt_.identity + 8) * 4) + few + 2048;
+        return static_cast<size_t>(tokens) * ((up_.out_features() + down_.in_features() + up_.in_features()) * dtype_size(dtype_) + (E_ + opt_.identity + 8) * 4) + few + 2048 +
+               grouped_bytes(std::min(tokens, 65535));
     }
-    void reserve(int, hipStream_t s) const override { reserve_linear_scratch(s); }
+    void reserve(int, hipStream_t s) const override {
+        reserve_linear_scratch(s);
+        if (gated_ && dtype_ == BF16) reserve_moe_scratch(s);
+    }
+    size_t grouped_bytes(int tokens) const {           // (steps of more tokens multiply densely)
+        if (!gated_ || dtype_ != BF16 || !moe_grouped_fits(tokens, up_.in_features(), glu_)) return 0;
+        return moe_grouped_bytes(tokens, up_.in_features(), glu_) + static_cast<size_t>(tokens) * (E_ + 8) * 4;
+    }
     void add_cost(StepCost& c) const override {
         up_.add_cost(c);
         down_.add_cost(c);

@@ -298,6 +298,47 @@ void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, co
     stream_add(add, nullptr, nullptr, a.dtype == F32, stream);
 }
 
+// Counters of the grouped experts' routing: zero at first, left zero by every use.
+static int* moe_counts(hipStream_t s) { return static_cast<int*>(scratch("moe_counts", 256 * sizeof(int), true, s)); }
+void reserve_moe_scratch(hipStream_t stream) { moe_counts(stream); }
+
+bool moe_grouped_fits(int T, int D, const MoeGlu& m) {
+    const int from = tuning().grouped_experts_rows;
+    return from > 0 && T >= from && T <= 65535 && m.shared_ff == 0 && !m.weight_on_input && 2 * m.top <= m.experts && m.top <= 8 && m.experts <= 256 && D % 8 == 0 && m.ff % 8 == 0;
+}
+
+size_t moe_grouped_bytes(int T, int D, const MoeGlu& m) {
+    const size_t slots = static_cast<size_t>(T) * m.top;
+    return slots * D * 4 + slots * m.ff * 2 + slots * 4 + static_cast<size_t>(m.experts) * T * 4 + 4 * 256;
+}
+
+bool moe_grouped(const Tensor2& h, const Tensor2& logits, const MoeGlu& m, const Tensor2& up, const Tensor2& down, const Tensor2& x, bool add_to,
+                 const StreamAdd* through, void* room, hipStream_t stream) {
+    const int T = static_cast<int>(h.rows), D = static_cast<int>(h.cols);
+    if (!moe_grouped_fits(T, D, m)) return false;
+    if (h.dtype != BF16 || up.dtype != BF16 || down.dtype != BF16 || logits.dtype != F32) return false;
+    if (logits.rows != T || logits.cols != m.experts || up.rows != 2ll * m.experts * m.ff || up.cols != D || down.rows != D || down.cols != static_cast<int64_t>(m.experts) * m.ff)
+        fail("moe_grouped: the experts' matrices do not fit %d experts of %d at width %d", m.experts, m.ff, D);
+    if (x.dtype != F32 || !x.contiguous() || x.rows != T || x.cols != D) fail("moe_grouped: the result must be contiguous float32 [%d, %d]", T, D);
+    if (through != nullptr) check_stream_add(*through, "moe_grouped");
+    char* at = static_cast<char*>(room);
+    auto take = [&](size_t bytes) { char* p = at; at += (bytes + 255) & ~static_cast<size_t>(255); return p; };
+    const size_t slots = static_cast<size_t>(T) * m.top;
+    float* y = reinterpret_cast<float*>(take(slots * D * 4));
+    void* act = take(slots * m.ff * 2);
+    float* weights = reinterpret_cast<float*>(take(slots * 4));
+    int* lists = reinterpret_cast<int*>(at);
+    MllmStreamAdd add{{nullptr, nullptr, nullptr}, {nullptr, nullptr, nullptr}, nullptr, 0};
+    if (through != nullptr) add = MllmStreamAdd{through->norm, through->next, through->copy.data, static_cast<int>(through->copy.stride)};
+    const int rc = mllm_moe_grouped_glu(h.data, static_cast<int>(h.stride), static_cast<const float*>(logits.data), static_cast<int>(logits.stride), T, D, m.experts, m.ff,
+                                        m.top, m.scale, m.router, m.limit, m.alpha, m.up_shift, up.data, static_cast<int>(up.stride), down.data,
+                                        static_cast<int>(down.stride), moe_counts(stream), lists, weights, act, y, static_cast<float*>(x.data),
+                                        add_to || through != nullptr ? 1 : 0, add, stream);
+    if (rc == -1 || rc == -2) return false;
+    check(rc, "moe_grouped");
+    return true;
+}
+
 void merge_splits(const AttentionSplits& a, const Tensor2& out, hipStream_t stream) {
     if (out.rows != a.n_tokens || out.cols != static_cast<int64_t>(a.n_heads) * a.head_dim)
         fail("merge_splits: out must be [%d, %d]", a.n_tokens, a.n_heads * a.head_dim);

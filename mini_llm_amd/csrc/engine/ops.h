@@ -105,6 +105,7 @@ struct AttentionArgs {
 void reserve_attention_scratch(int rows, int n_heads, int head_dim, hipStream_t stream);
 void reserve_sampling_scratch(int rows, int vocab, hipStream_t stream);
 void reserve_linear_scratch(hipStream_t stream);
+void reserve_moe_scratch(hipStream_t stream);
 void release_scratch(hipStream_t stream);
 void* scratch_address(const char* name, hipStream_t stream);      // nullptr if not allocated yet (tests)
 size_t scratch_bytes();                                            // all streams of the current device (tests)
@@ -118,6 +119,7 @@ struct Tuning {
     int ln_fuse_max_rows = 32;                        // rows up to which the norm is fused into the few-row product
     int latent_tiles = 1;                             // 1: latent attention's prompt portions may run on the matrix cores
     int scored_shared_kernels = 1;                    // 1: attention with shaped scores may run on the kernels the plain attention runs on
+    int grouped_experts_rows = 192;                   // tokens from which routed experts of which at most half are chosen run as grouped products (0: never)
     int through_products = 1;                         // 1: a product may take its result into the stream through norms itself
     int halves_max_width = 1024;                      // stream widths up to which a block whose sub-layers read one stream runs the
                                                       // feed-forward's first products, with the norm inside, in front of the mixer
@@ -391,6 +393,7 @@ void softcap(const Tensor2& x, float cap, hipStream_t stream);
 // x is stored behind them as stream n_old, and x <- sum_(j <= n_old) w[j] stream_j (w: n_old + 1 floats on the device).
 void depth_mix(const Tensor2& x, const Tensor2& kept, int n_old, const float* w, hipStream_t stream);
 
+struct StreamAdd;
 // -- mixture of experts -----------------------------------------------------------------------------
 // From a token's router logits ([T, E] fp32): scores softmax(logits) over all experts, the `top` largest chosen (the
 // lower index wins a tie), weight_e = scale * score_e for them and 0 for the others. Then
@@ -421,6 +424,15 @@ struct MoeGlu {
     bool weight_on_input = false, shared_gate = false;
 };
 void moe_glu_act(const Tensor2& up, const Tensor2& logits, const MoeGlu& m, const Tensor2& out, hipStream_t stream);
+
+// The same experts by grouped products, for many tokens of which each chooses few experts (bfloat16, no shared expert, the weight
+// on the result): every expert multiplies the tokens that chose it only. up [2 E ff, D] and down [D, E ff] as joined for the
+// dense products. x (fp32) is set to the result, grows by it, or (through given) takes it through norms; `room` holds
+// moe_grouped_bytes(T, D, m) bytes. False (and nothing done): sizes the kernels do not take.
+bool moe_grouped_fits(int T, int D, const MoeGlu& m);
+size_t moe_grouped_bytes(int T, int D, const MoeGlu& m);
+bool moe_grouped(const Tensor2& h, const Tensor2& logits, const MoeGlu& m, const Tensor2& up, const Tensor2& down, const Tensor2& x, bool add_to,
+                 const StreamAdd* through, void* room, hipStream_t stream);
 
 // -- the dynamic tanh norm, things added to the stream ------------------------------------------------
 // out[i, :] = tanh(alpha x[rows ? rows[i] : i, :]) * weight + bias

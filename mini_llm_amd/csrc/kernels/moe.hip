@@ -7,9 +7,13 @@
 // block by the token's weight for that expert (zero for an expert that was not chosen, one for the shared expert), so that the experts' second products are
 // one joined product as well: sum_e w_e W_down,e a_e = [W_down,0 | W_down,1 | ...] [w_0 a_0; w_1 a_1; ...].
 // Experts that hand on their input (the identity, times the weight) have no rows; the kernel adds them up by itself.
+// For many tokens and experts of which few are chosen the products are grouped instead (moe_route_kernel and what follows):
+// every expert multiplies the tokens that chose it and no others.
 // A second kernel serves experts that are gated and clamped, chosen by sigmoid or softmax scores, whose weight may
 // stand on the expert's input, beside a shared expert that a sigmoid of the input scales.
 #include "common.h"
+
+#include <type_traits>
 
 #define MOE_MAX_EXPERTS 256
 
@@ -306,6 +310,263 @@ moe_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ log
     }
 }
 
+// ---------------------------------------------------------------------------------------------
+// Grouped products: a slot is a (token, choice) pair, slot = token * top + choice. Routing writes, per expert, the list of
+// the slots that chose it (in any order: a row's arithmetic does not depend on its neighbours) and every slot's weight; the
+// first products gather the tokens' rows and leave act(gate, up) * weight per slot, the second products multiply those, and
+// a last kernel adds a token's slots in their order and takes the sum into the stream.
+// ---------------------------------------------------------------------------------------------
+
+// A workgroup takes `tokens` tokens, a thread each; counts are gathered in LDS first, so that an expert's counter sees one
+// addition a workgroup. LDS: tokens * (E + 1) logits, then 2 E counters.
+__global__ void __launch_bounds__(256)
+moe_route_kernel(const float* __restrict__ logits, int ldl, int T, int E, int top, float scale, int kind, int tokens, int* __restrict__ counts,
+                 int* __restrict__ lists, int cap, float* __restrict__ weights) {
+    extern __shared__ float mr_smem[];
+    const int tid = threadIdx.x, first = blockIdx.x * tokens, n = min(tokens, T - first), stride = E + 1;
+    int* mine = reinterpret_cast<int*>(mr_smem + tokens * stride);       // [E] slots of this workgroup, then [E] where they start
+    for (int i = tid; i < n * E; i += 256) mr_smem[(i / E) * stride + i % E] = logits[static_cast<size_t>(first + i / E) * ldl + i % E];
+    for (int i = tid; i < E; i += 256) mine[i] = 0;
+    __syncthreads();
+    constexpr int KEEP = 8;                          // choices whose places stay in registers; further ones are chosen again
+    int chosen[KEEP], place[KEEP];
+    float* z = mr_smem + tid * stride;
+    float m = -INFINITY, all = 0.f, sum = 0.f;
+    if (tid < n) {
+        for (int e = 0; e < E; ++e) m = fmaxf(m, z[e]);
+        if (kind == ROUTER_SOFTMAX)
+            for (int e = 0; e < E; ++e) all += expf(z[e] - m);
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            if (j >= top) break;
+            int best = 0;
+            float value = -INFINITY;
+            for (int e = 0; e < E; ++e)
+                if (z[e] > value) { value = z[e]; best = e; }
+            z[best] = -INFINITY;
+            chosen[j] = best;
+            place[j] = atomicAdd(&mine[best], 1);
+            const float ex = kind == ROUTER_SIGMOID ? 1.f / (1.f + expf(-value)) : expf(value - m);
+            sum += ex;
+            weights[static_cast<size_t>(first + tid) * top + j] = ex;
+        }
+    }
+    __syncthreads();
+    for (int e = tid; e < E; e += 256) mine[E + e] = mine[e] > 0 ? atomicAdd(&counts[e], mine[e]) : 0;
+    __syncthreads();
+    if (tid >= n) return;
+    const float over = kind == ROUTER_SOFTMAX ? all : (kind == ROUTER_SOFTMAX_CHOSEN ? sum : 1.f);
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) {
+        if (j >= top) break;
+        const size_t slot = static_cast<size_t>(first + tid) * top + j;
+        weights[slot] = scale * (weights[slot] / over);
+        const int at = mine[E + chosen[j]] + place[j];
+        if (at < cap) lists[static_cast<size_t>(chosen[j]) * cap + at] = static_cast<int>(slot);
+    }
+}
+
+typedef __bf16 mbf16x8 __attribute__((ext_vector_type(8)));
+typedef float mf32x16 __attribute__((ext_vector_type(16)));
+#define MG_BM 64
+#define MG_BK 64
+#define MG_STRIDE (MG_BK + 8)
+
+struct GroupedArgs {
+    const bf16_t* A;             // rows of K: tokens' (FIRST) or slots'
+    int lda;
+    const bf16_t* W;             // FIRST: expert e's rows [gate: ff | up: ff] from row 2 ff e; else columns ff e .. of [N, ldw]
+    int ldw, ff, N, K, E, top, cap;
+    const int* counts;
+    const int* lists;
+    const float* weights;        // per slot (FIRST)
+    bf16_t* act;                 // FIRST: [slots, ld_out]
+    float* y;                    // else: [slots, ld_out]
+    int ld_out;
+    float limit, alpha, up_shift;
+};
+
+// A tile of 64 slots of one expert x 128 columns (FIRST: 64 gates and the 64 ups of the same columns): four wavefronts, each 32
+// slots x 2 tiles of 32. v_mfma_f32_32x32x16_bf16 with the weights as the first operand; LDS double buffer, two k tiles in
+// flight in registers. The k loop has no conditions: columns of A beyond K are multiplied with zeros put in for W.
+template <bool FIRST>
+__global__ void __launch_bounds__(256)
+moe_grouped_kernel(GroupedArgs g) {
+    constexpr int BN = 128;
+    __shared__ __attribute__((aligned(16))) bf16_t As[2][MG_BM * MG_STRIDE];
+    __shared__ __attribute__((aligned(16))) bf16_t Ws[2][BN * MG_STRIDE];
+    __shared__ int slot_s[MG_BM];
+    const int tid = threadIdx.x, lane = tid % MLLM_WAVE, wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
+    // which expert's row tile this is: a prefix sum over the experts' tiles, 64 experts at a time
+    int e = -1, tile = blockIdx.x, count = 0;
+    for (int e0 = 0; e0 < g.E && e < 0; e0 += MLLM_WAVE) {
+        const int its = e0 + lane < g.E ? min(g.counts[e0 + lane], g.cap) : 0;
+        const int nt = (its + MG_BM - 1) / MG_BM;
+        int upto = nt;
+#pragma unroll
+        for (int off = 1; off < MLLM_WAVE; off *= 2) {
+            const int other = __shfl_up(upto, off, MLLM_WAVE);
+            if (lane >= off) upto += other;
+        }
+        const unsigned long long here = __ballot(tile < upto);
+        if (here != 0) {
+            const int l = __ffsll(here) - 1;
+            e = e0 + l;
+            count = __shfl(its, l, MLLM_WAVE);
+            tile -= __shfl(upto, l, MLLM_WAVE) - __shfl(nt, l, MLLM_WAVE);
+        } else {
+            tile -= __shfl(upto, MLLM_WAVE - 1, MLLM_WAVE);
+        }
+    }
+    if (e < 0) return;                               // (the grid is an upper bound)
+    e = __builtin_amdgcn_readfirstlane(e);
+    tile = __builtin_amdgcn_readfirstlane(tile);
+    count = __builtin_amdgcn_readfirstlane(count);
+    const int first = tile * MG_BM, rows = min(MG_BM, count - first), n0 = blockIdx.y * (FIRST ? BN / 2 : BN);
+    if (tid < MG_BM) slot_s[tid] = g.lists[static_cast<size_t>(e) * g.cap + first + min(tid, rows - 1)];
+    __syncthreads();
+    // loads: 16-byte pieces, eight neighbouring threads a row's 128 bytes
+    const bf16_t* a_row[2];
+    const bf16_t* w_row[4];
+    const int piece = (tid % 8) * 8;
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int slot = slot_s[tid / 8 + 32 * u];
+        a_row[u] = g.A + static_cast<size_t>(FIRST ? slot / g.top : slot) * g.lda;
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+        const int r = tid / 8 + 32 * u;
+        if (FIRST) w_row[u] = g.W + (static_cast<size_t>(e) * 2 * g.ff + (r < 64 ? min(n0 + r, g.ff - 1) : g.ff + min(n0 + r - 64, g.ff - 1))) * g.ldw;
+        else w_row[u] = g.W + static_cast<size_t>(min(n0 + r, g.N - 1)) * g.ldw + static_cast<size_t>(e) * g.ff;
+    }
+    mbf16x8 ra[2][2], rw[2][4];
+    const int KT = (g.K + MG_BK - 1) / MG_BK;
+    auto fetch = [&](auto ring, int kt) {
+        constexpr int R = decltype(ring)::value;
+        const int k = min(kt * MG_BK + piece, g.K - 8);
+#pragma unroll
+        for (int u = 0; u < 2; ++u) ra[R][u] = *reinterpret_cast<const mbf16x8*>(a_row[u] + k);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) rw[R][u] = *reinterpret_cast<const mbf16x8*>(w_row[u] + k);
+        __builtin_amdgcn_sched_barrier(0);
+    };
+    auto stage = [&](auto ring, int kt) {            // tile kt from its registers into its LDS buffer
+        constexpr int R = decltype(ring)::value;
+        const bool inside = kt * MG_BK + piece < g.K;
+        const mbf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+        for (int u = 0; u < 2; ++u) *reinterpret_cast<mbf16x8*>(&As[R][(tid / 8 + 32 * u) * MG_STRIDE + piece]) = ra[R][u];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) *reinterpret_cast<mbf16x8*>(&Ws[R][(tid / 8 + 32 * u) * MG_STRIDE + piece]) = inside ? rw[R][u] : zero;
+    };
+    const int wm = wave / 2, wn = wave % 2;
+    const int col[2] = {FIRST ? 32 * wn : 64 * wn, FIRST ? 64 + 32 * wn : 64 * wn + 32};      // this wavefront's rows of Ws
+    mf32x16 acc[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) acc[j][r] = 0.f;
+    auto multiply = [&](auto ring) {
+        constexpr int R = decltype(ring)::value;
+#pragma unroll
+        for (int ks = 0; ks < MG_BK / 16; ++ks) {
+            const int k = ks * 16 + 8 * (lane / 32);
+            const mbf16x8 a = *reinterpret_cast<const mbf16x8*>(&As[R][(32 * wm + lane % 32) * MG_STRIDE + k]);
+#pragma unroll
+            for (int j = 0; j < 2; ++j) {
+                const mbf16x8 w = *reinterpret_cast<const mbf16x8*>(&Ws[R][(col[j] + lane % 32) * MG_STRIDE + k]);
+                acc[j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(w, a, acc[j], 0, 0, 0);
+            }
+        }
+    };
+    std::integral_constant<int, 0> R0;
+    std::integral_constant<int, 1> R1;
+    fetch(R0, 0);
+    fetch(R1, 1);
+    stage(R0, 0);
+    for (int kt = 0; kt < KT; kt += 2) {
+        lds_barrier();                               // tile kt is in LDS, and everybody is done with tile kt - 1
+        fetch(R0, kt + 2);
+        multiply(R0);
+        stage(R1, kt + 1);
+        if (kt + 1 >= KT) break;
+        lds_barrier();
+        fetch(R1, kt + 3);
+        multiply(R1);
+        stage(R0, kt + 2);
+    }
+    lds_barrier();                                   // the tiles' LDS is free
+    // (register r of lane l: column 8 (r / 4) + 4 (l / 32) + r % 4 of slot l % 32) through LDS into stores of whole rows
+    float* epi = reinterpret_cast<float*>(&Ws[0][0]) + wave * (32 * 36);
+    constexpr int PASSES = FIRST ? 1 : 2;
+    const float my_weight = FIRST ? g.weights[slot_s[32 * wm + lane % 32]] : 1.f;
+#pragma unroll
+    for (int p = 0; p < PASSES; ++p) {
+        wave_lds_sync();
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+            float v[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                if (FIRST) {
+                    const float gk = fminf(acc[0][4 * q + i], g.limit), uk = fminf(fmaxf(acc[1][4 * q + i], -g.limit), g.limit);
+                    v[i] = gk / (1.f + __expf(-g.alpha * gk)) * (uk + g.up_shift) * my_weight;
+                } else {
+                    v[i] = acc[p][4 * q + i];
+                }
+            }
+            *reinterpret_cast<float4*>(&epi[(lane % 32) * 36 + 8 * q + 4 * (lane / 32)]) = make_float4(v[0], v[1], v[2], v[3]);
+        }
+        wave_lds_sync();
+        const int nb = n0 + (FIRST ? 32 * wn : 64 * wn + 32 * p), last = FIRST ? g.ff : g.N;
+#pragma unroll
+        for (int it = 0; it < 4; ++it) {
+            const int r = it * 8 + lane / 8, n = nb + (lane % 8) * 4;
+            if (32 * wm + r >= rows || n >= last) continue;
+            const float4 v = *reinterpret_cast<const float4*>(&epi[r * 36 + (lane % 8) * 4]);
+            const size_t at = static_cast<size_t>(slot_s[32 * wm + r]) * g.ld_out + n;
+            if (FIRST) *reinterpret_cast<uint2*>(g.act + at) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+            else *reinterpret_cast<float4*>(g.y + at) = v;
+        }
+    }
+}
+
+// What a token's slots sum up to, into the stream: through add (tanh_norm.h; norm and copy) with add_to 1, or with add_to 0 set
+// as it is. Zeroes the counters for the next routing.
+__global__ void __launch_bounds__(256)
+moe_combine_kernel(const float* __restrict__ y, int top, int D, float* __restrict__ x, int add_to, MllmStreamAdd add, int* __restrict__ counts, int E) {
+    const int t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (t == 0 && blockIdx.x == 0)
+        for (int e = threadIdx.x; e < E; e += 256) counts[e] = 0;
+    if (c >= D) return;
+    const float* row = y + static_cast<size_t>(t) * top * D + c;
+    float* xr = x + static_cast<size_t>(t) * D + c;
+    float4 old = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (add_to) old = *reinterpret_cast<const float4*>(xr);
+    float4 sum = *reinterpret_cast<const float4*>(row);
+    for (int j = 1; j < top; ++j) {
+        const float4 more = *reinterpret_cast<const float4*>(row + static_cast<size_t>(j) * D);
+        sum.x += more.x; sum.y += more.y; sum.z += more.z; sum.w += more.w;
+    }
+    float o[4] = {sum.x, sum.y, sum.z, sum.w};
+    const bool has = add.norm.weight != nullptr, has_next = add.next.weight != nullptr;
+    if (has) {
+        const float a = add.norm.alpha[0];
+        const float4 w = *reinterpret_cast<const float4*>(add.norm.weight + c), b = *reinterpret_cast<const float4*>(add.norm.bias + c);
+        o[0] = fast_tanh(a * o[0]) * w.x + b.x; o[1] = fast_tanh(a * o[1]) * w.y + b.y; o[2] = fast_tanh(a * o[2]) * w.z + b.z; o[3] = fast_tanh(a * o[3]) * w.w + b.w;
+    }
+    o[0] += old.x; o[1] += old.y; o[2] += old.z; o[3] += old.w;
+    *reinterpret_cast<float4*>(xr) = make_float4(o[0], o[1], o[2], o[3]);
+    if (add.copy == nullptr) return;
+    if (has_next) {
+        const float a = add.next.alpha[0];
+        const float4 w = *reinterpret_cast<const float4*>(add.next.weight + c), b = *reinterpret_cast<const float4*>(add.next.bias + c);
+        o[0] = fast_tanh(a * o[0]) * w.x + b.x; o[1] = fast_tanh(a * o[1]) * w.y + b.y; o[2] = fast_tanh(a * o[2]) * w.z + b.z; o[3] = fast_tanh(a * o[3]) * w.w + b.w;
+    }
+    *reinterpret_cast<uint2*>(static_cast<bf16_t*>(add.copy) + static_cast<size_t>(t) * add.ld_copy + c) = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+}
+
 }  // namespace
 
 extern "C" {
@@ -367,6 +628,40 @@ int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int 
     else MOE_GLU(bf16_t, bf16_t);
 #undef MOE_GLU
 #undef MOE_GLU_V
+    MLLM_LAUNCH_CHECK();
+    return 0;
+}
+
+// Gated experts by grouped products (bfloat16). h [T, D] (row stride ldh); logits [T, >= E] fp32; up [2 E ff, D]: expert e's gates
+// and ups from row 2 ff e; down [D, E ff]: expert e's from column ff e. router_kind, scale, limit, alpha, up_shift as for
+// mllm_moe_glu_act. Room: counts [E] ints, zero (and left zero); lists [E * T] ints, weights [T * top] floats, act [T * top, ff]
+// bfloat16, y [T * top, D] fp32. x [T, D] fp32 is set to the result (add_to 0), or grows by it through `add` (add_to 1). -2: sizes
+// these kernels do not take (the caller then multiplies densely); -1: operands that are not aligned.
+int mllm_moe_grouped_glu(const void* h, int ldh, const float* logits, int ldl, int T, int D, int E, int ff, int top, float scale, int router_kind,
+                         float limit, float alpha, float up_shift, const void* up, int ldu, const void* down, int ldd, int* counts, int* lists,
+                         float* weights, void* act, float* y, float* x, int add_to, MllmStreamAdd add, hipStream_t stream) {
+    if (T <= 0) return 0;
+    if (E < 1 || E > MOE_MAX_EXPERTS || top < 1 || top > E || top > 8 || D % 8 != 0 || ff % 8 != 0 || T > 65535 || ldh % 8 != 0 || ldu % 8 != 0 || ldd % 8 != 0) return -2;
+    const auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+    if (!a16(h) || !a16(up) || !a16(down) || !a16(act) || !a16(y) || !a16(x) || (add.copy != nullptr && (add.ld_copy % 4 != 0 || (reinterpret_cast<uintptr_t>(add.copy) & 7)))) return -1;
+    for (const MllmTanhNorm* n : {&add.norm, &add.next})
+        if (n->weight != nullptr && (n->alpha == nullptr || n->bias == nullptr || !a16(n->weight) || !a16(n->bias))) return -1;
+    if (router_kind < ROUTER_SOFTMAX || router_kind > ROUTER_SOFTMAX_CHOSEN || !(limit > 0.f)) return -1;
+    const int tokens = E <= 48 ? 256 : (E <= 128 ? 64 : 32);
+    const size_t lds = static_cast<size_t>(tokens) * (E + 1) * 4 + static_cast<size_t>(2) * E * 4;
+    moe_route_kernel<<<(T + tokens - 1) / tokens, 256, lds, stream>>>(logits, ldl, T, E, top, scale, router_kind, tokens, counts, lists, T, weights);
+    MLLM_LAUNCH_CHECK();
+    GroupedArgs g{};
+    g.A = static_cast<const bf16_t*>(h); g.lda = ldh; g.W = static_cast<const bf16_t*>(up); g.ldw = ldu; g.ff = ff; g.N = 2 * ff; g.K = D; g.E = E;
+    g.top = top; g.cap = T; g.counts = counts; g.lists = lists; g.weights = weights; g.act = static_cast<bf16_t*>(act); g.y = y; g.ld_out = ff;
+    g.limit = limit; g.alpha = alpha; g.up_shift = up_shift;
+    const int row_tiles = static_cast<int>((static_cast<long long>(T) * top) / MG_BM) + E;          // an upper bound
+    moe_grouped_kernel<true><<<dim3(row_tiles, (ff + 63) / 64), 256, 0, stream>>>(g);
+    MLLM_LAUNCH_CHECK();
+    g.A = static_cast<const bf16_t*>(act); g.lda = ff; g.W = static_cast<const bf16_t*>(down); g.ldw = ldd; g.N = D; g.K = ff; g.ld_out = D;
+    moe_grouped_kernel<false><<<dim3(row_tiles, (D + 127) / 128), 256, 0, stream>>>(g);
+    MLLM_LAUNCH_CHECK();
+    moe_combine_kernel<<<dim3((D + 1023) / 1024, T), 256, 0, stream>>>(y, top, D, x, add_to, add, counts, E);
     MLLM_LAUNCH_CHECK();
     return 0;
 }
