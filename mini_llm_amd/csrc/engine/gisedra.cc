@@ -24,6 +24,7 @@
 // Tensors: embed, head, side.embed, loop.step, final.norm[.alpha, .b], l<i>.{norm1, norm1b, norm2, norm2b}[.alpha, .b],
 // l<i>.mix.{q, dkv, dkv.norm, uk, uv, o} or l<i>.mix.left.{q, k, v}[.conv], l<i>.mix.left.{g, o}, l<i>.mix.right.{q, k, v, g, o},
 // l<i>.mlp.{router, router.b}, l<i>.mlp.e<k>.{gate, up, down}, l<i>.side.{gate, proj, norm}; linear weights are stored [out, in].
+#include <algorithm>
 #include <cmath>
 
 #include "arch.h"
@@ -325,19 +326,53 @@ std::unique_ptr<Mixer> latent_mixer(const LatentConfig& a, const std::string& M,
     return build_mixer("latent_attention", p);
 }
 
+// How the left mixer's heads lie in the engine. The attention kernels that every model shares take keys and values of one
+// width, and their matrix-core tiles widths of 32, 64 and 128. In bfloat16 a head's values are cut into `parts` of at most 128
+// columns, each with the head's queries and keys once more, and both widths are filled up with zeros to the next of those sizes:
+// a part's scores are the head's, and its result is the part of the head's. Within a key/value head the parts come one after the
+// other, each with all of that head's queries. Otherwise (32-bit; keys wider than 128) the narrower of the two widths is filled
+// up to the wider one.
+struct HeadLayout {
+    int64_t parts = 1, keys = 0, values = 0;          // columns of a head's keys and values as they are laid out
+    std::vector<int64_t> query_rows, key_rows, value_rows, result_rows;      // which stored row (or -1) each laid-out one is
+    HeadLayout(const AttentionConfig& a, int dtype) {
+        keys = (a.vdim > a.dim && a.vdim % 16 == 0) ? a.vdim : a.dim;
+        values = (a.vdim < a.dim && a.dim % 16 == 0) ? a.dim : a.vdim;
+        int64_t width = a.vdim;                       // stored value columns of a part
+        if (dtype == BF16 && a.dim <= 128) {
+            int64_t n = (a.vdim + 127) / 128;
+            while (n <= 8 && a.vdim % n != 0) ++n;
+            if (n <= 8) {
+                parts = n;
+                width = a.vdim / n;
+                const int64_t need = std::max(a.dim, width);
+                keys = values = need <= 32 ? 32 : (need <= 64 ? 64 : 128);
+            }
+        }
+        const int64_t group = a.heads / a.kv_heads;
+        auto add = [](std::vector<int64_t>& to, int64_t first, int64_t n, int64_t padded) {
+            for (int64_t i = 0; i < padded; ++i) to.push_back(i < n ? first + i : -1);
+        };
+        for (int64_t g = 0; g < a.kv_heads; ++g)
+            for (int64_t p = 0; p < parts; ++p) {
+                add(key_rows, g * a.dim, a.dim, keys);
+                add(value_rows, g * a.vdim + p * width, width, values);
+                for (int64_t r = 0; r < group; ++r) {
+                    add(query_rows, (g * group + r) * a.dim, a.dim, keys);
+                    add(result_rows, (g * group + r) * a.vdim + p * width, width, values);
+                }
+            }
+    }
+};
+
 std::unique_ptr<Mixer> pair_mixer(const LayerConfig& l, const std::string& M, int width, double eps, int dtype, const Tensors& t, DeviceTensors& store) {
     const AttentionConfig& a = l.left;
     const RetentionConfig& r = l.right;
     const std::string A = M + "left.", R = M + "right.";
-    // The attention kernels that every model shares take keys and values of one width: the narrower of the two is widened with
-    // zeros (rows of the projections and taps, columns of the output projection), which changes no score and no result.
-    const int64_t e = (a.vdim < a.dim && a.dim % 16 == 0) ? a.dim : a.vdim;
-    const int64_t d = (a.vdim > a.dim && a.vdim % 16 == 0) ? a.vdim : a.dim;
-    auto keys = [&](const std::string& n) { return d == a.dim ? t.at(n) : store.pad_row_blocks(t.at(n), a.dim, d); };
-    auto values = [&](const Tensor2& w) { return e == a.vdim ? w : store.pad_row_blocks(w, a.vdim, e); };
+    const HeadLayout lay(a, dtype);
     Params p;
-    p.num["heads"] = static_cast<double>(a.heads); p.num["kv_heads"] = static_cast<double>(a.kv_heads);
-    p.num["dim"] = static_cast<double>(d); p.num["value_dim"] = static_cast<double>(e);
+    p.num["heads"] = static_cast<double>(a.heads * lay.parts); p.num["kv_heads"] = static_cast<double>(a.kv_heads * lay.parts);
+    p.num["dim"] = static_cast<double>(lay.keys); p.num["value_dim"] = static_cast<double>(lay.values);
     p.num["scale"] = a.scale; p.num["eps"] = eps; p.num["dtype"] = dtype; p.num["gated"] = 1;
     p.num["window"] = static_cast<double>(a.window); p.num["keep_first"] = static_cast<double>(a.window > 0 ? a.keep_first : 0);
     p.num["rot_dims"] = static_cast<double>(a.rot.dims); p.num["rot_base"] = a.rot.base;
@@ -364,11 +399,11 @@ std::unique_ptr<Mixer> pair_mixer(const LayerConfig& l, const std::string& M, in
             tv = store.upload(std::vector<float>(static_cast<size_t>(nv), 1.f), nv, 1, F32);
         }
         const Tensor2 scaled(store.scaled(tv, static_cast<float>(l.left_scale)).data, F32, nv, taps);
-        p.tensor["qkv_conv"] = store.join_rows({d == a.dim ? tq : store.pad_row_blocks(tq, a.dim, d), d == a.dim ? tk : store.pad_row_blocks(tk, a.dim, d),
-                                                values(scaled)});
+        p.tensor["qkv_conv"] = store.join_rows({store.pick_rows(tq, lay.query_rows), store.pick_rows(tk, lay.key_rows), store.pick_rows(scaled, lay.value_rows)});
     }
-    const Tensor2 left_in = store.join_rows({keys(A + "q"), keys(A + "k"), values(t.at(A + "v")), values(t.at(A + "g"))});
-    const Tensor2 left_out = e == a.vdim ? t.at(A + "o") : store.pad_col_blocks(t.at(A + "o"), a.vdim, e);
+    const Tensor2 left_in = store.join_rows({store.pick_rows(t.at(A + "q"), lay.query_rows), store.pick_rows(t.at(A + "k"), lay.key_rows),
+                                             store.pick_rows(t.at(A + "v"), lay.value_rows), store.pick_rows(t.at(A + "g"), lay.result_rows)});
+    const Tensor2 left_out = store.pick_cols(t.at(A + "o"), lay.result_rows);
     // One input product and one output product for both mixers.
     Params pair;
     pair.num["size"] = width; pair.num["eps"] = eps; pair.num["dtype"] = dtype;

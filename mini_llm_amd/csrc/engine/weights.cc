@@ -373,6 +373,45 @@ Tensor2 DeviceTensors::pad_row_parts(const Tensor2& t, const std::vector<int64_t
     return Tensor2(base, t.dtype, n * out_block, t.cols);
 }
 
+// Runs of neighbours among the picked indices are copied together: f(first in the result, first in the source, length).
+template <typename F>
+static void runs_of(const std::vector<int64_t>& picked, int64_t limit, const char* what, F&& f) {
+    for (size_t i = 0; i < picked.size();) {
+        if (picked[i] < -1 || picked[i] >= limit) throw WeightsError(std::string(what) + ": an index beyond the tensor");
+        size_t n = 1;
+        if (picked[i] >= 0)
+            while (i + n < picked.size() && picked[i + n] == picked[i] + static_cast<int64_t>(n)) ++n;
+        if (picked[i] >= 0) {
+            if (picked[i] + static_cast<int64_t>(n) > limit) throw WeightsError(std::string(what) + ": an index beyond the tensor");
+            f(i, picked[i], n);
+        }
+        i += n;
+    }
+}
+
+Tensor2 DeviceTensors::pick_rows(const Tensor2& t, const std::vector<int64_t>& rows) {
+    if (!t.contiguous()) throw WeightsError("pick_rows: a contiguous tensor is needed");
+    const size_t row_bytes = static_cast<size_t>(t.cols) * t.esz();
+    char* base = static_cast<char*>(allocate(rows.size() * row_bytes, true));
+    runs_of(rows, t.rows, "pick_rows", [&](size_t to, int64_t from, size_t n) {
+        if (hipMemcpy(base + to * row_bytes, static_cast<const char*>(t.data) + static_cast<size_t>(from) * row_bytes, n * row_bytes, hipMemcpyDeviceToDevice) != hipSuccess)
+            throw WeightsError("pick_rows: the copy on the device failed");
+    });
+    return Tensor2(base, t.dtype, static_cast<int64_t>(rows.size()), t.cols);
+}
+
+Tensor2 DeviceTensors::pick_cols(const Tensor2& t, const std::vector<int64_t>& cols) {
+    if (!t.contiguous()) throw WeightsError("pick_cols: a contiguous tensor is needed");
+    const size_t esz = t.esz(), to_pitch = cols.size() * esz, from_pitch = static_cast<size_t>(t.cols) * esz;
+    char* base = static_cast<char*>(allocate(static_cast<size_t>(t.rows) * to_pitch, true));
+    runs_of(cols, t.cols, "pick_cols", [&](size_t to, int64_t from, size_t n) {
+        if (t.rows > 0 && hipMemcpy2D(base + to * esz, to_pitch, static_cast<const char*>(t.data) + static_cast<size_t>(from) * esz, from_pitch, n * esz, static_cast<size_t>(t.rows),
+                                      hipMemcpyDeviceToDevice) != hipSuccess)
+            throw WeightsError("pick_cols: the copy on the device failed");
+    });
+    return Tensor2(base, t.dtype, t.rows, static_cast<int64_t>(cols.size()));
+}
+
 Tensor2 DeviceTensors::operand_tiles(const Tensor2& t, int64_t rows, int64_t cols) {
     if (t.dtype != BF16 || !t.contiguous() || rows % 16 != 0 || cols % 32 != 0 || rows < t.rows || cols < t.cols)
         throw WeightsError("operand_tiles: a contiguous bfloat16 matrix and sizes in whole tiles are needed");

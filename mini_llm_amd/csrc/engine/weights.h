@@ -166,6 +166,10 @@ public:
     // The same for blocks made of several parts: a block's part i has parts[i] rows (their sum is the block), each followed by
     // zero rows up to padded[i].
     Tensor2 pad_row_parts(const Tensor2& t, const std::vector<int64_t>& parts, const std::vector<int64_t>& padded);
+    // The rows (columns) named one after the other ([n, cols] or [rows, n], a copy on the device; -1: a row or column of zeros):
+    // heads reordered, repeated, split or made wider.
+    Tensor2 pick_rows(const Tensor2& t, const std::vector<int64_t>& rows);
+    Tensor2 pick_cols(const Tensor2& t, const std::vector<int64_t>& cols);
     // A bfloat16 matrix [rows, cols] as 16 x 32 tiles in the matrix cores' operand order, [rows / 16][cols / 32][lane][8]: lane l holds
     // row l % 16, columns 8 (l / 16) to 8 (l / 16) + 7 of its tile. Rows and columns are filled up with zeros to `rows` and
     // `cols` (multiples of 16 and 32).
