@@ -494,6 +494,7 @@ void gisedra_assemble(const Json& config, const Tensors& t, int dtype, LoadedMod
                 const int64_t dim = token_side_padded(static_cast<int>(c.side_dim));
                 p.tensor["gate.tiles"] = out.store.operand_tiles(t.at(L + "side.gate"), dim, D);
                 p.tensor["proj.tiles"] = out.store.operand_tiles(t.at(L + "side.proj"), D, (dim + 31) / 32 * 32);
+                p.tensor["proj.gram"] = out.store.gram_tiles(t.at(L + "side.proj"), dim);
             }
             m.stream_steps.push_back(build_stream_step("token_side", p));          // step i stands behind layer i
         }

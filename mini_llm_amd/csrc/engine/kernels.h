@@ -129,7 +129,7 @@ int mllm_latent_expand(const void* o_lat, int ldo, const void* w_uv, int ldw, vo
 int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, int T, int H, int G, int d, int dv,
                     int norm_mode, const float* wq, const float* wk, float eps, int rot_dims, double rot_base,
                     const int* positions, const int* slots, void* q_out, int ldq, void* k_pages, void* v_pages, int dtype,
-                    hipStream_t stream, int interleaved = 0, const float* rot_freqs = nullptr);
+                    hipStream_t stream, int interleaved = 0, const float* rot_freqs = nullptr, const MllmConvSingle* conv = nullptr);
 int mllm_scored_attention_rows(const void* q, int ldq, const void* k_pages, const void* v_pages, const int* block_tables,
                                int max_blocks, const int* token_seq, const int* positions, int n_tokens, int H, int G, int d,
                                int dv, int page_size, float scale, float softcap, int window, int chunk, const float* r1,
@@ -188,7 +188,7 @@ int mllm_stream_add(float* x, const float* y, const float* x0, const float* step
 int mllm_token_gate(const float* z, int ldz, const int* ids, const int* src, const int* prev, int n_prev, const void* table, int ldt, int col0,
                     int dim, void* out, int ldo, int T, int dtype, hipStream_t stream);
 int mllm_token_side_fits(int D, int dim);
-int mllm_token_side(float* x, int T, int D, const void* gate, const void* proj, const float* weight, float eps, const int* ids, const int* src,
+int mllm_token_side(float* x, const void* xb, int T, int D, const void* gate, const void* proj, const float* gram, const float* weight, float eps, const int* ids, const int* src,
                     const int* prev, int n_prev, const void* table, int ldt, int col0, int dim, MllmStreamAdd add, hipStream_t stream);
 
 // sampling.hip

@@ -319,8 +319,11 @@ struct ScoredShape {
 // values are the keys before their norm): q [T, heads * dim] normed and turned, and the keys and values written
 // to their page rows (slots[t]). k_col < 0: queries only (the keys and values are another layer's; the pages are
 // not touched and may be empty tensors).
+// conv (optional; steps of single tokens where qk_prepare_takes_conv): the rows' convolution is done on the way.
 void qk_prepare(const Tensor2& proj, int q_col, int k_col, int v_col, const ScoredShape& sh, const int* positions,
-                const int* slots, const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, hipStream_t stream);
+                const int* slots, const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, hipStream_t stream,
+                const MllmConvSingle* conv = nullptr);
+bool qk_prepare_takes_conv(const ScoredShape& sh, int tokens, int taps);
 struct ScoredStep {
     const int* block_tables = nullptr;     // [n_seqs, max_blocks]
     int max_blocks = 0, n_seqs = 0, max_q_len = 0, max_ctx_len = 0, page_size = 0;
@@ -454,11 +457,12 @@ void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, co
 void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Tensor2& table, int col0, const Tensor2& out, hipStream_t stream);
 // The whole of it in one kernel, where token_side_fits (bfloat16): with e the columns col0 .. col0 + dim of the token's row of
 // the table, g = gelu_tanh(W_gate x) * e, y = W_proj g, x += y / sqrt(mean(y^2) + eps) * weight, then add's copy (add.x is the
-// stream, add.norm is not used). gate and proj: the maps' bfloat16 tiles in operand order (DeviceTensors::operand_tiles), dim
-// filled up to the next of 16, 32 and 64 rows and to whole tiles of 32 inputs.
+// stream, add.norm is not used). xb: the stream in bfloat16 (another tensor than add.copy). gate and proj: the maps' bfloat16 tiles
+// in operand order (DeviceTensors::operand_tiles), dim filled up to the next of 16, 32 and 64 rows and to whole tiles of 32 inputs;
+// gram: W_proj^T W_proj in fp32 operand tiles (DeviceTensors::gram_tiles).
 bool token_side_fits(int width, int dim);
 int token_side_padded(int dim);         // 16, 32 or 64
-void token_side(const StreamAdd& add, const Tensor2& gate, const Tensor2& proj, const float* weight, float eps, const int* ids, const FedTokens* fed,
+void token_side(const StreamAdd& add, const Tensor2& xb, const Tensor2& gate, const Tensor2& proj, const Tensor2& gram, const float* weight, float eps, const int* ids, const FedTokens* fed,
                 const Tensor2& table, int col0, int dim, hipStream_t stream);
 
 // out = [a | b] row by row in out's dtype (a, b fp32 [T, D])

@@ -107,9 +107,19 @@ void rmsnorm_add_many(const Tensor2& ys, const float* weights, int n, float mult
                                 static_cast<float*>(x.data), i32(x.rows), i32(x.cols), stream), "rmsnorm_add_many");
 }
 
+static int64_t nq_nk_nv(const ScoredShape& sh, bool values) {
+    return (static_cast<int64_t>(sh.n_heads) + sh.n_kv_heads) * sh.dim + (values ? static_cast<int64_t>(sh.n_kv_heads) * sh.value_dim : 0);
+}
+bool qk_prepare_takes_conv(const ScoredShape& sh, int tokens, int taps) {
+    return tokens <= 64 && sh.dim <= 256 && sh.norm_mode != 2 && taps >= 2 && taps <= 4;
+}
+
 void qk_prepare(const Tensor2& proj, int q_col, int k_col, int v_col, const ScoredShape& sh, const int* positions,
-                const int* slots, const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, hipStream_t stream) {
+                const int* slots, const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, hipStream_t stream, const MllmConvSingle* conv) {
     check_shape(sh, "qk_prepare");
+    if (conv != nullptr && (k_col < 0 || q_col != 0 || !qk_prepare_takes_conv(sh, i32(proj.rows), conv->taps) || conv->w == nullptr || conv->state == nullptr || conv->state_slots == nullptr ||
+                            conv->channels != nq_nk_nv(sh, v_col >= 0) || conv->slot_floats < static_cast<unsigned long long>(conv->taps - 1) * conv->channels))
+        fail("qk_prepare: the convolution does not fit queries, keys and values");
     need_f32(proj, "qk_prepare: the projection");
     need_act(q, "qk_prepare: q");
     const int64_t nq = static_cast<int64_t>(sh.n_heads) * sh.dim, nk = static_cast<int64_t>(sh.n_kv_heads) * sh.dim,
@@ -136,7 +146,7 @@ void qk_prepare(const Tensor2& proj, int q_col, int k_col, int v_col, const Scor
         fail("qk_prepare: %d turned columns of %d (even, at most the head) and a positive base are needed", sh.rot_dims, sh.dim);
     check(mllm_qk_prepare(static_cast<const float*>(proj.data), i32(proj.stride), q_col, k_col, v_col, i32(proj.rows), sh.n_heads, sh.n_kv_heads,
                           sh.dim, sh.value_dim, sh.norm_mode, sh.q_norm, sh.k_norm, sh.eps, sh.rot_dims, sh.rot_base, positions, slots, q.data,
-                          i32(q.stride), k_pages.data, v_pages.data, q.dtype, stream, sh.rot_interleaved ? 1 : 0, sh.rot_freqs), "qk_prepare");
+                          i32(q.stride), k_pages.data, v_pages.data, q.dtype, stream, sh.rot_interleaved ? 1 : 0, sh.rot_freqs, conv), "qk_prepare");
 }
 
 void scored_attention(const Tensor2& q, const Tensor2& k_pages, const Tensor2& v_pages, const ScoredStep& step,
@@ -384,7 +394,7 @@ void token_gate(const Tensor2& z, const int* ids, const FedTokens* fed, const Te
 bool token_side_fits(int width, int dim) { return mllm_token_side_fits(width, dim) != 0; }
 int token_side_padded(int dim) { return dim <= 16 ? 16 : (dim <= 32 ? 32 : 64); }
 
-void token_side(const StreamAdd& add, const Tensor2& gate, const Tensor2& proj, const float* weight, float eps, const int* ids, const FedTokens* fed,
+void token_side(const StreamAdd& add, const Tensor2& xb, const Tensor2& gate, const Tensor2& proj, const Tensor2& gram, const float* weight, float eps, const int* ids, const FedTokens* fed,
                 const Tensor2& table, int col0, int dim, hipStream_t stream) {
     check_stream_add(add, "token_side");
     const int D = i32(add.x.cols);
@@ -393,10 +403,12 @@ void token_side(const StreamAdd& add, const Tensor2& gate, const Tensor2& proj, 
     if (gate.dtype != BF16 || proj.dtype != BF16 || !gate.contiguous() || !proj.contiguous() || gate.rows * gate.cols != rows * D ||
         proj.rows * proj.cols != inputs * 32 * D || weight == nullptr)
         fail("token_side: the maps' tiles do not fit a width of %d and %d columns", D, dim);
+    if (gram.dtype != F32 || gram.rows * gram.cols != rows * rows) fail("token_side: the second map's square must be [%lld, %lld] in tiles", (long long)rows, (long long)rows);
+    if (xb.dtype != BF16 || !xb.contiguous() || xb.rows != add.x.rows || xb.cols != D || xb.data == add.copy.data) fail("token_side: a bfloat16 copy of the stream is needed, apart from the one it leaves");
     if (table.dtype != BF16 || col0 < 0 || col0 + dim > table.cols || ids == nullptr) fail("token_side: columns %d.. of a table of %lld", col0, (long long)table.cols);
     const bool feeds = fed != nullptr && fed->src != nullptr;
     if (feeds && (fed->prev == nullptr || fed->n_prev < 1)) fail("token_side: fed tokens need the earlier step's sampled tokens");
-    check(mllm_token_side(static_cast<float*>(add.x.data), i32(add.x.rows), D, gate.data, proj.data, weight, eps, ids, feeds ? fed->src : nullptr,
+    check(mllm_token_side(static_cast<float*>(add.x.data), xb.data, i32(add.x.rows), D, gate.data, proj.data, static_cast<const float*>(gram.data), weight, eps, ids, feeds ? fed->src : nullptr,
                           feeds ? fed->prev : nullptr, feeds ? fed->n_prev : 0, table.data, i32(table.stride), col0, dim, kernel_side(add), stream), "token_side");
 }
 

@@ -428,7 +428,7 @@ public:
     int hidden_size() const override { return static_cast<int>(table_.cols); }
     void forward(const StepView& step, const PositionEncoding* position, const Tensor2& x, hipStream_t s) const override {
         embed(step.token_ids, step.positions, table_, position ? position->table() : nullptr, x, s, &step.fed, scale_,
-              step.leave.wanted ? &step.stream_copy : nullptr, step.leave.wanted ? &step.leave.norm : nullptr);
+              step.leave.wanted ? &step.leave.into : nullptr, step.leave.wanted ? &step.leave.norm : nullptr);
     }
     bool resolves_fed_tokens() const override { return true; }
     bool writes_stream_copy() const override { return true; }
@@ -664,6 +664,8 @@ size_t DecoderModel::workspace_bytes(int tokens, int n_logits) const {
     for (const auto& st : stream_steps) {
         if (st->wants_embedding_output()) { stream += one; break; }
     }
+    for (const auto& st : stream_steps)
+        if (st->wants_copy()) { stream += one / 2 + 256; break; }
     {
         int kept = 0;
         for (const auto& st : stream_steps) kept = std::max(kept, st->kept_streams());
@@ -688,7 +690,12 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         with_rows.stream_copy = arena.tensor(BF16, step.n_tokens, hidden_size());
         break;
     }
-    // What the block of call i finds in the copy as it is entered, and what is in it now. Whoever runs in front of a block
+    for (const auto& st : stream_steps) {
+        if (!st->wants_copy()) continue;
+        with_rows.step_copy = arena.tensor(BF16, step.n_tokens, hidden_size());
+        break;
+    }
+    // What the block of call i (or a stream step) finds in its copy as it is entered, and what is there now. Whoever runs in front of a block
     // is told (StepView::leave) and leaves it if it can; otherwise it is made here.
     using Leave = StepView::Leave;
     auto wanted_by = [&](size_t i, bool behind_its_step) {
@@ -696,10 +703,22 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         if (i >= order.size() || (order[i].before >= 0 && !behind_its_step)) return w;
         const Block& b = *layers[order[i].layer];
         w.wanted = b.wants_stream_copy();
-        if (w.wanted) b.entry_norm(w.norm);
+        if (w.wanted) { b.entry_norm(w.norm); w.into = with_rows.stream_copy; }
         return w;
     };
-    with_rows.leave = wanted_by(0, false);
+    auto wanted_by_step = [&](int which) {
+        Leave w;
+        w.wanted = which >= 0 && stream_steps[which]->wants_copy();
+        if (w.wanted) w.into = with_rows.step_copy;
+        return w;
+    };
+    auto make = [&](const Leave& w) {
+        if (w.norm.weight != nullptr) tanh_norm(x, w.norm, w.into, nullptr, s);
+        else cast_stream(x, w.into, s);
+    };
+    // (in front of a call: its stream step's copy if it has one, else its block's)
+    auto wanted_in_front = [&](size_t i) { return i < order.size() && order[i].before >= 0 ? wanted_by_step(order[i].before) : wanted_by(i, false); };
+    with_rows.leave = wanted_in_front(0);
     embedding->forward(with_rows, position.get(), x, s);
     Leave have = embedding->writes_stream_copy() ? with_rows.leave : Leave();
     // a stream step that mixes the embedding's output back in later: a copy of it stays for the step
@@ -731,6 +750,8 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
         auto stream_step = [&](int which, int pass, const char* stage) {
             const size_t mark = arena.mark();
             const StreamStep& st = *stream_steps[which];
+            const Leave reads = wanted_by_step(which);
+            if (reads.wanted && !have.same(reads)) make(reads);
             st.forward(x, st.kept_streams() > 0 ? x0_and_kept : x0, pass, with_rows, arena, s);
             arena.release(mark);
             have = st.leaves_copy() ? with_rows.leave : Leave();
@@ -741,20 +762,17 @@ void DecoderModel::forward(const StepView& step, const std::vector<CacheView>& c
             with_rows.leave = enters;
             stream_step(c.before, c.pass, "stream_step");
         }
-        if (enters.wanted && !have.same(enters)) {
-            if (enters.norm.weight != nullptr) tanh_norm(x, enters.norm, with_rows.stream_copy, nullptr, s);
-            else cast_stream(x, with_rows.stream_copy, s);
-        }
+        if (enters.wanted && !have.same(enters)) make(enters);
         const Block& b = *layers[c.layer];
-        with_rows.leave = c.after >= 0 ? Leave() : wanted_by(i + 1, false);
+        with_rows.leave = c.after >= 0 ? wanted_by_step(c.after) : wanted_in_front(i + 1);
         b.forward(x, with_rows, caches[c.cache], c.write, arena, s);
         // (a block that keeps a copy of the stream itself keeps it whether it is asked or not)
         const bool normed = with_rows.leave.norm.weight != nullptr;
         have = Leave();
         if (b.leaves_copy(normed)) have = with_rows.leave;
-        if (b.leaves_copy(false) && !b.leaves_copy(true)) { have = Leave(); have.wanted = true; }
+        if (b.leaves_copy(false) && !b.leaves_copy(true)) { have = Leave(); have.wanted = true; have.into = with_rows.stream_copy; }
         if (c.after >= 0) {
-            with_rows.leave = wanted_by(i + 1, false);
+            with_rows.leave = wanted_in_front(i + 1);
             stream_step(c.after, c.after_pass, "stream_step_after");
         }
     }

@@ -97,11 +97,15 @@ struct StepView {
                                        // room for a sub-layer's result; whoever uses it leaves it zero again
     Tensor2 stream_copy;               // the stream in bfloat16 as a block is entered, if a block asked for it
                                        // (Block::wants_stream_copy): the stream itself, or the block's entry norm of it
-    // What the part that runs now is asked to leave in stream_copy for the block behind it (parts that can: leaves_copy).
+    Tensor2 step_copy;                 // the stream in bfloat16 as a stream step is entered, if one asked for it
+                                       // (StreamStep::wants_copy); another tensor than stream_copy
+    // What the part that runs now is asked to leave for the part behind it (parts that can: leaves_copy): the stream's norm, or
+    // the stream itself, in bfloat16, in `into` (stream_copy or step_copy).
     struct Leave {
         bool wanted = false;
         MllmTanhNorm norm{nullptr, nullptr, nullptr};      // weight null: the stream itself
-        bool same(const Leave& o) const { return wanted == o.wanted && norm.weight == o.norm.weight; }
+        Tensor2 into;
+        bool same(const Leave& o) const { return wanted == o.wanted && norm.weight == o.norm.weight && into.data == o.into.data; }
     } leave;
     int n_groups = 0;
     const int* const* block_tables = nullptr;   // per group [B, max_blocks[g]]
@@ -353,7 +357,7 @@ public:
     virtual bool wants_stream_copy() const { return false; }
     // with wants_stream_copy: true and the norm if the copy is to be the block's first norm of the stream
     virtual bool entry_norm(MllmTanhNorm& n) const { (void)n; return false; }
-    // true: the block leaves in the copy what StepView::leave asks for (the stream's norm, or the stream itself)
+    // true: the block leaves what StepView::leave asks for (the stream's norm, or the stream itself)
     virtual bool leaves_copy(bool normed) const { return wants_stream_copy() && !normed; }
     virtual void reserve(int max_seqs, hipStream_t s) const = 0;
     virtual void add_cost(StepCost&) const = 0;
@@ -371,7 +375,8 @@ public:
     virtual size_t workspace_bytes(int tokens) const = 0;
     virtual bool wants_embedding_output() const { return false; }
     virtual int kept_streams() const { return 0; }         // > 0 goes with wants_embedding_output()
-    virtual bool leaves_copy() const { return false; }     // true: it leaves in the copy what StepView::leave asks for
+    virtual bool leaves_copy() const { return false; }     // true: it leaves what StepView::leave asks for
+    virtual bool wants_copy() const { return false; }      // true: it reads the stream's bfloat16 copy, StepView::step_copy
     virtual void reserve(int max_seqs, hipStream_t s) const { (void)max_seqs; (void)s; }
     virtual void add_cost(StepCost&) const {}
 };

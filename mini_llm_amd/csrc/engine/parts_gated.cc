@@ -102,7 +102,7 @@ public:
         add.y = arena.tensor(F32, x.rows, x.cols);        // room for results that a product cannot add by itself
         const size_t mark = arena.mark();
         add.norm = n_post1_;
-        add.copy = copies && (ff_ || step.leave.wanted) ? step.stream_copy : none;
+        add.copy = !copies ? none : ff_ ? step.stream_copy : step.leave.wanted ? step.leave.into : none;
         add.next = ff_ ? n_pre2_ : step.leave.norm;
         {
             NormedInput h = copies ? NormedInput(step.stream_copy) : NormedInput(*pre1_, x);
@@ -111,7 +111,7 @@ public:
         arena.release(mark);
         if (ff_) {
             add.norm = n_post2_;
-            add.copy = copies && step.leave.wanted ? step.stream_copy : none;
+            add.copy = copies && step.leave.wanted ? step.leave.into : none;
             add.next = step.leave.norm;
             NormedInput h = copies ? NormedInput(step.stream_copy) : NormedInput(*pre2_, x);
             ff_->forward_through(h, step, add, arena, s);

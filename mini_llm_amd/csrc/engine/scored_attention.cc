@@ -139,7 +139,14 @@ public:
                                                  : "scored_attention writes its own keys and values: it cannot read another call's cache");
         const int T = step.n_tokens, g = cache.group;
         Tensor2 q = arena.tensor(dtype_, T, sh_.n_heads * sh_.dim);
-        if (conv_.data != nullptr) {
+        const bool one_each = step.max_q_len == 1 && step.n_tokens == step.n_seqs;
+        if (conv_.data != nullptr && one_each && cache.has_state() && qk_prepare_takes_conv(sh_, T, static_cast<int>(conv_.cols)) && (conv_values_ || v_col_ < 0)) {
+            // single tokens: the convolution on the way
+            if (cache.state_bytes < conv_bytes_) fail("scored_attention with a convolution needs %zu bytes of state per request", conv_bytes_);
+            const MllmConvSingle cv{static_cast<const float*>(conv_.data), static_cast<int>(conv_.cols), static_cast<int>(conv_.rows), step.state_slots,
+                                    static_cast<float*>(cache.state), cache.slot_bytes / 4, write ? 1 : 0};
+            qk_prepare(proj, 0, k_col_, v_col_, sh_, step.positions, step.slots[g], q, cache.k_pages, cache.v_pages, s, &cv);
+        } else if (conv_.data != nullptr) {
             // the convolution over the projected queries and keys (and values), which lie side by side in front of the rows
             if (conv_bytes_ > 0 && (!cache.has_state() || cache.state_bytes < conv_bytes_)) fail("scored_attention with a convolution needs %zu bytes of state per request", conv_bytes_);
             const int C = static_cast<int>(conv_.rows);

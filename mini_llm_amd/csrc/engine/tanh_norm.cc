@@ -63,7 +63,7 @@ public:
         if (pass > 0 && x0.data == nullptr) fail("embedding_add needs the embedding's output");
         StreamAdd add;
         add.x = x;
-        if (step.leave.wanted) { add.copy = step.stream_copy; add.next = step.leave.norm; }
+        if (step.leave.wanted) { add.copy = step.leave.into; add.next = step.leave.norm; }
         stream_add(add, pass > 0 ? &x0 : nullptr, static_cast<const float*>(steps_.data) + static_cast<size_t>(pass) * steps_.cols, dtype_ == F32, s);
     }
     size_t workspace_bytes(int) const override { return 0; }
@@ -79,8 +79,8 @@ private:
 // Behind a layer: with e the `dim` columns from column `column` on of the token's row of a second table,
 //   g = gelu_tanh(W_gate x) * e,  y = W_proj g,  x += y / sqrt(mean(y^2) + eps) * weight.
 // Parameters: dtype, column, eps; tensors table [vocab, columns], gate.weight [dim, width], proj.weight [width, dim],
-// norm.weight [width]; and, for one kernel that does it all, gate.tiles and proj.tiles (the two maps in operand order, see
-// ops.h).
+// norm.weight [width]; and, for one kernel that does it all, gate.tiles, proj.tiles and proj.gram (the two maps and the second
+// one's square in operand order, see ops.h).
 class TokenSide final : public StreamStep {
 public:
     explicit TokenSide(const Params& p) : table_(p.weights("table")), gate_(p.weights("gate.weight"), nullptr), proj_(p.weights("proj.weight"), nullptr) {
@@ -94,6 +94,7 @@ public:
         if (const Tensor2* g = p.weights_or_null("gate.tiles")) {
             gate_tiles_ = *g;
             proj_tiles_ = p.weights("proj.tiles");
+            gram_tiles_ = p.weights("proj.gram");
             if (dtype_ != BF16 || !token_side_fits(proj_.out_features(), dim_)) fail("token_side: tiles for a width of %d and %d columns: no kernel takes them", proj_.out_features(), dim_);
         }
     }
@@ -103,8 +104,8 @@ public:
         if (gate_tiles_.data != nullptr) {
             StreamAdd add;
             add.x = x;
-            if (step.leave.wanted) { add.copy = step.stream_copy; add.next = step.leave.norm; }
-            token_side(add, gate_tiles_, proj_tiles_, norm_, eps_, step.token_ids, &step.fed, table_, column_, dim_, s);
+            if (step.leave.wanted) { add.copy = step.leave.into; add.next = step.leave.norm; }
+            token_side(add, step.step_copy, gate_tiles_, proj_tiles_, gram_tiles_, norm_, eps_, step.token_ids, &step.fed, table_, column_, dim_, s);
             return;
         }
         Tensor2 h = x;
@@ -121,11 +122,12 @@ public:
         return static_cast<size_t>(tokens) * (proj_.out_features() * 6 + (dim_ + 8) * 8) + 2048;
     }
     bool leaves_copy() const override { return gate_tiles_.data != nullptr; }
+    bool wants_copy() const override { return gate_tiles_.data != nullptr; }
     void reserve(int, hipStream_t s) const override { reserve_linear_scratch(s); }
     void add_cost(StepCost& c) const override { gate_.add_cost(c); proj_.add_cost(c); c.weight_bytes += 4.0 * proj_.out_features(); }
 
 private:
-    Tensor2 table_, gate_tiles_, proj_tiles_;
+    Tensor2 table_, gate_tiles_, proj_tiles_, gram_tiles_;
     Linear gate_, proj_;
     const float* norm_ = nullptr;
     int dtype_ = BF16, column_ = 0, dim_ = 0;

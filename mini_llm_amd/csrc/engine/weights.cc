@@ -430,6 +430,28 @@ Tensor2 DeviceTensors::operand_tiles(const Tensor2& t, int64_t rows, int64_t col
     return Tensor2(dev, BF16, rows, cols);
 }
 
+Tensor2 DeviceTensors::gram_tiles(const Tensor2& w, int64_t n) {
+    if (w.dtype != BF16 || !w.contiguous() || n % 16 != 0 || n < w.cols) throw WeightsError("gram_tiles: a contiguous bfloat16 matrix and a size in whole tiles are needed");
+    std::vector<uint16_t> from(static_cast<size_t>(w.rows) * w.cols);
+    if (!from.empty() && hipMemcpy(from.data(), w.data, from.size() * 2, hipMemcpyDeviceToHost) != hipSuccess) throw WeightsError("gram_tiles: the copy from the device failed");
+    const size_t C = static_cast<size_t>(w.cols);
+    std::vector<double> g(C * C, 0.0), row(C);
+    for (int64_t r = 0; r < w.rows; ++r) {
+        for (size_t c = 0; c < C; ++c) row[c] = bf16_bits_to_float(from[static_cast<size_t>(r) * C + c]);
+        for (size_t a = 0; a < C; ++a)
+            for (size_t b = 0; b < C; ++b) g[a * C + b] += row[a] * row[b];
+    }
+    std::vector<float> tiles(static_cast<size_t>(n) * n, 0.f);
+    size_t at = 0;
+    for (int64_t r0 = 0; r0 < n; r0 += 16)
+        for (int64_t c0 = 0; c0 < n; c0 += 4)
+            for (int lane = 0; lane < 64; ++lane, ++at) {
+                const int64_t r = r0 + lane % 16, c = c0 + lane / 16;
+                if (r < w.cols && c < w.cols) tiles[at] = static_cast<float>(g[static_cast<size_t>(r) * C + static_cast<size_t>(c)]);
+            }
+    return upload(tiles, n, n, F32);
+}
+
 Tensor2 DeviceTensors::scaled(const Tensor2& v, float factor) {
     const size_t n = static_cast<size_t>(v.rows) * v.cols;
     if (v.dtype != F32 || !v.contiguous()) throw WeightsError("scaled: a contiguous float32 vector is needed");

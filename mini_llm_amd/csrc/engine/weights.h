@@ -174,6 +174,9 @@ public:
     // row l % 16, columns 8 (l / 16) to 8 (l / 16) + 7 of its tile. Rows and columns are filled up with zeros to `rows` and
     // `cols` (multiples of 16 and 32).
     Tensor2 operand_tiles(const Tensor2& t, int64_t rows, int64_t cols);
+    // W^T W of a bfloat16 matrix W [rows, cols], in fp32 (sums in double), filled up with zeros to [n, n] (n a multiple of 16), as 16
+    // x 4 tiles in operand order, [n / 16][n / 4][lane]: lane l holds row l % 16, column l / 16 of its tile.
+    Tensor2 gram_tiles(const Tensor2& w, int64_t n);
     // A vector times a number ([1, n] fp32, a copy on the device).
     Tensor2 scaled(const Tensor2& vector, float factor);
     size_t bytes() const { return bytes_; }

@@ -647,7 +647,7 @@ int mllm_moe_grouped_glu(const void* h, int ldh, const float* logits, int ldl, i
     for (const MllmTanhNorm* n : {&add.norm, &add.next})
         if (n->weight != nullptr && (n->alpha == nullptr || n->bias == nullptr || !a16(n->weight) || !a16(n->bias))) return -1;
     if (router_kind < ROUTER_SOFTMAX || router_kind > ROUTER_SOFTMAX_CHOSEN || !(limit > 0.f)) return -1;
-    const int tokens = E <= 48 ? 256 : (E <= 128 ? 64 : 32);
+    const int tokens = E <= 128 ? 64 : 32;
     const size_t lds = static_cast<size_t>(tokens) * (E + 1) * 4 + static_cast<size_t>(2) * E * 4;
     moe_route_kernel<<<(T + tokens - 1) / tokens, 256, lds, stream>>>(logits, ldl, T, E, top, scale, router_kind, tokens, counts, lists, T, weights);
     MLLM_LAUNCH_CHECK();

@@ -22,3 +22,15 @@ struct MllmScoreShape {
     const float* sink;       // per head, or null: nothing added to the denominator (softmax weights only)
     int keep_first;          // with a window: the first positions that stay visible; <= 0: none
 };
+
+// A short causal convolution that a kernel applies to the projected rows of single tokens as it reads them: channel c of the
+// rows' first `channels` columns becomes sum_j w[c, j] u(t - taps + 1 + j), the earlier inputs carried in the request's slot
+// ([taps - 1][channels], the oldest first), which move up by one.
+struct MllmConvSingle {
+    const float* w;              // [channels, taps]
+    int taps, channels;
+    const int* state_slots;      // per token
+    float* state;
+    unsigned long long slot_floats;
+    int write;
+};

@@ -122,15 +122,33 @@ qk_prepare_kernel(const float* __restrict__ proj, int ld, int q_col, int k_col, 
     }
 }
 
+// Channel ch of a single token's row behind the convolution; with `mine` its carried inputs move up.
+template <int TAPS>
+__device__ __forceinline__ float conv_value(const MllmConvSingle& cv, float* carried, int ch, float now, bool mine) {
+    float v[TAPS], acc = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) v[j] = carried[static_cast<size_t>(j) * cv.channels + ch];
+    v[TAPS - 1] = now;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) acc += cv.w[static_cast<size_t>(ch) * TAPS + j] * v[j];
+    if (mine && cv.write) {
+#pragma unroll
+        for (int j = 1; j < TAPS; ++j) carried[static_cast<size_t>(j - 1) * cv.channels + ch] = v[j];
+    }
+    return acc;
+}
+
 // The same for steps of few rows (decoding), one wavefront per (token, head): queries, then keys. A head of the
 // whole-row norm adds up the whole row itself (a few loads a lane) instead of waiting for the other heads. A lane has
 // up to 4 columns of its head (d <= 256); rotation partners meet through the wavefront's LDS.
-template <typename T>
+// TAPS > 0: the rows are convolved as they are read (a channel's value belongs to one lane, which also moves its carried inputs
+// up).
+template <typename T, int TAPS>
 __global__ void __launch_bounds__(256)
 qk_prepare_heads_kernel(const float* __restrict__ proj, int ld, int q_col, int k_col, int v_col, int n_tokens, int H, int G, int d,
                         int dv, int norm_mode, const float* __restrict__ wq, const float* __restrict__ wk, float eps, int rot_dims,
                         double rot_base, const float* __restrict__ rot_freqs, int interleaved, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
-                        int ldq, T* __restrict__ k_pages, T* __restrict__ v_pages) {
+                        int ldq, T* __restrict__ k_pages, T* __restrict__ v_pages, MllmConvSingle cv) {
     __shared__ float normed_s[4][256];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lane = threadIdx.x % 64;
     const int pair = blockIdx.x * 4 + wave;
@@ -143,6 +161,17 @@ qk_prepare_heads_kernel(const float* __restrict__ proj, int ld, int q_col, int k
     float raw[4];
 #pragma unroll
     for (int u = 0; u < 4; ++u) raw[u] = row[h * d + min(lane + 64 * u, d - 1)];
+    float* carried = nullptr;
+    if constexpr (TAPS > 0) {
+        const int state_slot = cv.state_slots[t];
+        if (state_slot < 0) return;                   // (a padding row: the whole wavefront)
+        carried = cv.state + static_cast<size_t>(state_slot) * cv.slot_floats;
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            if (64 * u >= d) continue;                // (uniform: no lane has such a column)
+            raw[u] = conv_value<TAPS>(cv, carried, (is_k ? k_col : q_col) + h * d + min(lane + 64 * u, d - 1), raw[u], lane + 64 * u < d);
+        }
+    }
     float inv = 1.f;
     if (norm_mode == NORM_HEAD) {
         float ss = 0.f;
@@ -213,7 +242,11 @@ qk_prepare_heads_kernel(const float* __restrict__ proj, int ld, int q_col, int k
             if (lane + 64 * u < d) vp[lane + 64 * u] = from_float<T>(raw[u]);
     } else {
         const float* vr = proj + static_cast<size_t>(t) * ld + v_col + h * dv;
-        for (int i = lane; i < dv; i += 64) vp[i] = from_float<T>(vr[i]);
+        for (int i = lane; i < dv; i += 64) {
+            float v = vr[i];
+            if constexpr (TAPS > 0) v = conv_value<TAPS>(cv, carried, v_col + h * dv + i, v, true);
+            vp[i] = from_float<T>(v);
+        }
     }
 }
 
@@ -382,7 +415,7 @@ int mllm_gate_mul(void* x, int ldx, const float* gate, int ldg, int T, int N, in
 int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, int T, int H, int G, int d, int dv,
                     int norm_mode, const float* wq, const float* wk, float eps, int rot_dims, double rot_base,
                     const int* positions, const int* slots, void* q_out, int ldq, void* k_pages, void* v_pages, int dtype,
-                    hipStream_t stream, int interleaved, const float* rot_freqs) {
+                    hipStream_t stream, int interleaved, const float* rot_freqs, const MllmConvSingle* conv) {
     if (T <= 0) return 0;
     // (G == 0: queries only; the keys and values are another layer's)
     if (H < 1 || G < 0 || d < 1 || dv < 1 || rot_dims < 0 || rot_dims % 2 != 0 || rot_dims > d || rot_dims / 2 > 256) return -1;
@@ -392,17 +425,25 @@ int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, 
     if (T <= 64 && d <= 256) {
         // few rows: one wavefront per (token, head) instead of one workgroup per token
         const int blocks = (T * (H + G) + 3) / 4;
-        if (dtype == MLLM_F32)
-            qk_prepare_heads_kernel<float><<<blocks, 256, 0, stream>>>(proj, ld, q_col, k_col, v_col, T, H, G, d, dv, norm_mode, wq, wk, eps,
-                                                                       rot_dims, rot_base, rot_freqs, interleaved, positions, slots, static_cast<float*>(q_out), ldq,
-                                                                       static_cast<float*>(k_pages), static_cast<float*>(v_pages));
-        else
-            qk_prepare_heads_kernel<bf16_t><<<blocks, 256, 0, stream>>>(proj, ld, q_col, k_col, v_col, T, H, G, d, dv, norm_mode, wq, wk, eps,
-                                                                        rot_dims, rot_base, rot_freqs, interleaved, positions, slots, static_cast<bf16_t*>(q_out), ldq,
-                                                                        static_cast<bf16_t*>(k_pages), static_cast<bf16_t*>(v_pages));
+        const int taps = conv != nullptr ? conv->taps : 0;
+        const MllmConvSingle cv = conv != nullptr ? *conv : MllmConvSingle{nullptr, 0, 0, nullptr, nullptr, 0, 0};
+#define QK_HEADS(TYPE, TAPS)                                                                                                        \
+    qk_prepare_heads_kernel<TYPE, TAPS><<<blocks, 256, 0, stream>>>(proj, ld, q_col, k_col, v_col, T, H, G, d, dv, norm_mode, wq, wk, eps, \
+                                                                    rot_dims, rot_base, rot_freqs, interleaved, positions, slots,   \
+                                                                    static_cast<TYPE*>(q_out), ldq, static_cast<TYPE*>(k_pages),    \
+                                                                    static_cast<TYPE*>(v_pages), cv)
+#define QK_HEADS_T(TYPE)                                                                                                            \
+    do {                                                                                                                            \
+        if (taps == 0) QK_HEADS(TYPE, 0); else if (taps == 2) QK_HEADS(TYPE, 2); else if (taps == 3) QK_HEADS(TYPE, 3);              \
+        else if (taps == 4) QK_HEADS(TYPE, 4); else return -1;                                                                       \
+    } while (0)
+        if (dtype == MLLM_F32) QK_HEADS_T(float); else QK_HEADS_T(bf16_t);
+#undef QK_HEADS_T
+#undef QK_HEADS
         MLLM_LAUNCH_CHECK();
         return 0;
     }
+    if (conv != nullptr) return -1;                   // (only the kernel above convolves)
     const size_t smem = (static_cast<size_t>(H + G) * d + rot_dims + (H + G) + 2) * sizeof(float);
     if (smem > 60 * 1024) return -1;
     if (dtype == MLLM_F32)

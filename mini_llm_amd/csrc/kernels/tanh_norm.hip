@@ -102,16 +102,21 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // [8]: lane l holds row l % 16, inputs 8 (l / 16) ..), so a wavefront's load is one kilobyte in a row; both are asked for at the
 // start. The weights are the matrix cores' first operand: a lane then holds four consecutive columns of one token. The inputs of
 // the first map (the stream, rounded to bfloat16) are dealt over the wavefronts, whose sums meet in LDS in the order of their
-// index; of the second the columns are. DT: tiles of 16 over dim; KPW: tiles of 32 over the width a wavefront takes of the
-// first map; CPW: tiles of 16 columns it takes of the second.
-template <int DT, int KPW, int CPW>
+// index; of the second the columns are. The first map reads the stream from `xb`, its bfloat16 copy. DT: tiles of 16 over dim; KPW: tiles
+// of 32 over the width a wavefront takes of the first map; CPW: tiles of 16 columns it takes of the second.
+// SPLIT (few tokens): several workgroups (blockIdx.y) share a token's columns, 16 tiles each; every one works out the first map
+// for itself, and the sum of squares comes from g alone, |W_proj g|^2 = g^T (W_proj^T W_proj) g, with that matrix in `gram`:
+// fp32 operand tiles [tile of 16 rows][4 inputs][lane] (lane l: row l % 16, input l / 16).
+template <int DT, int KPW, int CPW, bool SPLIT>
 __global__ void __launch_bounds__(SIDE_WAVES * 64)
-token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* __restrict__ gate, const bf16x8* __restrict__ proj,
-                  const float* __restrict__ weight, float eps, const int* __restrict__ ids, const int* __restrict__ src,
+token_side_kernel(float* __restrict__ x, const bf16_t* __restrict__ xb, int T, int rows, int D, const bf16x8* __restrict__ gate,
+                  const bf16x8* __restrict__ proj, const float* __restrict__ gram, const float* __restrict__ weight, float eps, const int* __restrict__ ids, const int* __restrict__ src,
                   const int* __restrict__ prev, int n_prev, const bf16_t* __restrict__ table, int ldt, int col0, int dim, MllmStreamAdd add) {
     constexpr int DIM = DT * 16, DK = (DIM + 31) / 32, GS = DK * 32 + 8, ZS = DIM + 4;
     // (wide streams: the second map's tiles are asked for behind the first map's products, whose registers they take)
-    constexpr bool EARLY = KPW * (DT * 4 + 8) + CPW * (DK * 4 + 4) <= 96;
+    constexpr bool EARLY = KPW * (DT * 4 + 4) + CPW * (DK * 4 + 4) <= 96;
+    static_assert(!SPLIT || CPW == 1, "shared columns: one tile a wavefront");
+    constexpr int GU = DT == 4 ? 4 : 1;              // products of g with gram a wavefront takes (DT 1: four wavefronts have one)
     __shared__ __attribute__((aligned(16))) float z_s[SIDE_WAVES][ZS * 16];
     __shared__ __attribute__((aligned(16))) bf16_t g_s[16 * GS];
     __shared__ float ss_s[SIDE_WAVES][16];
@@ -121,12 +126,11 @@ token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* _
     // everything the kernel reads is asked for here: the first map's tiles with the stream, then the table's columns, the
     // second map's tiles and the stream again as the result is laid out
     bf16x8 wg[KPW][DT];
-    float4 xa[KPW][2];
+    bf16x8 xa[KPW];
 #pragma unroll
     for (int u = 0; u < KPW; ++u) {
         const int kb = min(wave + SIDE_WAVES * u, KB - 1);
-        xa[u][0] = *reinterpret_cast<const float4*>(x + row_at + kb * 32 + 8 * q);
-        xa[u][1] = *reinterpret_cast<const float4*>(x + row_at + kb * 32 + 8 * q + 4);
+        xa[u] = *reinterpret_cast<const bf16x8*>(xb + row_at + kb * 32 + 8 * q);
 #pragma unroll
         for (int d = 0; d < DT; ++d) wg[u][d] = gate[(static_cast<size_t>(d) * KB + kb) * 64 + lane];
     }
@@ -147,7 +151,7 @@ token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* _
     auto fetch_second = [&]() {
 #pragma unroll
         for (int c = 0; c < CPW; ++c) {
-            const int cb = min(wave + SIDE_WAVES * c, CB - 1);
+            const int cb = min(static_cast<int>(blockIdx.y) * SIDE_WAVES + wave + SIDE_WAVES * c, CB - 1);
 #pragma unroll
             for (int k = 0; k < DK; ++k) wp[c][k] = proj[(static_cast<size_t>(cb) * DK + k) * 64 + lane];
             xv[c] = *reinterpret_cast<const float4*>(x + row_at + cb * 16 + 4 * q);
@@ -155,17 +159,29 @@ token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* _
         __builtin_amdgcn_sched_barrier(0);
     };
     if (EARLY) fetch_second();
+    // (SPLIT: the end's vectors and this wavefront's tiles of gram: row tile, first of its steps of four inputs)
+    const int g_row = DT == 1 ? 0 : wave % DT, g_step = DT == 4 ? (wave / 4) * 4 : wave / DT;
+    float gm[GU];
+    float4 w_first = make_float4(0.f, 0.f, 0.f, 0.f), nw_first = w_first, nb_first = w_first;
+    if constexpr (SPLIT) {
+#pragma unroll
+        for (int u = 0; u < GU; ++u) gm[u] = gram[(static_cast<size_t>(g_row) * (DT * 4) + min(g_step + u, DT * 4 - 1)) * 64 + lane];
+        const int n = min(static_cast<int>(blockIdx.y) * SIDE_WAVES + wave, CB - 1) * 16 + 4 * q;
+        w_first = *reinterpret_cast<const float4*>(weight + n);
+        if (add.copy != nullptr && add.next.weight != nullptr) {
+            nw_first = *reinterpret_cast<const float4*>(add.next.weight + n);
+            nb_first = *reinterpret_cast<const float4*>(add.next.bias + n);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+    }
     f32x4 acc[DT];
 #pragma unroll
     for (int d = 0; d < DT; ++d) acc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int u = 0; u < KPW; ++u) {
         if (wave + SIDE_WAVES * u >= KB) continue;
-        union { uint32_t w[4]; bf16x8 v; } b;
-        b.w[0] = pack_bf16x2(xa[u][0].x, xa[u][0].y); b.w[1] = pack_bf16x2(xa[u][0].z, xa[u][0].w);
-        b.w[2] = pack_bf16x2(xa[u][1].x, xa[u][1].y); b.w[3] = pack_bf16x2(xa[u][1].z, xa[u][1].w);
 #pragma unroll
-        for (int d = 0; d < DT; ++d) acc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wg[u][d], b.v, acc[d], 0, 0, 0);
+        for (int d = 0; d < DT; ++d) acc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wg[u][d], xa[u], acc[d], 0, 0, 0);
     }
     // (register r of lane l: column of dim 4 (l / 16) + r, token l % 16)
 #pragma unroll
@@ -190,7 +206,17 @@ token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* _
         y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int k = 0; k < DK; ++k) y[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wp[c][k], gb[k], y[c], 0, 0, 0);
-        if (wave + SIDE_WAVES * c < CB) ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+        if (!SPLIT && wave + SIDE_WAVES * c < CB) ss += y[c][0] * y[c][0] + y[c][1] * y[c][1] + y[c][2] * y[c][2] + y[c][3] * y[c][3];
+    }
+    if constexpr (SPLIT) {
+        f32x4 t = f32x4{0.f, 0.f, 0.f, 0.f};
+        const bool has = DT > 1 || wave < 4;
+#pragma unroll
+        for (int u = 0; u < GU; ++u)
+            t = __builtin_amdgcn_mfma_f32_16x16x4f32(gm[u], to_float(g_s[tok * GS + 4 * (has ? g_step + u : 0) + q]), t, 0, 0, 0);
+        // (register r: row 16 g_row + 4 q + r of gram g, of token `tok`)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) ss += has ? t[r] * to_float(g_s[tok * GS + 16 * g_row + 4 * q + r]) : 0.f;
     }
     ss = rows_sum(ss);
     if (lane < 16) ss_s[wave][lane] = ss;
@@ -198,21 +224,21 @@ token_side_kernel(float* __restrict__ x, int T, int rows, int D, const bf16x8* _
     float total = 0.f;
 #pragma unroll
     for (int w = 0; w < SIDE_WAVES; ++w) total += ss_s[w][tok];
-    const float inv = 1.f / sqrtf(total / static_cast<float>(D) + eps);
+    const float inv = 1.f / sqrtf(fmaxf(total, 0.f) / static_cast<float>(D) + eps);
     if (tok >= n_rows) return;
     const bool has_next = add.next.weight != nullptr;
     const float alpha = has_next ? add.next.alpha[0] : 0.f;
 #pragma unroll
     for (int c = 0; c < CPW; ++c) {
-        const int cb = wave + SIDE_WAVES * c;
+        const int cb = static_cast<int>(blockIdx.y) * SIDE_WAVES + wave + SIDE_WAVES * c;
         if (cb >= CB) continue;
         const int n = cb * 16 + 4 * q;
-        const float4 w4 = *reinterpret_cast<const float4*>(weight + n);
+        const float4 w4 = SPLIT ? w_first : *reinterpret_cast<const float4*>(weight + n);
         float o[4] = {xv[c].x + y[c][0] * inv * w4.x, xv[c].y + y[c][1] * inv * w4.y, xv[c].z + y[c][2] * inv * w4.z, xv[c].w + y[c][3] * inv * w4.w};
         *reinterpret_cast<float4*>(x + row_at + n) = make_float4(o[0], o[1], o[2], o[3]);
         if (add.copy == nullptr) continue;
         if (has_next) {
-            const float4 nw = *reinterpret_cast<const float4*>(add.next.weight + n), nb = *reinterpret_cast<const float4*>(add.next.bias + n);
+            const float4 nw = SPLIT ? nw_first : *reinterpret_cast<const float4*>(add.next.weight + n), nb = SPLIT ? nb_first : *reinterpret_cast<const float4*>(add.next.bias + n);
             o[0] = fast_tanh(alpha * o[0]) * nw.x + nb.x; o[1] = fast_tanh(alpha * o[1]) * nw.y + nb.y;
             o[2] = fast_tanh(alpha * o[2]) * nw.z + nb.z; o[3] = fast_tanh(alpha * o[3]) * nw.w + nb.w;
         }
@@ -287,25 +313,30 @@ int mllm_token_gate(const float* z, int ldz, const int* ids, const int* src, con
 int mllm_token_side_fits(int D, int dim) { return D >= 32 && D % 32 == 0 && D <= 2048 && dim >= 1 && dim <= 64 ? 1 : 0; }
 
 // x fp32 [T, D] contiguous; gate and proj bfloat16 in tiles (see the kernel; dim filled up with zeros to a multiple of 16 in the
-// gate's rows and of 32 in proj's inputs); weight [D]; ids, src, prev, table as for mllm_token_gate. Tokens up to
+// gate's rows and of 32 in proj's inputs); xb: the stream's bfloat16 copy [T, D], which add.copy must not be; gram: see the kernel;
+// weight [D]; ids, src, prev, table as for mllm_token_gate. Tokens up to
 // 2,048 take 8 a workgroup, more take 16. -2: sizes the kernel is not built for; -1: operands that are not aligned.
-int mllm_token_side(float* x, int T, int D, const void* gate, const void* proj, const float* weight, float eps, const int* ids, const int* src,
+int mllm_token_side(float* x, const void* xb, int T, int D, const void* gate, const void* proj, const float* gram, const float* weight, float eps, const int* ids, const int* src,
                     const int* prev, int n_prev, const void* table, int ldt, int col0, int dim, MllmStreamAdd add, hipStream_t stream) {
     if (T <= 0) return 0;
     if (!mllm_token_side_fits(D, dim)) return -2;
-    if (ids == nullptr || (src != nullptr && prev == nullptr) || !on16(x) || !on16(gate) || !on16(proj) || !on16(weight) || !norm_on16(add.next) ||
+    if (ids == nullptr || (src != nullptr && prev == nullptr) || !on16(x) || !on16(xb) || xb == add.copy || gram == nullptr || !on16(gate) || !on16(proj) || !on16(weight) || !norm_on16(add.next) ||
         (add.copy != nullptr && (add.ld_copy % 4 != 0 || (reinterpret_cast<uintptr_t>(add.copy) & 7))))
         return -1;
     const int rows = T <= 2048 ? 8 : 16, blocks = (T + rows - 1) / rows;
-    const int dt = dim <= 16 ? 1 : (dim <= 32 ? 2 : 4), kpw = D <= 512 ? 1 : (D <= 1024 ? 2 : 4);
-#define TOKEN_SIDE(DT, KPW, CPW)                                                                                                        \
-    token_side_kernel<DT, KPW, CPW><<<blocks, SIDE_WAVES * 64, 0, stream>>>(x, T, rows, D, static_cast<const bf16x8*>(gate),              \
-        static_cast<const bf16x8*>(proj), weight, eps, ids, src, prev, n_prev, static_cast<const bf16_t*>(table), ldt, col0, dim, add)
-#define TOKEN_SIDE_D(DT) do { if (kpw == 1) TOKEN_SIDE(DT, 1, 2); else if (kpw == 2) TOKEN_SIDE(DT, 2, 4); else TOKEN_SIDE(DT, 4, 8); } while (0)
+    const int dt = dim <= 16 ? 1 : (dim <= 32 ? 2 : 4), kpw = D <= 512 ? 1 : (D <= 1024 ? 2 : 4), parts = (D / 16 + SIDE_WAVES - 1) / SIDE_WAVES;
+    const bool split = blocks * parts <= 128;
+#define TOKEN_SIDE(DT, KPW, CPW, SPLIT)                                                                                                 \
+    token_side_kernel<DT, KPW, CPW, SPLIT><<<dim3(blocks, SPLIT ? parts : 1), SIDE_WAVES * 64, 0, stream>>>(x, static_cast<const bf16_t*>(xb), T, rows, D, \
+        static_cast<const bf16x8*>(gate), static_cast<const bf16x8*>(proj), gram, weight, eps, ids, src, prev, n_prev,                  \
+        static_cast<const bf16_t*>(table), ldt, col0, dim, add)
+#define TOKEN_SIDE_K(DT, KPW, CPW) do { if (split) TOKEN_SIDE(DT, KPW, 1, true); else TOKEN_SIDE(DT, KPW, CPW, false); } while (0)
+#define TOKEN_SIDE_D(DT) do { if (kpw == 1) TOKEN_SIDE_K(DT, 1, 2); else if (kpw == 2) TOKEN_SIDE_K(DT, 2, 4); else TOKEN_SIDE_K(DT, 4, 8); } while (0)
     if (dt == 1) TOKEN_SIDE_D(1);
     else if (dt == 2) TOKEN_SIDE_D(2);
     else TOKEN_SIDE_D(4);
 #undef TOKEN_SIDE_D
+#undef TOKEN_SIDE_K
 #undef TOKEN_SIDE
     MLLM_LAUNCH_CHECK();
     return 0;
