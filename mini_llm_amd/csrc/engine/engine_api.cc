@@ -60,7 +60,7 @@ unsigned long long mllm_scratch_bytes(void) {
 }
 int mllm_release_scratch(hipStream_t stream) { return guarded([&] { release_scratch(stream); }); }
 // name: "decode_shape" (nsplit, waves; 0, 0 = automatic), "unmerged_shape", "merge_max_rows" (a), "ln_fuse_max_rows" (a), "long_context_splits" (a: 0 off, 1 on),
-// "latent_tiles", "scored_shared_kernels" (a: 0 off, 1 on), "halves_max_width" (a)
+// "latent_tiles", "scored_shared_kernels" (a: 0 off, 1 on), "halves_max_width" (a), "through_products" (a: 0 off, 1 on), "grouped_experts_rows" (a)
 int mllm_set_tuning(const char* name, int a, int b) {
     return guarded([&] {
         Tuning& t = tuning();
@@ -73,6 +73,8 @@ int mllm_set_tuning(const char* name, int a, int b) {
         else if (n == "latent_tiles") t.latent_tiles = a;
         else if (n == "scored_shared_kernels") t.scored_shared_kernels = a;
         else if (n == "halves_max_width") t.halves_max_width = a;
+        else if (n == "through_products") t.through_products = a;
+        else if (n == "grouped_experts_rows") t.grouped_experts_rows = a;
         else if (n == "reset_seen") t.seen = Tuning::Seen();
         else fail("unknown tuning value '%s'", name);
     });
@@ -80,7 +82,8 @@ int mllm_set_tuning(const char* name, int a, int b) {
 // What the ops chose since the last "reset_seen": "max_decode_splits" (most workgroups a (token, head) pair's keys
 // were split over), "merge_kernel_launches", "prefill_tile_launches" (the bfloat16 matrix-core kernel), "tiled_f32_launches" (the 32-bit one),
 // "generic_attention_launches", "latent_tile_launches" and "latent_token_launches" (latent attention on the matrix cores / one
-// workgroup per token). -1: unknown name.
+// workgroup per token), "through_products" (products that took their result into the stream themselves), "grouped_experts"
+// (feed-forwards of routed experts run as grouped products). -1: unknown name.
 long long mllm_get_seen(const char* name) {
     const Tuning::Seen& s = tuning().seen;
     const std::string n(name);
@@ -91,6 +94,8 @@ long long mllm_get_seen(const char* name) {
     if (n == "generic_attention_launches") return s.generic_attention_launches;
     if (n == "latent_tile_launches") return s.latent_tile_launches;
     if (n == "latent_token_launches") return s.latent_token_launches;
+    if (n == "through_products") return s.through_products;
+    if (n == "grouped_experts") return s.grouped_experts;
     return -1;
 }
 
@@ -137,6 +142,44 @@ int mllm_op_ln_linear(const Tensor2* x, const float* gamma, const float* beta, f
 // *unmerged = 1 and *splits filled when the result was left as splits (only with may_split)
 int mllm_op_paged_attention(const AttentionArgs* a, AttentionSplits* splits, int* unmerged, hipStream_t s) {
     return guarded([&] { *unmerged = paged_attention(*a, splits, s) ? 1 : 0; });
+}
+// A norm is {alpha, weight, bias} (weight null: none). copy, y, x0 and step may be null.
+int mllm_op_tanh_norm(const Tensor2* x, const MllmTanhNorm* norm, const Tensor2* out, const int* rows, hipStream_t s) {
+    return guarded([&] { tanh_norm(*x, *norm, *out, rows, s); });
+}
+static StreamAdd stream_add_of(const Tensor2* x, const Tensor2* y, const Tensor2* copy, const MllmTanhNorm* norm, const MllmTanhNorm* next) {
+    StreamAdd add;
+    add.x = *x;
+    if (y != nullptr) add.y = *y;
+    if (copy != nullptr) add.copy = *copy;
+    if (norm != nullptr) add.norm = *norm;
+    if (next != nullptr) add.next = *next;
+    return add;
+}
+int mllm_op_stream_add(const Tensor2* x, const Tensor2* y, const Tensor2* x0, const float* step, const Tensor2* copy, const MllmTanhNorm* norm,
+                       const MllmTanhNorm* next, int precise, hipStream_t s) {
+    return guarded([&] { stream_add(stream_add_of(x, y, copy, norm, next), x0, step, precise != 0, s); });
+}
+int mllm_op_linear_stream_add(const Tensor2* a, const Tensor2* w, const float* bias, const Tensor2* x, const Tensor2* y, const Tensor2* copy,
+                              const MllmTanhNorm* norm, const MllmTanhNorm* next, hipStream_t s) {
+    return guarded([&] { linear_stream_add(*a, *w, bias, stream_add_of(x, y, copy, norm, next), s); });
+}
+// gate [dim, D] and proj [D, dim] bfloat16 as they are stored (brought into operand order here).
+int mllm_op_token_side(const Tensor2* x, const Tensor2* xb, const Tensor2* gate, const Tensor2* proj, const float* weight, float eps, const int* ids,
+                       const int* src, const int* prev, int n_prev, const Tensor2* table, int col0, const Tensor2* copy, const MllmTanhNorm* next,
+                       hipStream_t s) {
+    return guarded([&] {
+        DeviceTensors store;
+        const int dim = static_cast<int>(gate->rows);
+        const int64_t padded = token_side_padded(dim);
+        if (!token_side_fits(static_cast<int>(gate->cols), dim)) fail("token_side: no kernel for a width of %lld and %d columns", (long long)gate->cols, dim);
+        const Tensor2 g = store.operand_tiles(*gate, padded, gate->cols), p = store.operand_tiles(*proj, proj->rows, (padded + 31) / 32 * 32),
+                      m = store.gram_tiles(*proj, padded);
+        FedTokens fed;
+        fed.src = src; fed.prev = prev; fed.n_prev = n_prev;
+        token_side(stream_add_of(x, nullptr, copy, nullptr, next), *xb, g, p, m, weight, eps, ids, src ? &fed : nullptr, *table, col0, dim, s);
+        if (hipStreamSynchronize(s) != hipSuccess) fail("token_side: the kernel failed");
+    });
 }
 int mllm_op_argmax(const Tensor2* logits, int* out, hipStream_t s) { return guarded([&] { argmax(*logits, out, s); }); }
 int mllm_op_sample(const Tensor2* logits, const float* temperature, const float* u, int* out, hipStream_t s) {

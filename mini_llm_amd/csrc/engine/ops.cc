@@ -290,7 +290,7 @@ void linear_stream_add(const Tensor2& a, const Tensor2& w, const float* bias, co
         const int rc = mllm_gemm_bf16_through(a.data, static_cast<int>(a.stride), w.data, static_cast<int>(w.stride), bias, static_cast<float*>(add.x.data),
                                               static_cast<int>(add.x.stride), static_cast<int>(M), static_cast<int>(w.rows), static_cast<int>(K), k, ws,
                                               ws ? GEMM_WORKSPACE_BYTES : 0, stream);
-        if (rc == 0) return;
+        if (rc == 0) { tuning().seen.through_products += 1; return; }
         if (rc != -1) check(rc, "linear_stream_add");
     }
     if (add.y.data == nullptr) fail("linear_stream_add: these sizes need room for the result");
@@ -336,6 +336,7 @@ bool moe_grouped(const Tensor2& h, const Tensor2& logits, const MoeGlu& m, const
                                         add_to || through != nullptr ? 1 : 0, add, stream);
     if (rc == -1 || rc == -2) return false;
     check(rc, "moe_grouped");
+    tuning().seen.grouped_experts += 1;
     return true;
 }
 

@@ -130,6 +130,7 @@ struct Tuning {
         int max_decode_splits = 0;                    // most workgroups a (token, head) pair's keys were split over
         long long merge_kernel_launches = 0, prefill_tile_launches = 0, tiled_f32_launches = 0, generic_attention_launches = 0;
         long long latent_tile_launches = 0, latent_token_launches = 0;      // latent attention: matrix-core kernel, one workgroup per token
+        long long through_products = 0, grouped_experts = 0;                // products that took their result into the stream; routed experts as grouped products
     } seen;
 };
 Tuning& tuning();

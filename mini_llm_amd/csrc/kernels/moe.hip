@@ -65,7 +65,8 @@ __device__ __forceinline__ float wave_expert_weight(float mine, int lane, int E,
 // router's product then has one more row). One workgroup per token. VEC: eight columns a thread at a time (16-byte
 // loads of bfloat16, two of float; ff, shared_ff and the strides are then multiples of 8 and the rows aligned), all of
 // one expert.
-template <typename TI, typename T, bool VEC>
+// AHEAD (few tokens): a thread's first columns are asked for before the weights are worked out, chosen expert or not.
+template <typename TI, typename T, bool VEC, bool AHEAD>
 __global__ void __launch_bounds__(256)
 moe_glu_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__ logits, int ldl, int E, int ff, int shared_ff, int top,
                    float scale, int router_kind, float limit, float shared_limit, float alpha, float up_shift, int weight_on_input,
@@ -75,6 +76,14 @@ moe_glu_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__
     const int t = blockIdx.x, tid = threadIdx.x, lane = tid % MLLM_WAVE;
     const int wave = __builtin_amdgcn_readfirstlane(tid / MLLM_WAVE);
     const float* lr = logits + static_cast<size_t>(t) * ldl;
+    float g_first[8], u_first[8];
+    if (VEC && AHEAD) {
+        const int c = min(tid * 8, E * ff + shared_ff - 8), e = c / ff, j = c - e * ff;
+        const TI* p = up + static_cast<size_t>(t) * ldu + (c < E * ff ? static_cast<size_t>(e) * 2 * ff + j : static_cast<size_t>(E) * ff * 2 + (c - E * ff));
+        load8(p, g_first);
+        load8(p + (c < E * ff ? ff : shared_ff), u_first);
+        __builtin_amdgcn_sched_barrier(0);
+    }
     const float sg = shared_gate ? 1.f / (1.f + expf(-lr[E])) : 1.f;
     float* wgt = weights[E <= MLLM_WAVE ? wave : 0];
     if (E <= MLLM_WAVE) {
@@ -129,8 +138,13 @@ moe_glu_act_kernel(const TI* __restrict__ up, int ldu, const float* __restrict__
                 w_out = sg;
             }
             if (live) {
-                load8(gp, g);
-                load8(upp, u);
+                if (AHEAD && c < 256 * 8) {
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) { g[k] = g_first[k]; u[k] = u_first[k]; }
+                } else {
+                    load8(gp, g);
+                    load8(upp, u);
+                }
 #pragma unroll
                 for (int k = 0; k < 8; ++k) {
                     const float gk = fminf(g[k] * w_in, lim), uk = fminf(fmaxf(u[k] * w_in, -lim), lim);
@@ -619,10 +633,14 @@ int mllm_moe_glu_act(const void* up, int ldu, const float* logits, int ldl, int 
     const int isz = up_dtype == MLLM_F32 ? 4 : 2;
     const bool vec = ff % 8 == 0 && shared_ff % 8 == 0 && ldo % 8 == 0 &&
                      ((reinterpret_cast<uintptr_t>(up) | reinterpret_cast<uintptr_t>(out)) & 15) == 0 && (static_cast<size_t>(ldu) * isz) % 16 == 0;
-#define MOE_GLU_V(TI, TYPE, VEC)                                                                                                               \
-    moe_glu_act_kernel<TI, TYPE, VEC><<<T, 256, 0, stream>>>(static_cast<const TI*>(up), ldu, logits, ldl, E, ff, shared_ff, top, scale, router_kind, \
+#define MOE_GLU_V(TI, TYPE, VEC, AHEAD)                                                                                                               \
+    moe_glu_act_kernel<TI, TYPE, VEC, AHEAD><<<T, 256, 0, stream>>>(static_cast<const TI*>(up), ldu, logits, ldl, E, ff, shared_ff, top, scale, router_kind, \
                                                              limit, shared_limit, alpha, up_shift, weight_on_input, shared_gate, static_cast<TYPE*>(out), ldo)
-#define MOE_GLU(TI, TYPE) do { if (vec) MOE_GLU_V(TI, TYPE, true); else MOE_GLU_V(TI, TYPE, false); } while (0)
+#define MOE_GLU(TI, TYPE)                                                                                                                     \
+    do {                                                                                                                                       \
+        if (vec && T <= 64) MOE_GLU_V(TI, TYPE, true, true); else if (vec) MOE_GLU_V(TI, TYPE, true, false);                                     \
+        else MOE_GLU_V(TI, TYPE, false, false);                                                                                                  \
+    } while (0)
     if (dtype == MLLM_F32) MOE_GLU(float, float);
     else if (up_dtype == MLLM_F32) MOE_GLU(float, bf16_t);
     else MOE_GLU(bf16_t, bf16_t);

@@ -55,6 +55,11 @@ class ScoreShapeC(ctypes.Structure):
                 ("slope", _vp), ("sink", _vp), ("keep_first", _i)]
 
 
+class TanhNormC(ctypes.Structure):
+    # (field for field the kernels' MllmTanhNorm, csrc/kernels/tanh_norm.h)
+    _fields_ = [("alpha", _vp), ("weight", _vp), ("bias", _vp)]
+
+
 _lib = None
 
 
@@ -77,6 +82,10 @@ def engine_library():
         "mllm_op_ln_linear": (_i, [T2p, _vp, _vp, _f, T2p, _vp, T2p, _i, _vp, _vp, _vp, _vp]),
         "mllm_op_paged_attention": (_i, [ctypes.POINTER(AttentionArgsC), ctypes.POINTER(AttentionSplitsC),
                                          ctypes.POINTER(_i), _vp]),
+        "mllm_op_tanh_norm": (_i, [T2p, ctypes.POINTER(TanhNormC), T2p, _vp, _vp]),
+        "mllm_op_stream_add": (_i, [T2p, T2p, T2p, _vp, T2p, ctypes.POINTER(TanhNormC), ctypes.POINTER(TanhNormC), _i, _vp]),
+        "mllm_op_linear_stream_add": (_i, [T2p, T2p, _vp, T2p, T2p, T2p, ctypes.POINTER(TanhNormC), ctypes.POINTER(TanhNormC), _vp]),
+        "mllm_op_token_side": (_i, [T2p, T2p, T2p, T2p, _vp, _f, _vp, _vp, _vp, _i, T2p, _i, T2p, ctypes.POINTER(TanhNormC), _vp]),
         "mllm_op_argmax": (_i, [T2p, _vp, _vp]),
         "mllm_op_sample": (_i, [T2p, _vp, _vp, _vp, _vp]),
     }
@@ -183,6 +192,16 @@ def set_scored_shared_kernels(on: bool) -> None:
     """Whether attention with shaped scores may run on the kernels that plain attention runs on (default: on);
     off: every row goes through the one-wavefront-per-row kernel that takes any sizes."""
     _ok(engine_library().mllm_set_tuning(b"scored_shared_kernels", 1 if on else 0, 0))
+
+
+def set_through_products(on: bool) -> None:
+    """Whether a product may take its result into the stream through norms by itself (otherwise it passes through memory)."""
+    _ok(engine_library().mllm_set_tuning(b"through_products", 1 if on else 0, 0))
+
+
+def set_grouped_experts_rows(rows: int) -> None:
+    """Tokens from which routed experts may run as grouped products (0: never)."""
+    _ok(engine_library().mllm_set_tuning(b"grouped_experts_rows", int(rows), 0))
 
 
 # Tuning hooks: tests and tuning scripts set these module attributes; they reach the native side at the
@@ -510,3 +529,71 @@ def sample(logits: torch.Tensor, temperature: torch.Tensor, u: torch.Tensor, out
     _i32(out, "out", n)
     _ok(engine_library().mllm_op_sample(ctypes.byref(t2(logits, "logits")), _p(temperature), _p(u), _p(out), _stream()))
     return out
+
+
+# -- the dynamic tanh norm, things added to the stream --------------------------------------------------
+def _norm(n):
+    """(alpha [1], weight [D], bias [D]) fp32 tensors, or None."""
+    if n is None:
+        return None
+    alpha, weight, bias = n
+    _gpu(alpha, weight, bias)
+    _f32vec(alpha, "alpha", 1)
+    _f32vec(weight, "weight", weight.numel())
+    _f32vec(bias, "bias", weight.numel())
+    return ctypes.byref(TanhNormC(alpha.data_ptr(), weight.data_ptr(), bias.data_ptr()))
+
+
+def _ref(t, name):
+    return None if t is None else ctypes.byref(t2(t, name))
+
+
+def _norm_fits(n, columns):
+    if n is not None and n[1].numel() != columns:
+        raise KernelError(f"a norm of {n[1].numel()} columns for rows of {columns}")
+
+
+def tanh_norm(x, norm, out, rows=None):
+    """out[i,:] = tanh(alpha x[rows[i] if rows else i,:]) * weight + bias"""
+    _gpu(x, out, rows)
+    _norm_fits(norm, x.shape[1])
+    if rows is not None:
+        _i32(rows, "rows", out.shape[0])
+    _ok(engine_library().mllm_op_tanh_norm(_ref(x, "x"), _norm(norm), _ref(out, "out"), _p(rows), _stream()))
+    return out
+
+
+def stream_add(x, y=None, norm=None, x0=None, step=None, copy=None, next=None, precise=False):
+    """x += norm(y) + x0 + step (each optional; without a norm y itself), then copy = next(x) (or x) in bfloat16."""
+    _gpu(x, y, x0, step, copy)
+    _norm_fits(norm, x.shape[1])
+    _norm_fits(next, x.shape[1])
+    _f32vec(step, "step", x.shape[1])
+    _ok(engine_library().mllm_op_stream_add(_ref(x, "x"), _ref(y, "y"), _ref(x0, "x0"), _p(step), _ref(copy, "copy"), _norm(norm), _norm(next),
+                                            1 if precise else 0, _stream()))
+    return x
+
+
+def linear_stream_add(a, w, x, bias=None, y=None, norm=None, copy=None, next=None):
+    """x += norm(a w^T + bias), then copy = next(x) in bfloat16; y: room for the product where it passes through memory."""
+    _gpu(a, w, x, bias, y, copy)
+    _norm_fits(norm, x.shape[1])
+    _norm_fits(next, x.shape[1])
+    _f32vec(bias, "bias", w.shape[0])
+    _ok(engine_library().mllm_op_linear_stream_add(_ref(a, "a"), _ref(w, "w"), _p(bias), _ref(x, "x"), _ref(y, "y"), _ref(copy, "copy"), _norm(norm),
+                                                   _norm(next), _stream()))
+    return x
+
+
+def token_side(x, xb, gate, proj, weight, eps, ids, table, col0, copy=None, next=None, src=None, prev=None):
+    """x += rmsnorm(proj (gelu_tanh(gate xb) * table[ids, col0:col0 + dim])) * weight, then copy = next(x) in bfloat16."""
+    _gpu(x, xb, gate, proj, weight, ids, table, copy, src, prev)
+    _norm_fits(next, x.shape[1])
+    _f32vec(weight, "weight", x.shape[1])
+    _i32(ids, "ids", x.shape[0])
+    if src is not None:
+        _i32(src, "src", x.shape[0])
+        _i32(prev, "prev")
+    _ok(engine_library().mllm_op_token_side(_ref(x, "x"), _ref(xb, "xb"), _ref(gate, "gate"), _ref(proj, "proj"), _p(weight), eps, _p(ids), _p(src), _p(prev),
+                                            0 if prev is None else prev.numel(), _ref(table, "table"), col0, _ref(copy, "copy"), _norm(next), _stream()))
+    return x

@@ -72,7 +72,7 @@ class FeedForward(_Part):
 
     def forward(self, h, x):
         """x += feed_forward(h)"""
-        a = _arena()
+        a = _arena(1 << 25)
         native.check(self._lib.mllm_feed_forward_forward(self.h, ctypes.byref(ops.t2(h)), ctypes.byref(ops.t2(x)),
                                                          a.data_ptr(), a.numel(), ops._stream()))
         return x

@@ -99,6 +99,35 @@ def test_the_matrix_core_kernels_serve_the_larger_sizes(dirs):
     gc.check_against_plain(d, reqs, steps, ru.run_in_process(runner, steps), "bfloat16", cfg["vocab"], "kernels used")
     assert ops.seen("latent_tile_launches") > 0 and ops.seen("latent_token_launches") == 0
     assert ops.seen("prefill_tile_launches") > 0 and ops.seen("generic_attention_launches") == 0
+    assert ops.seen("through_products") > 0
+
+
+@pytest.mark.parametrize("name", ["MIXED_A", "LARGER", "ODD"])
+def test_the_same_logits_with_and_without_fused_steps(dirs, name):
+    """Products that take their result through the norms into the stream, and experts as grouped products however few the
+    tokens, against the same model with every step a kernel of its own: the same rows up to rounding, in bfloat16."""
+    from mini_llm_amd.kernels import ops
+    cfg, d = getattr(gc, name), dirs(name)
+    reqs = gc.decisive_requests(d, cfg["vocab"], [5, 50, 18], seed=43)
+    steps = _families(reqs, seed=4)["mixed"] + [dict(s, step=1000 + s["step"]) for s in ru.trace_whole({"w" + r: t for r, t in reqs.items()})]
+    got = {}
+    try:
+        for fused in (True, False):
+            ops.set_through_products(fused)
+            ops.set_grouped_experts_rows(2 if fused else 0)
+            ops.reset_seen()
+            runner = _runner(d, "bfloat16", n_pages=ru.peak_tokens(steps) // 16, page=16)
+            got[fused] = ru.collect(steps, ru.run_in_process(runner, steps), cfg["vocab"])
+            if fused and name != "ODD":              # (ODD's sizes are no multiple of 8: nothing to group)
+                assert ops.seen("grouped_experts") > 0 and ops.seen("through_products") > 0
+            if not fused:
+                assert ops.seen("grouped_experts") == 0 and ops.seen("through_products") == 0
+    finally:
+        ops.set_through_products(True)
+        ops.set_grouped_experts_rows(192)
+    errs = sorted(gc.row_error(got[True][r][p], got[False][r][p].astype("float64")) for r in got[True] for p in got[True][r])
+    print(f"fused against unfused {name}: worst {errs[-1]:.3e}, median {errs[len(errs) // 2]:.3e} of {len(errs)}")
+    assert errs[-1] <= 3e-2 and errs[len(errs) // 2] <= 1e-2
 
 
 @pytest.mark.parametrize("page", [2, 4, 16])
