@@ -445,7 +445,12 @@ int mllm_qk_prepare(const float* proj, int ld, int q_col, int k_col, int v_col, 
     }
     if (conv != nullptr) return -1;                   // (only the kernel above convolves)
     const size_t smem = (static_cast<size_t>(H + G) * d + rot_dims + (H + G) + 2) * sizeof(float);
-    if (smem > 60 * 1024) return -1;
+    if (smem > 150 * 1024) return -1;
+    if (smem > 60 * 1024) {                           // (many wide heads: more than the usual 64 KB of LDS has to be asked for)
+        const void* kernel = dtype == MLLM_F32 ? reinterpret_cast<const void*>(qk_prepare_kernel<float>) : reinterpret_cast<const void*>(qk_prepare_kernel<bf16_t>);
+        const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);
+        if (e != hipSuccess) return static_cast<int>(e);
+    }
     if (dtype == MLLM_F32)
         qk_prepare_kernel<float><<<T, 256, smem, stream>>>(proj, ld, q_col, k_col, v_col, H, G, d, dv, norm_mode, wq, wk, eps, rot_dims,
                                                            rot_base, rot_freqs, interleaved, positions, slots, static_cast<float*>(q_out), ldq,

@@ -78,6 +78,7 @@ PAIR_KEEPS_MORE = model([pair(left(window=4, keep_first=9))], side=None)        
 PAIR_KEEPS_NONE = model([pair(left(window=12, keep_first=0))], side=None)
 PAIR_ONE_HEAD = model([pair(left(heads=1, kv_heads=1, dim=32, vdim=16), right(heads=1, dim=24, vdim=40))], width=48, side=None)
 PAIR_TWICE_AS_WIDE = model([pair(left(heads=4, kv_heads=2, dim=32, vdim=64), right(heads=3, dim=40, vdim=16))], side=None)
+PAIR_VERY_MANY_HEADS = model([pair(left(heads=64, kv_heads=64, dim=136, vdim=8), right(heads=1, dim=8, vdim=8))], width=32, side=None)   # 70 KB of heads a token
 PAIR_UNALIGNED = model([pair(left(heads=3, kv_heads=1, dim=10, vdim=7, rot=rotation(6, scaling=SCALING)), right(heads=3, dim=5, vdim=9))], width=40, side=None)
 PAIR_MANY_KEY_COLUMNS = model([pair(left(), right(heads=2, dim=72, vdim=80))], width=48, side=None)
 ONLY_EXPERTS = model([latent(mlp=moe())], side=None)
