@@ -194,9 +194,9 @@ def gisedra_config(n_layer, size="gpt2-small", n_positions=1024):
         else:
             layers.append({"type": "parallel", "mlp": mlp, "mixer": {
                 "left": {"heads": h, "kv_heads": kv, "dim": 64, "vdim": 64, "conv": 4, "scale": 0.125, "mask": {"size": 512, "keep_first": 16},
-                         "rot": {"base": 10000.0, "dims": 32, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 512}}},
+                         "rot": {"base": 10000.0, "dims": 32, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 1024}}},
                 "right": {"heads": rh, "dim": 64, "vdim": 64, "decay": [1.0 - 2.0 ** -(5 + 5 * k / rh) for k in range(rh)]},
-                "left_scale": 0.8, "right_scale": 0.9}})
+                "left_scale": 0.6, "right_scale": 1.2}})
     at = distinct // 2
     return {"architecture": "Gisedra", "vocab": 50257, "width": d, "norm": {"eps": 1e-6}, "token_side": {"dim": 64},
             "loop": {"start": at - 1, "stop": at + 1, "times": 2}, "layers": layers,
